@@ -158,6 +158,22 @@ int    raven_linear(const void* x0, const void* x1, const void* w, const void* r
                     int32_t M, int32_t N, int32_t K0, int32_t K1, int32_t swiglu, int32_t out_f32,
                     int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
 
+/* The products of models whose residual stream is kept in fp32: z = concat(x0, x1) W^T as in raven_linear (same kernels, same
+ * choice between them), then
+ *     y = act(scale * z + bias) + residual
+ * on the unrounded fp32 sums; y is float when out_f32 != 0, else T (one rounding).  bias [N] and residual [M, N] are float
+ * and may be NULL; residual may be y itself (out_f32).  act: RAVEN_ACT_*. */
+enum { RAVEN_ACT_NONE = 0, RAVEN_ACT_GELU = 1 /* exact: z (1 + erf(z / sqrt 2)) / 2 */, RAVEN_ACT_TANH = 2 };
+typedef struct raven_epilogue {
+    const float* bias;
+    const float* residual;
+    float        scale;
+    int32_t      act;
+    int32_t      out_f32;
+} raven_epilogue;
+int raven_linear_epilogue(const void* x0, const void* x1, const void* w, void* y, int32_t M, int32_t N, int32_t K0, int32_t K1,
+                          const raven_epilogue* epi, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
+
 /* Line-aligned copies of bf16 weight matrices for products over 33 and more token rows.  No counterpart in the reference
  * (its nn.Linear weights are [out, in] with rows K elements apart, RMM:463, 493, 507-509, and stay the layout every entry point
  * takes).  Where K * 2 bytes is not a multiple of 128 (K = 5280: every second row starts 64 bytes into a cache line) the
@@ -374,6 +390,90 @@ int raven_core_iterations(const raven_dims* dims, const void* adapter_w, const r
                           void* state_out, const float* freqs, const raven_kv_cache* cache, const int32_t* slots,
                           int32_t n_iterations, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev,
                           void* workspace, size_t workspace_bytes, void* stream);
+
+/* ---- Layer kinds of decoders with an fp32 residual stream (the Gitipel design; no counterpart in the reference) -----------
+ * Rows of width channels are stored `ld` elements apart, ld = width rounded up to a multiple of 8 with zeros behind the true
+ * width; heads likewise have head_dim elements, head_dim = dim rounded up to a multiple of 8 (the caller pads the weights).
+ *
+ * raven_norm_conv: h = RMSNorm(x) over rows x [B*S, ld] float, mean over `dim` channels; y = T(h) when conv is NULL, else
+ *   y_t = T(h_t + sum_j conv[j] * h_(t - taps + 1 + j)), conv [taps, ld] float, zeros before a sequence's start.  ring
+ *   [B, taps, ld] float carries the rows h between calls (position p in row p mod taps; never needs clearing).
+ * raven_embed_stream: x[m] = table[ids[m]] * scale as float, and the same rows rounded to T (x_rounded, may be NULL).
+ * raven_round_rows: n floats to T. */
+int raven_norm_conv(const float* x, const float* weight, const float* conv, float* ring, void* y, int32_t B, int32_t S, int32_t dim,
+                    int32_t ld, int32_t taps, float eps, int32_t pos0, const int32_t* pos_dev, int32_t dtype, void* stream);
+int raven_embed_stream(const void* table, const int64_t* ids, float* x, void* x_rounded, int32_t M, int32_t ld, int64_t vocab, float scale,
+                       int32_t dtype, void* stream);
+int raven_round_rows(const float* x, void* y, int64_t n, int32_t dtype, void* stream);
+
+/* Attention whose keys are its values, over a cache of keys alone ([batch, n_kv_heads, t_max, head_dim] of T; query head h reads
+ * key head h / (n_heads / n_kv_heads)).  Score of query position i and key position j <= i:
+ *     s = softcap * tanh(scale * q.k / softcap) - r1[h] * ln(1 + r2[h] * (i - j))      (softcap <= 0: no cap; r1, r2 NULL: no bias)
+ * qk [B*S, (n_heads + n_kv_heads) * head_dim] holds q | k of the new rows; their keys are appended at positions pos0 (or
+ * *pos_dev) .. + S - 1, y [B*S, n_heads * head_dim].  Scores and weights are fp32.  workspace as for raven_decode_attention. */
+typedef struct raven_key_cache {
+    void*   k;
+    int32_t batch, n_kv_heads, head_dim, t_max;
+} raven_key_cache;
+typedef struct raven_score {
+    float        scale, softcap;
+    const float* r1;
+    const float* r2;
+} raven_score;
+size_t raven_capped_attention_workspace_bytes(int32_t M, int32_t n_heads, int32_t n_kv_heads, int32_t head_dim);
+int    raven_capped_attention(const void* qk, void* y, const raven_key_cache* cache, const raven_score* score, int32_t B, int32_t S,
+                              int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dtype, void* workspace,
+                              size_t workspace_bytes, void* stream);
+
+/* The generalised delta rule with its output stage: per head, u = k / sqrt(|k|^2 + 1e-6), w = exp(-exp(-1/2) sigmoid(decay_logits)),
+ * a = sigmoid(z_a + a_bias),
+ *     S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T,   o_t = S_t^T r,   y = T(o / rms(o) * norm * sigmoid(g))
+ * z [B*S, ldz] float: r | k | v | g | a, sections of n_heads * head_dim; decay_logits [B*S, n_heads * head_dim] float; a_bias, norm
+ * [n_heads * head_dim] float; state [batch, n_heads, head_dim, head_dim] float (value channel, key channel), taken as zero when
+ * the call starts at position 0; y [B*S, n_heads * head_dim] of T.  The mean of rms runs over `dim` channels.  workspace
+ * (nullable, raven_delta_rule_workspace_bytes): long chunks run chunk-parallel with it, token by token without. */
+size_t raven_delta_rule_workspace_bytes(int32_t B, int32_t S, int32_t n_heads, int32_t head_dim);
+int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const float* a_bias, const float* norm, float* state, void* y,
+                     int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim, int32_t head_dim, float eps,
+                     int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
+
+/* One pre-norm layer on the stream x [B*S, ld] (in place):
+ *     h = norm1(x) [+ causal convolution];  x += mixer(h);  x += down(gelu(up(norm2(x))))      (up NULL: no feed-forward)
+ * mixer RAVEN_MIXER_ATTENTION: w_in = q | k rows [(heads + kv_heads) * head_dim, ld].  RAVEN_MIXER_GENERAL_DELTA: w_in = r | k | v | g | a
+ * [5 * heads * head_dim, ld], w_low = [rank, ld] (rank a multiple of 8), w_decay = [heads * head_dim, rank]: decay logits =
+ * w_decay tanh(w_low h) + decay_bias.  w_out [ld, heads * head_dim], up [ff, ld], down [ld, ff].  Weights of T, vectors float. */
+enum { RAVEN_MIXER_ATTENTION = 0, RAVEN_MIXER_GENERAL_DELTA = 1 };
+typedef struct raven_mixer_layer {
+    const float* norm1;
+    const float* conv;        /* [taps, ld] or NULL */
+    const void*  w_in;
+    const void*  w_low;
+    const void*  w_decay;
+    const float* decay_bias;  /* [heads * head_dim] */
+    const float* a_bias;      /* [heads * head_dim] */
+    const float* out_norm;    /* [heads * head_dim] */
+    const void*  w_out;
+    const float* norm2;
+    const void*  up;
+    const void*  down;
+    raven_score  score;
+    int32_t      mixer, heads, kv_heads, dim, head_dim, rank, taps, ff;
+} raven_mixer_layer;
+typedef struct raven_stream_dims {
+    int32_t width, ld;
+    float   eps;
+    int32_t dtype;
+} raven_stream_dims;
+/* What one run of a layer keeps of a batch of sequences: ring [B, taps, ld]; keys (attention) or state (delta rule). */
+typedef struct raven_mixer_state {
+    float*          ring;
+    float*          state;
+    raven_key_cache keys;
+} raven_mixer_state;
+size_t raven_mixer_layer_workspace_bytes(const raven_stream_dims* dims, const raven_mixer_layer* layer, int32_t B, int32_t S);
+int    raven_mixer_layer_forward(const raven_stream_dims* dims, const raven_mixer_layer* layer, const raven_mixer_state* state, float* x,
+                                 int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, void* workspace, size_t workspace_bytes,
+                                 void* stream);
 
 #ifdef __cplusplus
 }

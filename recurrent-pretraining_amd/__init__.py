@@ -20,8 +20,9 @@ from .adaptive import (  # noqa: F401
     PerIterationExitEvaluator,
     get_adaptive_exit_evaluator,
 )
-from .cache import HuginnDynamicCache, HuginnStaticCache, remap_step  # noqa: F401
-from .config import RavenConfig  # noqa: F401
+from .cache import HuginnDynamicCache, HuginnStaticCache, MixerStateCache, RequestCaches, remap_step  # noqa: F401
+from .config import GitipelConfig, RavenConfig  # noqa: F401
+from .gitipel import GitipelForCausalLM, MixerDecodeRunner  # noqa: F401
 from .modeling import (  # noqa: F401
     CausalLMOutputRecurrentLatents,
     DecodeRunner,
@@ -30,11 +31,13 @@ from .modeling import (  # noqa: F401
     precompute_freqs_cis,
 )
 from .paged import PagedDecoder  # noqa: F401
+from .registry import family_of, load_model  # noqa: F401
 
 __all__ = [
     "hip", "HuginnDynamicCache", "HuginnStaticCache", "remap_step", "RavenConfig", "RavenForCausalLM", "DecodeRunner",
     "CausalLMOutputRecurrentLatents", "GenerationSettings", "precompute_freqs_cis", "adaptive", "vllm_binding",
     "PerIterationExitEvaluator", "NoOpExitEvaluator", "EntropyDiffExitEvaluator", "LatentDiffExitEvaluator",
     "KLExitEvaluator", "MinKLExitEvaluator", "ArgmaxStabilityExitEvaluator", "CosineExitEvaluator", "NumStepsGenerator",
-    "get_adaptive_exit_evaluator", "PagedDecoder",
+    "get_adaptive_exit_evaluator", "PagedDecoder", "GitipelConfig", "GitipelForCausalLM", "MixerDecodeRunner", "MixerStateCache",
+    "RequestCaches", "family_of", "load_model",
 ]

@@ -11,7 +11,8 @@ ROOT = os.path.dirname(PKG_DIR)
 CSRC = os.path.join(PKG_DIR, "csrc")
 LIB_DIR = os.path.join(PKG_DIR, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libraven_hip.so")
-SOURCES = ["rmsnorm.hip", "gemm_skinny.hip", "gemm_splitk.hip", "gemm_tiled.hip", "gemv_decode.hip", "attention.hip", "attention_prefill.hip", "misc.hip", "exit_stats.hip", "compose.hip"]
+SOURCES = ["rmsnorm.hip", "gemm_skinny.hip", "gemm_splitk.hip", "gemm_tiled.hip", "gemv_decode.hip", "attention.hip", "attention_prefill.hip", "misc.hip", "exit_stats.hip", "compose.hip",
+           "tuning.hip", "norm_conv.hip", "attention_capped.hip", "delta_rule.hip", "compose_mixer.hip"]
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC",
@@ -27,11 +28,12 @@ def hipcc() -> str:
     return exe
 
 
-def build_library(verbose: bool = True) -> str:
+def build_library(verbose: bool = True, sources=None, path: str = LIB_PATH) -> str:
+    """Compiles `sources` (all by default) in parallel and links them into `path`."""
     os.makedirs(LIB_DIR, exist_ok=True)
     objs = []
     procs = []
-    for src in SOURCES:
+    for src in (SOURCES if sources is None else sources):
         obj = os.path.join(LIB_DIR, src.replace(".hip", ".o"))
         cmd = [hipcc(), *HIPCC_FLAGS, "-I", os.path.join(ROOT, "include"), "-I", CSRC, "-c", os.path.join(CSRC, src), "-o", obj]
         procs.append((src, subprocess.Popen(cmd, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)))
@@ -43,11 +45,24 @@ def build_library(verbose: bool = True) -> str:
             raise RuntimeError(f"hipcc failed on {src}:\n{out}")
         if verbose and out.strip():
             print(out, file=sys.stderr)
-    link = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-o", LIB_PATH, *objs]
+    part = f"{path}.{os.getpid()}.tmp"  # a process that loads the library meanwhile sees the old one or the new one
+    link = [hipcc(), "--offload-arch=gfx950", "-shared", "-fPIC", "-Wl,-z,defs", "-o", part, *objs]
     r = subprocess.run(link, stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)
     if r.returncode != 0:
         raise RuntimeError(f"link failed:\n{r.stdout}")
-    return LIB_PATH
+    os.replace(part, path)
+    return path
+
+
+def ensure_library(name: str, sources=None) -> str:
+    """Path of a built library that serves the model family `name`: the whole one when it has been built, else one of only the
+    family's kernel sources, compiled now if need be."""
+    if os.path.exists(LIB_PATH):
+        return LIB_PATH
+    if sources is None:
+        return build_library(verbose=False)
+    path = os.path.join(LIB_DIR, f"libraven_hip_{name}.so")
+    return path if os.path.exists(path) else build_library(verbose=False, sources=sources, path=path)
 
 
 if __name__ == "__main__":

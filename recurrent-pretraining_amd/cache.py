@@ -458,3 +458,103 @@ class HuginnStaticCache(HuginnDynamicCache):
     def get_memory_usage(self) -> float:
         """Allocated MiB, as the reference's static cache reports (RMM:432-433)."""
         return self.get_allocated_mb()
+
+
+class MixerStateCache:
+    """What a decoder with a list of mixers keeps of a batch of sequences that share their length: per layer RUN (a looped layer
+    has a state per pass) the last rows of the input convolution, and either the keys of every position or the recurrent state
+    matrices.  `plan` describes the runs: dicts with taps, ld, heads, head_dim and, for attention, kv_heads.
+
+    Only the token count says what is in it: rows and states before position 0 are taken as zero by the kernels and keys past
+    the length are never read, so a cache is given back and used again by resetting the count.  A recurrent state cannot be
+    rolled back, so positions are only ever added."""
+
+    is_compileable = False
+
+    def __init__(self, plan: list, max_length: Optional[int] = None):
+        self.plan = plan
+        self.max_length = max_length
+        self._seen_tokens = 0
+        self.batch = 0
+        self.t_max = 0
+        self.dtype: Optional[torch.dtype] = None
+        self.rings: list = []
+        self.keys: list = []      # per run [batch, kv_heads, t_max, head_dim], or None
+        self.states: list = []    # per run [batch, heads, head_dim, head_dim] float, or None
+        self._structs: list = []
+        self.generation = 0       # grows with every reallocation: captured launches hold pointers
+
+    def ensure(self, batch: int, t_needed: int, dtype: torch.dtype, device) -> None:
+        """Room for t_needed positions of `batch` sequences; contents survive growth."""
+        if self.max_length is not None and t_needed > self.max_length:
+            raise ValueError(f"sequence of {t_needed} positions exceeds the cache's max_length {self.max_length}")
+        if self.batch and (batch != self.batch or dtype != self.dtype):
+            if self._seen_tokens:
+                raise ValueError(f"cache holds {self.batch} sequences in {self.dtype}; asked for {batch} in {dtype}")
+            self.batch = 0
+        if self.batch and t_needed <= self.t_max:
+            return
+        if self.max_length is not None:
+            new_t = self.max_length
+        else:
+            new_t = max(256, self.t_max)
+            while new_t < t_needed:
+                new_t *= 2
+        new_t = (new_t + 15) // 16 * 16  # whole cache lines per head, whatever the head size (a multiple of 8 elements)
+        old = self.keys if self.batch else None
+        keys = [torch.zeros(batch, p["kv_heads"], new_t, p["head_dim"], dtype=dtype, device=device) if p.get("kv_heads") else None
+                for p in self.plan]
+        if old is not None:
+            for k, o in zip(keys, old):
+                if k is not None:
+                    k[:, :, :o.shape[2]] = o
+        else:
+            self.rings = [torch.zeros(batch, p["taps"], p["ld"], dtype=torch.float32, device=device) for p in self.plan]
+            self.states = [None if p.get("kv_heads") else
+                           torch.zeros(batch, p["heads"], p["head_dim"], p["head_dim"], dtype=torch.float32, device=device) for p in self.plan]
+        self.keys, self.batch, self.t_max, self.dtype = keys, batch, new_t, dtype
+        self._structs = [hip.MixerState(r.data_ptr(), None if s is None else s.data_ptr(),
+                                        hip.KeyCache() if k is None else hip.KeyCache(k.data_ptr(), *[k.shape[i] for i in (0, 1, 3, 2)]))
+                         for r, s, k in zip(self.rings, self.states, self.keys)]
+        self.generation += 1
+
+    def native(self, run: int) -> "hip.MixerState":
+        return self._structs[run]
+
+    def advance(self, n: int) -> None:
+        self._seen_tokens += n
+
+    def reset(self) -> None:
+        self._seen_tokens = 0
+
+    def get_seq_length(self, layer_idx: int = 0) -> int:
+        return self._seen_tokens
+
+    def get_memory_usage(self) -> float:
+        """MiB allocated."""
+        return sum(t.nelement() * t.element_size() for group in (self.rings, self.keys, self.states) for t in group if t is not None) / 2 ** 20
+
+
+class RequestCaches:
+    """Caches by request id.  A finished request's cache is reset and kept for the next one (its storage, and with it every
+    captured launch over it, stays valid)."""
+
+    def __init__(self, make):
+        self._make = make
+        self._live: dict = {}
+        self._free: list = []
+
+    def get(self, request):
+        """The cache of a request; a request that has none yet takes a free one or a new one."""
+        if request not in self._live:
+            self._live[request] = self._free.pop() if self._free else self._make()
+        return self._live[request]
+
+    def release(self, request) -> None:
+        cache = self._live.pop(request, None)
+        if cache is not None:
+            cache.reset()
+            self._free.append(cache)
+
+    def __len__(self) -> int:
+        return len(self._live)

@@ -73,3 +73,63 @@ class RavenConfig(PretrainedConfig):
         """The CPU-runnable plumbing shape."""
         return cls(n_embd=256, n_heads=4, n_layers=4, n_layers_in_prelude=1, n_layers_in_recurrent_block=2,
                    n_layers_in_coda=1, intermediate_size=704, vocab_size=1024, mean_recurrence=4)
+
+
+class GitipelConfig(PretrainedConfig):
+    """Shape of a Gitipel decoder, with the field names of its `config.json`: an embedding scale, a list of layers (each a mixer
+    with its sizes and a feed-forward or none), an optional stretch of layers that runs several times with a state per
+    pass, and the constants of norm, input convolution and output.  Every size comes from here, except the rank of the delta
+    rule's decay projection, which the weights give (`mixer["rank"]`)."""
+
+    model_type = "gitipel"
+    attribute_map = {"vocab_size": "vocab", "hidden_size": "width", "n_embd": "width"}
+
+    architecture: str = "Gitipel"
+    vocab: int = 256
+    width: int = 64
+    layers: list | None = None
+    embedding: dict | None = None
+    norm: dict | None = None
+    canon: dict | None = None
+    loop: dict | None = None
+    logit_scale: float = 1.0
+
+    def __post_init__(self, **kwargs):
+        for alias, field in self.attribute_map.items():
+            if kwargs.get(alias) is not None:
+                setattr(self, field, kwargs[alias])
+            kwargs.pop(alias, None)
+        kwargs.pop("model_type", None)
+        kwargs.pop("num_hidden_layers", None)
+        self.layers = [dict(x) for x in (self.layers or [])]
+        self.embedding = self.embedding or {"scale": 1.0}
+        self.norm = self.norm or {"eps": 1e-5}
+        self.canon = self.canon or {"taps": 1}
+        if self.architecture != "Gitipel":
+            raise ValueError(f"not a Gitipel configuration: architecture {self.architecture!r}")
+        for i, layer in enumerate(self.layers):
+            m = layer["mixer"]
+            if layer["type"] == "attention":
+                if m["heads"] % m["kv_heads"]:
+                    raise ValueError(f"layer {i}: {m['heads']} query heads over {m['kv_heads']} key heads")
+                if m.get("vdim", m["dim"]) != m["dim"]:
+                    raise ValueError(f"layer {i}: the keys are the values, so vdim {m['vdim']} must be dim {m['dim']}")
+            elif layer["type"] != "general_delta":
+                raise ValueError(f"layer {i}: unknown mixer {layer['type']!r}")
+            if layer.get("mlp") is not None and layer["mlp"]["kind"] != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward {layer['mlp']['kind']!r}")
+        if self.loop is not None and not 0 <= self.loop["start"] < self.loop["stop"] <= len(self.layers):
+            raise ValueError(f"loop {self.loop} over {len(self.layers)} layers")
+        self.num_hidden_layers = len(self.layers)
+        kwargs["tie_word_embeddings"] = False
+        if self.dtype is None and kwargs.get("torch_dtype") is None:
+            self.dtype = "bfloat16"
+        super().__post_init__(**kwargs)
+
+    def runs(self) -> list:
+        """(layer, pass) in the order they run; pass is None outside the loop."""
+        n, loop = len(self.layers), self.loop
+        if loop is None:
+            return [(i, None) for i in range(n)]
+        inside = [(i, t) for t in range(loop["times"]) for i in range(loop["start"], loop["stop"])]
+        return [(i, None) for i in range(loop["start"])] + inside + [(i, None) for i in range(loop["stop"], n)]

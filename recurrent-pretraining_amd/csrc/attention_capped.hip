@@ -1,0 +1,301 @@
+// Attention with capped scores, a per-head distance bias, grouped query heads and keys that serve as values:
+//     s_ij = cap * tanh(scale * q_i . k_j / cap) - r1_h * ln(1 + r2_h * (i - j)),   j <= i        (cap <= 0: no cap; r1 null: no bias)
+//     y_i  = sum_j softmax_j(s_ij) k_j
+// The rows q | k come out of one fused product ([M, (n_heads + n_kv_heads) * head_dim], heads of head_dim elements, zero
+// past the head's true size); the cache holds keys only, [batch, n_kv_heads, t_max, head_dim] of T.
+//
+// Two kernels:
+//   capped_attention_kernel          any T, any number of rows: a workgroup takes one row, one key head and up to four of the
+//       query heads that read it, and a range of positions.  LPP lanes share a position (16 bytes each), so one 16-byte load
+//       per lane serves the score AND the weighted sum of all those query heads -- a cached position is read once per key
+//       head.  Ranges are merged by a second launch in range order.  A decode step reads its own position's key from
+//       the fused row and appends it to the cache on the way.
+//   capped_attention_prefill_kernel  bf16 chunks on the matrix cores (further down).
+
+#include <math.h>
+
+#include "raven_common.h"
+
+namespace raven {
+
+struct CappedArgs {
+    const void* qk;   // [M, ldq]
+    void* y;          // [M, ldy]
+    void* kc;         // [batch, G, t_max, hd]
+    int ldq, ldy;
+    int H, G, hd, t_max, S, pos0;
+    const int* pos_dev;
+    float scale, cap;
+    const float* r1;
+    const float* r2;
+    int append;       // S == 1: the row's own key comes from qk and goes to the cache
+    int splits;
+    float* part;      // [M, H, splits, hd + 2] when splits > 1
+};
+
+// The score behind the product, in natural-log units.  float: the library functions; bf16: hardware exp2 / log2 / reciprocal
+// (1 ulp each; the absolute error of the tanh form, 1.2e-7 of the cap, is far below what a bf16 q or k leaves in the product).
+template <typename T>
+__device__ __forceinline__ float capped_score(float dot, float scale, float cap, float inv_cap, float r1, float r2, float dist) {
+    float s = dot * scale;
+    if constexpr (sizeof(T) == 4) {
+        if (cap > 0.f) s = cap * tanhf(s / cap);
+        if (r1 != 0.f) s -= r1 * log1pf(r2 * dist);
+    } else {
+        if (cap > 0.f) s = cap * (1.0f - 2.0f * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(s * inv_cap * 2.8853900817779268f)));
+        if (r1 != 0.f) s -= r1 * 0.69314718055994531f * __builtin_amdgcn_logf(1.0f + r2 * dist);
+    }
+    return s;
+}
+template <typename T>
+__device__ __forceinline__ float exp_weight(float x) {
+    if constexpr (sizeof(T) == 4) return expf(x);
+    else return __builtin_amdgcn_exp2f(x * 1.4426950408889634f);
+}
+
+template <int LPP>
+__device__ __forceinline__ float lanes_sum(float v) {  // over groups of LPP neighbouring lanes
+    v += dpp_f<0xB1>(v);
+    v += dpp_f<0x4E>(v);
+    if (LPP >= 8) v += dpp_f<0x141>(v);
+    if (LPP >= 16) v += dpp_f<0x140>(v);
+    if (LPP >= 32) v += __shfl_xor(v, 16, 64);
+    if (LPP >= 64) v += __shfl_xor(v, 32, 64);
+    return v;
+}
+
+template <typename T, int LPP, int NQ>
+__global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
+    constexpr int E = Chunk<T>::N;
+    constexpr int U = 4;                 // positions in flight per lane group
+    constexpr int GPW = 64 / LPP, NG = 4 * GPW;
+    __shared__ float sm[NG][NQ], sl[NG][NQ];
+    __shared__ __align__(16) float so[NG][NQ][LPP * E];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int grp = wave * GPW + lane / LPP, c = lane % LPP;
+    const int group = a.H / a.G;
+    const int sub = (group + NQ - 1) / NQ;           // workgroups per key head
+    const int g = blockIdx.y / sub, q0 = (blockIdx.y % sub) * NQ;
+    const int m = blockIdx.z, b = m / a.S, s = m % a.S;
+    const int pos = (a.pos_dev ? *a.pos_dev : a.pos0) + s;
+    const int n_cached = a.append ? pos : pos + 1;
+    const int span = (n_cached + a.splits - 1) / a.splits;
+    const int lo = (int)blockIdx.x * span, hi = min(n_cached, lo + span);
+    const bool active = c * E < a.hd;
+    const int cc = active ? c : 0;
+
+    const T* row = static_cast<const T*>(a.qk) + (int64_t)m * a.ldq;
+    T* keys = static_cast<T*>(a.kc) + ((int64_t)b * a.G + g) * a.t_max * a.hd;
+    Chunk<T> q[NQ];
+    float r1[NQ], r2[NQ], mx[NQ], l[NQ], acc[NQ][E];
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+        const int h = g * group + min(q0 + i, group - 1);
+        q[i] = active ? load_chunk(row + h * a.hd + c * E) : zero_chunk<T>();
+        r1[i] = a.r1 ? a.r1[h] : 0.f;
+        r2[i] = a.r1 ? a.r2[h] : 0.f;
+        mx[i] = -INFINITY;
+        l[i] = 0.f;
+#pragma unroll
+        for (int e = 0; e < E; ++e) acc[i][e] = 0.f;
+    }
+    const float inv_cap = a.cap > 0.f ? 1.0f / a.cap : 0.f;
+
+    // U positions: their scores, one rescaling, their weighted sum
+    auto take = [&](const Chunk<T>* k, const int* p, const bool* ok) {
+#pragma unroll
+        for (int i = 0; i < NQ; ++i) {
+            float sc[U], top = mx[i];
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const float d = lanes_sum<LPP>(dot_chunk(q[i], k[u], 0.f));
+                sc[u] = ok[u] ? capped_score<T>(d, a.scale, a.cap, inv_cap, r1[i], r2[i], (float)(pos - p[u])) : -INFINITY;
+                top = fmaxf(top, sc[u]);
+            }
+            const float ref = top == -INFINITY ? 0.f : top;
+            const float corr = exp_weight<T>(mx[i] - ref);
+            mx[i] = top;
+            l[i] *= corr;
+#pragma unroll
+            for (int e = 0; e < E; ++e) acc[i][e] *= corr;
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const float w = exp_weight<T>(sc[u] - ref);
+                l[i] += w;
+#pragma unroll
+                for (int e = 0; e < E; ++e) acc[i][e] = __builtin_fmaf(w, to_f32(k[u].v[e]), acc[i][e]);
+            }
+        }
+    };
+    for (int p0 = lo; p0 < hi; p0 += NG * U) {
+        Chunk<T> k[U];
+        int p[U];
+        bool ok[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            p[u] = p0 + u * NG + grp;
+            ok[u] = p[u] < hi;
+            k[u] = load_chunk(keys + (int64_t)min(p[u], hi - 1) * a.hd + cc * E);  // hi > lo >= 0 here
+        }
+        take(k, p, ok);
+    }
+    if (a.append && (int)blockIdx.x == a.splits - 1) {  // the row's own position, from the fused row
+        const Chunk<T> own = load_chunk(row + (int64_t)(a.H + g) * a.hd + cc * E);
+        Chunk<T> k[U];
+        int p[U];
+        bool ok[U];
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            k[u] = own;
+            p[u] = pos;
+            ok[u] = u == 0 && grp == 0;
+        }
+        take(k, p, ok);
+        if (q0 == 0 && grp == 0 && active && pos < a.t_max) store_chunk(keys + (int64_t)pos * a.hd + c * E, own);
+    }
+
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+        if (c == 0) {
+            sm[grp][i] = mx[i];
+            sl[grp][i] = l[i];
+        }
+#pragma unroll
+        for (int e = 0; e < E; e += 4) *reinterpret_cast<f32x4*>(&so[grp][i][c * E + e]) = f32x4{acc[i][e], acc[i][e + 1], acc[i][e + 2], acc[i][e + 3]};
+    }
+    __syncthreads();
+    for (int t = threadIdx.x; t < NQ * a.hd; t += 256) {
+        const int i = t / a.hd, col = t - i * a.hd;
+        if (q0 + i >= group) break;
+        float top = -INFINITY;
+        for (int n = 0; n < NG; ++n) top = fmaxf(top, sm[n][i]);
+        const float ref = top == -INFINITY ? 0.f : top;
+        float sum = 0.f, o = 0.f;
+        for (int n = 0; n < NG; ++n) {
+            const float w = exp_weight<T>(sm[n][i] - ref);
+            sum += w * sl[n][i];
+            o += w * so[n][i][col];
+        }
+        const int h = g * group + q0 + i;
+        if (a.splits == 1) {
+            static_cast<T*>(a.y)[(int64_t)m * a.ldy + h * a.hd + col] = from_f32<T>(o / sum);
+        } else {
+            float* p = a.part + (((int64_t)m * a.H + h) * a.splits + blockIdx.x) * (a.hd + 2);
+            p[2 + col] = o;
+            if (col == 0) {
+                p[0] = top;
+                p[1] = sum;
+            }
+        }
+    }
+}
+
+template <typename T>
+__global__ __launch_bounds__(64) void capped_combine_kernel(CappedArgs a) {
+    const int h = blockIdx.x, m = blockIdx.y;
+    const float* p = a.part + ((int64_t)m * a.H + h) * a.splits * (a.hd + 2);
+    float top = -INFINITY;
+    for (int n = 0; n < a.splits; ++n) top = fmaxf(top, p[(int64_t)n * (a.hd + 2)]);
+    for (int col = threadIdx.x; col < a.hd; col += 64) {
+        float sum = 0.f, o = 0.f;
+        for (int n = 0; n < a.splits; ++n) {
+            const float* q = p + (int64_t)n * (a.hd + 2);
+            const float w = exp_weight<T>(q[0] - top);  // some range always holds a position, so top is finite
+            sum += w * q[1];
+            o += w * q[2 + col];
+        }
+        static_cast<T*>(a.y)[(int64_t)m * a.ldy + h * a.hd + col] = from_f32<T>(o / sum);
+    }
+}
+
+// keys of the fused rows -> cache positions pos0 .. pos0 + S - 1
+template <typename T>
+__global__ __launch_bounds__(256) void key_append_kernel(CappedArgs a, int M) {
+    constexpr int E = Chunk<T>::N;
+    const int cpr = a.hd / E;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= (int64_t)M * a.G * cpr) return;
+    const int c = (int)(i % cpr), g = (int)(i / cpr % a.G), m = (int)(i / cpr / a.G);
+    const int b = m / a.S, pos = (a.pos_dev ? *a.pos_dev : a.pos0) + m % a.S;
+    if (pos >= a.t_max) return;
+    store_chunk(static_cast<T*>(a.kc) + (((int64_t)b * a.G + g) * a.t_max + pos) * a.hd + c * E,
+                load_chunk(static_cast<const T*>(a.qk) + (int64_t)m * a.ldq + (int64_t)(a.H + g) * a.hd + c * E));
+}
+
+static int capped_nq(int group) { return group >= 4 ? 4 : group >= 2 ? 2 : 1; }
+
+// position ranges per (row, key head): enough workgroups for the chip, at least 128 positions each
+static int capped_splits(int rows, int H, int G, int n_pos) {
+    const int group = H / G, nq = capped_nq(group);
+    const int64_t wgs = (int64_t)rows * G * ((group + nq - 1) / nq);
+    int64_t n = (512 + wgs - 1) / wgs;
+    if (n > (n_pos + 127) / 128) n = (n_pos + 127) / 128;
+    if (n > 32) n = 32;
+    return n < 1 ? 1 : (int)n;
+}
+
+template <typename T, int LPP>
+static int launch_capped(const CappedArgs& a, int M, hipStream_t s) {
+    const int group = a.H / a.G, nq = capped_nq(group);
+    const dim3 grid(a.splits, a.G * ((group + nq - 1) / nq), M);
+    if (nq == 4) capped_attention_kernel<T, LPP, 4><<<grid, dim3(256), 0, s>>>(a);
+    else if (nq == 2) capped_attention_kernel<T, LPP, 2><<<grid, dim3(256), 0, s>>>(a);
+    else capped_attention_kernel<T, LPP, 1><<<grid, dim3(256), 0, s>>>(a);
+    if (a.splits > 1) capped_combine_kernel<T><<<dim3(a.H, M), dim3(64), 0, s>>>(a);
+    return raven_host::check_launch("capped_attention");
+}
+
+template <typename T>
+static int run_capped(CappedArgs a, int M, hipStream_t s) {
+    constexpr int E = Chunk<T>::N;
+    if (!a.append) {
+        const int64_t n = (int64_t)M * a.G * (a.hd / E);
+        key_append_kernel<T><<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s>>>(a, M);
+        if (const int rc = raven_host::check_launch("capped_attention (append)")) return rc;
+    }
+    const int chunks = a.hd / E;
+    if (chunks <= 4) return launch_capped<T, 4>(a, M, s);
+    if (chunks <= 8) return launch_capped<T, 8>(a, M, s);
+    if (chunks <= 16) return launch_capped<T, 16>(a, M, s);
+    if (chunks <= 32) return launch_capped<T, 32>(a, M, s);
+    return launch_capped<T, 64>(a, M, s);
+}
+
+}  // namespace raven
+
+extern "C" size_t raven_capped_attention_workspace_bytes(int32_t M, int32_t n_heads, int32_t n_kv_heads, int32_t head_dim) {
+    if (M <= 0 || n_heads <= 0 || n_kv_heads <= 0 || head_dim <= 0) return 0;
+    const int splits = raven::capped_splits(M, n_heads, n_kv_heads, 1 << 30);
+    return splits > 1 ? raven_host::align_up((size_t)M * n_heads * splits * (head_dim + 2) * sizeof(float)) : 0;
+}
+
+extern "C" int raven_capped_attention(const void* qk, void* y, const raven_key_cache* cache, const raven_score* score, int32_t B, int32_t S,
+                                      int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dtype, void* workspace,
+                                      size_t workspace_bytes, void* stream) {
+    using namespace raven;
+    RAVEN_REQUIRE(dtype == RAVEN_F32 || dtype == RAVEN_BF16, "capped_attention: unknown dtype %d", dtype);
+    RAVEN_REQUIRE(cache && score && cache->k, "capped_attention: null pointer");
+    RAVEN_REQUIRE(B >= 0 && S >= 0 && pos0 >= 0 && n_heads > 0, "capped_attention: bad B=%d S=%d pos0=%d", B, S, pos0);
+    if (B == 0 || S == 0) return 0;
+    RAVEN_REQUIRE(qk && y, "capped_attention: null pointer");
+    RAVEN_REQUIRE(B <= cache->batch, "capped_attention: batch %d exceeds the cache's %d", B, cache->batch);
+    RAVEN_REQUIRE((int64_t)B * S <= 65535, "capped_attention: %d x %d rows in one call", B, S);
+    RAVEN_REQUIRE(cache->n_kv_heads > 0 && n_heads % cache->n_kv_heads == 0, "capped_attention: %d query heads for %d key heads", n_heads,
+                  cache->n_kv_heads);
+    RAVEN_REQUIRE(cache->head_dim > 0 && cache->head_dim % 8 == 0 && cache->head_dim <= 256, "capped_attention: head_dim %d is not a multiple of 8 up to 256",
+                  cache->head_dim);
+    RAVEN_REQUIRE(pos0 + S <= cache->t_max, "capped_attention: positions up to %d exceed the cache length %d", pos0 + S - 1, cache->t_max);
+    RAVEN_REQUIRE((score->r1 == nullptr) == (score->r2 == nullptr), "capped_attention: r1 and r2 must be given together");
+    CappedArgs a{};
+    a.qk = qk; a.y = y; a.kc = cache->k;
+    a.H = n_heads; a.G = cache->n_kv_heads; a.hd = cache->head_dim; a.t_max = cache->t_max; a.S = S; a.pos0 = pos0; a.pos_dev = pos_dev;
+    a.ldq = (a.H + a.G) * a.hd; a.ldy = a.H * a.hd;
+    a.scale = score->scale; a.cap = score->softcap; a.r1 = score->r1; a.r2 = score->r2;
+    a.append = S == 1;
+    const int M = B * S;
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    a.splits = capped_splits(M, a.H, a.G, pos0 + S);
+    while (a.splits > 1 && (workspace == nullptr || (size_t)M * a.H * a.splits * (a.hd + 2) * sizeof(float) > workspace_bytes)) --a.splits;
+    a.part = static_cast<float*>(workspace);
+    return dtype == RAVEN_BF16 ? run_capped<bf16>(a, M, s) : run_capped<float>(a, M, s);
+}

@@ -23,15 +23,13 @@ extern "C" int raven_gemv_fused(const void* x0, const void* x1, const void* norm
 
 namespace raven {
 
-int set_gemv1_tuning(const char* key, int value);
-extern int g_linear_ks;
-extern int g_tiled_min_rows, g_tiled_variant, g_tiled_split_tail;
+extern int g_tiled_min_rows;
 bool tiled_gemm_fits(int M, int N, int K0, int K1, int dtype);
 int tiled_gemm(const void* x0, const void* x1, const void* w, const void* residual, void* y, int M, int N, int K0, int K1, int swiglu,
                int out_f32, hipStream_t s);
-extern int g_attn_split_target, g_attn_big_grid, g_attn_wide, g_linear_min_rows, g_attn_nosplit_pairs, g_attn_nosplit_len, g_rope_tiled_rows, g_prefill_waves, g_norm_early, g_fuse_sums_norm, g_attn_prefetch, g_fuse_qkv_rope, g_pad_chunk_rows, g_pad_decode_rows;
 
-enum { EPI_PLAIN = 0, EPI_SWIGLU = 1 };
+int gemv1_free(const void* x0, const void* x1, const void* w, void* y, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
+               hipStream_t s);
 
 struct GemmArgs {
     const void* w;         // [N_total, K]
@@ -45,6 +43,7 @@ struct GemmArgs {
     int interleave;        // gemv: unit = u * total_waves + wave (1) or wave * units_per_wave + u (0)
     int row_stride;        // mfma: 1 = a tile is 16 neighbouring weight rows, 2 = every second row (see mfma_kernel)
     int line_aligned;      // mfma: the rows of a tile all start at the same offset inside a 128-byte line
+    raven_epilogue epi;    // EPI_FREE only (residual and y already offset to the pass)
     int rows_per_unit;     // mfma, ragged variants: weight rows (per side for SwiGLU) a workgroup owns; its last tile is partly empty
 };
 
@@ -60,6 +59,19 @@ struct Tuning {
 };
 static Tuning g_tuning;
 
+int set_skinny_tuning(const char* key, int value) {
+    const std::string k(key);
+    if (k == "gemv_units_per_wave") g_tuning.gemv_units_per_wave = value;
+    else if (k == "gemv_interleave") g_tuning.gemv_interleave = value;
+    else if (k == "gemv_nontemporal") g_tuning.gemv_nontemporal = value;
+    else if (k == "gemv_wgs_per_cu") g_tuning.gemv_wgs_per_cu = value;
+    else if (k == "gemm_four_tiles") g_tuning.gemm_four_tiles = value;
+    else if (k == "gemm_ragged") g_tuning.gemm_ragged = value;
+    else if (k == "gemm_mfma_min_rows" && value >= 2) g_tuning.gemm_mfma_min_rows = value;
+    else return -1;
+    return 0;
+}
+
 // weight rows are read exactly once: stream them past the caches
 template <bool NT, typename T>
 __device__ __forceinline__ Chunk<T> load_weight(const T* p) {
@@ -70,8 +82,12 @@ __device__ __forceinline__ Chunk<T> load_weight(const T* p) {
     return c;
 }
 
-template <typename T>
+template <typename T, int EPI = EPI_PLAIN>
 __device__ __forceinline__ void store_out(const GemmArgs& a, int m, int n, float acc) {
+    if (EPI == EPI_FREE) {
+        store_free<T>(a.epi, a.y, (int64_t)m * a.N + n, n, acc);
+        return;
+    }
     float r = round_to<T>(acc);
     if (a.residual) r = round_to<T>(r + to_f32(static_cast<const T*>(a.residual)[(int64_t)m * a.N + n]));
     if (a.out_f32)
@@ -171,8 +187,8 @@ __global__ __launch_bounds__(256) void gemv_kernel(GemmArgs a) {
                     if (EPI == EPI_SWIGLU) {
                         static_cast<T*>(a.y)[(int64_t)m * a.N + unit] = from_f32<T>(swiglu<T>(acc0[m], acc1[m]));
                     } else {
-                        store_out<T>(a, m, r0, acc0[m]);
-                        if (r1_ok) store_out<T>(a, m, r1, acc1[m]);
+                        store_out<T, EPI>(a, m, r0, acc0[m]);
+                        if (r1_ok) store_out<T, EPI>(a, m, r1, acc1[m]);
                     }
                 }
             }
@@ -402,7 +418,7 @@ __global__ __launch_bounds__(256) void mfma_kernel(GemmArgs a) {
                 if (!tile_ok[t]) continue;
 #pragma unroll
                 for (int v = 0; v < 4; ++v)
-                    if (!RAG || kq * 4 + v < tile_rows[t]) store_out<bf16>(a, m, tile_out0[t] + (kq * 4 + v) * rs, acc[t][mt][v]);
+                    if (!RAG || kq * 4 + v < tile_rows[t]) store_out<bf16, EPI>(a, m, tile_out0[t] + (kq * 4 + v) * rs, acc[t][mt][v]);
             }
         }
     }
@@ -536,6 +552,11 @@ static int run_gemm(GemmArgs a, int dtype, hipStream_t s) {
             const char* x1 = a.x1 ? static_cast<const char*>(a.x1) + (size_t)m0 * a.k1 * es : nullptr;
             const char* res = a.residual ? static_cast<const char*>(a.residual) + (size_t)m0 * a.N * es : nullptr;
             char* y = static_cast<char*>(a.y) + (size_t)m0 * a.N * out_es;
+            if (EPI == EPI_FREE) {
+                raven_epilogue e = a.epi;
+                if (e.residual) e.residual += (size_t)m0 * a.N;
+                return gemv1_free(x0, x1, a.w, y, a.N, a.k0, a.k1, e, dtype, s);
+            }
             return raven_gemv_fused(x0, x1, nullptr, nullptr, nullptr, a.w, res, y, a.N, a.k0, a.k1, 0.f, EPI == EPI_SWIGLU, a.out_f32,
                                     dtype, s);
         }
@@ -554,6 +575,7 @@ static int run_gemm(GemmArgs a, int dtype, hipStream_t s) {
         if (a.x1) p.x1 = static_cast<const char*>(a.x1) + (size_t)m0 * a.k1 * es;
         if (a.residual) p.residual = static_cast<const char*>(a.residual) + (size_t)m0 * a.N * es;
         p.y = static_cast<char*>(a.y) + (size_t)m0 * a.N * out_es;
+        if (a.epi.residual) p.epi.residual = a.epi.residual + (size_t)m0 * a.N;
         int rc;
         if (use_mfma) rc = dispatch_mfma<EPI>(p, s);
         else if (dtype == RAVEN_BF16) rc = dispatch_gemv<bf16, EPI>(p, s);
@@ -562,6 +584,15 @@ static int run_gemm(GemmArgs a, int dtype, hipStream_t s) {
         m0 += pass;
     }
     return 0;
+}
+
+// The skinny kernels with the free epilogue (raven_linear_epilogue, which has checked the arguments)
+int gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
+              hipStream_t s) {
+    GemmArgs a{};
+    a.w = w; a.x0 = x0; a.x1 = x1; a.y = y;
+    a.M = M; a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.out_f32 = epi.out_f32; a.epi = epi;
+    return run_gemm<EPI_FREE>(a, dtype, s);
 }
 
 static int check_common(const char* who, int M, int N, int K, int dtype) {
@@ -573,39 +604,6 @@ static int check_common(const char* who, int M, int N, int K, int dtype) {
 }
 
 }  // namespace raven
-
-extern "C" int raven_set_tuning(const char* key, int32_t value) {
-    using namespace raven;
-    RAVEN_REQUIRE(key != nullptr, "set_tuning: null key");
-    const std::string k(key);
-    if (k == "gemv_units_per_wave") g_tuning.gemv_units_per_wave = value;
-    else if (k == "gemv_interleave") g_tuning.gemv_interleave = value;
-    else if (k == "gemv_nontemporal") g_tuning.gemv_nontemporal = value;
-    else if (k == "gemv_wgs_per_cu") g_tuning.gemv_wgs_per_cu = value;
-    else if (k == "linear_ks") g_linear_ks = value;
-    else if (k == "gemm_four_tiles") g_tuning.gemm_four_tiles = value;
-    else if (k == "gemm_ragged") g_tuning.gemm_ragged = value;
-    else if (k == "gemm_mfma_min_rows" && value >= 2) g_tuning.gemm_mfma_min_rows = value;
-    else if (k == "attn_split_target" && value > 0) g_attn_split_target = value;
-    else if (k == "attn_big_grid" && value > 0) g_attn_big_grid = value;
-    else if (k == "attn_wide") g_attn_wide = value;
-    else if (k == "attn_prefetch" && value >= 0 && value <= 2) g_attn_prefetch = value;
-    else if (k == "prefill_waves" && (value == 0 || value == 4 || value == 6)) g_prefill_waves = value;
-    else if (k == "rope_tiled_rows" && value > 0) g_rope_tiled_rows = value;
-    else if (k == "fuse_qkv_rope" && (value == 0 || value == 1)) g_fuse_qkv_rope = value;
-    else if (k == "pad_chunk_rows" && (value == 0 || value == 1)) g_pad_chunk_rows = value;
-    else if (k == "pad_decode_rows" && (value == 0 || value == 1)) g_pad_decode_rows = value;
-    else if (k == "attn_nosplit_pairs" && value > 0 && value <= 1024) g_attn_nosplit_pairs = value;
-    else if (k == "attn_nosplit_len" && value >= 0) g_attn_nosplit_len = value;
-    else if (k == "linear_min_rows" && value >= 1) g_linear_min_rows = value;
-    else if (k == "norm_early" && value >= -1 && value <= 1) g_norm_early = value;
-    else if (k == "fuse_sums_norm" && (value == 0 || value == 1)) g_fuse_sums_norm = value;
-    else if (k == "gemm_tiled_min_rows" && value >= 33) g_tiled_min_rows = value;
-    else if (k == "gemm_tiled_variant" && value >= 0 && value <= 3) g_tiled_variant = value;
-    else if (k == "gemm_tiled_split_tail" && (value == 0 || value == 1)) g_tiled_split_tail = value;
-    else RAVEN_REQUIRE(set_gemv1_tuning(key, value) == 0, "set_tuning: unknown key %s", key);
-    return 0;
-}
 
 extern "C" int raven_gemm(const void* x, const void* w, const void* residual, void* y, int32_t M, int32_t N, int32_t K,
                           int32_t dtype, int32_t out_f32, void* stream) {

@@ -30,6 +30,10 @@ extern int g_tiled_min_rows;
 bool tiled_gemm_fits(int M, int N, int K0, int K1, int dtype);
 int tiled_gemm(const void* x0, const void* x1, const void* w, const void* residual, void* y, int M, int N, int K0, int K1, int swiglu,
                int out_f32, hipStream_t s);
+int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi,
+                    hipStream_t s);
+int gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
+              hipStream_t s);
 
 constexpr int kNsPitch = 136;  // bf16 elements per LDS row: 128 + 8 (272 bytes)
 typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
@@ -48,10 +52,16 @@ struct NsArgs {
     int ldw;               // elements between two weight rows: K, or more for a column block of a wider matrix
     const float* extra;    // [M, N] or null: fp32 sums of the remaining columns, added with the K-slice partials
     int raw_out;           // y receives the unrounded fp32 sums (what `extra` of a later call holds)
+    raven_epilogue epi;    // EPI_FREE only
 };
 
-template <bool SWIGLU>
+template <int EPI>
 __device__ __forceinline__ void ns_epilogue(const NsArgs& a, int m, int n, float v0, float v1) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
+    if (EPI == EPI_FREE) {
+        store_free<bf16>(a.epi, a.y, (int64_t)m * a.N + n, n, v0);
+        return;
+    }
     if (SWIGLU) {
         const float g = round_to<bf16>(v0), u = round_to<bf16>(v1);
         static_cast<bf16*>(a.y)[(int64_t)m * a.N + n] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
@@ -63,8 +73,9 @@ __device__ __forceinline__ void ns_epilogue(const NsArgs& a, int m, int n, float
     }
 }
 
-template <int MT, bool SWIGLU>
+template <int MT, int EPI>
 __global__ __launch_bounds__(256) void mfma_ns_kernel(NsArgs a) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int NT = SWIGLU ? 2 : 1;
     __shared__ __align__(16) bf16 xs[2][16 * MT][kNsPitch];
     __shared__ __align__(16) bf16 wsm[4][16 * NT][kNsPitch];
@@ -234,7 +245,7 @@ __global__ __launch_bounds__(256) void mfma_ns_kernel(NsArgs a) {
         for (int v = 0; v < 4; ++v) {
             const int n = out0 + (kq * 4 + v) * rs;
             if (a.ks == 1) {
-                ns_epilogue<SWIGLU>(a, m, n, acc[0][mt][v], acc[NT - 1][mt][v]);
+                ns_epilogue<EPI>(a, m, n, acc[0][mt][v], acc[NT - 1][mt][v]);
             } else {
                 float* p = a.partial + ((int64_t)blockIdx.y * a.M + m) * n_total;
                 p[n] = acc[0][mt][v];
@@ -245,8 +256,9 @@ __global__ __launch_bounds__(256) void mfma_ns_kernel(NsArgs a) {
 }
 
 // adds the K-slice partials in slice order and applies the epilogue; one thread per output element
-template <bool SWIGLU>
+template <int EPI>
 __global__ __launch_bounds__(256) void splitk_finalize_kernel(NsArgs a) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     const int64_t idx = (int64_t)blockIdx.x * 256 + threadIdx.x;
     if (idx >= (int64_t)a.M * a.N) return;
     const int m = (int)(idx / a.N), n = (int)(idx - (int64_t)m * a.N);
@@ -258,7 +270,7 @@ __global__ __launch_bounds__(256) void splitk_finalize_kernel(NsArgs a) {
         if (SWIGLU) v1 += p[a.N + n];
     }
     if (a.raw_out) static_cast<float*>(a.y)[idx] = v0;
-    else ns_epilogue<SWIGLU>(a, m, n, v0, v1);
+    else ns_epilogue<EPI>(a, m, n, v0, v1);
 }
 
 static int ns_cus() {
@@ -277,8 +289,9 @@ int g_linear_ks = 0;  // raven_set_tuning("linear_ks"): K slices per weight tile
 
 // ks_left (may be null): the caller adds the K slices itself (rmsnorm.hip, splitk_sums_then_norm); receives their number,
 // 0 when the product was finished here
-template <bool SWIGLU>
+template <int EPI>
 static int launch_ns(NsArgs a, void* workspace, size_t workspace_bytes, hipStream_t s, int* ks_left = nullptr) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     // tiles of one row parity when the row pitch is an odd multiple of 64 bytes (needs whole pairs of tiles)
     if (a.ldw == 0) a.ldw = a.K;
     a.row_stride = ((a.ldw * 2) % 128 == 64 && a.N % 32 == 0) ? 2 : 1;
@@ -306,12 +319,12 @@ static int launch_ns(NsArgs a, void* workspace, size_t workspace_bytes, hipStrea
     a.ks = ks;
     a.partial = ks > 1 ? static_cast<float*>(workspace) : nullptr;
     const dim3 grid(blocks, ks);
-    if (a.M <= 16) mfma_ns_kernel<1, SWIGLU><<<grid, dim3(256), 0, s>>>(a);
-    else mfma_ns_kernel<2, SWIGLU><<<grid, dim3(256), 0, s>>>(a);
+    if (a.M <= 16) mfma_ns_kernel<1, EPI><<<grid, dim3(256), 0, s>>>(a);
+    else mfma_ns_kernel<2, EPI><<<grid, dim3(256), 0, s>>>(a);
     if (ks_left) *ks_left = ks > 1 ? ks : 0;
     if (ks > 1 && !ks_left) {
         const int64_t n_out = (int64_t)a.M * a.N;
-        splitk_finalize_kernel<SWIGLU><<<dim3((unsigned)((n_out + 255) / 256)), dim3(256), 0, s>>>(a);
+        splitk_finalize_kernel<EPI><<<dim3((unsigned)((n_out + 255) / 256)), dim3(256), 0, s>>>(a);
     }
     return raven_host::check_launch("linear (split-K MFMA)");
 }
@@ -331,7 +344,7 @@ int linear_column_block(const void* x, const void* w_block, int ldw, const float
     a.x0 = static_cast<const bf16*>(x);
     a.y = y;
     a.M = M; a.N = N; a.K = K; a.k0 = K; a.k1 = 0; a.ldw = ldw; a.extra = extra; a.raw_out = raw_out;
-    return launch_ns<false>(a, workspace, workspace_bytes, s);
+    return launch_ns<EPI_PLAIN>(a, workspace, workspace_bytes, s);
 }
 
 int g_fuse_sums_norm = 1;  // raven_set_tuning("fuse_sums_norm"): 0 = a K-split product always adds its slices in a launch of its own
@@ -358,7 +371,7 @@ int linear_leave_sums(const void* x0, const void* x1, const void* w, int ldw, co
     a.residual = static_cast<const bf16*>(residual);
     a.y = y;
     a.M = M; a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.ldw = ldw; a.extra = extra;
-    return launch_ns<false>(a, workspace, workspace_bytes, s, ks_left);
+    return launch_ns<EPI_PLAIN>(a, workspace, workspace_bytes, s, ks_left);
 }
 
 }  // namespace raven
@@ -416,8 +429,42 @@ extern "C" int raven_linear(const void* x0, const void* x1, const void* w, const
         a.residual = residual ? static_cast<const bf16*>(residual) + (size_t)m0 * N : nullptr;
         a.y = static_cast<char*>(y) + (size_t)m0 * N * out_es;
         a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.out_f32 = out_f32;
-        const int rc = swiglu ? launch_ns<true>(a, workspace, workspace_bytes, s) : launch_ns<false>(a, workspace, workspace_bytes, s);
+        const int rc = swiglu ? launch_ns<EPI_SWIGLU>(a, workspace, workspace_bytes, s) : launch_ns<EPI_PLAIN>(a, workspace, workspace_bytes, s);
         if (rc) return rc;
+    }
+    return 0;
+}
+
+extern "C" int raven_linear_epilogue(const void* x0, const void* x1, const void* w, void* y, int32_t M, int32_t N, int32_t K0, int32_t K1,
+                                     const raven_epilogue* epi, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream) {
+    using namespace raven;
+    RAVEN_REQUIRE(dtype == RAVEN_F32 || dtype == RAVEN_BF16, "linear_epilogue: unknown dtype %d", dtype);
+    const int elts = 16 / (int)raven_host::elt_size(dtype);
+    RAVEN_REQUIRE(M >= 0 && N > 0 && K0 > 0 && K1 >= 0 && K0 % elts == 0 && K1 % elts == 0, "linear_epilogue: bad shape M=%d N=%d K0=%d K1=%d", M, N,
+                  K0, K1);
+    if (M == 0) return 0;
+    RAVEN_REQUIRE(x0 && w && y && epi, "linear_epilogue: null pointer");
+    RAVEN_REQUIRE((K1 == 0) == (x1 == nullptr), "linear_epilogue: x1 and K1 must be given together");
+    RAVEN_REQUIRE(epi->act >= RAVEN_ACT_NONE && epi->act <= RAVEN_ACT_TANH, "linear_epilogue: unknown activation %d", epi->act);
+    RAVEN_REQUIRE(((uintptr_t)epi->residual & 15) == 0 && ((uintptr_t)epi->bias & 15) == 0, "linear_epilogue: residual and bias must be 16-byte aligned");
+    hipStream_t s = static_cast<hipStream_t>(stream);
+    if (M >= g_tiled_min_rows && tiled_gemm_fits(M, N, K0, K1, dtype)) return tiled_gemm_free(x0, x1, w, y, M, N, K0, K1, *epi, s);
+    // the same choice between the kernels with and without a K split as raven_linear
+    const bool split = dtype == RAVEN_BF16 && M > g_linear_min_rows && N % 16 == 0 && K0 % 32 == 0 && K1 % 32 == 0 && workspace != nullptr &&
+                       ((uintptr_t)workspace & 255) == 0 && K0 / 128 + K1 / 128 >= 1 &&
+                       (g_linear_ks != 0 || (N / 16 < 2 * ns_cus() && (M > 16 || K0 + K1 >= 8192)));
+    if (!split) return gemm_free(x0, x1, w, y, M, N, K0, K1, *epi, dtype, s);
+    const size_t out_es = epi->out_f32 ? 4 : 2;
+    for (int m0 = 0; m0 < M; m0 += 32) {
+        NsArgs a{};
+        a.M = (M - m0) < 32 ? (M - m0) : 32;
+        a.w = static_cast<const bf16*>(w);
+        a.x0 = static_cast<const bf16*>(x0) + (size_t)m0 * K0;
+        a.x1 = x1 ? static_cast<const bf16*>(x1) + (size_t)m0 * K1 : nullptr;
+        a.y = static_cast<char*>(y) + (size_t)m0 * N * out_es;
+        a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.epi = *epi;
+        if (epi->residual) a.epi.residual = epi->residual + (size_t)m0 * N;
+        if (const int rc = launch_ns<EPI_FREE>(a, workspace, workspace_bytes, s)) return rc;
     }
     return 0;
 }

@@ -62,6 +62,7 @@ struct TiledArgs {
     int up_off;            // SwiGLU: weight rows between a gate row and its up row (the whole matrix's I)
     int out_f32;
     int tiles_m, tiles_n;
+    raven_epilogue epi;    // EPI_FREE only (y and residual [M, ldy])
     int rope_on;           // the epilogue below instead of y
     // The product is a chunk's fused q | k | v rows (3 * nh * hd columns): instead of y, the epilogue adds the q / k bias,
     // rotates q and k (RoPE on adjacent pairs) and writes q to q_out and k, v to their cache rows -- what
@@ -95,9 +96,10 @@ __device__ __forceinline__ void static_for(F&& f) {
 // Epilogue of both kernels.  Accumulator tile [ta][tb] (16 weight rows x 16 token rows) leaves a lane with token row
 // 16 tb + l16 and output columns 16 ta + 4 q4 + (0 .. 3); under SwiGLU tile 2 t holds gate columns and 2 t + 1 the
 // matching up columns.
-template <bool SWIGLU, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
 __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_m, int tile_n, int wm, int wn,
                                             int l16, int q4) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr int NA = 2 * TN, NB = 2 * TM, NT = SWIGLU ? TN : NA;
 #pragma unroll
@@ -116,6 +118,17 @@ __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&ac
                     o[i] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
                 }
                 *reinterpret_cast<u32x2*>(static_cast<bf16*>(a.y) + (int64_t)m * a.ldy + n) = *reinterpret_cast<const u32x2*>(o);
+            } else if (EPI == EPI_FREE) {  // float outputs; N is a multiple of 8, so the four columns exist together
+                const int64_t at = (int64_t)m * a.ldy + n;
+                f32x4 v = acc[t][tb] * a.epi.scale;
+                if (a.epi.bias) v += *reinterpret_cast<const f32x4*>(a.epi.bias + n);
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    if (a.epi.act == RAVEN_ACT_GELU) v[i] = 0.5f * v[i] * (1.0f + erff(v[i] * 0.70710678118654752f));
+                    else if (a.epi.act == RAVEN_ACT_TANH) v[i] = tanhf(v[i]);
+                }
+                if (a.epi.residual) v += *reinterpret_cast<const f32x4*>(a.epi.residual + at);
+                *reinterpret_cast<f32x4*>(static_cast<float*>(a.y) + at) = v;
             } else {
                 float r[4];
 #pragma unroll
@@ -141,8 +154,10 @@ __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&ac
 
 // The accumulators of a workgroup laid down in LDS as the output tile (rows of BN_OUT columns, 16-byte unit u of row r at
 // position u ^ (r mod units per row)), between two workgroup barriers: the first because the K loop's stages are reused.
-template <bool SWIGLU, int TM, int TN, int WM, int WN>
-__device__ __forceinline__ void lay_tiles_lds(const f32x4 (&acc)[2 * TN][2 * TM], int wave, int lane, unsigned lds_base) {
+template <int EPI, int TM, int TN, int WM, int WN>
+__device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_m, int tile_n, int wave, int lane,
+                                              unsigned lds_base) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr int NA = 2 * TN, NB = 2 * TM, NT = SWIGLU ? TN : NA;
     constexpr int RB = BN_OUT * 2, U = RB / 16;
@@ -164,6 +179,9 @@ __device__ __forceinline__ void lay_tiles_lds(const f32x4 (&acc)[2 * TN][2 * TM]
                 if (SWIGLU) {
                     const float g = round_to<bf16>(acc[2 * t][tb][i]), u = round_to<bf16>(acc[2 * t + 1][tb][i]);
                     o[i] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
+                } else if (EPI == EPI_FREE) {  // bf16 outputs of the free epilogue; bias columns past N are not read
+                    const int m = tile_m * (WM * TM * 32) + row, n = tile_n * BN_OUT + (wn * NT + t) * 16 + 4 * q4 + i;
+                    o[i] = from_f32<bf16>(m < a.M && n < a.N ? free_epilogue(a.epi, (int64_t)m * a.ldy + n, n, acc[t][tb][i]) : 0.f);
                 } else {
                     o[i] = from_f32<bf16>(acc[t][tb][i]);
                 }
@@ -183,9 +201,10 @@ __device__ __forceinline__ void lay_tiles_lds(const f32x4 (&acc)[2 * TN][2 * TM]
 // residual is fetched the same way, before the tile is laid down, so that its latency hides behind the transposition.
 // 16-byte unit u of tile row r sits at position u ^ (r mod units per row): the 16 rows a store instruction spreads over
 // then fall on different banks.
-template <bool SWIGLU, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
 __device__ __forceinline__ void store_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_m, int tile_n, int wave,
                                                 int lane, unsigned lds_base) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr int NA = 2 * TN, NB = 2 * TM, NT = SWIGLU ? TN : NA;
     constexpr int RB = BN_OUT * 2, U = RB / 16;      // bytes and 16-byte units per tile row
@@ -200,15 +219,15 @@ __device__ __forceinline__ void store_tiles_lds(const TiledArgs& a, const f32x4 
         const int m = tile_m * BM + idx / U, n = tile_n * BN_OUT + (idx % U) * 8;
         goff[it] = (m < a.M && n < a.N) ? (int64_t)m * a.ldy + n : -1;
         res[it] = u32x4{0, 0, 0, 0};
-        if (!SWIGLU && a.residual && goff[it] >= 0) res[it] = *reinterpret_cast<const u32x4*>(a.residual + goff[it]);
+        if (EPI == EPI_PLAIN && a.residual && goff[it] >= 0) res[it] = *reinterpret_cast<const u32x4*>(a.residual + goff[it]);
     }
-    lay_tiles_lds<SWIGLU, TM, TN, WM, WN>(acc, wave, lane, lds_base);
+    lay_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int idx = (wave * ITERS + it) * 64 + lane;
         const int row = idx / U, unit = idx % U;
         u32x4 v = *reinterpret_cast<const lds_u32x4*>(lds_base + row * RB + ((unit ^ (row & (U - 1))) * 16));
-        if (!SWIGLU && a.residual) {
+        if (EPI == EPI_PLAIN && a.residual) {
             bf16 o[8], r[8];
             *reinterpret_cast<u32x4*>(o) = v;
             *reinterpret_cast<u32x4*>(r) = res[it];
@@ -279,7 +298,7 @@ __device__ __forceinline__ void store_tiles_rope(const TiledArgs& a, const f32x4
     };
 #pragma unroll
     for (int it = 0; it < PD; ++it) request(fq[it]);
-    lay_tiles_lds<false, TM, TN, WM, WN>(acc, wave, lane, lds_base);
+    lay_tiles_lds<EPI_PLAIN, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int row = row0 + it * RS;
@@ -308,8 +327,9 @@ __device__ __forceinline__ void store_tiles_rope(const TiledArgs& a, const f32x4
 
 __device__ __align__(16) unsigned int g_zero_piece[4];  // what a 16-byte piece past the end of K is loaded from
 
-template <bool SWIGLU, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
 __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32;
     constexpr int NWAVES = WM * WN;
     constexpr int ROWS = BN + BM;              // LDS rows of a stage: the W tile, then the X tile
@@ -531,14 +551,14 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
     run(e1, e2, std::false_type{});
     run(e2, e3, std::true_type{});
     run(e3, nk, std::false_type{});
-    if constexpr (!SWIGLU) {
+    if constexpr (EPI == EPI_PLAIN) {
         if (a.rope_on) {  // uniform over the launch
             store_tiles_rope<TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
             return;
         }
     }
-    if (a.out_f32) store_tiles<SWIGLU, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
-    else store_tiles_lds<SWIGLU, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    if (a.out_f32) store_tiles<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
+    else store_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -557,8 +577,9 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
 //     of step k + 1 have landed, and its slice 0 is read under the last products.  A request has between 1.4 and 2.4
 //     steps to land.
 // Same products in the same order per accumulator as the eight-wave kernel: bit-identical results.
-template <bool SWIGLU>
+template <int EPI>
 __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int TM = 4, TN = 4, WM = 2, WN = 2;
     constexpr int BM = 256, BN = 256, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr int NA = 8, NB = 8, NP = NA * NB;   // 16-row tiles of a wave along the weight / token rows; products of a k-slice
@@ -737,23 +758,24 @@ __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
     run(e3, nk, std::false_type{});
     // requests past the last step still write into the ring, and the last products must land before their tiles are read
     asm volatile("s_waitcnt vmcnt(0)\n\ts_nop 15\n\ts_nop 15" ::: "memory");
-    if constexpr (!SWIGLU) {
+    if constexpr (EPI == EPI_PLAIN) {
         if (a.rope_on) {  // uniform over the launch
             store_tiles_rope<TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
             return;
         }
     }
-    if (a.out_f32) store_tiles<SWIGLU, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
-    else store_tiles_lds<SWIGLU, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    if (a.out_f32) store_tiles<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
+    else store_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 }
 
-template <bool SWIGLU>
+template <int EPI>
 static int launch_ring(TiledArgs a, hipStream_t s) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = 256, BN_OUT = SWIGLU ? 128 : 256;
     constexpr size_t lds = 5 * 32768;
     static bool attr_set = false;
     if (!attr_set) {
-        hipError_t e = hipFuncSetAttribute((const void*)gemm_ring_kernel<SWIGLU>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        hipError_t e = hipFuncSetAttribute((const void*)gemm_ring_kernel<EPI>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) {
             raven_host::set_error("gemm (ring): hipFuncSetAttribute failed: %s", hipGetErrorString(e));
             return (int)e;
@@ -765,7 +787,7 @@ static int launch_ring(TiledArgs a, hipStream_t s) {
     const int64_t n_tiles = (int64_t)a.tiles_m * a.tiles_n;
     RAVEN_REQUIRE(n_tiles < (1 << 28), "gemm (ring): too many tiles (M=%d N=%d)", a.M, a.N);
     const unsigned grid = (unsigned)((n_tiles + 7) / 8 * 8);
-    gemm_ring_kernel<SWIGLU><<<dim3(grid), dim3(256), lds, s>>>(a);
+    gemm_ring_kernel<EPI><<<dim3(grid), dim3(256), lds, s>>>(a);
     return raven_host::check_launch("gemm (ring MFMA)");
 }
 
@@ -773,13 +795,14 @@ int g_tiled_min_rows = 33;  // raven_set_tuning("gemm_tiled_min_rows"): fewest r
 int g_tiled_variant = 0;    // raven_set_tuning("gemm_tiled_variant"): 0 = by shape, 1 = 256 x 256 tiles, 2 = 128 x 128 tiles, 3 = 256 x 256 tiles by the eight-wave kernel
 int g_tiled_split_tail = 1; // raven_set_tuning("gemm_tiled_split_tail"): 0 = never hand the last round's tile columns to 128 x 128 tiles
 
-template <bool SWIGLU, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
 static int launch_tiled(TiledArgs a, hipStream_t s) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr size_t lds = (size_t)2 * (BM + BN) * 128;
     static bool attr_set = false;
     if (!attr_set) {
-        hipError_t e = hipFuncSetAttribute((const void*)gemm_tiled_kernel<SWIGLU, TM, TN, WM, WN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        hipError_t e = hipFuncSetAttribute((const void*)gemm_tiled_kernel<EPI, TM, TN, WM, WN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) {
             raven_host::set_error("gemm (tiled): hipFuncSetAttribute failed: %s", hipGetErrorString(e));
             return (int)e;
@@ -791,7 +814,7 @@ static int launch_tiled(TiledArgs a, hipStream_t s) {
     const int64_t n_tiles = (int64_t)a.tiles_m * a.tiles_n;
     RAVEN_REQUIRE(n_tiles < (1 << 28), "gemm (tiled): too many tiles (M=%d N=%d)", a.M, a.N);
     const unsigned grid = (unsigned)((n_tiles + 7) / 8 * 8);
-    gemm_tiled_kernel<SWIGLU, TM, TN, WM, WN><<<dim3(grid), dim3(64 * WM * WN), lds, s>>>(a);
+    gemm_tiled_kernel<EPI, TM, TN, WM, WN><<<dim3(grid), dim3(64 * WM * WN), lds, s>>>(a);
     return raven_host::check_launch("gemm (tiled MFMA)");
 }
 
@@ -837,7 +860,7 @@ __global__ __launch_bounds__(256) void pack_rows_kernel(const bf16* __restrict__
 }
 
 static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* w, const void* residual, void* y, int M, int N, int K0,
-                           int K1, int swiglu, int out_f32, const TiledArgs::RopeAppend* rope, hipStream_t s) {
+                           int K1, int swiglu, int out_f32, const TiledArgs::RopeAppend* rope, hipStream_t s, const raven_epilogue* epi = nullptr) {
     RAVEN_REQUIRE(tiled_gemm_fits(M, N, K0, K1, RAVEN_BF16), "gemm (tiled): unsupported shape M=%d N=%d K0=%d K1=%d", M, N, K0, K1);
     RAVEN_REQUIRE(!(swiglu && (residual || out_f32)), "gemm (tiled): the SwiGLU epilogue has no residual and stores bf16");
     RAVEN_REQUIRE(((uintptr_t)x0 & 15) == 0 && ((uintptr_t)x1 & 15) == 0 && ((uintptr_t)w & 15) == 0 && ((uintptr_t)y & 15) == 0 &&
@@ -862,6 +885,7 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
             a.ldw = it->second.ld;
         }
     }
+    if (epi) a.epi = *epi;
     if (rope) {
         a.rope = *rope;
         a.rope_on = 1;
@@ -874,9 +898,10 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
     auto launch = [&](const TiledArgs& t, bool as_big) {
         // 256 x 256 tiles: four waves, operands straight into an LDS ring (5 to 8 % faster than eight waves with staging
         // registers at the model's shapes, same bits); the eight-wave kernel stays selectable and serves the small tiles
-        if (as_big && g_tiled_variant != 3) return swiglu ? launch_ring<true>(t, s) : launch_ring<false>(t, s);
-        if (swiglu) return as_big ? launch_tiled<true, 4, 2>(t, s) : launch_tiled<true, 2, 1>(t, s);
-        return as_big ? launch_tiled<false, 4, 2>(t, s) : launch_tiled<false, 2, 1>(t, s);
+        if (epi) return as_big ? launch_ring<EPI_FREE>(t, s) : launch_tiled<EPI_FREE, 2, 1>(t, s);
+        if (as_big && g_tiled_variant != 3) return swiglu ? launch_ring<EPI_SWIGLU>(t, s) : launch_ring<EPI_PLAIN>(t, s);
+        if (swiglu) return as_big ? launch_tiled<EPI_SWIGLU, 4, 2>(t, s) : launch_tiled<EPI_SWIGLU, 2, 1>(t, s);
+        return as_big ? launch_tiled<EPI_PLAIN, 4, 2>(t, s) : launch_tiled<EPI_PLAIN, 2, 1>(t, s);
     };
     // The last round of 256 x 256 tiles: when it would fill at most half of the 256 CUs and is whole tile columns, those
     // columns are multiplied as 128 x 128 tiles instead -- four times as many workgroups, a quarter of the time each
@@ -893,6 +918,8 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
         tail.residual = a.residual ? a.residual + n_big : nullptr;
         tail.y = out_f32 ? static_cast<void*>(static_cast<float*>(y) + n_big) : static_cast<void*>(static_cast<bf16*>(y) + n_big);
         tail.rope.col0 = n_big;
+        if (tail.epi.bias) tail.epi.bias += n_big;
+        if (tail.epi.residual) tail.epi.residual += n_big;
         const int rc = launch(head, true);
         return rc ? rc : launch(tail, false);
     }
@@ -902,6 +929,12 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
 int tiled_gemm(const void* x0, const void* x1, const void* w, const void* residual, void* y, int M, int N, int K0, int K1, int swiglu,
                int out_f32, hipStream_t s) {
     return tiled_gemm_impl(x0, 0, x1, w, residual, y, M, N, K0, K1, swiglu, out_f32, nullptr, s);
+}
+
+// The product with the free epilogue: y = act(scale * z + bias) + residual, float or bf16
+int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi,
+                    hipStream_t s) {
+    return tiled_gemm_impl(x0, 0, x1, w, nullptr, y, M, N, K0, K1, 0, epi.out_f32, nullptr, s, &epi);
 }
 
 // The same with the rows of x `ldx` elements apart (>= K, one segment): activations whose rows are padded to whole cache lines

@@ -36,6 +36,7 @@ struct Gemv1Args {
     int ldw;               // elements between two weight rows (K, or more for a column block of a wider matrix)
     const float* acc_in;   // [N] or null: fp32 sums of the remaining columns, added before the result is rounded
     int raw_out;           // y receives the unrounded fp32 sums (the other half of acc_in)
+    raven_epilogue epi;    // EPI_FREE only
 };
 
 template <bool NT, typename T>
@@ -59,8 +60,9 @@ __device__ __forceinline__ float wg_sum(float v, float* red) {
 constexpr int kMaxPairsPerWg = 16;
 
 // MULTI: the workgroup walks several row pairs and double-buffers their weights in registers
-template <typename T, int C, bool SWIGLU, bool NORM, bool MULTI>
+template <typename T, int C, int EPI, bool NORM, bool MULTI>
 __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int E = Chunk<T>::N;
     __shared__ float red[4];
     __shared__ float part[kMaxPairsPerWg][4][2];
@@ -187,7 +189,7 @@ __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
         const int unit = unit_of(p);
         float s0 = part[p][0][0] + part[p][1][0] + part[p][2][0] + part[p][3][0];
         float s1 = part[p][0][1] + part[p][1][1] + part[p][2][1] + part[p][3][1];
-        if (!SWIGLU && (a.acc_in || a.raw_out)) {
+        if (EPI == EPI_PLAIN && (a.acc_in || a.raw_out)) {
             const int r0 = 2 * unit, r1 = r0 + 1;
             if (a.acc_in) {
                 s0 += a.acc_in[r0];
@@ -198,6 +200,12 @@ __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
                 if (r1 < a.N) static_cast<float*>(a.y)[r1] = s1;
                 return;
             }
+        }
+        if (EPI == EPI_FREE) {
+            const int r0 = 2 * unit;
+            store_free<T>(a.epi, a.y, r0, r0, s0);
+            if (r0 + 1 < a.N) store_free<T>(a.epi, a.y, r0 + 1, r0 + 1, s1);
+            return;
         }
         if (SWIGLU) {
             const float g = round_to<T>(s0), u = round_to<T>(s1);
@@ -239,8 +247,9 @@ static int gemv1_cus() {
     return cus;
 }
 
-template <typename T, bool SWIGLU>
+template <typename T, int EPI>
 static int launch_gemv1(Gemv1Args a, hipStream_t s) {
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int E = Chunk<T>::N;
     const int n_chunks = a.K / E;
     const int per_wave = (n_chunks + 3) / 4 + 1;  // a quarter, rounded up
@@ -259,12 +268,12 @@ static int launch_gemv1(Gemv1Args a, hipStream_t s) {
     const int wgs = (units + ppw - 1) / ppw;
 #define RAVEN_GEMV1(CC)                                                                            \
     do {                                                                                           \
-        if (norm) gemv1_kernel<T, CC, SWIGLU, true, false><<<dim3(wgs), dim3(256), 0, s>>>(a);     \
-        else gemv1_kernel<T, CC, SWIGLU, false, false><<<dim3(wgs), dim3(256), 0, s>>>(a);         \
+        if (norm) gemv1_kernel<T, CC, EPI, true, false><<<dim3(wgs), dim3(256), 0, s>>>(a);     \
+        else gemv1_kernel<T, CC, EPI, false, false><<<dim3(wgs), dim3(256), 0, s>>>(a);         \
     } while (0)
     if (c <= 3 && ppw > 1) {
-        if (norm) gemv1_kernel<T, 3, SWIGLU, true, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
-        else gemv1_kernel<T, 3, SWIGLU, false, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
+        if (norm) gemv1_kernel<T, 3, EPI, true, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
+        else gemv1_kernel<T, 3, EPI, false, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
     } else if (c <= 3) RAVEN_GEMV1(3);
     else if (c <= 6) RAVEN_GEMV1(6);
     else if (c <= 9) RAVEN_GEMV1(9);
@@ -293,7 +302,15 @@ int gemv1_column_block(const void* x, const void* norm_a, const void* w_block, i
     Gemv1Args a{};
     a.w = w_block; a.x0 = x; a.norm_a = norm_a; a.y = y; a.N = N; a.K = K; a.k0 = K; a.eps = eps;
     a.ldw = ldw; a.acc_in = acc_in; a.raw_out = raw_out;
-    return dtype == RAVEN_BF16 ? launch_gemv1<bf16, false>(a, s) : launch_gemv1<float, false>(a, s);
+    return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_PLAIN>(a, s) : launch_gemv1<float, EPI_PLAIN>(a, s);
+}
+
+// One row with the free epilogue; longest K as launch_gemv1
+int gemv1_free(const void* x0, const void* x1, const void* w, void* y, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
+               hipStream_t s) {
+    Gemv1Args a{};
+    a.w = w; a.x0 = x0; a.x1 = x1; a.y = y; a.N = N; a.K = K0 + K1; a.k0 = K0; a.ldw = a.K; a.epi = epi;
+    return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_FREE>(a, s) : launch_gemv1<float, EPI_FREE>(a, s);
 }
 
 }  // namespace raven
@@ -315,6 +332,6 @@ extern "C" int raven_gemv_fused(const void* x0, const void* x1, const void* norm
     a.residual = residual; a.y = y; a.N = N; a.K = K0 + K1; a.k0 = K0; a.out_f32 = out_f32; a.eps = eps;
     a.ldw = a.K;
     hipStream_t s = static_cast<hipStream_t>(stream);
-    if (dtype == RAVEN_BF16) return swiglu ? launch_gemv1<bf16, true>(a, s) : launch_gemv1<bf16, false>(a, s);
-    return swiglu ? launch_gemv1<float, true>(a, s) : launch_gemv1<float, false>(a, s);
+    if (dtype == RAVEN_BF16) return swiglu ? launch_gemv1<bf16, EPI_SWIGLU>(a, s) : launch_gemv1<bf16, EPI_PLAIN>(a, s);
+    return swiglu ? launch_gemv1<float, EPI_SWIGLU>(a, s) : launch_gemv1<float, EPI_PLAIN>(a, s);
 }

@@ -114,6 +114,29 @@ __device__ __forceinline__ float wave_max(float v) {
 // inside the fp32 bar, and a true division costs five times the instructions in the SwiGLU epilogue of a 256 x 256 tile.
 __device__ __forceinline__ float silu_f32(float x) { return x * __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }
 
+__device__ __forceinline__ float sigmoid_f32(float x) { return 1.0f / (1.0f + expf(-x)); }
+
+// ---- the free epilogue of the linear kernels (raven_linear_epilogue) --------------------------------------------
+// which epilogue a linear kernel is compiled with: the nn.Linear one (rounded to T, then a residual in T), SwiGLU, or the
+// free one below, whose sums stay unrounded until they are stored
+enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_FREE = 2 };
+
+// act(scale * z + bias[n]) + residual[at], z an fp32 sum and `at` its element offset in the output
+__device__ __forceinline__ float free_epilogue(const raven_epilogue& e, int64_t at, int n, float z) {
+    float v = z * e.scale;
+    if (e.bias) v += e.bias[n];
+    if (e.act == RAVEN_ACT_GELU) v = 0.5f * v * (1.0f + erff(v * 0.70710678118654752f));
+    else if (e.act == RAVEN_ACT_TANH) v = tanhf(v);
+    if (e.residual) v += e.residual[at];
+    return v;
+}
+template <typename T>
+__device__ __forceinline__ void store_free(const raven_epilogue& e, void* y, int64_t at, int n, float z) {
+    const float v = free_epilogue(e, at, n, z);
+    if (e.out_f32) static_cast<float*>(y)[at] = v;
+    else static_cast<T*>(y)[at] = from_f32<T>(v);
+}
+
 // One RoPE pair, adjacent elements (recpre/raven_modeling_minimal.py:118-131): products and sums rounded one by one in
 // fp32, as the reference's separate elementwise kernels do; every kernel that rotates uses this one function, so that
 // the fused and the two-launch paths write the same bits.

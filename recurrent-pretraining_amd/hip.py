@@ -46,7 +46,35 @@ class PagedKV(C.Structure):
                 ("kv_layout", C.c_int32)]
 
 
+class Epilogue(C.Structure):
+    _fields_ = [("bias", C.c_void_p), ("residual", C.c_void_p), ("scale", C.c_float), ("act", C.c_int32), ("out_f32", C.c_int32)]
+
+
+class KeyCache(C.Structure):
+    _fields_ = [("k", C.c_void_p), ("batch", C.c_int32), ("n_kv_heads", C.c_int32), ("head_dim", C.c_int32), ("t_max", C.c_int32)]
+
+
+class Score(C.Structure):
+    _fields_ = [("scale", C.c_float), ("softcap", C.c_float), ("r1", C.c_void_p), ("r2", C.c_void_p)]
+
+
+class MixerLayer(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("norm1", "conv", "w_in", "w_low", "w_decay", "decay_bias", "a_bias", "out_norm", "w_out", "norm2",
+                                          "up", "down")] + [("score", Score)] + [
+        (n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "head_dim", "rank", "taps", "ff")]
+
+
+class StreamDims(C.Structure):
+    _fields_ = [("width", C.c_int32), ("ld", C.c_int32), ("eps", C.c_float), ("dtype", C.c_int32)]
+
+
+class MixerState(C.Structure):
+    _fields_ = [("ring", C.c_void_p), ("state", C.c_void_p), ("keys", KeyCache)]
+
+
 PAGED_NHD, PAGED_HND = 0, 1
+ACT_NONE, ACT_GELU, ACT_TANH = 0, 1, 2
+MIXER_ATTENTION, MIXER_GENERAL_DELTA = 0, 1
 
 
 def _paged_dims(cache: torch.Tensor, layout: int):
@@ -113,22 +141,46 @@ SIGNATURES = {
     "raven_paged_prefill_attention": (C.c_int, [_VP, _VP, _VP, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _I32, _VP]),
     "raven_paged_decode_blocks": (C.c_int, [C.POINTER(Dims), _VP, C.POINTER(BlockWeights), _I32, _VP, _VP, _VP, _VP, _VP,
                                             C.POINTER(PagedKV), _I32, _I32, _VP, _SZ, _VP]),
+    "raven_linear_epilogue": (C.c_int, [_VP, _VP, _VP, _VP, _I32, _I32, _I32, _I32, C.POINTER(Epilogue), _I32, _VP, _SZ, _VP]),
+    "raven_norm_conv": (C.c_int, [_VP, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _I32, _I32, _F, _I32, _VP, _I32, _VP]),
+    "raven_embed_stream": (C.c_int, [_VP, _VP, _VP, _VP, _I32, _I32, _I64, _F, _I32, _VP]),
+    "raven_round_rows": (C.c_int, [_VP, _VP, _I64, _I32, _VP]),
+    "raven_capped_attention_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
+    "raven_capped_attention": (C.c_int, [_VP, _VP, C.POINTER(KeyCache), C.POINTER(Score), _I32, _I32, _I32, _VP, _I32, _I32, _VP, _SZ, _VP]),
+    "raven_delta_rule_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
+    "raven_delta_rule": (C.c_int, [_VP, _I32, _VP, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _VP, _I32, _I32, _I32, _F, _I32, _VP, _SZ, _VP]),
+    "raven_mixer_layer_workspace_bytes": (_SZ, [C.POINTER(StreamDims), C.POINTER(MixerLayer), _I32, _I32]),
+    "raven_mixer_layer_forward": (C.c_int, [C.POINTER(StreamDims), C.POINTER(MixerLayer), C.POINTER(MixerState), _VP, _I32, _I32, _I32, _VP,
+                                            _VP, _SZ, _VP]),
 }
 
 _lib: Optional[C.CDLL] = None
+_lib_path = LIB_PATH
+
+
+def use_library(path: str) -> None:
+    """Binds another build of the library (build.ensure_library) before the first call: one family's kernels, say."""
+    global _lib_path
+    if _lib is not None and path != _lib_path:
+        raise RavenHipError("the library is already loaded")
+    _lib_path = path
 
 
 def load() -> C.CDLL:
     """Loads the library (once).  Raises when it has not been built: there is no other code path."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
+        if not os.path.exists(_lib_path):
             raise RavenHipError(
-                f"{LIB_PATH} is missing: build it with `python -c 'import __graft_entry__ as e; e.build()'` "
+                f"{_lib_path} is missing: build it with `python -c 'import __graft_entry__ as e; e.build()'` "
                 "(hipcc, gfx950).  This package has no CPU or PyTorch fallback.")
-        lib = C.CDLL(LIB_PATH)
+        lib = C.CDLL(_lib_path)
         for name, (res, args) in SIGNATURES.items():
-            fn = getattr(lib, name)
+            fn = getattr(lib, name, None)
+            if fn is None and _lib_path != LIB_PATH:
+                continue  # a family's library lacks the others' entry points: calling one raises
+            if fn is None:
+                raise RavenHipError(f"{_lib_path} does not export {name}: build it again")
             fn.restype = res
             fn.argtypes = args
         _lib = lib
@@ -568,3 +620,109 @@ def paged_decode_blocks(dims: Dims, blocks, x_in, x_out, freqs, kv: PagedKV, B, 
         int(n_iterations), B, _ptr(workspace, "workspace", torch.uint8), workspace.numel(), _stream())
     _check(rc, "raven_paged_decode_blocks")
     return x_out
+
+
+# ---------------------------------------------------------------------------------------------
+# layers over an fp32 residual stream
+# ---------------------------------------------------------------------------------------------
+def _workspace(n: int, device) -> Optional[torch.Tensor]:
+    return torch.empty(n, dtype=torch.uint8, device=device) if n else None
+
+
+def linear_epilogue(x0, w, x1=None, bias=None, residual=None, scale=1.0, act=ACT_NONE, out_f32=True, out=None, workspace=None):
+    """act(scale * concat(x0, x1) W^T + bias) + residual on unrounded sums; x0 [M, K0], w [N, K0 + K1], bias [N] / residual [M, N] float."""
+    dt = x0.dtype
+    M, K0 = x0.shape
+    K1 = 0 if x1 is None else x1.shape[1]
+    N = w.shape[0]
+    if w.shape[1] != K0 + K1 or (bias is not None and bias.shape != (N,)) or (residual is not None and residual.shape != (M, N)):
+        raise RavenHipError("linear_epilogue: operand shapes do not fit together")
+    y = out if out is not None else torch.empty(M, N, device=x0.device, dtype=torch.float32 if out_f32 else dt)
+    if y.shape != (M, N):
+        raise RavenHipError(f"linear_epilogue: output {tuple(y.shape)}, expected {(M, N)}")
+    e = Epilogue(_ptr(bias, "bias", torch.float32), _ptr(residual, "residual", torch.float32), float(scale), int(act), int(out_f32))
+    rc = load().raven_linear_epilogue(_ptr(x0, "x0"), _ptr(x1, "x1", dt), _ptr(w, "w", dt), _ptr(y, "y", torch.float32 if out_f32 else dt), M, N, K0, K1,
+                                      C.byref(e), dtype_code(dt), _ptr(workspace, "workspace", torch.uint8),
+                                      0 if workspace is None else workspace.numel(), _stream())
+    _check(rc, "raven_linear_epilogue")
+    return y
+
+
+def norm_conv(x, weight, dim, eps, B, S, dtype, conv=None, ring=None, pos0=0, pos_dev=None, out=None):
+    """x [B*S, ld] float -> T [B*S, ld]; conv [taps, ld] and ring [B, taps, ld] float, or None."""
+    ld = x.shape[1]
+    taps = 0 if conv is None else conv.shape[0]
+    if x.shape[0] != B * S or weight.shape != (ld,) or (conv is not None and (conv.shape[1] != ld or ring.shape != (B, taps, ld))):
+        raise RavenHipError("norm_conv: operand shapes do not fit together")
+    y = out if out is not None else torch.empty(B * S, ld, device=x.device, dtype=dtype)
+    rc = load().raven_norm_conv(_ptr(x, "x", torch.float32), _ptr(weight, "weight", torch.float32), _ptr(conv, "conv", torch.float32),
+                                _ptr(ring, "ring", torch.float32), _ptr(y, "y", dtype), B, S, dim, ld, taps, float(eps), int(pos0),
+                                _ptr(pos_dev, "pos_dev", torch.int32), dtype_code(dtype), _stream())
+    _check(rc, "raven_norm_conv")
+    return y
+
+
+def embed_stream(table, ids, scale, x, x_rounded=None):
+    if x.shape != (ids.numel(), table.shape[1]) or (x_rounded is not None and x_rounded.shape != x.shape):
+        raise RavenHipError("embed_stream: output rows do not fit the ids")
+    rc = load().raven_embed_stream(_ptr(table, "table"), _ptr(ids, "ids", torch.int64), _ptr(x, "x", torch.float32),
+                                   _ptr(x_rounded, "x_rounded", table.dtype), ids.numel(), table.shape[1], table.shape[0], float(scale),
+                                   dtype_code(table.dtype), _stream())
+    _check(rc, "raven_embed_stream")
+
+
+def round_rows(x, out):
+    _check(load().raven_round_rows(_ptr(x, "x", torch.float32), _ptr(out, "out"), x.numel(), dtype_code(out.dtype), _stream()), "raven_round_rows")
+    return out
+
+
+def make_key_cache(k: torch.Tensor) -> KeyCache:
+    """k: [batch, n_kv_heads, t_max, head_dim]."""
+    b, g, t, hd = k.shape
+    return KeyCache(_ptr(k, "keys"), b, g, hd, t)
+
+
+def make_score(scale: float, softcap: float = 0.0, r1: Optional[torch.Tensor] = None, r2: Optional[torch.Tensor] = None) -> Score:
+    return Score(float(scale), float(softcap), _ptr(r1, "r1", torch.float32), _ptr(r2, "r2", torch.float32))
+
+
+def capped_attention(qk, keys: torch.Tensor, score: Score, B, S, pos0, n_heads, pos_dev=None):
+    """qk [B*S, (n_heads + n_kv_heads) * hd]; appends the rows' keys to `keys` and attends.  Returns [B*S, n_heads * hd]."""
+    _, g, _, hd = keys.shape
+    if qk.shape != (B * S, (n_heads + g) * hd):
+        raise RavenHipError(f"capped_attention: q | k rows {tuple(qk.shape)} for {n_heads} + {g} heads of {hd}")
+    y = torch.empty(B * S, n_heads * hd, device=qk.device, dtype=qk.dtype)
+    ws = _workspace(load().raven_capped_attention_workspace_bytes(B * S, n_heads, g, hd), qk.device)
+    cache = make_key_cache(keys)
+    rc = load().raven_capped_attention(_ptr(qk, "qk", keys.dtype), _ptr(y, "y"), C.byref(cache), C.byref(score), B, S, int(pos0),
+                                       _ptr(pos_dev, "pos_dev", torch.int32), n_heads, dtype_code(qk.dtype), _ptr(ws, "ws"),
+                                       0 if ws is None else ws.numel(), _stream())
+    _check(rc, "raven_capped_attention")
+    return y
+
+
+def delta_rule(z, decay_logits, a_bias, norm, state, B, S, pos0, dim, eps, dtype, pos_dev=None, parallel=True):
+    """z [B*S, >= 5 * H * hd] float; state [B, H, hd, hd] float, updated in place.  Returns [B*S, H * hd] of dtype.  parallel=False
+    walks the tokens one by one whatever the chunk's length."""
+    _, H, hd, _ = state.shape
+    if z.shape[0] != B * S or decay_logits.shape != (B * S, H * hd) or a_bias.shape != (H * hd,) or norm.shape != (H * hd,) or state.shape[0] < B:
+        raise RavenHipError("delta_rule: operand shapes do not fit together")
+    y = torch.empty(B * S, H * hd, device=z.device, dtype=dtype)
+    ws = _workspace(load().raven_delta_rule_workspace_bytes(B, S, H, hd), z.device) if parallel else None
+    f = torch.float32
+    rc = load().raven_delta_rule(_ptr(z, "z", f), z.shape[1], _ptr(decay_logits, "decay_logits", f), _ptr(a_bias, "a_bias", f), _ptr(norm, "norm", f),
+                                 _ptr(state, "state", f), _ptr(y, "y"), B, S, int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), H, int(dim), hd,
+                                 float(eps), dtype_code(dtype), _ptr(ws, "ws"), 0 if ws is None else ws.numel(), _stream())
+    _check(rc, "raven_delta_rule")
+    return y
+
+
+def mixer_layer_workspace_bytes(dims: StreamDims, layer: MixerLayer, B: int, S: int) -> int:
+    return load().raven_mixer_layer_workspace_bytes(C.byref(dims), C.byref(layer), B, S)
+
+
+def mixer_layer(dims: StreamDims, layer: MixerLayer, state: MixerState, x, B, S, pos0, workspace, pos_dev=None):
+    rc = load().raven_mixer_layer_forward(C.byref(dims), C.byref(layer), C.byref(state), _ptr(x, "x", torch.float32), B, S, int(pos0),
+                                          _ptr(pos_dev, "pos_dev", torch.int32), _ptr(workspace, "workspace", torch.uint8),
+                                          workspace.numel(), _stream())
+    _check(rc, "raven_mixer_layer_forward")

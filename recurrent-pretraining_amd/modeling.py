@@ -20,53 +20,15 @@ from __future__ import annotations
 
 import math
 import weakref
-from dataclasses import dataclass
-from typing import Any, Callable, Optional, Union
+from typing import Optional, Union
 
 import torch
 from transformers import AutoConfig, AutoModel, AutoModelForCausalLM, GenerationMixin, PreTrainedModel
-from transformers.utils import ModelOutput
 
-from . import hip
+from . import checkpoint, hip
 from .cache import HuginnDynamicCache, HuginnStaticCache, remap_step
 from .config import RavenConfig
-
-
-@dataclass
-class CausalLMOutputRecurrentLatents(ModelOutput):  # RMM:113-123
-    loss: Optional[torch.Tensor] = None
-    log_ppl: Optional[torch.Tensor] = None
-    logits: Optional[torch.Tensor] = None
-    past_key_values: Optional[HuginnDynamicCache] = None
-    latent_states: Optional[torch.Tensor] = None
-    hidden_states: Optional[torch.Tensor] = None
-    attention_maps: Optional[dict] = None
-    stats: Optional[dict] = None
-
-
-@dataclass
-class GenerationSettings:
-    """The fields of transformers.GenerationConfig that the generate loops read."""
-    max_length: int = 4096
-    max_new_tokens: Optional[int] = None
-    do_sample: bool = False
-    temperature: Optional[float] = None
-    top_k: Optional[int] = None
-    top_p: Optional[float] = None
-    min_p: Optional[float] = None
-    repetition_penalty: Optional[float] = None
-    dry_multiplier: float = 0.0        # > 0 selects the n-gram penalty instead (RMM:2003-2046)
-    dry_base: float = 1.75
-    dry_allowed_length: int = 2
-    eos_token_id: Any = None
-    return_dict_in_generate: bool = False
-
-
-@dataclass
-class GenerateOutput:
-    sequences: torch.Tensor
-    past_key_values: Optional[HuginnDynamicCache] = None
-    scores: Optional[dict] = None
+from .generation import CausalLMOutputRecurrentLatents, GenerateOutput, GenerationSettings, GraphedStep, MinimalGeneration  # noqa: F401
 
 
 # ------------------------------------------------------------------------------------------------
@@ -211,7 +173,9 @@ class RavenPreTrainedModel(PreTrainedModel):
                 normal(module.weight, iv["std"])
 
 
-class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
+class RavenForCausalLM(MinimalGeneration, RavenPreTrainedModel, GenerationMixin):
+    DEFAULT_STOPS = frozenset({65504, 65505, 65508})  # begin_text, end_text, end_turn (RMM:1929-1931)
+
     def __init__(self, config: RavenConfig, device: Union[str, torch.device, None] = None, dtype: Optional[torch.dtype] = None):
         """`device` None: wherever torch currently creates tensors (a `with torch.device(...)` block, transformers'
         loaders), else the GPU when there is one.  The parameters may live on the CPU; the forward needs them on the GPU."""
@@ -315,8 +279,6 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
         Replaces transformers' loader (one shard in host memory at a time, straight into the parameters) and takes its
         call shape: `config=` from an Auto class, `torch_dtype` / `dtype`, `device_map` as one device; the other loader
         keywords are accepted and have nothing to act on; any remaining keyword overrides a configuration field."""
-        import json
-        import os
         if dtype is None:
             dtype = kwargs.pop("torch_dtype", None)
         else:
@@ -333,46 +295,22 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
             device = "cuda" if device_map == "auto" else device_map
         for k in cls._LOADER_KWARGS:
             kwargs.pop(k, None)
-        path = str(path)
-        if not os.path.isdir(path):
-            raise FileNotFoundError(f"{path} is not a local directory (nothing is downloaded)")
-        with open(os.path.join(path, "config.json")) as f:
-            cfg_dict = json.load(f)
+        cfg_dict = checkpoint.read_config(path)
         if config is not None:
             cfg_dict = config.to_dict()
         cfg_dict.update(kwargs)
         config = RavenConfig(**cfg_dict)
         model = cls(config, device=device, dtype=dtype)
-        index = os.path.join(path, "model.safetensors.index.json")
-        single = os.path.join(path, "model.safetensors")
-        legacy = os.path.join(path, "pytorch_model.bin")
-        if os.path.exists(index):
-            with open(index) as f:
-                shards = sorted(set(json.load(f)["weight_map"].values()))
-            files = [os.path.join(path, s) for s in shards]
-        elif os.path.exists(single):
-            files = [single]
-        elif os.path.exists(legacy):
-            files = [legacy]
-        else:
-            raise FileNotFoundError(f"no model.safetensors(.index.json) or pytorch_model.bin under {path}")
         own = model.state_dict()
         seen, unexpected = set(), []
-        for file in files:  # shard by shard: at most one shard is held besides the model
-            if file.endswith(".safetensors"):
-                from safetensors.torch import load_file
-                part = load_file(file, device="cpu")
-            else:
-                part = torch.load(file, map_location="cpu", weights_only=True)
-            for name, tensor in part.items():
-                if name not in own:
-                    unexpected.append(name)
-                    continue
-                if own[name].shape != tensor.shape:
-                    raise ValueError(f"{name}: checkpoint shape {tuple(tensor.shape)} != model shape {tuple(own[name].shape)}")
-                own[name].copy_(tensor)
-                seen.add(name)
-            del part
+        for name, tensor in checkpoint.tensors(path):
+            if name not in own:
+                unexpected.append(name)
+                continue
+            if own[name].shape != tensor.shape:
+                raise ValueError(f"{name}: checkpoint shape {tuple(tensor.shape)} != model shape {tuple(own[name].shape)}")
+            own[name].copy_(tensor)
+            seen.add(name)
         optional = {"freqs_cis"} | ({"lm_head.weight", "transformer.wte.weight"} if config.tie_embeddings else set())
         missing = [n for n in own if n not in seen and n not in optional]
         if config.tie_embeddings and not ({"lm_head.weight", "transformer.wte.weight"} & seen):
@@ -385,38 +323,11 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
     def save_pretrained(self, path: str, max_shard_bytes: int = 5 * 2 ** 30, **unused) -> None:
         """Writes `config.json` and safetensors shards (with an index when there are several) that from_pretrained and
         the reference's loader read.  The tied head is stored once, under the embedding's name."""
-        import json
-        import os
-        from safetensors.torch import save_file
-        path = str(path)
-        os.makedirs(path, exist_ok=True)
         cfg = self.config.to_dict()
         cfg.update(architectures=["RavenForCausalLM"], torch_dtype=str(self.dtype).replace("torch.", ""))
         cfg["dtype"] = cfg["torch_dtype"]
-        with open(os.path.join(path, "config.json"), "w") as f:
-            json.dump(cfg, f, indent=1, sort_keys=True)
-        sd = {k: v.detach().to("cpu").contiguous() for k, v in self.state_dict().items()
-              if not (self.config.tie_embeddings and k == "lm_head.weight")}
-        shards, cur, size = [], {}, 0
-        for name, t in sd.items():
-            nbytes = t.numel() * t.element_size()
-            if cur and size + nbytes > max_shard_bytes:
-                shards.append(cur)
-                cur, size = {}, 0
-            cur[name] = t
-            size += nbytes
-        shards.append(cur)
-        if len(shards) == 1:
-            save_file(shards[0], os.path.join(path, "model.safetensors"), metadata={"format": "pt"})
-            return
-        weight_map = {}
-        for i, part in enumerate(shards):
-            fname = f"model-{i + 1:05d}-of-{len(shards):05d}.safetensors"
-            save_file(part, os.path.join(path, fname), metadata={"format": "pt"})
-            weight_map.update({k: fname for k in part})
-        with open(os.path.join(path, "model.safetensors.index.json"), "w") as f:
-            json.dump({"metadata": {"total_size": sum(t.numel() * t.element_size() for t in sd.values())}, "weight_map": weight_map}, f,
-                      indent=1)
+        sd = {k: v for k, v in self.state_dict().items() if not (self.config.tie_embeddings and k == "lm_head.weight")}
+        checkpoint.write(path, cfg, sd, max_shard_bytes)
 
     def _natives(self) -> dict:
         """ctypes views of the weights; rebuilt when a parameter's storage has moved."""
@@ -846,48 +757,6 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
                 model_inputs[key] = value
         return model_inputs
 
-    def _get_stops(self, generation_config, model_kwargs=None) -> set:
-        stops = {65504, 65505, 65508}  # begin_text, end_text, end_turn (RMM:1929-1931)
-        eos = getattr(generation_config, "eos_token_id", None)
-        if eos is not None:
-            try:
-                stops.update(eos)
-            except TypeError:
-                stops.add(eos)
-        return stops
-
-    def _sample_next_token(self, next_token_logits: torch.Tensor, input_ids, generation_config) -> torch.Tensor:
-        """RMM:1944-1989.  Greedy selection runs in the HIP argmax kernel."""
-        gc = generation_config
-        if getattr(gc, "repetition_penalty", None) is not None and gc.repetition_penalty != 1.0:
-            next_token_logits = self._apply_repetition_penalty(next_token_logits, input_ids, gc)
-        if not getattr(gc, "do_sample", False):
-            return hip.argmax(next_token_logits.float().contiguous()).unsqueeze(-1)
-        logits = next_token_logits.to(torch.float32)
-        if gc.temperature:
-            logits = logits / gc.temperature
-        probs = torch.softmax(logits, dim=-1)
-        if gc.top_k:
-            kth = torch.topk(probs, gc.top_k, dim=-1).values[:, -1:]
-            probs = torch.where(probs < kth, torch.zeros_like(probs), probs)
-        if gc.top_p:
-            sp, si = torch.sort(probs, descending=True, dim=-1)
-            remove = torch.cumsum(sp, dim=-1) > gc.top_p
-            remove[:, 0] = False
-            mask = torch.zeros_like(probs, dtype=torch.bool).scatter(1, si, remove)
-            probs = torch.where(mask, torch.zeros_like(probs), probs)
-        if gc.min_p:
-            probs = torch.where(probs < gc.min_p * probs.max(dim=-1, keepdim=True).values, torch.zeros_like(probs), probs)
-        probs = probs / probs.sum(dim=-1, keepdim=True).clamp(min=1e-10)
-        return torch.multinomial(probs, num_samples=1)
-
-    def _default_max_length(self, gc) -> int:
-        """`max_length` of the generation settings; transformers 5 leaves it unset by default, then the RoPE table's length."""
-        for src in (gc, self.generation_config):
-            if getattr(src, "max_length", None):
-                return src.max_length
-        return self.config.block_size
-
     def _generation_cache(self, model_kwargs: dict, cache_lookup_strategy: str, batch: int, max_length: Optional[int] = None):
         """The cache a generate loop works on (RMM:1146-1160): the caller's `past_key_values`, or a new one --
         HuginnStaticCache when `cache_implementation="static"` is asked for, else HuginnDynamicCache."""
@@ -903,11 +772,6 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
                                      lookup_strategy=cache_lookup_strategy)
         return HuginnDynamicCache(cache_lookup_strategy, max_length=max_length)
 
-    def _apply_repetition_penalty(self, original_logits, input_ids, generation_config, use_candidates: bool = False):
-        """RMM:1991-2070; see sampling.apply_repetition_penalty."""
-        from .sampling import apply_repetition_penalty
-        return apply_repetition_penalty(original_logits, input_ids, generation_config, use_candidates)
-
     def get_stats(self, logits, x, latent_states, xk, input_embeds, num_steps_no_grad, num_steps_with_grad) -> dict:
         """RMM:1037-1049: entropy of the predictive distribution and the distance between two latent states."""
         probs = torch.softmax(logits.float(), dim=-1)
@@ -915,8 +779,6 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
         return {"entropy": torch.where(probs > 0, -probs * probs.log(), 0).sum(dim=-1), "residual_diff": residual_diff,
                 "rel_residual": residual_diff / latent_states.norm(dim=-1), "num_steps_no_grad": num_steps_no_grad,
                 "num_steps_with_grad": num_steps_with_grad}
-
-    _MINIMAL_LOOP_KEYS = ("continuous_compute", "input_states_fn", "stop_tokens", "use_graph")
 
     @torch.no_grad()
     def generate(self, input_ids: Optional[torch.Tensor] = None, generation_config=None, **kwargs):
@@ -963,90 +825,19 @@ class RavenForCausalLM(RavenPreTrainedModel, GenerationMixin):
         from . import adaptive
         return adaptive.prefill_with_varied_exit_steps(self, input_ids, exit_evaluator, past_key_values, init_scale, **kwargs)
 
-    @torch.no_grad()
-    def generate_minimal(self, input_ids: torch.Tensor, generation_config=None, tokenizer=None, streamer=None,
-                         continuous_compute: bool = False, init_scale: float = 1.0, cache_lookup_strategy: str = "full",
-                         input_states_fn: Optional[Callable] = None, stop_tokens: Optional[set] = None,
-                         use_graph: bool = True, **model_kwargs):
-        """RMM:1165-1232.  Prefill through forward(), then one token per step through the decode
-        runner (all kernels of a token on one stream, optionally replayed as a HIP graph).
+    # ---- hooks of the shared decode loop (generation.MinimalGeneration) -----------------------------------------------
+    @property
+    def max_positions(self) -> int:
+        return self.config.block_size  # rows of the RoPE table
 
-        input_states_fn(call_index, (B, S, h)) -> latent state to inject into that forward (an
-        extension for reproducible runs: the reference re-draws the state from the device RNG on
-        every call, RMM:738).  stop_tokens overrides the reference's fixed stop set."""
-        gc = generation_config if generation_config is not None else self.generation_config
-        B, prompt_len = input_ids.shape
-        if "max_new_tokens" in model_kwargs and model_kwargs["max_new_tokens"] is not None:
-            max_new = model_kwargs["max_new_tokens"]
-            if "max_length" in model_kwargs:
-                max_new = min(max_new, model_kwargs["max_length"] - prompt_len)
-        elif getattr(gc, "max_new_tokens", None):
-            max_new = gc.max_new_tokens
-        else:
-            max_new = model_kwargs.get("max_length", self._default_max_length(gc)) - prompt_len
-        num_steps = model_kwargs.get("num_steps", None)
-        stops = self._get_stops(gc) if stop_tokens is None else set(stop_tokens)
-        input_ids = input_ids.to(self.device)
-        if max_new <= 0:
-            return input_ids
-        total = min(prompt_len + max_new, self.config.block_size)
-        cache = self._generation_cache(model_kwargs, cache_lookup_strategy, B, total)
+    def decode_runner(self, cache, batch: int, num_steps, greedy: bool, use_graph: bool) -> "DecodeRunner":
+        return DecodeRunner(self, cache, batch, self._split_steps(num_steps), greedy=greedy, use_graph=use_graph)
 
-        def state_for(call: int, S: int, embeds_like=None):
-            if input_states_fn is not None:
-                return input_states_fn(call, (B, S, self.config.n_embd)).to(self.device, self.dtype)
-            return None
-
-        # prefill
-        seen = cache.get_seq_length()
-        pos = torch.arange(seen, prompt_len, device=self.device)
-        out = self.forward(input_ids=input_ids[:, seen:], input_states=state_for(0, prompt_len - seen), num_steps=num_steps,
-                           past_key_values=cache, use_cache=True, cache_position=pos, init_scale=init_scale)
-        next_tok = self._sample_next_token(out.logits[:, -1, :], input_ids, gc)
-        carried = out.latent_states[:, -1:, :] if continuous_compute else None
-        tokens = [next_tok]
-        alive = torch.ones(B, dtype=torch.bool)
-        if streamer:
-            streamer.put(next_tok.cpu())
-
-        def update_alive(tok) -> bool:
-            if stops:
-                for b, v in enumerate(tok.view(-1).tolist()):
-                    if alive[b] and v in stops:
-                        alive[b] = False
-            return bool(alive.any())
-
-        runner = None
-        call = 1
-        # the penalties look at the growing sequence on every step (RMM:1198-1201, 1946-1947); with one configured the
-        # pick is made from the penalised logits on the greedy path too
-        penalised = getattr(gc, "repetition_penalty", None) is not None and gc.repetition_penalty != 1.0
-        pick_on_host = bool(getattr(gc, "do_sample", False)) or penalised
-        all_ids = torch.cat([input_ids, next_tok], dim=-1) if pick_on_host else None
-        while len(tokens) < max_new and update_alive(tokens[-1]) and cache.get_seq_length() + 1 <= total:
-            if runner is None:
-                runner = DecodeRunner(self, cache, B, self._split_steps(num_steps), greedy=not getattr(gc, "do_sample", False),
-                                      use_graph=use_graph)
-            state = carried if continuous_compute else state_for(call, 1)
-            logits, nxt, latents = runner.step(tokens[-1].view(-1), state, init_scale)
-            if pick_on_host:
-                nxt = self._sample_next_token(logits, all_ids, gc).view(-1)
-                all_ids = torch.cat([all_ids, nxt.view(B, 1)], dim=-1)
-            tokens.append(nxt.view(B, 1).clone())
-            if continuous_compute:
-                carried = latents.view(B, 1, -1).clone()
-            if streamer:
-                streamer.put(tokens[-1].cpu())
-            call += 1
-        if streamer:
-            streamer.end()
-        sequences = torch.cat([input_ids] + tokens, dim=-1)
-        if getattr(gc, "return_dict_in_generate", False):
-            return GenerateOutput(sequences=sequences, past_key_values=cache, scores={})
-        return sequences
+    def new_cache(self, max_length: Optional[int] = None) -> HuginnDynamicCache:
+        return HuginnDynamicCache(max_length=max_length)
 
 
-class DecodeRunner:
+class DecodeRunner(GraphedStep):
     """One decode step (S = 1) with every buffer preallocated: embedding, prelude, r recurrences,
     coda, ln_f, LM head and greedy argmax are enqueued back to back on the current stream.  The
     position is read by the kernels from a device counter, so the identical launch sequence serves
@@ -1062,7 +853,8 @@ class DecodeRunner:
         need_t = cache.max_length if cache.max_length is not None else cache.get_seq_length() + 1
         cache.ensure(max(n_pos, 1), cfg.n_layers_in_coda, batch, cfg.n_heads, cfg.head_dim, need_t, dt, dev)
         self.ids = torch.zeros(batch, dtype=torch.int64, device=dev)
-        self.pos = torch.zeros(1, dtype=torch.int32, device=dev)
+        # the noise draws are not part of a replayable launch sequence
+        super().__init__(use_graph and cfg.test_time_noise <= 0, dev)
         self.state = torch.zeros(batch, h, dtype=dt, device=dev)
         self.embeds = torch.empty(batch, h, dtype=dt, device=dev)
         self.x = torch.empty(batch, h, dtype=dt, device=dev)
@@ -1073,10 +865,6 @@ class DecodeRunner:
         if batch >= 17 and model.dtype == torch.bfloat16 and model.pack_chunk_weights:
             model.pack_weights()  # decode steps of 17..32 rows read Wqkv and mlp.fc through their line-aligned copies
         self.ws = hip.block_workspace(model._natives()["dims"], batch, dev)
-        self.use_graph = use_graph and cfg.test_time_noise <= 0  # the noise draws are not part of a replayable launch sequence
-        self.graph: Optional[torch.cuda.CUDAGraph] = None
-        self._graph_key = None
-        self._warm = False
 
     def _slots(self):
         """(prelude slots, first core slot per recurrence or per-block slots, coda slots) for one token."""
@@ -1164,7 +952,6 @@ class DecodeRunner:
         if self.B >= 17 and m.dtype == torch.bfloat16 and m.pack_chunk_weights:
             m.pack_weights()  # no work unless a weight changed since the copies were made (in place: the copies keep their addresses)
         self.ids.copy_(ids.view(-1))
-        self.pos.fill_(pos0)
         if state is None:
             if init_scale > 0:
                 self.state.copy_(m.initialize_state(self.embeds, init_scale))
@@ -1172,20 +959,9 @@ class DecodeRunner:
                 self.state.zero_()
         else:
             self.state.copy_(state.reshape(self.B, -1))
-        if self.use_graph and self._warm:
-            # the captured launches hold the cache's pointers, slot numbers and capacity: any reallocation (more
-            # positions, more step slots) makes them stale
-            key = (c._k.data_ptr(), c._v.data_ptr(), tuple(c._k.shape), c._neg_slots, hint)
-            if self.graph is None or self._graph_key != key:
-                self.graph = torch.cuda.CUDAGraph()
-                with torch.cuda.graph(self.graph):
-                    self._enqueue(hint)
-                self._graph_key = key
-                self.pos.fill_(pos0)  # capture does not execute; make sure the counter is what this step needs
-            self.graph.replay()
-        else:
-            self._enqueue(hint)
-            self._warm = True
+        # the captured launches hold the cache's pointers, slot numbers and capacity: any reallocation (more positions, more
+        # step slots) makes them stale
+        self.launch(pos0, hint, (c._k.data_ptr(), c._v.data_ptr(), tuple(c._k.shape), c._neg_slots, hint))
         # bookkeeping the reference does inside cache.update (RMM:188-196)
         cfg = m.config
         c._seen_tokens += 1
