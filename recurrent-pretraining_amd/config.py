@@ -104,7 +104,6 @@ class GitipelConfig(PretrainedConfig):
         self.layers = [dict(x) for x in (self.layers or [])]
         self.embedding = self.embedding or {"scale": 1.0}
         self.norm = self.norm or {"eps": 1e-5}
-        self.canon = self.canon or {"taps": 1}
         if self.architecture != "Gitipel":
             raise ValueError(f"not a Gitipel configuration: architecture {self.architecture!r}")
         for i, layer in enumerate(self.layers):

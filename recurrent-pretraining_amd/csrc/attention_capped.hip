@@ -10,7 +10,7 @@
 //       per lane serves the score AND the weighted sum of all those query heads -- a cached position is read once per key
 //       head.  Ranges are merged by a second launch in range order.  A decode step reads its own position's key from
 //       the fused row and appends it to the cache on the way.
-//   capped_attention_prefill_kernel  bf16 chunks on the matrix cores (further down).
+//   capped_attention_prefill_kernel  bf16 chunks of 16 and more rows on the matrix cores (further down).
 
 #include <math.h>
 
@@ -222,6 +222,227 @@ __global__ __launch_bounds__(256) void key_append_kernel(CappedArgs a, int M) {
                 load_chunk(static_cast<const T*>(a.qk) + (int64_t)m * a.ldq + (int64_t)(a.H + g) * a.hd + c * E));
 }
 
+// ------------------------------------------------------------------------------------------------
+// bf16 chunks on the matrix cores, the scheme of attention_prefill.hip: a wave owns RG groups of 16 query rows and walks tiles
+// of 64 keys; S^T = K Q^T leaves a lane with the scores of 16 keys of ONE query per group, in the layout the A operand of
+// P V wants; the weights' row sums come from one more product against ones; the reference maximum moves only when a tile
+// exceeds it by 2^8.  Keys are values, so ONE staged tile serves both products: read by rows for the scores and
+// through the transposing loads for P V.  Heads of up to HD channels (multiples of 8) sit zero-padded in the tile.
+//
+// A score costs four quarter-rate instructions (exp2 and reciprocal for the cap, log2 for the distance, exp2 for the weight)
+// where plain attention has one: the kernel is bound by vector work, not by the products.
+// ------------------------------------------------------------------------------------------------
+constexpr int kCpKeys = 64;
+
+template <int HD, int RG>
+__global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(CappedArgs a) {
+    constexpr int KS = HD / 32, NT = HD / 16;
+    constexpr int KP = HD + 16;          // an odd multiple of 8 banks: the transposing reads of 8 key rows hit 64 banks
+    constexpr int WR = 16 * RG, ROWS = 4 * WR;
+    constexpr int CPR = HD / 8, KCH = kCpKeys * CPR / 256;
+    static_assert(kCpKeys * CPR % 256 == 0, "staging shape");
+    __shared__ __align__(16) bf16 sk[2][kCpKeys][KP];
+    typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
+    typedef short s16x4 __attribute__((ext_vector_type(4)));
+
+    const int qb = gridDim.x - 1 - blockIdx.x;  // the blocks with the most keys start first
+    const int head = blockIdx.y, b = blockIdx.z, g = head / (a.H / a.G);
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    const int qc = lane & 15, s4 = lane >> 4;
+    const int pos0 = a.pos_dev ? *a.pos_dev : a.pos0;
+    const int hd = a.hd, row0 = qb * ROWS + wave * WR;
+    const bf16* keys = static_cast<const bf16*>(a.kc) + ((int64_t)b * a.G + g) * a.t_max * hd;
+    const bf16* q = static_cast<const bf16*>(a.qk) + (int64_t)b * a.S * a.ldq + head * hd;
+
+    bf16x8 qf[RG][KS];
+    int my_pos[RG];
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+        const int row = row0 + 16 * r + qc;
+        my_pos[r] = pos0 + row;
+        const bf16* qp = q + (int64_t)min(row, a.S - 1) * a.ldq;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            const int d = 32 * ks + 8 * s4;
+            const u32x4 v = *reinterpret_cast<const u32x4*>(qp + (d < hd ? d : 0));
+            qf[r][ks] = __builtin_bit_cast(bf16x8, d < hd ? v : u32x4{0, 0, 0, 0});
+        }
+    }
+    f32x4 o[RG][NT + 1];
+    float ref[RG];
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+        ref[r] = -INFINITY;
+#pragma unroll
+        for (int nt = 0; nt <= NT; ++nt) o[r][nt] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    bf16x8 ones;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ones[e] = static_cast<bf16>(1.0f);
+    // scores in log2 units: with a cap, cap2 - 2 cap2 / (1 + exp2(x in_scale)) and in_scale = 2 log2(e) scale / cap
+    const float log2e = 1.4426950408889634f;
+    const bool capped = a.cap > 0.f;
+    const float in_scale = capped ? 2.f * log2e * a.scale / a.cap : a.scale * log2e;
+    const float cap2 = a.cap * log2e;
+    const bool biased = a.r1 != nullptr;
+    const float r1 = biased ? a.r1[head] : 0.f, r2 = biased ? a.r2[head] : 0.f;
+
+    const int n_keys = min(pos0 + min(qb * ROWS + ROWS, a.S), a.t_max);
+    const int wave_last = pos0 + row0 + WR - 1;
+    u32x4 reg[KCH];
+    auto fetch = [&](int kt) {
+#pragma unroll
+        for (int i = 0; i < KCH; ++i) {
+            const int c = threadIdx.x + 256 * i;
+            const int key = min(kt + c / CPR, a.t_max - 1), d = (c % CPR) * 8;
+            const u32x4 v = *reinterpret_cast<const u32x4*>(keys + (int64_t)key * hd + (d < hd ? d : 0));
+            reg[i] = d < hd ? v : u32x4{0, 0, 0, 0};
+        }
+    };
+    // keys past the last row's own position may never have been written: weight 0 times whatever lies there must stay 0
+    auto park = [&](int kt, int buf) {
+#pragma unroll
+        for (int i = 0; i < KCH; ++i) {
+            const int c = threadIdx.x + 256 * i;
+            *reinterpret_cast<u32x4*>(&sk[buf][c / CPR][(c % CPR) * 8]) = kt + c / CPR < n_keys ? reg[i] : u32x4{0, 0, 0, 0};
+        }
+    };
+
+    auto tile = [&](int kt, int buf, bool masked) {
+        f32x4 sc[RG][4];
+#pragma unroll
+        for (int r = 0; r < RG; ++r)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) sc[r][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const bf16x8 kf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(&sk[buf][16 * t + qc][32 * ks + 8 * s4]));
+#pragma unroll
+                for (int r = 0; r < RG; ++r) sc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[r][ks], sc[r][t], 0, 0, 0);
+            }
+        bool moved = false;
+        float next[RG];
+#pragma unroll
+        for (int r = 0; r < RG; ++r) {
+            const float d0 = (float)(my_pos[r] - kt - 4 * s4);
+            float mx = -INFINITY;
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    float s = sc[r][t][v] * in_scale;
+                    if (capped) s = __builtin_fmaf(-2.f * cap2, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s)), cap2);
+                    // a key behind the query has a negative distance: clamped, and hidden below
+                    if (biased) s = __builtin_fmaf(-r1, __builtin_amdgcn_logf(__builtin_fmaf(r2, fmaxf(d0 - (float)(16 * t + v), 0.f), 1.f)), s);
+                    if (masked && kt + 16 * t + 4 * s4 + v > my_pos[r]) s = -INFINITY;
+                    sc[r][t][v] = s;
+                    mx = fmaxf(mx, s);
+                }
+            mx = max_over_quarters(mx);
+            const bool up = mx > ref[r] + 8.f;
+            next[r] = up ? mx : ref[r];
+            moved |= up;
+        }
+        if (__builtin_amdgcn_ballot_w64(moved) != 0) {
+#pragma unroll
+            for (int r = 0; r < RG; ++r) {
+                const float corr = next[r] == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(ref[r] - next[r]);
+#pragma unroll
+                for (int v = 0; v < 4; ++v) {
+                    const float cv = __shfl(corr, 4 * s4 + v, 64);
+#pragma unroll
+                    for (int nt = 0; nt <= NT; ++nt) o[r][nt][v] *= cv;
+                }
+                ref[r] = next[r];
+            }
+        }
+        const bf16* vtr = &sk[buf][4 * s4 + (qc >> 2)][4 * (qc & 3)];
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+            bf16x8 pf[RG];
+#pragma unroll
+            for (int r = 0; r < RG; ++r) {
+                const float m = ref[r] == -INFINITY ? 0.f : ref[r];
+#pragma unroll
+                for (int e = 0; e < 8; ++e) pf[r][e] = static_cast<bf16>(__builtin_amdgcn_exp2f(sc[r][2 * c + e / 4][e % 4] - m));
+            }
+#pragma unroll
+            for (int nt = 0; nt < NT; ++nt) {
+                const bf16* p0 = vtr + (32 * c) * KP + 16 * nt;
+                const s16x4 lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4 __attribute__((address_space(3)))*)(p0));
+                const s16x4 hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4 __attribute__((address_space(3)))*)(p0 + 16 * KP));
+                const bf16x8 vf = __builtin_bit_cast(bf16x8, __builtin_shufflevector(lo, hi, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                for (int r = 0; r < RG; ++r) o[r][nt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[r], vf, o[r][nt], 0, 0, 0);
+            }
+#pragma unroll
+            for (int r = 0; r < RG; ++r) o[r][NT] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[r], ones, o[r][NT], 0, 0, 0);
+        }
+    };
+
+    fetch(0);
+    park(0, 0);
+    if (kCpKeys < n_keys) fetch(kCpKeys);
+    __syncthreads();
+    int buf = 0;
+    for (int kt = 0; kt < n_keys; kt += kCpKeys, buf ^= 1) {
+        if (kt + kCpKeys - 1 <= pos0 + row0) tile(kt, buf, false);
+        else if (kt <= wave_last) tile(kt, buf, true);
+        if (kt + kCpKeys < n_keys) {
+            park(kt + kCpKeys, buf ^ 1);  // last read two tiles ago; every wave has passed the barrier since
+            if (kt + 2 * kCpKeys < n_keys) fetch(kt + 2 * kCpKeys);
+        }
+        __syncthreads();
+    }
+
+    // rows leave through LDS (free after the last barrier) as 16-byte pieces; each wave has its own 16 rows
+    bf16* ot = &sk[0][0][0] + wave * (16 * KP);
+    static_assert(2 * kCpKeys >= 4 * 16, "the output pass fits the staging buffers");
+    bf16* y = static_cast<bf16*>(a.y) + (int64_t)b * a.S * a.ldy + head * hd;
+#pragma unroll
+    for (int r = 0; r < RG; ++r) {
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const float inv = 1.0f / o[r][NT][v];
+#pragma unroll
+            for (int nt = 0; nt < NT; ++nt) ot[(4 * s4 + v) * KP + 16 * nt + qc] = from_f32<bf16>(o[r][nt][v] * inv);
+        }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+        for (int c = lane; c < 16 * CPR; c += 64) {
+            const int rr = c / CPR, d = (c % CPR) * 8, row = row0 + 16 * r + rr;
+            if (row < a.S && d < hd) *reinterpret_cast<u32x4*>(y + (int64_t)row * a.ldy + d) = *reinterpret_cast<const u32x4*>(ot + rr * KP + d);
+        }
+        __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+        __builtin_amdgcn_wave_barrier();
+        __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    }
+}
+
+template <int HD>
+static int launch_capped_prefill(const CappedArgs& a, int B, hipStream_t s) {
+    const int rg = (int64_t)((a.S + 127) / 128) * a.H * B >= 512 ? 2 : 1;
+    const dim3 grid((a.S + 64 * rg - 1) / (64 * rg), a.H, B);
+    if (rg == 2) capped_attention_prefill_kernel<HD, 2><<<grid, dim3(256), 0, s>>>(a);
+    else capped_attention_prefill_kernel<HD, 1><<<grid, dim3(256), 0, s>>>(a);
+    return raven_host::check_launch("capped_attention (prefill)");
+}
+
+constexpr int kCpMinRows = 16;  // fewer new rows per sequence go to the row kernel
+
+static int run_capped_prefill(const CappedArgs& a, int B, hipStream_t s) {
+    const int64_t n = (int64_t)B * a.S * a.G * (a.hd / 8);
+    key_append_kernel<bf16><<<dim3((unsigned)((n + 255) / 256)), dim3(256), 0, s>>>(a, B * a.S);
+    if (const int rc = raven_host::check_launch("capped_attention (append)")) return rc;
+    if (a.hd <= 32) return launch_capped_prefill<32>(a, B, s);
+    if (a.hd <= 64) return launch_capped_prefill<64>(a, B, s);
+    if (a.hd <= 96) return launch_capped_prefill<96>(a, B, s);
+    return launch_capped_prefill<128>(a, B, s);
+}
+
 static int capped_nq(int group) { return group >= 4 ? 4 : group >= 2 ? 2 : 1; }
 
 // position ranges per (row, key head): enough workgroups for the chip, at least 128 positions each
@@ -279,7 +500,6 @@ extern "C" int raven_capped_attention(const void* qk, void* y, const raven_key_c
     if (B == 0 || S == 0) return 0;
     RAVEN_REQUIRE(qk && y, "capped_attention: null pointer");
     RAVEN_REQUIRE(B <= cache->batch, "capped_attention: batch %d exceeds the cache's %d", B, cache->batch);
-    RAVEN_REQUIRE((int64_t)B * S <= 65535, "capped_attention: %d x %d rows in one call", B, S);
     RAVEN_REQUIRE(cache->n_kv_heads > 0 && n_heads % cache->n_kv_heads == 0, "capped_attention: %d query heads for %d key heads", n_heads,
                   cache->n_kv_heads);
     RAVEN_REQUIRE(cache->head_dim > 0 && cache->head_dim % 8 == 0 && cache->head_dim <= 256, "capped_attention: head_dim %d is not a multiple of 8 up to 256",
@@ -294,6 +514,11 @@ extern "C" int raven_capped_attention(const void* qk, void* y, const raven_key_c
     a.append = S == 1;
     const int M = B * S;
     hipStream_t s = static_cast<hipStream_t>(stream);
+    if (dtype == RAVEN_BF16 && S >= kCpMinRows && a.hd <= 128) {
+        RAVEN_REQUIRE(B <= 65535 && a.H <= 65535, "capped_attention: grid too large");
+        return run_capped_prefill(a, B, s);
+    }
+    RAVEN_REQUIRE((int64_t)B * S <= 65535, "capped_attention: %d x %d rows in one call", B, S);
     a.splits = capped_splits(M, a.H, a.G, pos0 + S);
     while (a.splits > 1 && (workspace == nullptr || (size_t)M * a.H * a.splits * (a.hd + 2) * sizeof(float) > workspace_bytes)) --a.splits;
     a.part = static_cast<float*>(workspace);

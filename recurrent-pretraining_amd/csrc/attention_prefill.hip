@@ -53,18 +53,6 @@ struct PrefillArgs {
 
 constexpr int kPfTable = 1024;  // block-table entries of a sequence held in LDS (beyond that they are read from memory)
 
-// Maximum over the four lanes l, l^16, l^32, l^48 (the lanes that share a query), in every lane, with the two row-swap
-// instructions of gfx950 instead of two round trips through the LDS crossbar: after v_permlane16_swap of a register
-// with a copy of itself the pair holds rows (0,0,2,2) and (1,1,3,3) of 16 lanes, after v_permlane32_swap the two halves.
-__device__ __forceinline__ float max_over_quarters(float x) {
-    typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
-    unsigned u = __builtin_bit_cast(unsigned, x);
-    const u32x2 r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-    u = __builtin_bit_cast(unsigned, fmaxf(__builtin_bit_cast(float, r[0]), __builtin_bit_cast(float, r[1])));
-    const u32x2 q = __builtin_amdgcn_permlane32_swap(u, u, false, false);
-    return fmaxf(__builtin_bit_cast(float, q[0]), __builtin_bit_cast(float, q[1]));
-}
-
 template <int HD, int RG, bool PAGED = false, int NW = 4>
 __global__ __launch_bounds__(NW * 64, NW == 6 ? 3 : 2) void attention_prefill_kernel(PrefillArgs a) {
     constexpr int NTH = NW * 64;     // threads; NW waves, each with its own query rows

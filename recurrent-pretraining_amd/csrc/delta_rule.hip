@@ -13,6 +13,25 @@
 //   delta_steps_kernel   one workgroup per (head, sequence) walks the tokens one by one, eight at a time: each of its eight
 //       waves prepares one token's vectors into LDS, then all columns advance through the eight tokens without a barrier, then
 //       each wave finishes one token's output row.  Decode steps and short chunks.
+//
+//   Long chunks run in blocks of 16 tokens.  With g_t the products of the block's decays up to token t (per key channel), S the
+//   state in front of the block, G = g_16, and rows
+//       U_t = u_t g_(t-1),  R_t = r_t g_t,  b_t = a_t u_t,  K_t = k_t / g_t,  B_t = b_t / g_t
+//   the removals p_t = u_t^T S_(t-1) of all 16 tokens solve one unit lower triangular system:
+//       (I + L) P = U S + M V,   L = stril(U B^T),  M = stril(U K^T)
+//       O = R S - tril(R B^T) P + tril(R K^T) V
+//       S' = G (S - B^T P + K^T V)
+//   (g stays above exp(-16 exp(-1/2)) = 6e-5, so the quotients are harmless in fp32.)  Everything but S and P is independent
+//   of the state:
+//   delta_block_kernel   one workgroup per (block, head, sequence): the four 16 x 16 products, T = (I + L)^-1 by forward
+//       substitution, T U and T M; operands of the next kernel to the workspace.
+//   delta_scan_kernel    walks the blocks: one workgroup per 16 columns of a head's state, one wave per 16 rows, the wave's
+//       16 x 16 piece of S in four registers per lane for the whole walk (the accumulator layout of the fp32 MFMA read as
+//       the B operand of the next product with the k slots permuted accordingly, so S and P never change layout).  The
+//       waves exchange their partial sums of P once per block, one barrier; partial sums of O ride along one block later.
+//       Operands are requested four blocks ahead.
+//   delta_output_kernel  the output stage.
+//   All matrix products are fp32 MFMA (16 x 16 x 4).
 
 #include <math.h>
 
@@ -153,6 +172,322 @@ __global__ __launch_bounds__(512) void delta_steps_kernel(DeltaArgs a) {
         }
 }
 
+// ---- blocks of 16 tokens ----------------------------------------------------------------------------------------
+constexpr int kBlk = 16;
+constexpr int kScanAhead = 4;        // blocks whose operands are in flight
+constexpr int kSegment = 64;         // blocks per (block, scan) launch pair: bounds the workspace and keeps it near the caches
+constexpr int kMinBlocked = 48;      // shorter chunks walk token by token
+constexpr int kMaxBlockedDim = 128;  // and so do wider heads (the scan's operands would not fit a wave's registers)
+
+// workspace of one (sequence, head, block), in floats; R = rows rounded up to 16
+__host__ __device__ constexpr int blk_floats(int R) { return 65 * R + 3 * kBlk * kBlk; }
+//   T U [16][R] | R [16][R] | -B^T G [R][16] | K^T G [R][16] | T M [16][16] | -tril(R B^T) | tril(R K^T) | G [R]
+
+struct DeltaBlockArgs {
+    DeltaArgs d;
+    float* ws;
+    float* o;         // [M, inner]
+    int first;        // first block of the segment
+    int n_blocks;     // blocks of the segment
+};
+
+// a 16 x 16 product over the channels of two row sets in LDS: acc[v] = X[4 q + v] . Y[l16]
+template <int R>
+__device__ __forceinline__ f32x4 block_product(const float (*X)[R + 4], const float (*Y)[R + 4], int l16, int q) {
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int kk = 0; kk < R / 16; ++kk) {
+        const f32x4 x = *reinterpret_cast<const f32x4*>(&X[l16][16 * kk + 4 * q]);
+        const f32x4 y = *reinterpret_cast<const f32x4*>(&Y[l16][16 * kk + 4 * q]);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[i], y[i], acc, 0, 0, 0);
+    }
+    return acc;
+}
+
+template <int R>
+__global__ __launch_bounds__(256) void delta_block_kernel(DeltaBlockArgs p) {
+    constexpr int KEEP = (R + 63) / 64;
+    __shared__ __align__(16) float U[kBlk][R + 4], Rt[kBlk][R + 4], Bt[kBlk][R + 4], Kt[kBlk][R + 4];
+    __shared__ float part[4][R];                            // each wave's sum of log decays
+    __shared__ __align__(16) float L[kBlk][kBlk], Mm[kBlk][kBlk], Ti[kBlk][kBlk + 4];
+    const DeltaArgs& a = p.d;
+    const int blk = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, q = lane >> 4;
+    const int hd = a.hd, inner = a.H * hd;
+    const int t0 = (p.first + blk) * kBlk;
+    float* ws = p.ws + (((int64_t)b * a.H + h) * kSegment + blk) * blk_floats(R);
+    float *wTU = ws, *wR = ws + 16 * R, *wB = ws + 32 * R, *wK = ws + 48 * R, *wTM = ws + 64 * R, *wRB = wTM + 256, *wRK = wRB + 256, *wG = wRK + 256;
+
+    // this wave's four tokens: channels lane, lane + 64, ...
+    float lw[4][KEEP], u[4][KEEP], bb[4][KEEP], k[4][KEEP], r[4][KEEP];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int t = t0 + 4 * wave + j;
+        const bool live = t < a.S;  // tokens past the chunk change nothing: zero rows, decay one
+        const int64_t m = (int64_t)b * a.S + (live ? t : 0);
+        const float* z = a.z + m * a.ldz + h * hd;
+        float kk = 0.f;
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+            const int c = lane + 64 * i;
+            const bool in = live && c < hd;
+            k[j][i] = in ? z[inner + c] : 0.f;
+            r[j][i] = in ? z[c] : 0.f;
+            bb[j][i] = in ? sigmoid_f32(z[4 * inner + c] + a.a_bias[h * hd + c]) : 0.f;
+            lw[j][i] = in ? -0.60653065971263342f * sigmoid_f32(a.decay[m * inner + h * hd + c]) : 0.f;
+            kk = __builtin_fmaf(k[j][i], k[j][i], kk);
+        }
+        const float inv = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+            u[j][i] = k[j][i] * inv;
+            bb[j][i] *= u[j][i];
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const int c = lane + 64 * i;
+        if (c < R) part[wave][c] = (lw[0][i] + lw[1][i]) + (lw[2][i] + lw[3][i]);
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) {
+        const int c = lane + 64 * i;
+        if (c >= R) continue;
+        float before = 0.f, total = 0.f;
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+            const float x = part[w][c];
+            if (w < wave) before += x;
+            total += x;
+        }
+        f32x4 bo, ko;
+        float log_g = before;  // of the token before
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int t = 4 * wave + j;
+            U[t][c] = u[j][i] * expf(log_g);
+            log_g += lw[j][i];
+            const float g = expf(log_g), rest = expf(total - log_g), back = expf(-log_g);
+            const float rr = r[j][i] * g;
+            Rt[t][c] = rr;
+            wR[t * R + c] = rr;
+            Bt[t][c] = bb[j][i] * back;
+            Kt[t][c] = k[j][i] * back;
+            bo[j] = -bb[j][i] * rest;
+            ko[j] = k[j][i] * rest;
+        }
+        *reinterpret_cast<f32x4*>(wB + c * 16 + 4 * wave) = bo;
+        *reinterpret_cast<f32x4*>(wK + c * 16 + 4 * wave) = ko;
+        if (wave == 3) wG[c] = expf(total);
+    }
+    __syncthreads();
+    // one of the four products per wave; rows are the later token, columns the earlier one
+    const f32x4 acc = block_product<R>(wave < 2 ? U : Rt, (wave & 1) ? Kt : Bt, l16, q);
+#pragma unroll
+    for (int v = 0; v < 4; ++v) {
+        const int t = 4 * q + v;
+        if (wave == 0) L[t][l16] = l16 < t ? acc[v] : 0.f;
+        else if (wave == 1) Mm[t][l16] = l16 < t ? acc[v] : 0.f;
+        else if (wave == 2) wRB[t * 16 + l16] = l16 <= t ? -acc[v] : 0.f;
+        else wRK[t * 16 + l16] = l16 <= t ? acc[v] : 0.f;
+    }
+    __syncthreads();
+    if (wave == 0) {  // column l16 of T, top down
+        float col[kBlk];
+#pragma unroll
+        for (int t = 0; t < kBlk; ++t) {
+            float x = t == l16 ? 1.f : 0.f;
+#pragma unroll
+            for (int i = 0; i < t; ++i) x = __builtin_fmaf(-L[t][i], col[i], x);
+            col[t] = x;
+        }
+#pragma unroll
+        for (int t = 0; t < kBlk; ++t)
+            if (q == (t & 3)) Ti[t][l16] = col[t];
+    }
+    __syncthreads();
+    const f32x4 ti = *reinterpret_cast<const f32x4*>(&Ti[l16][4 * q]);
+    for (int tile = wave; tile <= R / 16; tile += 4) {  // the column tiles of T U, then T M
+        f32x4 x = {0.f, 0.f, 0.f, 0.f};
+        const bool last = tile == R / 16;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            x = __builtin_amdgcn_mfma_f32_16x16x4f32(ti[i], last ? Mm[4 * q + i][l16] : U[4 * q + i][(last ? 0 : 16 * tile) + l16], x, 0, 0, 0);
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            if (last) wTM[(4 * q + v) * 16 + l16] = x[v];
+            else wTU[(4 * q + v) * R + 16 * tile + l16] = x[v];
+        }
+    }
+}
+
+template <int NB>  // waves = blocks of 16 rows
+__global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
+    constexpr int R = 16 * NB;
+    __shared__ __align__(16) f32x4 xp[2][NB][64], xo[2][NB][64];
+    const DeltaArgs& a = p.d;
+    const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+    const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, q = lane >> 4;
+    const int hd = a.hd, inner = a.H * hd;
+    const int col = 16 * tile + l16, row = 16 * wave + 4 * q;
+    const bool col_ok = col < hd, mine = col_ok && row < hd;  // hd is a multiple of 8: four rows exist together
+    const bool fresh = p.first == 0 && (a.pos_dev ? *a.pos_dev : a.pos0) == 0;
+    float* state = a.state + (((int64_t)b * a.H + h) * hd + min(col, hd - 1)) * hd + (row < hd ? row : 0);
+    const float* ws = p.ws + ((int64_t)b * a.H + h) * kSegment * blk_floats(R);
+    const float* vcol = a.z + (int64_t)b * a.S * a.ldz + 2 * inner + h * hd + min(col, hd - 1);
+    float* ocol = p.o + (int64_t)b * a.S * inner + h * hd + col;
+    constexpr int wGV = 0, wRKV = NB - 1, wRBP = NB / 2;  // which wave adds the 16 x 16 products
+
+    f32x4 S = {0.f, 0.f, 0.f, 0.f};
+    if (!fresh && mine) S = *reinterpret_cast<const f32x4*>(state);
+
+    struct Set {
+        f32x4 tu, r, bt, kt, g, tm, rb, rk;
+        float v[4];
+    };
+    Set st[kScanAhead];
+    auto fetch = [&](int c, Set& s) {
+        const int cc = min(c, p.n_blocks - 1);
+        const float* w = ws + (int64_t)cc * blk_floats(R);
+        s.tu = *reinterpret_cast<const f32x4*>(w + l16 * R + row);
+        s.r = *reinterpret_cast<const f32x4*>(w + 16 * R + l16 * R + row);
+        s.bt = *reinterpret_cast<const f32x4*>(w + 32 * R + (16 * wave + l16) * 16 + 4 * q);
+        s.kt = *reinterpret_cast<const f32x4*>(w + 48 * R + (16 * wave + l16) * 16 + 4 * q);
+        s.tm = *reinterpret_cast<const f32x4*>(w + 64 * R + l16 * 16 + 4 * q);
+        s.rb = *reinterpret_cast<const f32x4*>(w + 64 * R + 256 + l16 * 16 + 4 * q);
+        s.rk = *reinterpret_cast<const f32x4*>(w + 64 * R + 512 + l16 * 16 + 4 * q);
+        s.g = *reinterpret_cast<const f32x4*>(w + 64 * R + 768 + row);
+        const int t = (p.first + cc) * kBlk + 4 * q;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) s.v[i] = vcol[(int64_t)min(t + i, a.S - 1) * a.ldz];  // rows past the chunk meet zero factors
+    };
+    auto mac4 = [](const f32x4& x, const float* y, f32x4 acc) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[i], y[i], acc, 0, 0, 0);
+        return acc;
+    };
+    auto arr = [](const f32x4& x, float* y) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) y[i] = x[i];
+    };
+    // sums of the O parts that block c's barrier has published (they belong to block c - 1)
+    auto store_o = [&](int buf, int c) {
+        for (int v = wave; v < 4; v += NB) {
+            float sum = 0.f;
+#pragma unroll
+            for (int w = 0; w < NB; ++w) sum += reinterpret_cast<const float*>(&xo[buf][w][lane])[v];
+            const int t = (p.first + c) * kBlk + 4 * q + v;
+            if (col_ok && t < a.S) ocol[(int64_t)t * inner] = sum;
+        }
+    };
+#pragma unroll
+    for (int d = 0; d < kScanAhead; ++d) fetch(d, st[d]);
+    f32x4 O = {0.f, 0.f, 0.f, 0.f};
+    for (int c0 = 0; c0 < p.n_blocks; c0 += kScanAhead) {
+#pragma unroll
+        for (int d = 0; d < kScanAhead; ++d) {
+            const int c = c0 + d;
+            if (c < p.n_blocks) {  // the same for the whole workgroup
+                const Set& s = st[d];
+                const int buf = d & 1;
+                const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+                float sv[4];
+                arr(S, sv);
+                f32x4 P = wave == wGV ? mac4(s.tm, s.v, zero) : zero;
+                P = mac4(s.tu, sv, P);
+                xp[buf][wave][lane] = P;
+                xo[buf][wave][lane] = O;
+                O = wave == wRKV ? mac4(s.rk, s.v, zero) : zero;
+                O = mac4(s.r, sv, O);
+                S = mac4(s.kt, s.v, S * s.g);
+                __syncthreads();
+                P = xp[buf][0][lane];
+#pragma unroll
+                for (int w = 1; w < NB; ++w) P += xp[buf][w][lane];
+                float pv[4];
+                arr(P, pv);
+                S = mac4(s.bt, pv, S);
+                if (wave == wRBP) O = mac4(s.rb, pv, O);
+                if (c > 0) store_o(buf, c - 1);
+            }
+            fetch(c + kScanAhead, st[d]);
+        }
+    }
+    __syncthreads();
+    xo[0][wave][lane] = O;
+    __syncthreads();
+    store_o(0, p.n_blocks - 1);
+    if (mine) *reinterpret_cast<f32x4*>(state) = S;
+}
+
+// y = T(o / rms(o) * norm * sigmoid(g)); one wave per (row, head)
+template <typename T>
+__global__ __launch_bounds__(256) void delta_output_kernel(DeltaArgs a, const float* __restrict__ o, int64_t pairs) {
+    const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (i >= pairs) return;
+    const int lane = threadIdx.x & 63;
+    const int h = (int)(i % a.H);
+    const int64_t m = i / a.H;
+    const int inner = a.H * a.hd;
+    const float* row = o + m * inner + h * a.hd;
+    const float* gate = a.z + m * a.ldz + 3 * inner + h * a.hd;
+    float x[4], ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = lane + 64 * j;
+        x[j] = c < a.hd ? row[c] : 0.f;
+        ss = __builtin_fmaf(x[j], x[j], ss);
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+    T* y = static_cast<T*>(a.y) + m * inner + h * a.hd;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const int c = lane + 64 * j;
+        if (c < a.hd) y[c] = from_f32<T>(x[j] * inv * a.norm[h * a.hd + c] * sigmoid_f32(gate[c]));
+    }
+}
+
+static int scan_rows(int hd) {  // rows the block kernels are compiled for
+    return hd <= 32 ? 32 : hd <= 48 ? 48 : hd <= 64 ? 64 : hd <= 96 ? 96 : 128;
+}
+static size_t blocked_ws_floats(int B, int S, int H, int hd) {
+    return (size_t)B * H * kSegment * blk_floats(scan_rows(hd)) + (size_t)B * S * H * hd;
+}
+
+template <int R>
+static int launch_delta_segment(const DeltaBlockArgs& p, int B, hipStream_t s) {
+    delta_block_kernel<R><<<dim3(p.n_blocks, p.d.H, B), dim3(256), 0, s>>>(p);
+    if (const int rc = raven_host::check_launch("delta_rule (blocks)")) return rc;
+    delta_scan_kernel<R / 16><<<dim3((p.d.hd + 15) / 16, p.d.H, B), dim3(4 * R), 0, s>>>(p);
+    return raven_host::check_launch("delta_rule (scan)");
+}
+
+template <typename T>
+static int launch_delta_blocked(const DeltaArgs& a, int B, float* ws, hipStream_t s) {
+    DeltaBlockArgs p{};
+    p.d = a;
+    p.ws = ws;
+    p.o = ws + (size_t)B * a.H * kSegment * blk_floats(scan_rows(a.hd));
+    const int blocks = (a.S + kBlk - 1) / kBlk;
+    for (p.first = 0; p.first < blocks; p.first += kSegment) {
+        p.n_blocks = blocks - p.first < kSegment ? blocks - p.first : kSegment;
+        int rc;
+        switch (scan_rows(a.hd)) {
+            case 32: rc = launch_delta_segment<32>(p, B, s); break;
+            case 48: rc = launch_delta_segment<48>(p, B, s); break;
+            case 64: rc = launch_delta_segment<64>(p, B, s); break;
+            case 96: rc = launch_delta_segment<96>(p, B, s); break;
+            default: rc = launch_delta_segment<128>(p, B, s); break;
+        }
+        if (rc) return rc;
+    }
+    const int64_t pairs = (int64_t)B * a.S * a.H;
+    delta_output_kernel<T><<<dim3((unsigned)((pairs + 3) / 4)), dim3(256), 0, s>>>(a, p.o, pairs);
+    return raven_host::check_launch("delta_rule (output)");
+}
+
 template <typename T>
 static int launch_delta_steps(const DeltaArgs& a, int B, hipStream_t s) {
     const dim3 grid(a.H, B), block(512);
@@ -169,8 +504,8 @@ static int launch_delta_steps(const DeltaArgs& a, int B, hipStream_t s) {
 }  // namespace raven
 
 extern "C" size_t raven_delta_rule_workspace_bytes(int32_t B, int32_t S, int32_t n_heads, int32_t head_dim) {
-    (void)B; (void)S; (void)n_heads; (void)head_dim;
-    return 0;
+    if (B <= 0 || S < raven::kMinBlocked || n_heads <= 0 || head_dim <= 0 || head_dim > raven::kMaxBlockedDim) return 0;
+    return raven_host::align_up(raven::blocked_ws_floats(B, S, n_heads, head_dim) * sizeof(float));
 }
 
 extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const float* a_bias, const float* norm, float* state,
@@ -189,5 +524,11 @@ extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_
     a.z = z; a.decay = decay_logits; a.a_bias = a_bias; a.norm = norm; a.state = state; a.y = y;
     a.H = n_heads; a.dim = dim; a.hd = head_dim; a.ldz = ldz; a.S = S; a.pos0 = pos0; a.pos_dev = pos_dev; a.eps = eps;
     hipStream_t s = static_cast<hipStream_t>(stream);
+    const size_t need = raven_delta_rule_workspace_bytes(B, S, n_heads, head_dim);
+    if (need && workspace && need <= workspace_bytes) {
+        RAVEN_REQUIRE(((uintptr_t)workspace & 15) == 0 && ((uintptr_t)state & 15) == 0, "delta_rule: workspace and state must be 16-byte aligned");
+        float* ws = static_cast<float*>(workspace);
+        return dtype == RAVEN_BF16 ? launch_delta_blocked<bf16>(a, B, ws, s) : launch_delta_blocked<float>(a, B, ws, s);
+    }
     return dtype == RAVEN_BF16 ? launch_delta_steps<bf16>(a, B, s) : launch_delta_steps<float>(a, B, s);
 }

@@ -187,7 +187,7 @@ static int launch_norm_conv(const NormConvArgs& a, int B, hipStream_t s) {
     if (lds > 48 * 1024) {
         static bool attr_set = false;
         if (!attr_set) {
-            hipError_t e = hipFuncSetAttribute((const void*)norm_conv_kernel<T, P, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024);
+            hipError_t e = hipFuncSetAttribute((const void*)norm_conv_kernel<T, P, false>, hipFuncAttributeMaxDynamicSharedMemorySize, 156 * 1024);
             if (e != hipSuccess) {
                 raven_host::set_error("norm_conv: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
                 return (int)e;

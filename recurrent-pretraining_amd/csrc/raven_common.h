@@ -110,6 +110,18 @@ __device__ __forceinline__ float wave_max(float v) {
     return v;
 }
 
+// Maximum over the four lanes l, l^16, l^32, l^48 (the lanes that share a query), in every lane, with the two row-swap
+// instructions of gfx950 instead of two round trips through the LDS crossbar: after v_permlane16_swap of a register
+// with a copy of itself the pair holds rows (0,0,2,2) and (1,1,3,3) of 16 lanes, after v_permlane32_swap the two halves.
+__device__ __forceinline__ float max_over_quarters(float x) {
+    typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
+    unsigned u = __builtin_bit_cast(unsigned, x);
+    const u32x2 r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
+    u = __builtin_bit_cast(unsigned, fmaxf(__builtin_bit_cast(float, r[0]), __builtin_bit_cast(float, r[1])));
+    const u32x2 q = __builtin_amdgcn_permlane32_swap(u, u, false, false);
+    return fmaxf(__builtin_bit_cast(float, q[0]), __builtin_bit_cast(float, q[1]));
+}
+
 // x * sigmoid(x).  The reciprocal is the hardware's (1 ulp): its error vanishes in the bf16 rounding that follows and stays
 // inside the fp32 bar, and a true division costs five times the instructions in the SwiGLU epilogue of a 256 x 256 tile.
 __device__ __forceinline__ float silu_f32(float x) { return x * __builtin_amdgcn_rcpf(1.0f + __expf(-x)); }

@@ -56,13 +56,14 @@ class MixerLayer:
     def __init__(self, w: _Weights, cfg: GitipelConfig, index: int):
         spec = cfg.layers[index]
         m, p = spec["mixer"], f"l{index}."
-        D, Dp, taps = cfg.width, _pad8(cfg.width), cfg.canon["taps"]
+        D, Dp = cfg.width, _pad8(cfg.width)
+        taps = cfg.canon["taps"] if cfg.canon is not None else 0
         H, d = m["heads"], m["dim"]
         dp = _pad8(d)
         inner = H * dp
         attention = spec["type"] == "attention"
         G = m["kv_heads"] if attention else 0
-        self.plan = {"taps": taps, "ld": Dp, "heads": H, "head_dim": dp, "kv_heads": G}
+        self.plan = {"taps": max(taps, 1), "ld": Dp, "heads": H, "head_dim": dp, "kv_heads": G}
 
         def vec(name, n):
             t = w.vector(_pad8(n))
@@ -79,8 +80,9 @@ class MixerLayer:
             w.place(p + name, buf[first:first + n_heads * dp].view(n_heads, dp, buf.shape[1])[:, :d, :D], n_heads * d, D)
 
         self.norm1 = vec("norm1", D)
-        self.conv = w.vector(taps, Dp)
-        w.place(p + "canon1", self.conv.t()[:D], D, taps)
+        self.conv = w.vector(taps, Dp) if taps else None
+        if taps:
+            w.place(p + "canon1", self.conv.t()[:D], D, taps)
         self.w_out = w.matrix(Dp, inner)
         w.place(p + "mix.o", self.w_out[:D].view(D, H, dp)[:, :, :d], D, H * d)
         desc = hip.MixerLayer(heads=H, kv_heads=G, dim=d, head_dim=dp, taps=taps)
@@ -92,7 +94,7 @@ class MixerLayer:
             w.place(p + "mix.r1", self.r1, H)
             w.place(p + "mix.r2", self.r2, H)
             desc.mixer = hip.MIXER_ATTENTION
-            desc.score = hip.Score(m["scale"], m["softcap"], self.r1.data_ptr(), self.r2.data_ptr())
+            desc.score = hip.Score(m["scale"], m.get("softcap") or 0.0, self.r1.data_ptr(), self.r2.data_ptr())
         else:
             rank, rp = m["rank"], _pad8(m["rank"])
             self.w_in = w.matrix(5 * inner, Dp)
@@ -113,7 +115,8 @@ class MixerLayer:
             w.place(p + "mlp.up", self.up[:ff, :D], ff, D)
             w.place(p + "mlp.down", self.down[:D, :ff], D, ff)
             desc.norm2, desc.up, desc.down, desc.ff = self.norm2.data_ptr(), self.up.data_ptr(), self.down.data_ptr(), fp
-        desc.norm1, desc.conv, desc.w_in, desc.w_out = self.norm1.data_ptr(), self.conv.data_ptr(), self.w_in.data_ptr(), self.w_out.data_ptr()
+        desc.norm1, desc.w_in, desc.w_out = self.norm1.data_ptr(), self.w_in.data_ptr(), self.w_out.data_ptr()
+        desc.conv = self.conv.data_ptr() if taps else None
         self.native = desc
 
 
