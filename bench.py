@@ -66,6 +66,11 @@ def parse():
                     help="with --prefill: the tiled GEMMs read the weight matrices as given instead of line-aligned copies of them")
     ap.add_argument("--kernel-only", type=int, default=0, metavar="N",
                     help="run only N launches of the dominant kernel plus one 256 MiB device copy (for rocprofv3 --pmc runs)")
+    ap.add_argument("--gitipel", action="store_true",
+                    help="prompt and decode throughput of the Gitipel family beside Raven blocks of equal size (another line; --width, --part)")
+    ap.add_argument("--width", type=int, action="append", default=None, metavar="D", help="with --gitipel: model widths (default 2048 and 4096)")
+    ap.add_argument("--part", default="all", choices=["all", "gitipel-prompt", "gitipel-decode", "raven-prompt", "raven-decode"],
+                    help="with --gitipel: one family and phase only (for rocprofv3 runs)")
     return ap.parse_args()
 
 
@@ -446,6 +451,123 @@ def kernel_only(n_launches, batch=1):
                       "copy_bytes": src.numel()}))
 
 
+def gitipel_shapes(width, vocab=32768):
+    """A Gitipel and a Raven configuration of one size: 12 layer runs each (2 + 4 run twice + 2; two re-entry / adapter products), heads
+    of 64 channels, feed-forwards of 8 width^2 weights; Gitipel alternates its two mixers, attention with four query heads per
+    key head."""
+    heads = width // 64
+    attention = {"type": "attention", "mixer": {"heads": heads, "kv_heads": heads // 4, "dim": 64, "vdim": 64, "scale": 0.125, "softcap": 30.0},
+                 "mlp": {"kind": "dense", "ff": 4 * width}}
+    delta = {"type": "general_delta", "mixer": {"heads": heads, "dim": 64, "rank": 64}, "mlp": {"kind": "dense", "ff": 4 * width}}
+    gitipel = {"vocab": vocab, "width": width, "layers": [delta, attention] * 4, "canon": {"taps": 4}, "norm": {"eps": 1e-5},
+               "embedding": {"scale": 1.0}, "logit_scale": 1.0, "loop": {"start": 2, "stop": 6, "times": 2}}
+    raven = dict(n_embd=width, n_heads=heads, n_layers=8, n_layers_in_prelude=2, n_layers_in_recurrent_block=4, n_layers_in_coda=2,
+                 mean_recurrence=2, intermediate_size=(8 * width // 3 + 63) // 64 * 64, vocab_size=vocab, block_size=8192)
+    return gitipel, raven
+
+
+def gitipel_work(cfg, S, t_cached):
+    """(flops of a prompt of S tokens with all its logits, bytes a decode step reads with t_cached positions behind it)."""
+    D = cfg["width"]
+    flops = weights = state = 0.0
+    for i, t in [(i, None) for i in (0, 1)] + [(i, t) for t in (0, 1) for i in (2, 3, 4, 5)] + [(i, None) for i in (6, 7)]:
+        m = cfg["layers"][i]["mixer"]
+        inner = m["heads"] * m["dim"]
+        ff = 2 * D * cfg["layers"][i]["mlp"]["ff"]
+        if cfg["layers"][i]["type"] == "attention":
+            kv = m["kv_heads"] * m["dim"]
+            w = D * (2 * inner + kv) + ff
+            flops += 4.0 * m["heads"] * m["dim"] * S * (S + 1) / 2
+            state += 2 * kv * t_cached
+        else:
+            w = D * 6 * inner + D * m["rank"] + inner * m["rank"] + ff
+            flops += 12.0 * inner * m["dim"] * S
+            state += 2 * 4 * inner * m["dim"]
+        weights += w
+        flops += 2.0 * S * w
+    weights += 2 * 2 * D * D
+    flops += 2 * 2.0 * S * 2 * D * D + 2.0 * S * D * cfg["vocab"]
+    return flops, 2 * (weights + D * cfg["vocab"]) + state
+
+
+def raven_work(cfg, S, t_cached):
+    D, ff, runs = cfg.n_embd, 3 * cfg.n_embd * cfg.intermediate_size, 12
+    flops = runs * (2.0 * S * (4 * D * D + ff) + 4.0 * D * S * (S + 1) / 2) + 2 * 2.0 * S * 2 * D * D + 2.0 * S * D * cfg.vocab_size
+    return flops, 2 * (runs * (4 * D * D + ff) + 2 * 2 * D * D + D * cfg.vocab_size) + runs * 2 * 2 * D * t_cached
+
+
+def gitipel(args):
+    """Prompt (one sequence of 4096 tokens) and decode (one sequence, about 1024 positions cached, graph replay) of both families, timed
+    in turn in one process.  Random weights, random tokens."""
+    import statistics
+
+    import torch
+    import __graft_entry__ as entry
+    pkg = entry.import_package()
+    S, ctx, lines = 4096, 1024, {}
+    for width in args.width or [2048, 4096]:
+        gcfg, rcfg = gitipel_shapes(width)
+        models = {}
+        if args.part == "all" or args.part.startswith("gitipel"):
+            models["gitipel"] = pkg.GitipelForCausalLM(pkg.GitipelConfig(**gcfg), device="cuda:0", dtype=torch.bfloat16)
+            models["gitipel"].init_weights(seed=0)
+        if args.part == "all" or args.part.startswith("raven"):
+            models["raven"] = pkg.RavenForCausalLM(pkg.RavenConfig(**rcfg), device="cuda:0", dtype=torch.bfloat16)
+            fill_synthetic(models["raven"])
+        ids = torch.randint(0, gcfg["vocab"], (1, S), generator=torch.Generator().manual_seed(1)).cuda()
+        work = {"gitipel": gitipel_work(gcfg, S, ctx), "raven": raven_work(models["raven"].config, S, ctx) if "raven" in models else None}
+        runs, rec = {}, {}
+        for name, m in models.items():
+            cache, dcache = m.new_cache(S), m.new_cache(ctx + 256)
+            kw = {} if name == "gitipel" else {"num_steps": 2, "init_scale": 0.0}
+
+            def prompt(m=m, cache=cache, kw=kw):
+                cache.reset()
+                m.forward(input_ids=ids, past_key_values=cache, use_cache=True, **kw)
+
+            def decode(n, m=m, dcache=dcache, kw=kw, box={}):
+                if "runner" not in box:
+                    m.forward(input_ids=ids[:, :ctx - 64], past_key_values=dcache, use_cache=True, **kw)
+                    box["runner"] = m.decode_runner(dcache, 1, 2, greedy=True, use_graph=True)
+                for _ in range(n):
+                    box["runner"].step(ids[0, :1], None, 0.0)
+
+            runs[name] = (prompt, decode)
+
+        def timed(fn, *a):
+            torch.cuda.synchronize()
+            t = time.perf_counter()
+            fn(*a)
+            torch.cuda.synchronize()
+            return (time.perf_counter() - t) * 1e3
+
+        for phase in ("prompt", "decode"):
+            if args.part != "all" and not args.part.endswith(phase):
+                continue
+            k = 0 if phase == "prompt" else 1
+            got = {name: [] for name in runs}
+            for rep in range(7):
+                for name, fns in runs.items():
+                    ms = timed(fns[k]) if k == 0 else timed(fns[k], 20) / 20
+                    if rep >= 2:
+                        got[name].append(ms)
+            for name, ms in got.items():
+                t = statistics.median(ms)
+                flops, nbytes = work[name]
+                r = rec.setdefault(name, {})
+                if k == 0:
+                    r["prompt"] = {"ms": round(t, 3), "tokens_per_s": round(S / t * 1e3), "tflops": round(flops / t / 1e9, 1),
+                                   "of_mfma_peak": round(flops / t / 1e9 / MFMA_PEAK_TFLOPS, 4)}
+                else:
+                    r["decode"] = {"ms": round(t, 4), "tokens_per_s": round(1e3 / t, 1), "gb_per_s": round(nbytes / t / 1e6, 1),
+                                   "of_hbm_peak": round(nbytes / t / 1e6 / HBM_PEAK_GBS, 4)}
+        lines[str(width)] = rec
+        del models, runs
+        torch.cuda.empty_cache()
+    print(json.dumps({"metric": "Gitipel beside Raven blocks of equal size: one sequence, 4096-token prompt / decode at 1024 positions",
+                      "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "layer_runs": 12, "by_width": lines}))
+
+
 def event_time_ms(fn, reps, warm=3):
     import torch
     for _ in range(warm):
@@ -528,6 +650,9 @@ def main():
         return
     if args.paged:
         paged(args)
+        return
+    if args.gitipel:
+        gitipel(args)
         return
     if args.gpus != 1:
         print("bench.py measures one GPU: the decode path has no multi-GPU part (run with --gpus 1)", file=sys.stderr)

@@ -162,7 +162,7 @@ int    raven_linear(const void* x0, const void* x1, const void* w, const void* r
  * choice between them), then
  *     y = act(scale * z + bias) + residual
  * on the unrounded fp32 sums; y is float when out_f32 != 0, else T (one rounding).  bias [N] and residual [M, N] are float
- * and may be NULL; residual may be y itself (out_f32).  act: RAVEN_ACT_*. */
+ * and may be NULL; a residual needs out_f32 and may be y itself.  act: RAVEN_ACT_*. */
 enum { RAVEN_ACT_NONE = 0, RAVEN_ACT_GELU = 1 /* exact: z (1 + erf(z / sqrt 2)) / 2 */, RAVEN_ACT_TANH = 2 };
 typedef struct raven_epilogue {
     const float* bias;
@@ -173,6 +173,11 @@ typedef struct raven_epilogue {
 } raven_epilogue;
 int raven_linear_epilogue(const void* x0, const void* x1, const void* w, void* y, int32_t M, int32_t N, int32_t K0, int32_t K1,
                           const raven_epilogue* epi, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
+
+/* One row of it behind an RMSNorm of a float row: y = act(scale * T(x / rms(x) * norm) W^T + bias) + residual, x and norm [K] float with
+ * the mean over the first `dim` channels.  K up to 6144 - 32 bf16 or 3072 - 16 float elements. */
+int raven_gemv_stream(const float* x, const float* norm, int32_t dim, float eps, const void* w, void* y, int32_t N, int32_t K,
+                      const raven_epilogue* epi, int32_t dtype, void* stream);
 
 /* Line-aligned copies of bf16 weight matrices for products over 33 and more token rows.  No counterpart in the reference
  * (its nn.Linear weights are [out, in] with rows K elements apart, RMM:463, 493, 507-509, and stay the layout every entry point
@@ -425,29 +430,29 @@ int    raven_capped_attention(const void* qk, void* y, const raven_key_cache* ca
                               int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dtype, void* workspace,
                               size_t workspace_bytes, void* stream);
 
-/* The generalised delta rule with its output stage: per head, u = k / sqrt(|k|^2 + 1e-6), w = exp(-exp(-1/2) sigmoid(decay_logits)),
+/* The generalised delta rule with its output stage: per head, u = k / sqrt(|k|^2 + 1e-6), w = exp(-exp(-1/2) sigmoid(decay logits)),
  * a = sigmoid(z_a + a_bias),
  *     S_t = diag(w) S_(t-1) - (a u) (u^T S_(t-1)) + k v^T,   o_t = S_t^T r,   y = T(o / rms(o) * norm * sigmoid(g))
- * z [B*S, ldz] float: r | k | v | g | a, sections of n_heads * head_dim; decay_logits [B*S, n_heads * head_dim] float; a_bias, norm
- * [n_heads * head_dim] float; state [batch, n_heads, head_dim, head_dim] float (value channel, key channel), taken as zero when
+ * z [B*S, ldz] float: r | k | v | g | a [| low], sections of n_heads * head_dim (low: rank).  Decay logits: decay_logits [B*S, n_heads *
+ * head_dim] float, or, when that is NULL and S is at most 8, w_decay tanh(low) + decay_bias with w_decay [n_heads * head_dim, rank] of T,
+ * rank a multiple of 8 up to 256.  a_bias, norm, decay_bias [n_heads * head_dim] float; state [batch, n_heads, head_dim, head_dim] float (value channel, key channel), taken as zero when
  * the call starts at position 0; y [B*S, n_heads * head_dim] of T.  The mean of rms runs over `dim` channels.  workspace
  * (nullable, raven_delta_rule_workspace_bytes): long chunks run chunk-parallel with it, token by token without. */
 size_t raven_delta_rule_workspace_bytes(int32_t B, int32_t S, int32_t n_heads, int32_t head_dim);
-int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const float* a_bias, const float* norm, float* state, void* y,
-                     int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim, int32_t head_dim, float eps,
+int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const void* w_decay, const float* decay_bias, int32_t rank,
+                     const float* a_bias, const float* norm, float* state, void* y, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim, int32_t head_dim, float eps,
                      int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
 
 /* One pre-norm layer on the stream x [B*S, ld] (in place):
  *     h = norm1(x) [+ causal convolution];  x += mixer(h);  x += down(gelu(up(norm2(x))))      (up NULL: no feed-forward)
  * mixer RAVEN_MIXER_ATTENTION: w_in = q | k rows [(heads + kv_heads) * head_dim, ld].  RAVEN_MIXER_GENERAL_DELTA: w_in = r | k | v | g | a
- * [5 * heads * head_dim, ld], w_low = [rank, ld] (rank a multiple of 8), w_decay = [heads * head_dim, rank]: decay logits =
- * w_decay tanh(w_low h) + decay_bias.  w_out [ld, heads * head_dim], up [ff, ld], down [ld, ff].  Weights of T, vectors float. */
+ * | low [5 * heads * head_dim + rank, ld] (rank a multiple of 8), w_decay = [heads * head_dim, rank]: decay logits =
+ * w_decay tanh(low) + decay_bias.  w_out [ld, heads * head_dim], up [ff, ld], down [ld, ff].  Weights of T, vectors float. */
 enum { RAVEN_MIXER_ATTENTION = 0, RAVEN_MIXER_GENERAL_DELTA = 1 };
 typedef struct raven_mixer_layer {
     const float* norm1;
     const float* conv;        /* [taps, ld] or NULL */
     const void*  w_in;
-    const void*  w_low;
     const void*  w_decay;
     const float* decay_bias;  /* [heads * head_dim] */
     const float* a_bias;      /* [heads * head_dim] */

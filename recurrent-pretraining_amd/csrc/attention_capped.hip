@@ -190,21 +190,29 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
     }
 }
 
+// Lane n holds range n's reference and sum (at most 32 ranges); the columns then add eight ranges' partials per round, all
+// requested before the first is used.
 template <typename T>
 __global__ __launch_bounds__(64) void capped_combine_kernel(CappedArgs a) {
-    const int h = blockIdx.x, m = blockIdx.y;
-    const float* p = a.part + ((int64_t)m * a.H + h) * a.splits * (a.hd + 2);
-    float top = -INFINITY;
-    for (int n = 0; n < a.splits; ++n) top = fmaxf(top, p[(int64_t)n * (a.hd + 2)]);
-    for (int col = threadIdx.x; col < a.hd; col += 64) {
-        float sum = 0.f, o = 0.f;
-        for (int n = 0; n < a.splits; ++n) {
-            const float* q = p + (int64_t)n * (a.hd + 2);
-            const float w = exp_weight<T>(q[0] - top);  // some range always holds a position, so top is finite
-            sum += w * q[1];
-            o += w * q[2 + col];
+    const int h = blockIdx.x, m = blockIdx.y, lane = threadIdx.x;
+    const int ld = a.hd + 2;
+    const float* p = a.part + ((int64_t)m * a.H + h) * a.splits * ld;
+    const int mine = min(lane, a.splits - 1);
+    const float ref = p[(int64_t)mine * ld], sum = p[(int64_t)mine * ld + 1];
+    const float top = wave_max(ref);  // some range always holds a position, so it is finite
+    const float w = lane < a.splits ? exp_weight<T>(ref - top) : 0.f;
+    const float inv = 1.0f / wave_sum(w * sum);
+    for (int c0 = 0; c0 < a.hd; c0 += 64) {
+        const int col = min(c0 + lane, a.hd - 1);
+        float o = 0.f;
+        for (int n0 = 0; n0 < a.splits; n0 += 8) {
+            float x[8];
+#pragma unroll
+            for (int n = 0; n < 8; ++n) x[n] = p[(int64_t)min(n0 + n, a.splits - 1) * ld + 2 + col];
+#pragma unroll
+            for (int n = 0; n < 8; ++n) o = __builtin_fmaf(__shfl(w, n0 + n, 64), x[n], o);  // lanes past the last range hold 0
         }
-        static_cast<T*>(a.y)[(int64_t)m * a.ldy + h * a.hd + col] = from_f32<T>(o / sum);
+        if (c0 + lane < a.hd) static_cast<T*>(a.y)[(int64_t)m * a.ldy + h * a.hd + c0 + lane] = from_f32<T>(o * inv);
     }
 }
 
@@ -230,11 +238,19 @@ __global__ __launch_bounds__(256) void key_append_kernel(CappedArgs a, int M) {
 // through the transposing loads for P V.  Heads of up to HD channels (multiples of 8) sit zero-padded in the tile.
 //
 // A score costs four quarter-rate instructions (exp2 and reciprocal for the cap, log2 for the distance, exp2 for the weight)
-// where plain attention has one: the kernel is bound by vector work, not by the products.
+// where plain attention has one: the kernel is bound by vector work, not by the products.  The FIXED variant saves one of them
+// and the running maximum:
+//   * a capped score lies in [-cap, cap] and a row always sees its own position, whose bias is ln 1 = 0, so weights relative
+//     to the constant +cap never lose the row's sum below exp(-2 cap): for caps up to 35 (2^-101) nothing that matters
+//     underflows and no maximum is needed;
+//   * exp(-bias) = (1 + r2 d)^-r1 multiplies the weight and depends on the distance alone: the workgroup tabulates its tile's
+//     ROWS + 63 distances once per tile, zero for keys behind the query, which is the causal mask.  A lane's four
+//     consecutive keys are one 16-byte read; the table is stored four times, shifted by one element each, so that the
+//     read is aligned whatever the lane's query.
 // ------------------------------------------------------------------------------------------------
 constexpr int kCpKeys = 64;
 
-template <int HD, int RG>
+template <int HD, int RG, bool FIXED>
 __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(CappedArgs a) {
     constexpr int KS = HD / 32, NT = HD / 16;
     constexpr int KP = HD + 16;          // an odd multiple of 8 banks: the transposing reads of 8 key rows hit 64 banks
@@ -242,6 +258,8 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
     constexpr int CPR = HD / 8, KCH = kCpKeys * CPR / 256;
     static_assert(kCpKeys * CPR % 256 == 0, "staging shape");
     __shared__ __align__(16) bf16 sk[2][kCpKeys][KP];
+    constexpr int NE = ROWS + kCpKeys - 1;   // distances a tile holds
+    __shared__ __align__(16) float table[FIXED ? 2 : 1][FIXED ? 4 : 1][FIXED ? (NE + 7) / 4 * 4 : 1];
     typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
     typedef short s16x4 __attribute__((ext_vector_type(4)));
 
@@ -308,6 +326,22 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
         }
     };
 
+    // entry e: the key of distance d = (first row's position) - kt + ROWS - 1 - e; copy c holds entry e at place e - c
+    auto tabulate = [&](int kt, int buf) {
+        if constexpr (FIXED) {
+            const int e = threadIdx.x;
+            if (e < NE) {
+                const int d = pos0 + qb * ROWS - kt + ROWS - 1 - e;
+                float w = 1.f;
+                if (biased) w = __builtin_amdgcn_exp2f(-r1 * __builtin_amdgcn_logf(__builtin_fmaf(r2, (float)d, 1.f)));
+                if (d < 0) w = 0.f;
+#pragma unroll
+                for (int c = 0; c < 4; ++c)
+                    if (e >= c) table[buf][c][e - c] = w;
+            }
+        }
+    };
+
     auto tile = [&](int kt, int buf, bool masked) {
         f32x4 sc[RG][4];
 #pragma unroll
@@ -322,10 +356,24 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
 #pragma unroll
                 for (int r = 0; r < RG; ++r) sc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[r][ks], sc[r][t], 0, 0, 0);
             }
+        if constexpr (FIXED) {
+#pragma unroll
+            for (int r = 0; r < RG; ++r) {
+                const int e0 = ROWS - 1 - (wave * WR + 16 * r + qc) + 4 * s4, shift = (3 - qc) & 3;  // e0 = shift mod 4
+                const float* fac = &table[buf][shift][e0 - shift];
+#pragma unroll
+                for (int t = 0; t < 4; ++t) {
+                    const f32x4 w = *reinterpret_cast<const f32x4*>(fac + 16 * t);
+#pragma unroll
+                    for (int v = 0; v < 4; ++v)
+                        sc[r][t][v] = w[v] * __builtin_amdgcn_exp2f(-2.f * cap2 * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(sc[r][t][v] * in_scale)));
+                }
+            }
+        }
         bool moved = false;
         float next[RG];
 #pragma unroll
-        for (int r = 0; r < RG; ++r) {
+        for (int r = 0; r < RG && !FIXED; ++r) {
             const float d0 = (float)(my_pos[r] - kt - 4 * s4);
             float mx = -INFINITY;
 #pragma unroll
@@ -345,7 +393,7 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
             next[r] = up ? mx : ref[r];
             moved |= up;
         }
-        if (__builtin_amdgcn_ballot_w64(moved) != 0) {
+        if (!FIXED && __builtin_amdgcn_ballot_w64(moved) != 0) {
 #pragma unroll
             for (int r = 0; r < RG; ++r) {
                 const float corr = next[r] == -INFINITY ? 1.f : __builtin_amdgcn_exp2f(ref[r] - next[r]);
@@ -366,7 +414,10 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
             for (int r = 0; r < RG; ++r) {
                 const float m = ref[r] == -INFINITY ? 0.f : ref[r];
 #pragma unroll
-                for (int e = 0; e < 8; ++e) pf[r][e] = static_cast<bf16>(__builtin_amdgcn_exp2f(sc[r][2 * c + e / 4][e % 4] - m));
+                for (int e = 0; e < 8; ++e) {
+                    const float x = sc[r][2 * c + e / 4][e % 4];
+                    pf[r][e] = static_cast<bf16>(FIXED ? x : __builtin_amdgcn_exp2f(x - m));
+                }
             }
 #pragma unroll
             for (int nt = 0; nt < NT; ++nt) {
@@ -384,6 +435,7 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
 
     fetch(0);
     park(0, 0);
+    tabulate(0, 0);
     if (kCpKeys < n_keys) fetch(kCpKeys);
     __syncthreads();
     int buf = 0;
@@ -391,6 +443,7 @@ __global__ __launch_bounds__(256, 2) void capped_attention_prefill_kernel(Capped
         if (kt + kCpKeys - 1 <= pos0 + row0) tile(kt, buf, false);
         else if (kt <= wave_last) tile(kt, buf, true);
         if (kt + kCpKeys < n_keys) {
+            tabulate(kt + kCpKeys, buf ^ 1);
             park(kt + kCpKeys, buf ^ 1);  // last read two tiles ago; every wave has passed the barrier since
             if (kt + 2 * kCpKeys < n_keys) fetch(kt + 2 * kCpKeys);
         }
@@ -426,8 +479,14 @@ template <int HD>
 static int launch_capped_prefill(const CappedArgs& a, int B, hipStream_t s) {
     const int rg = (int64_t)((a.S + 127) / 128) * a.H * B >= 512 ? 2 : 1;
     const dim3 grid((a.S + 64 * rg - 1) / (64 * rg), a.H, B);
-    if (rg == 2) capped_attention_prefill_kernel<HD, 2><<<grid, dim3(256), 0, s>>>(a);
-    else capped_attention_prefill_kernel<HD, 1><<<grid, dim3(256), 0, s>>>(a);
+    const bool fixed = a.cap > 0.f && a.cap <= 35.f;
+    if (rg == 2) {
+        if (fixed) capped_attention_prefill_kernel<HD, 2, true><<<grid, dim3(256), 0, s>>>(a);
+        else capped_attention_prefill_kernel<HD, 2, false><<<grid, dim3(256), 0, s>>>(a);
+    } else {
+        if (fixed) capped_attention_prefill_kernel<HD, 1, true><<<grid, dim3(256), 0, s>>>(a);
+        else capped_attention_prefill_kernel<HD, 1, false><<<grid, dim3(256), 0, s>>>(a);
+    }
     return raven_host::check_launch("capped_attention (prefill)");
 }
 

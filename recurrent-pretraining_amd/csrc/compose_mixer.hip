@@ -13,6 +13,10 @@ struct MixerScratch {
     size_t attn_ws_bytes, delta_ws_bytes, lin_ws_bytes;
 };
 
+bool gemv1_stream_fits(int K, int dtype);
+int gemv1_stream(const float* x, const float* norm, int dim, float eps, const void* w, void* y, int N, int K, const raven_epilogue& epi, int dtype,
+                 hipStream_t s);
+
 static size_t carve_mixer(const raven_stream_dims* d, const raven_mixer_layer* l, int B, int S, char* base, MixerScratch* out) {
     const size_t es = raven_host::elt_size(d->dtype);
     const size_t M = (size_t)B * S;
@@ -26,7 +30,7 @@ static size_t carve_mixer(const raven_stream_dims* d, const raven_mixer_layer* l
     };
     MixerScratch s{};
     s.h = take(M * d->ld * es);
-    s.z = take(delta ? M * 5 * inner * sizeof(float) : M * (l->heads + l->kv_heads) * l->head_dim * es);
+    s.z = take(delta ? M * (5 * inner + l->rank) * sizeof(float) : M * (l->heads + l->kv_heads) * l->head_dim * es);
     s.low = take(delta ? M * l->rank * es : 0);
     s.decay = reinterpret_cast<float*>(take(delta ? M * inner * sizeof(float) : 0));
     s.y = take(M * inner * es);
@@ -35,7 +39,7 @@ static size_t carve_mixer(const raven_stream_dims* d, const raven_mixer_layer* l
     s.attn_ws = take(s.attn_ws_bytes);
     s.delta_ws_bytes = delta ? raven_delta_rule_workspace_bytes(B, S, l->heads, l->head_dim) : 0;
     s.delta_ws = take(s.delta_ws_bytes);
-    size_t widest = delta ? 5 * inner : (size_t)(l->heads + l->kv_heads) * l->head_dim;
+    size_t widest = delta ? 5 * inner + l->rank : (size_t)(l->heads + l->kv_heads) * l->head_dim;
     if ((size_t)d->ld > widest) widest = d->ld;
     if (l->up && (size_t)l->ff > widest) widest = l->ff;
     s.lin_ws_bytes = M > 1 ? raven_linear_workspace_bytes((int)M, (int)widest) : 0;
@@ -53,7 +57,7 @@ static int check_mixer_layer(const char* who, const raven_stream_dims* d, const 
                   l->dim, l->head_dim);
     RAVEN_REQUIRE(l->norm1 && l->w_in && l->w_out, "%s: null weight", who);
     if (l->mixer == RAVEN_MIXER_GENERAL_DELTA)
-        RAVEN_REQUIRE(l->w_low && l->w_decay && l->decay_bias && l->a_bias && l->out_norm && l->rank > 0 && l->rank % 8 == 0,
+        RAVEN_REQUIRE(l->w_decay && l->decay_bias && l->a_bias && l->out_norm && l->rank > 0 && l->rank % 8 == 0,
                       "%s: the delta rule needs its decay and output weights (rank %d)", who, l->rank);
     RAVEN_REQUIRE((l->up == nullptr) == (l->down == nullptr) && (l->up == nullptr || (l->norm2 && l->ff > 0 && l->ff % 8 == 0)),
                   "%s: a feed-forward needs norm2, up, down and ff a multiple of 8 (ff %d)", who, l->ff);
@@ -92,14 +96,27 @@ extern "C" int raven_mixer_layer_forward(const raven_stream_dims* dims, const ra
         if (int rc = product(w.h, l.w_in, w.z, (l.heads + l.kv_heads) * l.head_dim, ld, RAVEN_ACT_NONE, nullptr, nullptr, 0)) return rc;
         if (int rc = raven_capped_attention(w.z, w.y, &state->keys, &l.score, B, S, pos0, pos_dev, l.heads, dt, w.attn_ws, w.attn_ws_bytes, stream)) return rc;
     } else {
-        if (int rc = product(w.h, l.w_in, w.z, 5 * inner, ld, RAVEN_ACT_NONE, nullptr, nullptr, 1)) return rc;
-        if (int rc = product(w.h, l.w_low, w.low, l.rank, ld, RAVEN_ACT_TANH, nullptr, nullptr, 0)) return rc;
-        if (int rc = product(w.low, l.w_decay, w.decay, inner, l.rank, RAVEN_ACT_NONE, l.decay_bias, nullptr, 1)) return rc;
-        if (int rc = raven_delta_rule(reinterpret_cast<float*>(w.z), 5 * inner, w.decay, l.a_bias, l.out_norm, state->state, w.y, B, S, pos0, pos_dev,
-                                      l.heads, l.dim, l.head_dim, dims->eps, dt, w.delta_ws, w.delta_ws_bytes, stream)) return rc;
+        // a few tokens: the low-rank rows ride in the fused projection and the recurrence's kernel forms the decay logits;
+        // more: two small products of their own
+        const bool few = S <= 8 && l.rank <= 256;
+        const int ldz = 5 * inner + (few ? l.rank : 0);
+        if (int rc = product(w.h, l.w_in, w.z, ldz, ld, RAVEN_ACT_NONE, nullptr, nullptr, 1)) return rc;
+        if (!few) {
+            const char* w_low = static_cast<const char*>(l.w_in) + (size_t)5 * inner * ld * raven_host::elt_size(dt);
+            if (int rc = product(w.h, w_low, w.low, l.rank, ld, RAVEN_ACT_TANH, nullptr, nullptr, 0)) return rc;
+            if (int rc = product(w.low, l.w_decay, w.decay, inner, l.rank, RAVEN_ACT_NONE, l.decay_bias, nullptr, 1)) return rc;
+        }
+        if (int rc = raven_delta_rule(reinterpret_cast<float*>(w.z), ldz, few ? nullptr : w.decay, l.w_decay, l.decay_bias, l.rank, l.a_bias,
+                                      l.out_norm, state->state, w.y, B, S, pos0, pos_dev, l.heads, l.dim, l.head_dim, dims->eps, dt, w.delta_ws,
+                                      w.delta_ws_bytes, stream)) return rc;
     }
     if (int rc = product(w.y, l.w_out, x, ld, inner, RAVEN_ACT_NONE, nullptr, x, 1)) return rc;
-    if (l.up) {
+    if (l.up && M == 1 && gemv1_stream_fits(ld, dt)) {  // the norm rides in the product's prologue
+        raven_epilogue e{};
+        e.scale = 1.f; e.act = RAVEN_ACT_GELU;
+        if (int rc = gemv1_stream(x, l.norm2, dims->width, dims->eps, l.up, w.ff, l.ff, ld, e, dt, static_cast<hipStream_t>(stream))) return rc;
+        if (int rc = product(w.ff, l.down, x, ld, l.ff, RAVEN_ACT_NONE, nullptr, x, 1)) return rc;
+    } else if (l.up) {
         if (int rc = raven_norm_conv(x, l.norm2, nullptr, nullptr, w.h, B, S, dims->width, ld, 1, dims->eps, pos0, pos_dev, dt, stream)) return rc;
         if (int rc = product(w.h, l.up, w.ff, l.ff, ld, RAVEN_ACT_GELU, nullptr, nullptr, 0)) return rc;
         if (int rc = product(w.ff, l.down, x, ld, l.ff, RAVEN_ACT_NONE, nullptr, x, 1)) return rc;

@@ -41,7 +41,10 @@ namespace raven {
 
 struct DeltaArgs {
     const float* z;       // [M, ldz]: r | k | v | g | a
-    const float* decay;   // [M, inner] logits
+    const float* decay;   // [M, inner] logits, or null: w_decay tanh(low) + decay_bias, low = z's columns 5 * inner .. + rank - 1
+    const void* w_decay;  // [inner, rank] of T
+    const float* decay_bias;  // [inner]
+    int rank;
     const float* a_bias;  // [inner]
     const float* norm;    // [inner]
     float* state;         // [batch, H, hd columns, hd rows]
@@ -52,6 +55,7 @@ struct DeltaArgs {
 };
 
 constexpr int kDeltaTile = 8;  // tokens prepared together = waves of the workgroup
+constexpr int kMaxRank = 256;  // of the decay projection, where the kernel forms it
 
 __device__ __forceinline__ float delta_decay(float logit) { return expf(-0.60653065971263342f * sigmoid_f32(logit)); }
 
@@ -62,6 +66,7 @@ __global__ __launch_bounds__(512) void delta_steps_kernel(DeltaArgs a) {
     constexpr int KEEP = (R + 63) / 64;
     __shared__ __align__(16) float sw[kDeltaTile][R], su[kDeltaTile][R], sb[kDeltaTile][R], sk[kDeltaTile][R], sr[kDeltaTile][R];
     __shared__ __align__(16) float sv[kDeltaTile][32 * CP], so[kDeltaTile][32 * CP];
+    __shared__ __align__(16) float slow[kDeltaTile][kMaxRank];
     const int h = blockIdx.x, b = blockIdx.y;
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const int l16 = lane & 15, col0 = wave * 4 + (lane >> 4);
@@ -84,28 +89,51 @@ __global__ __launch_bounds__(512) void delta_steps_kernel(DeltaArgs a) {
         float g[KEEP];
         if (mine < a.S) {
             const float* z = a.z + m * a.ldz + h * hd;
-            float k[KEEP], kk = 0.f;
+            float k[KEEP], r[KEEP], v[KEEP], al[KEEP], dl[KEEP], kk = 0.f;
+#pragma unroll
+            for (int i = 0; i < KEEP; ++i) {  // every load unconditional, so that all are in flight together
+                const int c = min(lane + 64 * i, hd - 1);
+                k[i] = z[inner + c];
+                r[i] = z[c];
+                v[i] = z[2 * inner + c];
+                g[i] = z[3 * inner + c];
+                al[i] = z[4 * inner + c] + a.a_bias[h * hd + c];
+                dl[i] = a.decay ? a.decay[m * inner + h * hd + c] : a.decay_bias[h * hd + c];
+            }
+            if (!a.decay) {
+                for (int c = lane; c < a.rank; c += 64) slow[wave][c] = tanhf(a.z[m * a.ldz + 5 * inner + c]);
+                __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+                __builtin_amdgcn_wave_barrier();
+                __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+                constexpr int E = Chunk<T>::N;
+#pragma unroll
+                for (int i = 0; i < KEEP; ++i) {
+                    const T* w = static_cast<const T*>(a.w_decay) + (int64_t)(h * hd + min(lane + 64 * i, hd - 1)) * a.rank;
+                    for (int c = 0; c < a.rank; c += E) {
+                        const Chunk<T> x = load_chunk(w + c);
+#pragma unroll
+                        for (int e = 0; e < E; ++e) dl[i] = __builtin_fmaf(to_f32(x.v[e]), slow[wave][c + e], dl[i]);
+                    }
+                }
+            }
 #pragma unroll
             for (int i = 0; i < KEEP; ++i) {
-                const int r = lane + 64 * i;
-                const bool in = r < hd;
-                k[i] = in ? z[inner + r] : 0.f;
+                if (lane + 64 * i >= hd) k[i] = 0.f;
                 kk = __builtin_fmaf(k[i], k[i], kk);
-                g[i] = in ? z[3 * inner + r] : 0.f;
             }
             const float inv = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
 #pragma unroll
             for (int i = 0; i < KEEP; ++i) {
-                const int r = lane + 64 * i;
-                if (r >= R) continue;
-                const bool in = r < hd;
+                const int c = lane + 64 * i;
+                if (c >= R) continue;
+                const bool in = c < hd;
                 const float u = k[i] * inv;
-                sk[wave][r] = k[i];
-                su[wave][r] = u;
-                sb[wave][r] = in ? sigmoid_f32(z[4 * inner + r] + a.a_bias[h * hd + r]) * u : 0.f;
-                sw[wave][r] = in ? delta_decay(a.decay[m * inner + h * hd + r]) : 0.f;
-                sr[wave][r] = in ? z[r] : 0.f;
-                if (in) sv[wave][r] = z[2 * inner + r];
+                sk[wave][c] = k[i];
+                su[wave][c] = u;
+                sb[wave][c] = in ? sigmoid_f32(al[i]) * u : 0.f;
+                sw[wave][c] = in ? delta_decay(dl[i]) : 0.f;
+                sr[wave][c] = in ? r[i] : 0.f;
+                if (in) sv[wave][c] = v[i];
             }
         }
         __syncthreads();
@@ -186,9 +214,10 @@ __host__ __device__ constexpr int blk_floats(int R) { return 65 * R + 3 * kBlk *
 struct DeltaBlockArgs {
     DeltaArgs d;
     float* ws;
-    float* o;         // [M, inner]
+    float* o;         // [B, H, o_rows, R]: token t of the chunk in row 16 + t, columns past the head unused
+    int64_t o_rows;
     int first;        // first block of the segment
-    int n_blocks;     // blocks of the segment
+    int n_blocks;     // blocks of the segment, a multiple of kScanAhead (those past the chunk are empty)
 };
 
 // a 16 x 16 product over the channels of two row sets in LDS: acc[v] = X[4 q + v] . Y[l16]
@@ -219,23 +248,36 @@ __global__ __launch_bounds__(256) void delta_block_kernel(DeltaBlockArgs p) {
     float* ws = p.ws + (((int64_t)b * a.H + h) * kSegment + blk) * blk_floats(R);
     float *wTU = ws, *wR = ws + 16 * R, *wB = ws + 32 * R, *wK = ws + 48 * R, *wTM = ws + 64 * R, *wRB = wTM + 256, *wRK = wRB + 256, *wG = wRK + 256;
 
-    // this wave's four tokens: channels lane, lane + 64, ...
-    float lw[4][KEEP], u[4][KEEP], bb[4][KEEP], k[4][KEEP], r[4][KEEP];
+    // this wave's four tokens, channels lane, lane + 64, ...; every load is unconditional (a clamped address, the value dropped)
+    // so that all of them are in flight together
+    float lw[4][KEEP], u[4][KEEP], bb[4][KEEP], k[4][KEEP], r[4][KEEP], ab[KEEP];
+#pragma unroll
+    for (int i = 0; i < KEEP; ++i) ab[i] = a.a_bias[h * hd + min(lane + 64 * i, hd - 1)];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
-        const int t = t0 + 4 * wave + j;
-        const bool live = t < a.S;  // tokens past the chunk change nothing: zero rows, decay one
-        const int64_t m = (int64_t)b * a.S + (live ? t : 0);
+        const int64_t m = (int64_t)b * a.S + min(t0 + 4 * wave + j, a.S - 1);
         const float* z = a.z + m * a.ldz + h * hd;
+        const float* dl = a.decay + m * inner + h * hd;
+#pragma unroll
+        for (int i = 0; i < KEEP; ++i) {
+            const int c = min(lane + 64 * i, hd - 1);
+            k[j][i] = z[inner + c];
+            r[j][i] = z[c];
+            bb[j][i] = z[4 * inner + c];
+            lw[j][i] = dl[c];
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const bool live = t0 + 4 * wave + j < a.S;  // tokens past the chunk change nothing: zero rows, decay one
         float kk = 0.f;
 #pragma unroll
         for (int i = 0; i < KEEP; ++i) {
-            const int c = lane + 64 * i;
-            const bool in = live && c < hd;
-            k[j][i] = in ? z[inner + c] : 0.f;
-            r[j][i] = in ? z[c] : 0.f;
-            bb[j][i] = in ? sigmoid_f32(z[4 * inner + c] + a.a_bias[h * hd + c]) : 0.f;
-            lw[j][i] = in ? -0.60653065971263342f * sigmoid_f32(a.decay[m * inner + h * hd + c]) : 0.f;
+            const bool in = live && lane + 64 * i < hd;
+            k[j][i] = in ? k[j][i] : 0.f;
+            r[j][i] = in ? r[j][i] : 0.f;
+            bb[j][i] = in ? sigmoid_f32(bb[j][i] + ab[i]) : 0.f;
+            lw[j][i] = in ? -0.60653065971263342f * sigmoid_f32(lw[j][i]) : 0.f;
             kk = __builtin_fmaf(k[j][i], k[j][i], kk);
         }
         const float inv = 1.0f / sqrtf(wave_sum(kk) + 1e-6f);
@@ -337,7 +379,7 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     float* state = a.state + (((int64_t)b * a.H + h) * hd + min(col, hd - 1)) * hd + (row < hd ? row : 0);
     const float* ws = p.ws + ((int64_t)b * a.H + h) * kSegment * blk_floats(R);
     const float* vcol = a.z + (int64_t)b * a.S * a.ldz + 2 * inner + h * hd + min(col, hd - 1);
-    float* ocol = p.o + (int64_t)b * a.S * inner + h * hd + col;
+    float* orow = p.o + (((int64_t)b * a.H + h) * p.o_rows) * R + 16 * tile + l16;
     constexpr int wGV = 0, wRKV = NB - 1, wRBP = NB / 2;  // which wave adds the 16 x 16 products
 
     f32x4 S = {0.f, 0.f, 0.f, 0.f};
@@ -372,14 +414,17 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) y[i] = x[i];
     };
-    // sums of the O parts that block c's barrier has published (they belong to block c - 1)
-    auto store_o = [&](int buf, int c) {
-        for (int v = wave; v < 4; v += NB) {
+    // Sums of the O parts that block c's barrier has published: block c - 1's, one of the four rows of a lane per wave (with more
+    // than four waves some store the same value twice), to rows 16 c' .. of the walk-through numbering that has an empty block
+    // in front.  No condition anywhere: the stores and loads of an iteration can then be counted exactly.
+    auto store_o = [&](int buf, float* dst) {
+#pragma unroll
+        for (int n = 0; n < (4 + NB - 1) / NB; ++n) {
+            const int v = (wave + NB * n) & 3;
             float sum = 0.f;
 #pragma unroll
             for (int w = 0; w < NB; ++w) sum += reinterpret_cast<const float*>(&xo[buf][w][lane])[v];
-            const int t = (p.first + c) * kBlk + 4 * q + v;
-            if (col_ok && t < a.S) ocol[(int64_t)t * inner] = sum;
+            dst[(4 * q + v) * R] = sum;
         }
     };
 #pragma unroll
@@ -389,7 +434,7 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
 #pragma unroll
         for (int d = 0; d < kScanAhead; ++d) {
             const int c = c0 + d;
-            if (c < p.n_blocks) {  // the same for the whole workgroup
+            {
                 const Set& s = st[d];
                 const int buf = d & 1;
                 const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
@@ -410,7 +455,8 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
                 arr(P, pv);
                 S = mac4(s.bt, pv, S);
                 if (wave == wRBP) O = mac4(s.rb, pv, O);
-                if (c > 0) store_o(buf, c - 1);
+                // the first block of a segment has nothing to publish: it writes to the empty block in front
+                store_o(buf, orow + (int64_t)(c > 0 ? p.first + c : 0) * kBlk * R);
             }
             fetch(c + kScanAhead, st[d]);
         }
@@ -418,42 +464,60 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     __syncthreads();
     xo[0][wave][lane] = O;
     __syncthreads();
-    store_o(0, p.n_blocks - 1);
+    store_o(0, orow + (int64_t)(p.first + p.n_blocks) * kBlk * R);
     if (mine) *reinterpret_cast<f32x4*>(state) = S;
 }
 
-// y = T(o / rms(o) * norm * sigmoid(g)); one wave per (row, head)
-template <typename T>
-__global__ __launch_bounds__(256) void delta_output_kernel(DeltaArgs a, const float* __restrict__ o, int64_t pairs) {
-    const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (i >= pairs) return;
-    const int lane = threadIdx.x & 63;
-    const int h = (int)(i % a.H);
-    const int64_t m = i / a.H;
+// y = T(o / rms(o) * norm * sigmoid(g)); 16 lanes per (row, head), four channels per lane and round
+template <typename T, int J>
+__global__ __launch_bounds__(256) void delta_output_kernel(DeltaBlockArgs p, int R, int64_t pairs) {
+    const DeltaArgs& a = p.d;
+    const int64_t i = (int64_t)blockIdx.x * 16 + (threadIdx.x >> 4);
+    const int l16 = threadIdx.x & 15;
+    const bool ok = i < pairs;
+    const int64_t pair = ok ? i : pairs - 1;
+    const int h = (int)(pair % a.H);
+    const int64_t m = pair / a.H;
+    const int b = (int)(m / a.S), t = (int)(m % a.S);
     const int inner = a.H * a.hd;
-    const float* row = o + m * inner + h * a.hd;
+    const float* row = p.o + (((int64_t)b * a.H + h) * p.o_rows + kBlk + t) * R;
     const float* gate = a.z + m * a.ldz + 3 * inner + h * a.hd;
-    float x[4], ss = 0.f;
+    f32x4 x[J], g[J], w[J];
+    float ss = 0.f;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int c = lane + 64 * j;
-        x[j] = c < a.hd ? row[c] : 0.f;
-        ss = __builtin_fmaf(x[j], x[j], ss);
+    for (int j = 0; j < J; ++j) {
+        const int c = 4 * l16 + 64 * j, cc = min(c, a.hd - 4);
+        x[j] = *reinterpret_cast<const f32x4*>(row + cc);
+        g[j] = *reinterpret_cast<const f32x4*>(gate + cc);
+        w[j] = *reinterpret_cast<const f32x4*>(a.norm + h * a.hd + cc);
     }
-    const float inv = 1.0f / sqrtf(wave_sum(ss) / (float)a.dim + a.eps);
+#pragma unroll
+    for (int j = 0; j < J; ++j)
+        if (4 * l16 + 64 * j < a.hd) ss += x[j][0] * x[j][0] + x[j][1] * x[j][1] + x[j][2] * x[j][2] + x[j][3] * x[j][3];
+    const float inv = 1.0f / sqrtf(row16_sum(ss) / (float)a.dim + a.eps);
     T* y = static_cast<T*>(a.y) + m * inner + h * a.hd;
 #pragma unroll
-    for (int j = 0; j < 4; ++j) {
-        const int c = lane + 64 * j;
-        if (c < a.hd) y[c] = from_f32<T>(x[j] * inv * a.norm[h * a.hd + c] * sigmoid_f32(gate[c]));
+    for (int j = 0; j < J; ++j) {
+        const int c = 4 * l16 + 64 * j;
+        if (!ok || c >= a.hd) continue;
+        T o[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) o[e] = from_f32<T>(x[j][e] * inv * w[j][e] * sigmoid_f32(g[j][e]));
+        if constexpr (sizeof(T) == 4) *reinterpret_cast<f32x4*>(y + c) = *reinterpret_cast<const f32x4*>(o);
+        else *reinterpret_cast<uint2*>(y + c) = *reinterpret_cast<const uint2*>(o);
     }
 }
 
 static int scan_rows(int hd) {  // rows the block kernels are compiled for
     return hd <= 32 ? 32 : hd <= 48 ? 48 : hd <= 64 ? 64 : hd <= 96 ? 96 : 128;
 }
+static int64_t blocked_o_rows(int S) {  // an empty block in front, the chunk in whole rounds of blocks behind it
+    const int round = kBlk * kScanAhead;
+    return kBlk + (int64_t)(S + round - 1) / round * round;
+}
 static size_t blocked_ws_floats(int B, int S, int H, int hd) {
-    return (size_t)B * H * kSegment * blk_floats(scan_rows(hd)) + (size_t)B * S * H * hd;
+    const int R = scan_rows(hd);
+    return (size_t)B * H * kSegment * blk_floats(R) + (size_t)B * H * blocked_o_rows(S) * R;
 }
 
 template <int R>
@@ -470,7 +534,8 @@ static int launch_delta_blocked(const DeltaArgs& a, int B, float* ws, hipStream_
     p.d = a;
     p.ws = ws;
     p.o = ws + (size_t)B * a.H * kSegment * blk_floats(scan_rows(a.hd));
-    const int blocks = (a.S + kBlk - 1) / kBlk;
+    p.o_rows = blocked_o_rows(a.S);
+    const int blocks = (int)((p.o_rows - kBlk) / kBlk);
     for (p.first = 0; p.first < blocks; p.first += kSegment) {
         p.n_blocks = blocks - p.first < kSegment ? blocks - p.first : kSegment;
         int rc;
@@ -484,7 +549,9 @@ static int launch_delta_blocked(const DeltaArgs& a, int B, float* ws, hipStream_
         if (rc) return rc;
     }
     const int64_t pairs = (int64_t)B * a.S * a.H;
-    delta_output_kernel<T><<<dim3((unsigned)((pairs + 3) / 4)), dim3(256), 0, s>>>(a, p.o, pairs);
+    const dim3 grid((unsigned)((pairs + 15) / 16));
+    if (a.hd <= 64) delta_output_kernel<T, 1><<<grid, dim3(256), 0, s>>>(p, scan_rows(a.hd), pairs);
+    else delta_output_kernel<T, 2><<<grid, dim3(256), 0, s>>>(p, scan_rows(a.hd), pairs);
     return raven_host::check_launch("delta_rule (output)");
 }
 
@@ -508,8 +575,8 @@ extern "C" size_t raven_delta_rule_workspace_bytes(int32_t B, int32_t S, int32_t
     return raven_host::align_up(raven::blocked_ws_floats(B, S, n_heads, head_dim) * sizeof(float));
 }
 
-extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const float* a_bias, const float* norm, float* state,
-                                void* y, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim,
+extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, const void* w_decay, const float* decay_bias,
+                                int32_t rank, const float* a_bias, const float* norm, float* state, void* y, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim,
                                 int32_t head_dim, float eps, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream) {
     using namespace raven;
     RAVEN_REQUIRE(dtype == RAVEN_F32 || dtype == RAVEN_BF16, "delta_rule: unknown dtype %d", dtype);
@@ -519,9 +586,12 @@ extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_
                   dim, head_dim);
     RAVEN_REQUIRE(ldz >= 5 * n_heads * head_dim, "delta_rule: rows of %d elements hold less than five sections", ldz);
     if (B == 0 || S == 0) return 0;
-    RAVEN_REQUIRE(z && decay_logits && a_bias && norm && state && y, "delta_rule: null pointer");
+    RAVEN_REQUIRE(z && a_bias && norm && state && y, "delta_rule: null pointer");
+    RAVEN_REQUIRE(decay_logits || (w_decay && decay_bias && rank > 0 && rank % 8 == 0 && rank <= kMaxRank && S <= kDeltaTile && ldz >= 5 * n_heads * head_dim + rank),
+                  "delta_rule: without decay logits it needs the low-rank product's operands (rank %d, ldz %d) and at most %d tokens, not %d", rank, ldz,
+                  kDeltaTile, S);
     DeltaArgs a{};
-    a.z = z; a.decay = decay_logits; a.a_bias = a_bias; a.norm = norm; a.state = state; a.y = y;
+    a.z = z; a.decay = decay_logits; a.w_decay = w_decay; a.decay_bias = decay_bias; a.rank = rank; a.a_bias = a_bias; a.norm = norm; a.state = state; a.y = y;
     a.H = n_heads; a.dim = dim; a.hd = head_dim; a.ldz = ldz; a.S = S; a.pos0 = pos0; a.pos_dev = pos_dev; a.eps = eps;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const size_t need = raven_delta_rule_workspace_bytes(B, S, n_heads, head_dim);

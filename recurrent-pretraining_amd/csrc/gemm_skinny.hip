@@ -84,8 +84,8 @@ __device__ __forceinline__ Chunk<T> load_weight(const T* p) {
 
 template <typename T, int EPI = EPI_PLAIN>
 __device__ __forceinline__ void store_out(const GemmArgs& a, int m, int n, float acc) {
-    if (EPI == EPI_FREE) {
-        store_free<T>(a.epi, a.y, (int64_t)m * a.N + n, n, acc);
+    if (is_free(EPI)) {
+        store_free<T, EPI>(a.epi, a.y, (int64_t)m * a.N + n, n, acc);
         return;
     }
     float r = round_to<T>(acc);
@@ -552,7 +552,7 @@ static int run_gemm(GemmArgs a, int dtype, hipStream_t s) {
             const char* x1 = a.x1 ? static_cast<const char*>(a.x1) + (size_t)m0 * a.k1 * es : nullptr;
             const char* res = a.residual ? static_cast<const char*>(a.residual) + (size_t)m0 * a.N * es : nullptr;
             char* y = static_cast<char*>(a.y) + (size_t)m0 * a.N * out_es;
-            if (EPI == EPI_FREE) {
+            if (is_free(EPI)) {
                 raven_epilogue e = a.epi;
                 if (e.residual) e.residual += (size_t)m0 * a.N;
                 return gemv1_free(x0, x1, a.w, y, a.N, a.k0, a.k1, e, dtype, s);
@@ -592,7 +592,11 @@ int gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int
     GemmArgs a{};
     a.w = w; a.x0 = x0; a.x1 = x1; a.y = y;
     a.M = M; a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.out_f32 = epi.out_f32; a.epi = epi;
-    return run_gemm<EPI_FREE>(a, dtype, s);
+    switch (EPI_FREE + epi.act) {
+        case EPI_FREE_GELU: return run_gemm<EPI_FREE_GELU>(a, dtype, s);
+        case EPI_FREE_TANH: return run_gemm<EPI_FREE_TANH>(a, dtype, s);
+        default: return run_gemm<EPI_FREE>(a, dtype, s);
+    }
 }
 
 static int check_common(const char* who, int M, int N, int K, int dtype) {

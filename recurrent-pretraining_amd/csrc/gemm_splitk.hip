@@ -58,8 +58,8 @@ struct NsArgs {
 template <int EPI>
 __device__ __forceinline__ void ns_epilogue(const NsArgs& a, int m, int n, float v0, float v1) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
-    if (EPI == EPI_FREE) {
-        store_free<bf16>(a.epi, a.y, (int64_t)m * a.N + n, n, v0);
+    if (is_free(EPI)) {
+        store_free<bf16, EPI>(a.epi, a.y, (int64_t)m * a.N + n, n, v0);
         return;
     }
     if (SWIGLU) {
@@ -447,6 +447,7 @@ extern "C" int raven_linear_epilogue(const void* x0, const void* x1, const void*
     RAVEN_REQUIRE((K1 == 0) == (x1 == nullptr), "linear_epilogue: x1 and K1 must be given together");
     RAVEN_REQUIRE(epi->act >= RAVEN_ACT_NONE && epi->act <= RAVEN_ACT_TANH, "linear_epilogue: unknown activation %d", epi->act);
     RAVEN_REQUIRE(((uintptr_t)epi->residual & 15) == 0 && ((uintptr_t)epi->bias & 15) == 0, "linear_epilogue: residual and bias must be 16-byte aligned");
+    RAVEN_REQUIRE(!epi->residual || epi->out_f32, "linear_epilogue: a residual needs a float output");
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (M >= g_tiled_min_rows && tiled_gemm_fits(M, N, K0, K1, dtype)) return tiled_gemm_free(x0, x1, w, y, M, N, K0, K1, *epi, s);
     // the same choice between the kernels with and without a K split as raven_linear
@@ -464,7 +465,10 @@ extern "C" int raven_linear_epilogue(const void* x0, const void* x1, const void*
         a.y = static_cast<char*>(y) + (size_t)m0 * N * out_es;
         a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.epi = *epi;
         if (epi->residual) a.epi.residual = epi->residual + (size_t)m0 * N;
-        if (const int rc = launch_ns<EPI_FREE>(a, workspace, workspace_bytes, s)) return rc;
+        const int rc = epi->act == RAVEN_ACT_GELU   ? launch_ns<EPI_FREE_GELU>(a, workspace, workspace_bytes, s)
+                       : epi->act == RAVEN_ACT_TANH ? launch_ns<EPI_FREE_TANH>(a, workspace, workspace_bytes, s)
+                                                    : launch_ns<EPI_FREE>(a, workspace, workspace_bytes, s);
+        if (rc) return rc;
     }
     return 0;
 }

@@ -118,14 +118,14 @@ __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&ac
                     o[i] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
                 }
                 *reinterpret_cast<u32x2*>(static_cast<bf16*>(a.y) + (int64_t)m * a.ldy + n) = *reinterpret_cast<const u32x2*>(o);
-            } else if (EPI == EPI_FREE) {  // float outputs; N is a multiple of 8, so the four columns exist together
+            } else if (is_free(EPI)) {  // float outputs; N is a multiple of 8, so the four columns exist together
                 const int64_t at = (int64_t)m * a.ldy + n;
                 f32x4 v = acc[t][tb] * a.epi.scale;
                 if (a.epi.bias) v += *reinterpret_cast<const f32x4*>(a.epi.bias + n);
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    if (a.epi.act == RAVEN_ACT_GELU) v[i] = 0.5f * v[i] * (1.0f + erff(v[i] * 0.70710678118654752f));
-                    else if (a.epi.act == RAVEN_ACT_TANH) v[i] = tanhf(v[i]);
+                    if (EPI == EPI_FREE_GELU) v[i] = gelu_f32<bf16>(v[i]);
+                    if (EPI == EPI_FREE_TANH) v[i] = tanhf(v[i]);
                 }
                 if (a.epi.residual) v += *reinterpret_cast<const f32x4*>(a.epi.residual + at);
                 *reinterpret_cast<f32x4*>(static_cast<float*>(a.y) + at) = v;
@@ -155,13 +155,20 @@ __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&ac
 // The accumulators of a workgroup laid down in LDS as the output tile (rows of BN_OUT columns, 16-byte unit u of row r at
 // position u ^ (r mod units per row)), between two workgroup barriers: the first because the K loop's stages are reused.
 template <int EPI, int TM, int TN, int WM, int WN>
-__device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_m, int tile_n, int wave, int lane,
-                                              unsigned lds_base) {
+__device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_n, int wave, int lane, unsigned lds_base) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr int NA = 2 * TN, NB = 2 * TM, NT = SWIGLU ? TN : NA;
     constexpr int RB = BN_OUT * 2, U = RB / 16;
     const int wn = wave % WN, wm = wave / WN, l16 = lane & 15, q4 = lane >> 4;
+    f32x4 bias[is_free(EPI) ? NT : 1];  // free epilogue with bf16 outputs (no residual): the four columns of each tile
+    if constexpr (is_free(EPI)) {
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            const int n = min(tile_n * BN_OUT + (wn * NT + t) * 16 + 4 * q4, a.N - 4);
+            bias[t] = a.epi.bias ? *reinterpret_cast<const f32x4*>(a.epi.bias + n) : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    }
     // every wave has its last fragments; the stages are free
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
     __builtin_amdgcn_s_barrier();
@@ -179,9 +186,11 @@ __device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&
                 if (SWIGLU) {
                     const float g = round_to<bf16>(acc[2 * t][tb][i]), u = round_to<bf16>(acc[2 * t + 1][tb][i]);
                     o[i] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
-                } else if (EPI == EPI_FREE) {  // bf16 outputs of the free epilogue; bias columns past N are not read
-                    const int m = tile_m * (WM * TM * 32) + row, n = tile_n * BN_OUT + (wn * NT + t) * 16 + 4 * q4 + i;
-                    o[i] = from_f32<bf16>(m < a.M && n < a.N ? free_epilogue(a.epi, (int64_t)m * a.ldy + n, n, acc[t][tb][i]) : 0.f);
+                } else if (is_free(EPI)) {
+                    float v = __builtin_fmaf(acc[t][tb][i], a.epi.scale, bias[t][i]);
+                    if (EPI == EPI_FREE_GELU) v = gelu_f32<bf16>(v);
+                    if (EPI == EPI_FREE_TANH) v = tanhf(v);
+                    o[i] = from_f32<bf16>(v);
                 } else {
                     o[i] = from_f32<bf16>(acc[t][tb][i]);
                 }
@@ -221,7 +230,7 @@ __device__ __forceinline__ void store_tiles_lds(const TiledArgs& a, const f32x4 
         res[it] = u32x4{0, 0, 0, 0};
         if (EPI == EPI_PLAIN && a.residual && goff[it] >= 0) res[it] = *reinterpret_cast<const u32x4*>(a.residual + goff[it]);
     }
-    lay_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    lay_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_n, wave, lane, lds_base);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int idx = (wave * ITERS + it) * 64 + lane;
@@ -298,7 +307,7 @@ __device__ __forceinline__ void store_tiles_rope(const TiledArgs& a, const f32x4
     };
 #pragma unroll
     for (int it = 0; it < PD; ++it) request(fq[it]);
-    lay_tiles_lds<EPI_PLAIN, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    lay_tiles_lds<EPI_PLAIN, TM, TN, WM, WN>(a, acc, tile_n, wave, lane, lds_base);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int row = row0 + it * RS;
@@ -898,6 +907,8 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
     auto launch = [&](const TiledArgs& t, bool as_big) {
         // 256 x 256 tiles: four waves, operands straight into an LDS ring (5 to 8 % faster than eight waves with staging
         // registers at the model's shapes, same bits); the eight-wave kernel stays selectable and serves the small tiles
+        if (epi && epi->act == RAVEN_ACT_GELU) return as_big ? launch_ring<EPI_FREE_GELU>(t, s) : launch_tiled<EPI_FREE_GELU, 2, 1>(t, s);
+        if (epi && epi->act == RAVEN_ACT_TANH) return as_big ? launch_ring<EPI_FREE_TANH>(t, s) : launch_tiled<EPI_FREE_TANH, 2, 1>(t, s);
         if (epi) return as_big ? launch_ring<EPI_FREE>(t, s) : launch_tiled<EPI_FREE, 2, 1>(t, s);
         if (as_big && g_tiled_variant != 3) return swiglu ? launch_ring<EPI_SWIGLU>(t, s) : launch_ring<EPI_PLAIN>(t, s);
         if (swiglu) return as_big ? launch_tiled<EPI_SWIGLU, 4, 2>(t, s) : launch_tiled<EPI_SWIGLU, 2, 1>(t, s);

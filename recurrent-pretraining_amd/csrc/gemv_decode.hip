@@ -37,6 +37,7 @@ struct Gemv1Args {
     const float* acc_in;   // [N] or null: fp32 sums of the remaining columns, added before the result is rounded
     int raw_out;           // y receives the unrounded fp32 sums (the other half of acc_in)
     raven_epilogue epi;    // EPI_FREE only
+    int dim;               // PRO_STREAM: channels the mean runs over
 };
 
 template <bool NT, typename T>
@@ -60,9 +61,13 @@ __device__ __forceinline__ float wg_sum(float v, float* red) {
 constexpr int kMaxPairsPerWg = 16;
 
 // MULTI: the workgroup walks several row pairs and double-buffers their weights in registers
-template <typename T, int C, int EPI, bool NORM, bool MULTI>
+// PRO: prologue on x0 -- none, up to two RMSNorms in T (norm_a, norm_b), or one over a float row (a residual stream kept in fp32)
+// with a float weight norm_a, its mean over `dim` channels, rounded to T behind the weight
+enum { PRO_NONE = 0, PRO_NORM = 1, PRO_STREAM = 2 };
+
+template <typename T, int C, int EPI, int PRO, bool MULTI>
 __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
-    constexpr bool SWIGLU = EPI == EPI_SWIGLU;
+    constexpr bool SWIGLU = EPI == EPI_SWIGLU, NORM = PRO == PRO_NORM, STREAM = PRO == PRO_STREAM;
     constexpr int E = Chunk<T>::N;
     __shared__ float red[4];
     __shared__ float part[kMaxPairsPerWg][4][2];
@@ -99,8 +104,18 @@ __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
     // x first (older loads return first), then the first pair's weights
     Chunk<T> xc[C], na[NORM ? C : 1], nb[NORM ? C : 1];
     bool in0[C];
+    f32x4 xs[STREAM ? C : 1][E / 4], ns[STREAM ? C : 1][E / 4];
 #pragma unroll
-    for (int j = 0; j < C; ++j) {
+    for (int j = 0; j < C && STREAM; ++j) {
+        const int c = min(cb + lane + 64 * j, n_chunks - 1);
+#pragma unroll
+        for (int e = 0; e < E / 4; ++e) {
+            xs[j][e] = *reinterpret_cast<const f32x4*>(static_cast<const float*>(a.x0) + c * E + 4 * e);
+            ns[j][e] = *reinterpret_cast<const f32x4*>(static_cast<const float*>(a.norm_a) + c * E + 4 * e);
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < C && !STREAM; ++j) {
         const int c = cb + lane + 64 * j;
         in0[j] = c < ce && c < c0;
         xc[j] = zero_chunk<T>();
@@ -137,6 +152,25 @@ __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
                 for (int e = 0; e < E; ++e) xc[j].v[e] = from_f32<T>(round_to<T>(to_f32(xc[j].v[e]) * inv) * to_f32(na[NORM ? j : 0].v[e]));
                 if (a.xa_out && blockIdx.x == 0) store_chunk(static_cast<T*>(a.xa_out) + (cb + lane + 64 * j) * E, xc[j]);
             }
+    }
+    if constexpr (STREAM) {
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < C; ++j)
+#pragma unroll
+            for (int e = 0; e < E / 4; ++e) {
+                const f32x4 v = xs[j][e];
+                if (cb + lane + 64 * j < ce) ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+            }
+        const float inv = 1.0f / sqrtf(wg_sum(ss, red) / (float)a.dim + a.eps);
+#pragma unroll
+        for (int j = 0; j < C; ++j) {
+            xc[j] = zero_chunk<T>();
+            if (cb + lane + 64 * j < ce) {
+#pragma unroll
+                for (int e = 0; e < E; ++e) xc[j].v[e] = from_f32<T>(xs[j][e / 4][e % 4] * inv * ns[j][e / 4][e % 4]);
+            }
+        }
     }
     if (NORM && a.norm_b) {
         float ss = 0.f;
@@ -201,10 +235,10 @@ __global__ __launch_bounds__(256) void gemv1_kernel(Gemv1Args a) {
                 return;
             }
         }
-        if (EPI == EPI_FREE) {
+        if (is_free(EPI)) {
             const int r0 = 2 * unit;
-            store_free<T>(a.epi, a.y, r0, r0, s0);
-            if (r0 + 1 < a.N) store_free<T>(a.epi, a.y, r0 + 1, r0 + 1, s1);
+            store_free<T, EPI>(a.epi, a.y, r0, r0, s0);
+            if (r0 + 1 < a.N) store_free<T, EPI>(a.epi, a.y, r0 + 1, r0 + 1, s1);
             return;
         }
         if (SWIGLU) {
@@ -268,12 +302,18 @@ static int launch_gemv1(Gemv1Args a, hipStream_t s) {
     const int wgs = (units + ppw - 1) / ppw;
 #define RAVEN_GEMV1(CC)                                                                            \
     do {                                                                                           \
-        if (norm) gemv1_kernel<T, CC, EPI, true, false><<<dim3(wgs), dim3(256), 0, s>>>(a);     \
-        else gemv1_kernel<T, CC, EPI, false, false><<<dim3(wgs), dim3(256), 0, s>>>(a);         \
+        if (norm) gemv1_kernel<T, CC, EPI, PRO_NORM, false><<<dim3(wgs), dim3(256), 0, s>>>(a);     \
+        else gemv1_kernel<T, CC, EPI, PRO_NONE, false><<<dim3(wgs), dim3(256), 0, s>>>(a);         \
     } while (0)
-    if (c <= 3 && ppw > 1) {
-        if (norm) gemv1_kernel<T, 3, EPI, true, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
-        else gemv1_kernel<T, 3, EPI, false, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
+    if (a.dim > 0) {  // PRO_STREAM
+        RAVEN_REQUIRE(c <= 3, "gemv: K=%d is too long for the float-row norm prologue", a.K);
+        if constexpr (is_free(EPI)) {
+            if (ppw > 1) gemv1_kernel<T, 3, EPI, PRO_STREAM, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
+            else gemv1_kernel<T, 3, EPI, PRO_STREAM, false><<<dim3(wgs), dim3(256), 0, s>>>(a);
+        }
+    } else if (c <= 3 && ppw > 1) {
+        if (norm) gemv1_kernel<T, 3, EPI, PRO_NORM, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
+        else gemv1_kernel<T, 3, EPI, PRO_NONE, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
     } else if (c <= 3) RAVEN_GEMV1(3);
     else if (c <= 6) RAVEN_GEMV1(6);
     else if (c <= 9) RAVEN_GEMV1(9);
@@ -305,12 +345,32 @@ int gemv1_column_block(const void* x, const void* norm_a, const void* w_block, i
     return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_PLAIN>(a, s) : launch_gemv1<float, EPI_PLAIN>(a, s);
 }
 
+static int gemv1_free_dispatch(const Gemv1Args& a, int dtype, hipStream_t s) {
+    switch (EPI_FREE + a.epi.act) {
+        case EPI_FREE_GELU: return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_FREE_GELU>(a, s) : launch_gemv1<float, EPI_FREE_GELU>(a, s);
+        case EPI_FREE_TANH: return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_FREE_TANH>(a, s) : launch_gemv1<float, EPI_FREE_TANH>(a, s);
+        default: return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_FREE>(a, s) : launch_gemv1<float, EPI_FREE>(a, s);
+    }
+}
+
 // One row with the free epilogue; longest K as launch_gemv1
 int gemv1_free(const void* x0, const void* x1, const void* w, void* y, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
                hipStream_t s) {
     Gemv1Args a{};
     a.w = w; a.x0 = x0; a.x1 = x1; a.y = y; a.N = N; a.K = K0 + K1; a.k0 = K0; a.ldw = a.K; a.epi = epi;
-    return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_FREE>(a, s) : launch_gemv1<float, EPI_FREE>(a, s);
+    return gemv1_free_dispatch(a, dtype, s);
+}
+
+// The same behind an RMSNorm of a float row x [K] (weight float, mean over dim channels): true when K is short enough
+bool gemv1_stream_fits(int K, int dtype) {
+    const int n_chunks = K / (16 / (int)raven_host::elt_size(dtype));
+    return ((n_chunks + 3) / 4 + 1 + 63) / 64 <= 3;
+}
+int gemv1_stream(const float* x, const float* norm, int dim, float eps, const void* w, void* y, int N, int K, const raven_epilogue& epi, int dtype,
+                 hipStream_t s) {
+    Gemv1Args a{};
+    a.w = w; a.x0 = x; a.norm_a = norm; a.y = y; a.N = N; a.K = K; a.k0 = K; a.ldw = K; a.epi = epi; a.dim = dim; a.eps = eps;
+    return gemv1_free_dispatch(a, dtype, s);
 }
 
 }  // namespace raven
@@ -334,4 +394,15 @@ extern "C" int raven_gemv_fused(const void* x0, const void* x1, const void* norm
     hipStream_t s = static_cast<hipStream_t>(stream);
     if (dtype == RAVEN_BF16) return swiglu ? launch_gemv1<bf16, EPI_SWIGLU>(a, s) : launch_gemv1<bf16, EPI_PLAIN>(a, s);
     return swiglu ? launch_gemv1<float, EPI_SWIGLU>(a, s) : launch_gemv1<float, EPI_PLAIN>(a, s);
+}
+
+extern "C" int raven_gemv_stream(const float* x, const float* norm, int32_t dim, float eps, const void* w, void* y, int32_t N, int32_t K,
+                                 const raven_epilogue* epi, int32_t dtype, void* stream) {
+    using namespace raven;
+    RAVEN_REQUIRE(dtype == RAVEN_F32 || dtype == RAVEN_BF16, "gemv_stream: unknown dtype %d", dtype);
+    RAVEN_REQUIRE(x && norm && w && y && epi, "gemv_stream: null pointer");
+    RAVEN_REQUIRE(N > 0 && K > 0 && K % 8 == 0 && dim > 0 && dim <= K, "gemv_stream: bad shape N=%d K=%d dim=%d", N, K, dim);
+    RAVEN_REQUIRE(epi->act >= RAVEN_ACT_NONE && epi->act <= RAVEN_ACT_TANH && (!epi->residual || epi->out_f32), "gemv_stream: bad epilogue");
+    RAVEN_REQUIRE(gemv1_stream_fits(K, dtype), "gemv_stream: K=%d is too long", K);
+    return gemv1_stream(x, norm, dim, eps, w, y, N, K, *epi, dtype, static_cast<hipStream_t>(stream));
 }

@@ -129,22 +129,44 @@ __device__ __forceinline__ float silu_f32(float x) { return x * __builtin_amdgcn
 __device__ __forceinline__ float sigmoid_f32(float x) { return 1.0f / (1.0f + expf(-x)); }
 
 // ---- the free epilogue of the linear kernels (raven_linear_epilogue) --------------------------------------------
-// which epilogue a linear kernel is compiled with: the nn.Linear one (rounded to T, then a residual in T), SwiGLU, or the
-// free one below, whose sums stay unrounded until they are stored
-enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_FREE = 2 };
+// Which epilogue a linear kernel is compiled with: the nn.Linear one (rounded to T, then a residual in T), SwiGLU, or the
+// free one, whose sums stay unrounded until they are stored -- one value per activation, so that a tile's hundreds of
+// unrolled elements carry no code for the other activations (with all of them behind run-time branches the 256 x 256 kernel
+// outgrew the instruction cache and lost a third of its speed even without an activation).
+enum { EPI_PLAIN = 0, EPI_SWIGLU = 1, EPI_FREE = 2, EPI_FREE_GELU = EPI_FREE + RAVEN_ACT_GELU, EPI_FREE_TANH = EPI_FREE + RAVEN_ACT_TANH };
+constexpr bool is_free(int epi) { return epi >= EPI_FREE; }
+
+// z (1 + erf(z / sqrt 2)) / 2.  float: the library's erf.  bf16 results: erf by the rational approximation 7.1.26 of Abramowitz and
+// Stegun, Handbook of Mathematical Functions (absolute error 1.5e-7), in the form 1 - erf(x) = poly(t) exp(-x^2), t = 1 / (1 + p x).
+template <typename T>
+__device__ __forceinline__ float gelu_f32(float z) {
+    if constexpr (sizeof(T) == 4) {
+        return 0.5f * z * (1.0f + erff(z * 0.70710678118654752f));
+    } else {
+        const float x = fabsf(z) * 0.70710678118654752f;
+        const float t = __builtin_amdgcn_rcpf(__builtin_fmaf(0.3275911f, x, 1.0f));
+        float p = __builtin_fmaf(1.061405429f, t, -1.453152027f);
+        p = __builtin_fmaf(p, t, 1.421413741f);
+        p = __builtin_fmaf(p, t, -0.284496736f);
+        p = __builtin_fmaf(p, t, 0.254829592f);
+        const float tail = p * t * __builtin_amdgcn_exp2f(x * x * -1.4426950408889634f);  // erfc(x)
+        return 0.5f * z * (z < 0.f ? tail : 2.0f - tail);
+    }
+}
 
 // act(scale * z + bias[n]) + residual[at], z an fp32 sum and `at` its element offset in the output
+template <typename T, int EPI>
 __device__ __forceinline__ float free_epilogue(const raven_epilogue& e, int64_t at, int n, float z) {
     float v = z * e.scale;
     if (e.bias) v += e.bias[n];
-    if (e.act == RAVEN_ACT_GELU) v = 0.5f * v * (1.0f + erff(v * 0.70710678118654752f));
-    else if (e.act == RAVEN_ACT_TANH) v = tanhf(v);
+    if (EPI == EPI_FREE_GELU) v = gelu_f32<T>(v);
+    if (EPI == EPI_FREE_TANH) v = tanhf(v);
     if (e.residual) v += e.residual[at];
     return v;
 }
-template <typename T>
+template <typename T, int EPI>
 __device__ __forceinline__ void store_free(const raven_epilogue& e, void* y, int64_t at, int n, float z) {
-    const float v = free_epilogue(e, at, n, z);
+    const float v = free_epilogue<T, EPI>(e, at, n, z);
     if (e.out_f32) static_cast<float*>(y)[at] = v;
     else static_cast<T*>(y)[at] = from_f32<T>(v);
 }

@@ -97,16 +97,15 @@ class MixerLayer:
             desc.score = hip.Score(m["scale"], m.get("softcap") or 0.0, self.r1.data_ptr(), self.r2.data_ptr())
         else:
             rank, rp = m["rank"], _pad8(m["rank"])
-            self.w_in = w.matrix(5 * inner, Dp)
+            self.w_in = w.matrix(5 * inner + rp, Dp)
             for i, name in enumerate(("r", "k", "v", "g", "a")):
                 head_rows("mix." + name, self.w_in, i * inner, H)
-            self.w_low = w.matrix(rp, Dp)
-            w.place(p + "mix.w1", self.w_low[:rank, :D], rank, D)
+            w.place(p + "mix.w1", self.w_in[5 * inner:5 * inner + rank, :D], rank, D)
             self.w_decay = w.matrix(inner, rp)
             w.place(p + "mix.w2", self.w_decay.view(H, dp, rp)[:, :d, :rank], H * d, rank)
             self.decay_bias, self.a_bias, self.out_norm = head_vec("mix.w0"), head_vec("mix.a.b"), head_vec("mix.norm")
             desc.mixer, desc.rank = hip.MIXER_GENERAL_DELTA, rp
-            desc.w_low, desc.w_decay = self.w_low.data_ptr(), self.w_decay.data_ptr()
+            desc.w_decay = self.w_decay.data_ptr()
             desc.decay_bias, desc.a_bias, desc.out_norm = self.decay_bias.data_ptr(), self.a_bias.data_ptr(), self.out_norm.data_ptr()
         if spec.get("mlp") is not None:
             ff, fp = spec["mlp"]["ff"], _pad8(spec["mlp"]["ff"])
@@ -261,6 +260,8 @@ class GitipelForCausalLM(MinimalGeneration, PreTrainedModel, GenerationMixin):
 
     def _logits(self, x: torch.Tensor, h: torch.Tensor, out: torch.Tensor, ws) -> torch.Tensor:
         cfg = self.config
+        if x.shape[0] == 1 and hip.gemv_stream_fits(self.dims.ld, self.dtype):
+            return hip.gemv_stream(x, self.final_norm, cfg.width, cfg.norm["eps"], self.head, self.dtype, scale=cfg.logit_scale, out=out)
         hip.norm_conv(x, self.final_norm, cfg.width, cfg.norm["eps"], x.shape[0], 1, self.dtype, out=h)
         return hip.linear_epilogue(h, self.head, scale=cfg.logit_scale, out=out, workspace=ws)
 

@@ -59,7 +59,7 @@ class Score(C.Structure):
 
 
 class MixerLayer(C.Structure):
-    _fields_ = [(n, C.c_void_p) for n in ("norm1", "conv", "w_in", "w_low", "w_decay", "decay_bias", "a_bias", "out_norm", "w_out", "norm2",
+    _fields_ = [(n, C.c_void_p) for n in ("norm1", "conv", "w_in", "w_decay", "decay_bias", "a_bias", "out_norm", "w_out", "norm2",
                                           "up", "down")] + [("score", Score)] + [
         (n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "head_dim", "rank", "taps", "ff")]
 
@@ -142,13 +142,14 @@ SIGNATURES = {
     "raven_paged_decode_blocks": (C.c_int, [C.POINTER(Dims), _VP, C.POINTER(BlockWeights), _I32, _VP, _VP, _VP, _VP, _VP,
                                             C.POINTER(PagedKV), _I32, _I32, _VP, _SZ, _VP]),
     "raven_linear_epilogue": (C.c_int, [_VP, _VP, _VP, _VP, _I32, _I32, _I32, _I32, C.POINTER(Epilogue), _I32, _VP, _SZ, _VP]),
+    "raven_gemv_stream": (C.c_int, [_VP, _VP, _I32, _F, _VP, _VP, _I32, _I32, C.POINTER(Epilogue), _I32, _VP]),
     "raven_norm_conv": (C.c_int, [_VP, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _I32, _I32, _F, _I32, _VP, _I32, _VP]),
     "raven_embed_stream": (C.c_int, [_VP, _VP, _VP, _VP, _I32, _I32, _I64, _F, _I32, _VP]),
     "raven_round_rows": (C.c_int, [_VP, _VP, _I64, _I32, _VP]),
     "raven_capped_attention_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
     "raven_capped_attention": (C.c_int, [_VP, _VP, C.POINTER(KeyCache), C.POINTER(Score), _I32, _I32, _I32, _VP, _I32, _I32, _VP, _SZ, _VP]),
     "raven_delta_rule_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
-    "raven_delta_rule": (C.c_int, [_VP, _I32, _VP, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _VP, _I32, _I32, _I32, _F, _I32, _VP, _SZ, _VP]),
+    "raven_delta_rule": (C.c_int, [_VP, _I32, _VP, _VP, _VP, _I32, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _VP, _I32, _I32, _I32, _F, _I32, _VP, _SZ, _VP]),
     "raven_mixer_layer_workspace_bytes": (_SZ, [C.POINTER(StreamDims), C.POINTER(MixerLayer), _I32, _I32]),
     "raven_mixer_layer_forward": (C.c_int, [C.POINTER(StreamDims), C.POINTER(MixerLayer), C.POINTER(MixerState), _VP, _I32, _I32, _I32, _VP,
                                             _VP, _SZ, _VP]),
@@ -648,6 +649,24 @@ def linear_epilogue(x0, w, x1=None, bias=None, residual=None, scale=1.0, act=ACT
     return y
 
 
+def gemv_stream(x, norm, dim, eps, w, dtype, bias=None, residual=None, scale=1.0, act=ACT_NONE, out_f32=True, out=None):
+    """One row of linear_epilogue behind an RMSNorm of the float row x [K]."""
+    N, K = w.shape
+    if x.numel() != K or norm.shape != (K,) or (bias is not None and bias.shape != (N,)) or (residual is not None and residual.numel() != N):
+        raise RavenHipError("gemv_stream: operand shapes do not fit together")
+    y = out if out is not None else torch.empty(N, device=x.device, dtype=torch.float32 if out_f32 else dtype)
+    e = Epilogue(_ptr(bias, "bias", torch.float32), _ptr(residual, "residual", torch.float32), float(scale), int(act), int(out_f32))
+    rc = load().raven_gemv_stream(_ptr(x, "x", torch.float32), _ptr(norm, "norm", torch.float32), int(dim), float(eps), _ptr(w, "w", dtype),
+                                  _ptr(y, "y"), N, K, C.byref(e), dtype_code(dtype), _stream())
+    _check(rc, "raven_gemv_stream")
+    return y
+
+
+def gemv_stream_fits(K: int, dtype: torch.dtype) -> bool:
+    chunks = K * torch.empty((), dtype=dtype).element_size() // 16
+    return ((chunks + 3) // 4 + 1 + 63) // 64 <= 3
+
+
 def norm_conv(x, weight, dim, eps, B, S, dtype, conv=None, ring=None, pos0=0, pos_dev=None, out=None):
     """x [B*S, ld] float -> T [B*S, ld]; conv [taps, ld] and ring [B, taps, ld] float, or None."""
     ld = x.shape[1]
@@ -701,18 +720,22 @@ def capped_attention(qk, keys: torch.Tensor, score: Score, B, S, pos0, n_heads, 
     return y
 
 
-def delta_rule(z, decay_logits, a_bias, norm, state, B, S, pos0, dim, eps, dtype, pos_dev=None, parallel=True):
-    """z [B*S, >= 5 * H * hd] float; state [B, H, hd, hd] float, updated in place.  Returns [B*S, H * hd] of dtype.  parallel=False
-    walks the tokens one by one whatever the chunk's length."""
+def delta_rule(z, decay_logits, a_bias, norm, state, B, S, pos0, dim, eps, dtype, pos_dev=None, parallel=True, w_decay=None, decay_bias=None):
+    """z [B*S, >= 5 * H * hd] float; state [B, H, hd, hd] float, updated in place.  Returns [B*S, H * hd] of dtype.  decay_logits None: formed
+    from z's sixth section with w_decay [H * hd, rank] and decay_bias.  parallel=False walks the tokens one by one whatever the
+    chunk's length."""
     _, H, hd, _ = state.shape
-    if z.shape[0] != B * S or decay_logits.shape != (B * S, H * hd) or a_bias.shape != (H * hd,) or norm.shape != (H * hd,) or state.shape[0] < B:
+    n, rank = H * hd, 0 if w_decay is None else w_decay.shape[1]
+    if z.shape[0] != B * S or a_bias.shape != (n,) or norm.shape != (n,) or state.shape[0] < B or (
+            decay_logits.shape != (B * S, n) if decay_logits is not None else w_decay.shape[0] != n or decay_bias.shape != (n,)):
         raise RavenHipError("delta_rule: operand shapes do not fit together")
-    y = torch.empty(B * S, H * hd, device=z.device, dtype=dtype)
+    y = torch.empty(B * S, n, device=z.device, dtype=dtype)
     ws = _workspace(load().raven_delta_rule_workspace_bytes(B, S, H, hd), z.device) if parallel else None
     f = torch.float32
-    rc = load().raven_delta_rule(_ptr(z, "z", f), z.shape[1], _ptr(decay_logits, "decay_logits", f), _ptr(a_bias, "a_bias", f), _ptr(norm, "norm", f),
-                                 _ptr(state, "state", f), _ptr(y, "y"), B, S, int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), H, int(dim), hd,
-                                 float(eps), dtype_code(dtype), _ptr(ws, "ws"), 0 if ws is None else ws.numel(), _stream())
+    rc = load().raven_delta_rule(_ptr(z, "z", f), z.shape[1], _ptr(decay_logits, "decay_logits", f), _ptr(w_decay, "w_decay", dtype),
+                                 _ptr(decay_bias, "decay_bias", f), rank, _ptr(a_bias, "a_bias", f), _ptr(norm, "norm", f), _ptr(state, "state", f),
+                                 _ptr(y, "y"), B, S, int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), H, int(dim), hd, float(eps),
+                                 dtype_code(dtype), _ptr(ws, "ws"), 0 if ws is None else ws.numel(), _stream())
     _check(rc, "raven_delta_rule")
     return y
 

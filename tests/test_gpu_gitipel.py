@@ -67,6 +67,33 @@ def test_linear_epilogue_large_tiles(pkg, M, N, K):
     assert ((got - ref).abs() <= ref.abs() * 2 ** -8 + 1e-4).all()
 
 
+@DT
+@pytest.mark.parametrize("N,D,dim", [(77, 56, 50), (128, 320, 320), (4100, 2048, 2044)])
+def test_gemv_behind_a_norm(pkg, dtype, N, D, dim):
+    g = torch.Generator().manual_seed(D)
+    x, norm, w = torch.randn(D, generator=g) * 20, torch.rand(D, generator=g) + 0.5, (torch.randn(N, D, generator=g) / D ** 0.5).to(dtype)
+    x[dim:] = 0
+    bias, res = torch.randn(N, generator=g), torch.randn(N, generator=g)
+    h = (x / torch.sqrt((x * x).sum() / dim + 1e-3) * norm).to(dtype).double()
+    z = w.double() @ h + bias
+    run = lambda **kw: pkg.hip.gemv_stream(x.cuda(), norm.cuda(), dim, 1e-3, w.cuda(), dtype, bias=bias.cuda(), **kw).double().cpu()
+    tol = 3e-5 if dtype == F32 else 6e-3  # a row element on a tie of the bf16 grid may round the other way
+    assert (run(residual=res.cuda()) - (z + res)).abs().max() < tol
+    assert (run(act=pkg.hip.ACT_GELU, out_f32=False) - O.gelu_erf(z)).abs().max() < (3e-5 if dtype == F32 else 4e-2)
+
+
+def test_gelu_over_its_whole_range(pkg):
+    """bf16 results use an approximation of erf: every magnitude against the float64 function."""
+    z = torch.cat([torch.linspace(-12, 12, 4001), torch.tensor([0.0, -0.0, 1e-30, -1e-6, 100.0, -100.0])]).bfloat16()
+    eye = torch.zeros(z.numel(), 8).bfloat16()
+    eye[:, 0] = z
+    w = torch.zeros(8, 8).bfloat16()
+    w[0, 0] = 1
+    got = pkg.hip.linear_epilogue(eye.cuda(), w.cuda(), act=pkg.hip.ACT_GELU, out_f32=False)[:, 0].double().cpu()
+    want = O.gelu_erf(z.double())
+    assert ((got - want).abs() <= want.abs() * 2 ** -8 + 2e-6).all()
+
+
 # ---- norm and convolution ----------------------------------------------------------------------------
 @DT
 @pytest.mark.parametrize("D,taps", [(50, 3), (320, 2), (72, 1), (1032, 5), (4104, 4)])
@@ -122,6 +149,29 @@ def test_attention_prompts_portions_and_decoding(pkg, dtype, H, Gk, d):
     for cuts in ([T], [2, 61, 1, 64, 17, 3, 2], [100] + [1] * 50, [1] * 20 + [130]):
         got = run_attention(pkg, q, k, sc, cuts, dtype, t_max=T + 13)
         assert G.rel(got, want) < (1e-5 if dtype == F32 else 1.2e-2), cuts
+
+
+@DT
+@pytest.mark.parametrize("cap", [0.0, 1.5, 35.0, 60.0])
+@pytest.mark.parametrize("bias", [False, True])
+def test_attention_caps_and_bias(pkg, dtype, cap, bias):
+    """No cap, caps on either side of the bound up to which weights are taken relative to the cap itself, with scores that
+    reach it on both sides; without a bias."""
+    T, H, Gk, d = 170, 4, 2, 32
+    g = torch.Generator().manual_seed(int(cap))
+    q, k = (torch.randn(T, n, d, generator=g) for n in (H, Gk))
+    q[100:] *= 6
+    k[0] = -3 * k[0].abs()
+    q[160] = q[160].abs() * 3   # sees scores far below zero only at key 0
+    q, k = q.to(dtype).float(), k.to(dtype).float()
+    r1, r2 = torch.tensor([0.0, 3.0, 0.4, 1.0]), torch.tensor([1.0, 0.5, 0.01, 0.0])
+    if not bias:
+        r1, r2 = torch.zeros(H), torch.zeros(H)
+    r1c, r2c = r1.cuda(), r2.cuda()
+    sc = pkg.hip.make_score(0.5, cap, r1c, r2c) if bias else pkg.hip.make_score(0.5, cap)
+    want = O.attention(q.double(), k.double(), 0.5, cap if cap else 1e9, r1.double(), r2.double())
+    for cuts in ([T], [20, 2, 100, 1, 1, 46]):
+        assert G.rel(run_attention(pkg, q, k, sc, cuts, dtype), want) < (2e-5 if dtype == F32 else 1.5e-2), cuts
 
 
 @DT
@@ -219,6 +269,29 @@ def test_delta_rule_prompts_portions_and_decoding(pkg, H, d, kind):
             assert ((state - S).norm() / S.norm()) < 2e-5, (parallel, cuts)
     got, _ = run_delta(pkg, ins, [T], eps, BF16)
     assert ((got - want).abs() <= 2 ** -8 * want.abs() + 1e-3).all()
+
+
+@DT
+@pytest.mark.parametrize("rank", [8, 64, 120])
+def test_delta_rule_forms_its_decay_logits(pkg, dtype, rank):
+    T, H, d, eps = 21, 3, 40, 1e-4
+    r, k, v, gate, a, _, a_bias, norm = delta_inputs(T, H, d, rank)
+    g = torch.Generator().manual_seed(rank)
+    low, w0 = torch.randn(T, rank, generator=g), torch.randn(H * d, generator=g) - 2
+    w2 = (torch.randn(H * d, rank, generator=g) * 2 / rank ** 0.5).to(dtype)
+    decay = (torch.tanh(low) @ w2.float().T + w0).view(T, H, d)
+    want, _ = delta_want(r, k, v, gate, a, decay, a_bias, norm, eps)
+    z = torch.cat([t.reshape(T, -1) for t in (r, k, v, gate, a)] + [low], 1).cuda()
+    S = torch.zeros(1, H, d, d, device="cuda")
+    pos, out = 0, []
+    for n in (1, 8, 1, 5, 2, 4):
+        out.append(pkg.hip.delta_rule(z[pos:pos + n].contiguous(), None, a_bias.reshape(-1).cuda(), norm.reshape(-1).cuda(), S, 1, n, pos, d, eps, dtype,
+                                      w_decay=w2.cuda(), decay_bias=w0.cuda()))
+        pos += n
+    assert G.rel(torch.cat(out).float().view(T, H, d), want) < (1e-4 if dtype == F32 else 5e-3)
+    with pytest.raises(pkg.hip.RavenHipError):
+        pkg.hip.delta_rule(z[:9].contiguous(), None, a_bias.reshape(-1).cuda(), norm.reshape(-1).cuda(), S, 1, 9, 0, d, eps, dtype, w_decay=w2.cuda(),
+                           decay_bias=w0.cuda())
 
 
 def test_delta_rule_long_sequences(pkg):
