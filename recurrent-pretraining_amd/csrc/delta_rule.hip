@@ -235,7 +235,7 @@ __device__ __forceinline__ f32x4 block_product(const float (*X)[R + 4], const fl
 }
 
 template <int R>
-__global__ __launch_bounds__(256) void delta_block_kernel(DeltaBlockArgs p) {
+__global__ __launch_bounds__(256, R <= 64 ? 4 : 2) void delta_block_kernel(DeltaBlockArgs p) {
     constexpr int KEEP = (R + 63) / 64;
     __shared__ __align__(16) float U[kBlk][R + 4], Rt[kBlk][R + 4], Bt[kBlk][R + 4], Kt[kBlk][R + 4];
     __shared__ float part[4][R];                            // each wave's sum of log decays
@@ -378,7 +378,10 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     const bool fresh = p.first == 0 && (a.pos_dev ? *a.pos_dev : a.pos0) == 0;
     float* state = a.state + (((int64_t)b * a.H + h) * hd + min(col, hd - 1)) * hd + (row < hd ? row : 0);
     const float* ws = p.ws + ((int64_t)b * a.H + h) * kSegment * blk_floats(R);
-    const float* vcol = a.z + (int64_t)b * a.S * a.ldz + 2 * inner + h * hd + min(col, hd - 1);
+    const char* vbase = reinterpret_cast<const char*>(a.z + (int64_t)b * a.S * a.ldz + 2 * inner + h * hd);
+    // byte offsets below 2^32 (the host checks): uniform bases plus 32-bit lane offsets keep the address arithmetic off the loop
+    const unsigned vcol = 4u * min(col, hd - 1), vrow = 4u * a.ldz, vlast = (a.S - 1) * vrow;
+    const unsigned at_row = 4u * (l16 * R + row), at_tok = 4u * ((16 * wave + l16) * 16 + 4 * q), at_sq = 4u * (l16 * 16 + 4 * q), at_g = 4u * row;
     float* orow = p.o + (((int64_t)b * a.H + h) * p.o_rows) * R + 16 * tile + l16;
     constexpr int wGV = 0, wRKV = NB - 1, wRBP = NB / 2;  // which wave adds the 16 x 16 products
 
@@ -392,18 +395,19 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     Set st[kScanAhead];
     auto fetch = [&](int c, Set& s) {
         const int cc = min(c, p.n_blocks - 1);
-        const float* w = ws + (int64_t)cc * blk_floats(R);
-        s.tu = *reinterpret_cast<const f32x4*>(w + l16 * R + row);
-        s.r = *reinterpret_cast<const f32x4*>(w + 16 * R + l16 * R + row);
-        s.bt = *reinterpret_cast<const f32x4*>(w + 32 * R + (16 * wave + l16) * 16 + 4 * q);
-        s.kt = *reinterpret_cast<const f32x4*>(w + 48 * R + (16 * wave + l16) * 16 + 4 * q);
-        s.tm = *reinterpret_cast<const f32x4*>(w + 64 * R + l16 * 16 + 4 * q);
-        s.rb = *reinterpret_cast<const f32x4*>(w + 64 * R + 256 + l16 * 16 + 4 * q);
-        s.rk = *reinterpret_cast<const f32x4*>(w + 64 * R + 512 + l16 * 16 + 4 * q);
-        s.g = *reinterpret_cast<const f32x4*>(w + 64 * R + 768 + row);
-        const int t = (p.first + cc) * kBlk + 4 * q;
+        const char* w = reinterpret_cast<const char*>(ws + (int64_t)cc * blk_floats(R));
+        auto at = [&](int floats, unsigned off) { return *reinterpret_cast<const f32x4*>(w + 4 * floats + off); };
+        s.tu = at(0, at_row);
+        s.r = at(16 * R, at_row);
+        s.bt = at(32 * R, at_tok);
+        s.kt = at(48 * R, at_tok);
+        s.tm = at(64 * R, at_sq);
+        s.rb = at(64 * R + 256, at_sq);
+        s.rk = at(64 * R + 512, at_sq);
+        s.g = at(64 * R + 768, at_g);
+        const unsigned first = (unsigned)((p.first + cc) * kBlk) * vrow;  // rows past the chunk repeat its last one: they meet zero factors
 #pragma unroll
-        for (int i = 0; i < 4; ++i) s.v[i] = vcol[(int64_t)min(t + i, a.S - 1) * a.ldz];  // rows past the chunk meet zero factors
+        for (int i = 0; i < 4; ++i) s.v[i] = *reinterpret_cast<const float*>(vbase + (min(first + (4 * q + i) * vrow, vlast) + vcol));
     };
     auto mac4 = [](const f32x4& x, const float* y, f32x4 acc) {
 #pragma unroll
@@ -429,38 +433,45 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     };
 #pragma unroll
     for (int d = 0; d < kScanAhead; ++d) fetch(d, st[d]);
-    f32x4 O = {0.f, 0.f, 0.f, 0.f};
+    const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
+    f32x4 O = zero, rb = zero;             // of the block before: its outputs so far, its -tril(R B^T) ...
+    float pv[4] = {0.f, 0.f, 0.f, 0.f};    // ... and its removals
+    f32x4 P = wave == wGV ? mac4(st[0].tm, st[0].v, zero) : zero;
     for (int c0 = 0; c0 < p.n_blocks; c0 += kScanAhead) {
 #pragma unroll
         for (int d = 0; d < kScanAhead; ++d) {
             const int c = c0 + d;
-            {
-                const Set& s = st[d];
-                const int buf = d & 1;
-                const f32x4 zero = {0.f, 0.f, 0.f, 0.f};
-                float sv[4];
-                arr(S, sv);
-                f32x4 P = wave == wGV ? mac4(s.tm, s.v, zero) : zero;
-                P = mac4(s.tu, sv, P);
-                xp[buf][wave][lane] = P;
-                xo[buf][wave][lane] = O;
-                O = wave == wRKV ? mac4(s.rk, s.v, zero) : zero;
-                O = mac4(s.r, sv, O);
-                S = mac4(s.kt, s.v, S * s.g);
-                __syncthreads();
-                P = xp[buf][0][lane];
+            Set& s = st[d];
+            const Set& next = st[(d + 1) % kScanAhead];
+            const int buf = d & 1;
+            float sv[4];
+            arr(S, sv);
+            // the chain from block to block: P -> exchange -> S.  Everything else fills the time between P's products and the
+            // barrier (the fences keep it there)
+            P = mac4(s.tu, sv, P);
+            S = mac4(s.kt, s.v, S * s.g);
+            xp[buf][wave][lane] = P;
+            if (wave == wRBP) O = mac4(rb, pv, O);
+            __builtin_amdgcn_sched_barrier(0);
+            f32x4 O_next = wave == wRKV ? mac4(s.rk, s.v, zero) : zero;
+            O_next = mac4(s.r, sv, O_next);
+            xo[buf][wave][lane] = O;
+            P = wave == wGV ? mac4(next.tm, next.v, zero) : zero;
+            rb = s.rb;
+            __builtin_amdgcn_sched_barrier(0);
+            __syncthreads();
+            f32x4 sum = xp[buf][0][lane];
 #pragma unroll
-                for (int w = 1; w < NB; ++w) P += xp[buf][w][lane];
-                float pv[4];
-                arr(P, pv);
-                S = mac4(s.bt, pv, S);
-                if (wave == wRBP) O = mac4(s.rb, pv, O);
-                // the first block of a segment has nothing to publish: it writes to the empty block in front
-                store_o(buf, orow + (int64_t)(c > 0 ? p.first + c : 0) * kBlk * R);
-            }
-            fetch(c + kScanAhead, st[d]);
+            for (int w = 1; w < NB; ++w) sum += xp[buf][w][lane];
+            arr(sum, pv);
+            S = mac4(s.bt, pv, S);
+            // the first block of a segment has nothing to publish: it writes to the empty block in front
+            store_o(buf, orow + (int64_t)(c > 0 ? p.first + c : 0) * kBlk * R);
+            O = O_next;
+            fetch(c + kScanAhead, s);
         }
     }
+    if (wave == wRBP) O = mac4(rb, pv, O);
     __syncthreads();
     xo[0][wave][lane] = O;
     __syncthreads();
@@ -595,7 +606,7 @@ extern "C" int raven_delta_rule(const float* z, int32_t ldz, const float* decay_
     a.H = n_heads; a.dim = dim; a.hd = head_dim; a.ldz = ldz; a.S = S; a.pos0 = pos0; a.pos_dev = pos_dev; a.eps = eps;
     hipStream_t s = static_cast<hipStream_t>(stream);
     const size_t need = raven_delta_rule_workspace_bytes(B, S, n_heads, head_dim);
-    if (need && workspace && need <= workspace_bytes) {
+    if (need && (int64_t)S * ldz < (1ll << 30) && workspace && need <= workspace_bytes) {
         RAVEN_REQUIRE(((uintptr_t)workspace & 15) == 0 && ((uintptr_t)state & 15) == 0, "delta_rule: workspace and state must be 16-byte aligned");
         float* ws = static_cast<float*>(workspace);
         return dtype == RAVEN_BF16 ? launch_delta_blocked<bf16>(a, B, ws, s) : launch_delta_blocked<float>(a, B, ws, s);

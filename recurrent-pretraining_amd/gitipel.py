@@ -302,9 +302,13 @@ class GitipelForCausalLM(MinimalGeneration, PreTrainedModel, GenerationMixin):
                     rows = rows[:, torch.tensor([wanted[k] - lo for k in here], device=self.device)]
                 rows = rows.reshape(B * len(here), -1).contiguous()
                 h = torch.empty(rows.shape, dtype=self.dtype, device=self.device)
-                y = torch.empty(rows.shape[0], V, dtype=torch.float32, device=self.device)
                 lws = hip.linear_workspace(rows.shape[0], V, self.device) if 1 < rows.shape[0] <= 32 else None
-                logits[:, here] = self._logits(rows, h, y, lws).view(B, len(here), V)
+                straight = here == list(range(here[0], here[-1] + 1)) and (B == 1 or len(here) == len(wanted))
+                y = (logits[:, here[0]:here[-1] + 1].view(rows.shape[0], V) if straight else
+                     torch.empty(rows.shape[0], V, dtype=torch.float32, device=self.device))
+                self._logits(rows, h, y, lws)
+                if not straight:
+                    logits[:, here] = y.view(B, len(here), V)
         loss = torch.as_tensor(0.0)
         if labels is not None:
             loss = torch.nn.functional.cross_entropy(logits.view(-1, V), labels.to(self.device).view(-1), ignore_index=-100)
