@@ -164,26 +164,44 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
         for (int e = 0; e < E; e += 4) *reinterpret_cast<f32x4*>(&so[grp][i][c * E + e]) = f32x4{acc[i][e], acc[i][e + 1], acc[i][e + 2], acc[i][e + 3]};
     }
     __syncthreads();
+    // merge: the groups' factors first (group-major threads), then every output is one dot product over the groups
+    float top[NQ];
+#pragma unroll
+    for (int i = 0; i < NQ; ++i) {
+        float x = -INFINITY;
+        for (int n = lane; n < NG; n += 64) x = fmaxf(x, sm[n][i]);
+        top[i] = wave_max(x);
+    }
+    __syncthreads();
+    for (int t = threadIdx.x; t < NG * NQ; t += 256) {
+        const int n = t / NQ, i = t % NQ;
+        float ref = top[0];
+#pragma unroll
+        for (int k = 1; k < NQ; ++k) ref = i == k ? top[k] : ref;
+        sm[n][i] = exp_weight<T>(sm[n][i] - (ref == -INFINITY ? 0.f : ref));
+    }
+    __syncthreads();
     for (int t = threadIdx.x; t < NQ * a.hd; t += 256) {
         const int i = t / a.hd, col = t - i * a.hd;
         if (q0 + i >= group) break;
-        float top = -INFINITY;
-        for (int n = 0; n < NG; ++n) top = fmaxf(top, sm[n][i]);
-        const float ref = top == -INFINITY ? 0.f : top;
         float sum = 0.f, o = 0.f;
+#pragma unroll 8
         for (int n = 0; n < NG; ++n) {
-            const float w = exp_weight<T>(sm[n][i] - ref);
-            sum += w * sl[n][i];
-            o += w * so[n][i][col];
+            const float w = sm[n][i];
+            sum = __builtin_fmaf(w, sl[n][i], sum);
+            o = __builtin_fmaf(w, so[n][i][col], o);
         }
         const int h = g * group + q0 + i;
         if (a.splits == 1) {
             static_cast<T*>(a.y)[(int64_t)m * a.ldy + h * a.hd + col] = from_f32<T>(o / sum);
         } else {
             float* p = a.part + (((int64_t)m * a.H + h) * a.splits + blockIdx.x) * (a.hd + 2);
+            float ref = top[0];
+#pragma unroll
+            for (int k = 1; k < NQ; ++k) ref = i == k ? top[k] : ref;
             p[2 + col] = o;
             if (col == 0) {
-                p[0] = top;
+                p[0] = ref;
                 p[1] = sum;
             }
         }

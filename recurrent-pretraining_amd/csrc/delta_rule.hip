@@ -203,7 +203,8 @@ __global__ __launch_bounds__(512) void delta_steps_kernel(DeltaArgs a) {
 // ---- blocks of 16 tokens ----------------------------------------------------------------------------------------
 constexpr int kBlk = 16;
 constexpr int kScanAhead = 4;        // blocks whose operands are in flight
-constexpr int kSegment = 64;         // blocks per (block, scan) launch pair: bounds the workspace and keeps it near the caches
+constexpr int kSegment = 256;        // most blocks per (block, scan) launch pair: bounds the workspace.  A pair costs about 13 us beside its
+                                     // blocks (4096 tokens, 32 heads of 64: 307 us in segments of 64 blocks, 281 of 128)
 constexpr int kMinBlocked = 48;      // shorter chunks walk token by token
 constexpr int kMaxBlockedDim = 128;  // and so do wider heads (the scan's operands would not fit a wave's registers)
 
@@ -216,6 +217,7 @@ struct DeltaBlockArgs {
     float* ws;
     float* o;         // [B, H, o_rows, R]: token t of the chunk in row 16 + t, columns past the head unused
     int64_t o_rows;
+    int stride;       // blocks the workspace holds per (sequence, head)
     int first;        // first block of the segment
     int n_blocks;     // blocks of the segment, a multiple of kScanAhead (those past the chunk are empty)
 };
@@ -245,7 +247,7 @@ __global__ __launch_bounds__(256, R <= 64 ? 4 : 2) void delta_block_kernel(Delta
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, q = lane >> 4;
     const int hd = a.hd, inner = a.H * hd;
     const int t0 = (p.first + blk) * kBlk;
-    float* ws = p.ws + (((int64_t)b * a.H + h) * kSegment + blk) * blk_floats(R);
+    float* ws = p.ws + (((int64_t)b * a.H + h) * p.stride + blk) * blk_floats(R);
     float *wTU = ws, *wR = ws + 16 * R, *wB = ws + 32 * R, *wK = ws + 48 * R, *wTM = ws + 64 * R, *wRB = wTM + 256, *wRK = wRB + 256, *wG = wRK + 256;
 
     // this wave's four tokens, channels lane, lane + 64, ...; every load is unconditional (a clamped address, the value dropped)
@@ -370,14 +372,18 @@ __global__ __launch_bounds__(64 * NB) void delta_scan_kernel(DeltaBlockArgs p) {
     constexpr int R = 16 * NB;
     __shared__ __align__(16) f32x4 xp[2][NB][64], xo[2][NB][64];
     const DeltaArgs& a = p.d;
-    const int tile = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+    // workgroups go round the eight XCDs: the column tiles of one head, which read the same operands, land on one of them
+    const int tiles = (p.d.hd + 15) / 16, n_wgs = tiles * p.d.H;
+    const int logical = ((int)blockIdx.x & 7) * ((n_wgs + 7) >> 3) + ((int)blockIdx.x >> 3);
+    if (logical >= n_wgs) return;
+    const int tile = logical % tiles, h = logical / tiles, b = blockIdx.y;
     const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, q = lane >> 4;
     const int hd = a.hd, inner = a.H * hd;
     const int col = 16 * tile + l16, row = 16 * wave + 4 * q;
     const bool col_ok = col < hd, mine = col_ok && row < hd;  // hd is a multiple of 8: four rows exist together
     const bool fresh = p.first == 0 && (a.pos_dev ? *a.pos_dev : a.pos0) == 0;
     float* state = a.state + (((int64_t)b * a.H + h) * hd + min(col, hd - 1)) * hd + (row < hd ? row : 0);
-    const float* ws = p.ws + ((int64_t)b * a.H + h) * kSegment * blk_floats(R);
+    const float* ws = p.ws + ((int64_t)b * a.H + h) * p.stride * blk_floats(R);
     const char* vbase = reinterpret_cast<const char*>(a.z + (int64_t)b * a.S * a.ldz + 2 * inner + h * hd);
     // byte offsets below 2^32 (the host checks): uniform bases plus 32-bit lane offsets keep the address arithmetic off the loop
     const unsigned vcol = 4u * min(col, hd - 1), vrow = 4u * a.ldz, vlast = (a.S - 1) * vrow;
@@ -526,16 +532,20 @@ static int64_t blocked_o_rows(int S) {  // an empty block in front, the chunk in
     const int round = kBlk * kScanAhead;
     return kBlk + (int64_t)(S + round - 1) / round * round;
 }
+static int blocked_stride(int S) {
+    const int64_t blocks = (blocked_o_rows(S) - kBlk) / kBlk;
+    return blocks < kSegment ? (int)blocks : kSegment;
+}
 static size_t blocked_ws_floats(int B, int S, int H, int hd) {
     const int R = scan_rows(hd);
-    return (size_t)B * H * kSegment * blk_floats(R) + (size_t)B * H * blocked_o_rows(S) * R;
+    return (size_t)B * H * blocked_stride(S) * blk_floats(R) + (size_t)B * H * blocked_o_rows(S) * R;
 }
 
 template <int R>
 static int launch_delta_segment(const DeltaBlockArgs& p, int B, hipStream_t s) {
     delta_block_kernel<R><<<dim3(p.n_blocks, p.d.H, B), dim3(256), 0, s>>>(p);
     if (const int rc = raven_host::check_launch("delta_rule (blocks)")) return rc;
-    delta_scan_kernel<R / 16><<<dim3((p.d.hd + 15) / 16, p.d.H, B), dim3(4 * R), 0, s>>>(p);
+    delta_scan_kernel<R / 16><<<dim3(((p.d.hd + 15) / 16 * p.d.H + 7) / 8 * 8, B), dim3(4 * R), 0, s>>>(p);
     return raven_host::check_launch("delta_rule (scan)");
 }
 
@@ -544,7 +554,8 @@ static int launch_delta_blocked(const DeltaArgs& a, int B, float* ws, hipStream_
     DeltaBlockArgs p{};
     p.d = a;
     p.ws = ws;
-    p.o = ws + (size_t)B * a.H * kSegment * blk_floats(scan_rows(a.hd));
+    p.stride = blocked_stride(a.S);
+    p.o = ws + (size_t)B * a.H * p.stride * blk_floats(scan_rows(a.hd));
     p.o_rows = blocked_o_rows(a.S);
     const int blocks = (int)((p.o_rows - kBlk) / kBlk);
     for (p.first = 0; p.first < blocks; p.first += kSegment) {

@@ -144,6 +144,57 @@ __global__ __launch_bounds__(256) void norm_conv_kernel(NormConvArgs a) {
     }
 }
 
+// One token per sequence: the row, the weights and every row of the window are requested at once, one memory latency instead of one
+// per window row.  TAPS: window rows held (taps <= TAPS; the others are skipped).
+template <typename T, int P, int TAPS>
+__global__ __launch_bounds__(256) void norm_conv_step_kernel(NormConvArgs a) {
+    __shared__ float red[4];
+    const int b = blockIdx.x, tid = threadIdx.x;
+    const int pos = a.pos_dev ? *a.pos_dev : a.pos0;
+    const int pieces = a.ld / 4;
+    const float* row = a.x + (int64_t)b * a.ld;
+    float* ring = a.ring + (int64_t)b * a.taps * a.ld;
+    f32x4 h[P], w[P], c[TAPS][P], past[TAPS][P];
+#pragma unroll
+    for (int j = 0; j < P; ++j) {
+        const int at = 4 * min(tid + 256 * j, pieces - 1);
+        h[j] = *reinterpret_cast<const f32x4*>(row + at);
+        w[j] = *reinterpret_cast<const f32x4*>(a.w + at);
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) {  // t = tokens back; beyond the window or the sequence's start any row will do
+            const int back = min(t, a.taps - 1), p = max(pos - back, 0);
+            c[t][j] = *reinterpret_cast<const f32x4*>(a.conv + (int64_t)(a.taps - 1 - back) * a.ld + at);
+            past[t][j] = *reinterpret_cast<const f32x4*>(ring + (int64_t)(p % a.taps) * a.ld + at);
+        }
+    }
+    float ss = 0.f;
+#pragma unroll
+    for (int j = 0; j < P; ++j)
+        if (tid + 256 * j < pieces) ss += h[j][0] * h[j][0] + h[j][1] * h[j][1] + h[j][2] * h[j][2] + h[j][3] * h[j][3];
+    const float inv = 1.0f / sqrtf(wg_sum4(ss, red) / (float)a.dim + a.eps);
+    T* y = static_cast<T*>(a.y) + (int64_t)b * a.ld;
+    float* keep = ring + (int64_t)(pos % a.taps) * a.ld;  // not one of the rows read above, except as the ignored t = 0
+#pragma unroll
+    for (int j = 0; j < P; ++j) {
+        const int at = 4 * (tid + 256 * j);
+        if (tid + 256 * j >= pieces) continue;
+        const f32x4 n = h[j] * inv * w[j];
+        f32x4 o = n;
+        for (int t = TAPS - 1; t > 0; --t)  // oldest first, as over chunks
+            if (t < a.taps && t <= pos) o += c[t][j] * past[t][j];
+        o += c[0][j] * n;
+        *reinterpret_cast<f32x4*>(keep + at) = n;
+        if constexpr (sizeof(T) == 4) {
+            *reinterpret_cast<f32x4*>(y + at) = o;
+        } else {
+            bf16 q[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) q[i] = from_f32<bf16>(o[i]);
+            *reinterpret_cast<uint2*>(y + at) = *reinterpret_cast<const uint2*>(q);
+        }
+    }
+}
+
 // x[m] = float(table[ids[m]]) * scale, and the same row rounded to T
 template <typename T>
 __global__ __launch_bounds__(256) void embed_stream_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, float* __restrict__ x,
@@ -183,6 +234,12 @@ __global__ __launch_bounds__(256) void round_rows_kernel(const float* __restrict
 
 template <typename T, int P>
 static int launch_norm_conv(const NormConvArgs& a, int B, hipStream_t s) {
+    if constexpr (P <= 4) {
+        if (a.conv && a.S == 1 && a.taps <= 4) {
+            norm_conv_step_kernel<T, P, 4><<<dim3(B), dim3(256), 0, s>>>(a);
+            return raven_host::check_launch("norm_conv (step)");
+        }
+    }
     const size_t lds = a.conv ? (size_t)a.taps * a.ld * sizeof(float) : 0;
     if (lds > 48 * 1024) {
         static bool attr_set = false;
