@@ -14,9 +14,14 @@
 
 #include <math.h>
 
+#include <type_traits>
+
 #include "raven_common.h"
 
 namespace raven {
+
+// caps whose weights may be taken relative to the cap itself (see the chunk kernel)
+static bool fixed_reference(float cap) { return cap > 0.f && cap <= 35.f; }
 
 struct CappedArgs {
     const void* qk;   // [M, ldq]
@@ -64,7 +69,10 @@ __device__ __forceinline__ float lanes_sum(float v) {  // over groups of LPP nei
     return v;
 }
 
-template <typename T, int LPP, int NQ>
+// FIXED (bf16, caps up to 35): weights are taken relative to the constant +cap, as in the chunk kernel below (its comment says why
+// that is safe): no maximum, no rescaling, and ranges merge by plain sums.  The lanes that share a position then also share
+// the work behind the product: each turns NQ * U / LPP of the NQ * U scores into weights and hands them round.
+template <typename T, int LPP, int NQ, bool FIXED>
 __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
     constexpr int E = Chunk<T>::N;
     constexpr int U = 4;                 // positions in flight per lane group
@@ -78,9 +86,9 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
     const int g = blockIdx.y / sub, q0 = (blockIdx.y % sub) * NQ;
     const int m = blockIdx.z, b = m / a.S, s = m % a.S;
     const int pos = (a.pos_dev ? *a.pos_dev : a.pos0) + s;
-    const int n_cached = a.append ? pos : pos + 1;
-    const int span = (n_cached + a.splits - 1) / a.splits;
-    const int lo = (int)blockIdx.x * span, hi = min(n_cached, lo + span);
+    const int n_pos = pos + 1;
+    const int span = (n_pos + a.splits - 1) / a.splits;
+    const int lo = (int)blockIdx.x * span, hi = min(n_pos, lo + span);
     const bool active = c * E < a.hd;
     const int cc = active ? c : 0;
 
@@ -127,6 +135,48 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
             }
         }
     };
+    // FIXED: this lane's pairs (query head, position of the round): pair = c + LPP * j
+    constexpr int NP = NQ * U, PER = (NP + LPP - 1) / LPP;
+    float pr1[PER], pr2[PER];
+    if constexpr (FIXED) {
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            const int i = min((c + LPP * j) / U, NQ - 1);
+            pr1[j] = r1[0];
+            pr2[j] = r2[0];
+#pragma unroll
+            for (int k = 1; k < NQ; ++k) {
+                pr1[j] = i == k ? r1[k] : pr1[j];
+                pr2[j] = i == k ? r2[k] : pr2[j];
+            }
+        }
+    }
+    const float in_scale = 2.8853900817779268f * a.scale * inv_cap, drop = -2.8853900817779268f * a.cap;
+    auto take_fixed = [&](const Chunk<T>* k, int p0) {
+        float d[NP];
+#pragma unroll
+        for (int n = 0; n < NP; ++n) d[n] = lanes_sum<LPP>(dot_chunk(q[n / U], k[n % U], 0.f));
+        float w[PER];
+#pragma unroll
+        for (int j = 0; j < PER; ++j) {
+            float x = d[LPP * j < NP ? LPP * j : 0];
+#pragma unroll
+            for (int n = 1; n < LPP; ++n)
+                if (LPP * j + n < NP) x = c == n ? d[LPP * j + n] : x;
+            const int p = p0 + ((c + LPP * j) % U) * NG + grp;
+            const float e = drop * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * in_scale)) -
+                            pr1[j] * __builtin_amdgcn_logf(1.f + pr2[j] * fmaxf((float)(pos - p), 0.f));
+            w[j] = p < hi ? __builtin_amdgcn_exp2f(e) : 0.f;
+        }
+#pragma unroll
+        for (int n = 0; n < NP; ++n) {
+            const float wn = __shfl(w[n / LPP], (lane & ~(LPP - 1)) | (n % LPP), 64);
+            l[n / U] += wn;
+#pragma unroll
+            for (int e = 0; e < E; ++e) acc[n / U][e] = __builtin_fmaf(wn, to_f32(k[n % U].v[e]), acc[n / U][e]);
+        }
+    };
+    const T* own = row + (int64_t)(a.H + g) * a.hd;  // a decode step's own key is still in its fused row
     for (int p0 = lo; p0 < hi; p0 += NG * U) {
         Chunk<T> k[U];
         int p[U];
@@ -135,29 +185,19 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
         for (int u = 0; u < U; ++u) {
             p[u] = p0 + u * NG + grp;
             ok[u] = p[u] < hi;
-            k[u] = load_chunk(keys + (int64_t)min(p[u], hi - 1) * a.hd + cc * E);  // hi > lo >= 0 here
+            const int at = min(p[u], hi - 1);  // hi > lo >= 0 here
+            k[u] = load_chunk((a.append && at == pos ? own : keys + (int64_t)at * a.hd) + cc * E);
         }
-        take(k, p, ok);
+        if constexpr (FIXED) take_fixed(k, p0);
+        else take(k, p, ok);
     }
-    if (a.append && (int)blockIdx.x == a.splits - 1) {  // the row's own position, from the fused row
-        const Chunk<T> own = load_chunk(row + (int64_t)(a.H + g) * a.hd + cc * E);
-        Chunk<T> k[U];
-        int p[U];
-        bool ok[U];
-#pragma unroll
-        for (int u = 0; u < U; ++u) {
-            k[u] = own;
-            p[u] = pos;
-            ok[u] = u == 0 && grp == 0;
-        }
-        take(k, p, ok);
-        if (q0 == 0 && grp == 0 && active && pos < a.t_max) store_chunk(keys + (int64_t)pos * a.hd + c * E, own);
-    }
+    if (a.append && (int)blockIdx.x == a.splits - 1 && q0 == 0 && grp == 0 && active && pos < a.t_max)
+        store_chunk(keys + (int64_t)pos * a.hd + c * E, load_chunk(own + c * E));
 
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
         if (c == 0) {
-            sm[grp][i] = mx[i];
+            sm[grp][i] = FIXED ? 1.f : mx[i];
             sl[grp][i] = l[i];
         }
 #pragma unroll
@@ -167,27 +207,31 @@ __global__ __launch_bounds__(256) void capped_attention_kernel(CappedArgs a) {
     // merge: the groups' factors first (group-major threads), then every output is one dot product over the groups
     float top[NQ];
 #pragma unroll
-    for (int i = 0; i < NQ; ++i) {
-        float x = -INFINITY;
-        for (int n = lane; n < NG; n += 64) x = fmaxf(x, sm[n][i]);
-        top[i] = wave_max(x);
-    }
-    __syncthreads();
-    for (int t = threadIdx.x; t < NG * NQ; t += 256) {
-        const int n = t / NQ, i = t % NQ;
-        float ref = top[0];
+    for (int i = 0; i < NQ; ++i) top[i] = 0.f;
+    if constexpr (!FIXED) {
 #pragma unroll
-        for (int k = 1; k < NQ; ++k) ref = i == k ? top[k] : ref;
-        sm[n][i] = exp_weight<T>(sm[n][i] - (ref == -INFINITY ? 0.f : ref));
+        for (int i = 0; i < NQ; ++i) {
+            float x = -INFINITY;
+            for (int n = lane; n < NG; n += 64) x = fmaxf(x, sm[n][i]);
+            top[i] = wave_max(x);
+        }
+        __syncthreads();
+        for (int t = threadIdx.x; t < NG * NQ; t += 256) {
+            const int n = t / NQ, i = t % NQ;
+            float ref = top[0];
+#pragma unroll
+            for (int k = 1; k < NQ; ++k) ref = i == k ? top[k] : ref;
+            sm[n][i] = exp_weight<T>(sm[n][i] - (ref == -INFINITY ? 0.f : ref));
+        }
+        __syncthreads();
     }
-    __syncthreads();
     for (int t = threadIdx.x; t < NQ * a.hd; t += 256) {
         const int i = t / a.hd, col = t - i * a.hd;
         if (q0 + i >= group) break;
         float sum = 0.f, o = 0.f;
 #pragma unroll 8
         for (int n = 0; n < NG; ++n) {
-            const float w = sm[n][i];
+            const float w = FIXED ? 1.f : sm[n][i];
             sum = __builtin_fmaf(w, sl[n][i], sum);
             o = __builtin_fmaf(w, so[n][i][col], o);
         }
@@ -497,7 +541,7 @@ template <int HD>
 static int launch_capped_prefill(const CappedArgs& a, int B, hipStream_t s) {
     const int rg = (int64_t)((a.S + 127) / 128) * a.H * B >= 512 ? 2 : 1;
     const dim3 grid((a.S + 64 * rg - 1) / (64 * rg), a.H, B);
-    const bool fixed = a.cap > 0.f && a.cap <= 35.f;
+    const bool fixed = fixed_reference(a.cap);
     if (rg == 2) {
         if (fixed) capped_attention_prefill_kernel<HD, 2, true><<<grid, dim3(256), 0, s>>>(a);
         else capped_attention_prefill_kernel<HD, 2, false><<<grid, dim3(256), 0, s>>>(a);
@@ -536,9 +580,18 @@ template <typename T, int LPP>
 static int launch_capped(const CappedArgs& a, int M, hipStream_t s) {
     const int group = a.H / a.G, nq = capped_nq(group);
     const dim3 grid(a.splits, a.G * ((group + nq - 1) / nq), M);
-    if (nq == 4) capped_attention_kernel<T, LPP, 4><<<grid, dim3(256), 0, s>>>(a);
-    else if (nq == 2) capped_attention_kernel<T, LPP, 2><<<grid, dim3(256), 0, s>>>(a);
-    else capped_attention_kernel<T, LPP, 1><<<grid, dim3(256), 0, s>>>(a);
+    auto run = [&](auto fixed) {
+        constexpr bool F = decltype(fixed)::value;
+        if (nq == 4) capped_attention_kernel<T, LPP, 4, F><<<grid, dim3(256), 0, s>>>(a);
+        else if (nq == 2) capped_attention_kernel<T, LPP, 2, F><<<grid, dim3(256), 0, s>>>(a);
+        else capped_attention_kernel<T, LPP, 1, F><<<grid, dim3(256), 0, s>>>(a);
+    };
+    if constexpr (sizeof(T) == 2) {
+        if (fixed_reference(a.cap)) run(std::true_type{});
+        else run(std::false_type{});
+    } else {
+        run(std::false_type{});
+    }
     if (a.splits > 1) capped_combine_kernel<T><<<dim3(a.H, M), dim3(64), 0, s>>>(a);
     return raven_host::check_launch("capped_attention");
 }

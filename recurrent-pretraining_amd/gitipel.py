@@ -298,7 +298,7 @@ class GitipelForCausalLM(MinimalGeneration, PreTrainedModel, GenerationMixin):
             here = [k for k, p in enumerate(wanted) if lo <= p < lo + n]
             if here:
                 rows = x.view(B, n, -1)
-                if len(here) < n:
+                if [wanted[k] for k in here] != list(range(lo, lo + n)):
                     rows = rows[:, torch.tensor([wanted[k] - lo for k in here], device=self.device)]
                 rows = rows.reshape(B * len(here), -1).contiguous()
                 h = torch.empty(rows.shape, dtype=self.dtype, device=self.device)
