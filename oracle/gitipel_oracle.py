@@ -1,5 +1,5 @@
-"""CPU restatement of the Gitipel decoder, used as the checker by the tests only (nothing of the product path imports it, and
-it imports nothing of the product path).  One plain function per mechanism, token by token where the mechanism is a
+"""CPU restatement of the Gitipel decoder, for the tests only (nothing of the product path imports it, and it imports
+nothing of the product path).  One plain function per mechanism, token by token where the mechanism is a
 recurrence, in the dtype of its inputs (float32 or float64).  Sequences are processed whole, from position 0.
 
 `cfg` is the dictionary of a config.json; `w` maps tensor names to floating-point tensors.
