@@ -396,7 +396,7 @@ int raven_core_iterations(const raven_dims* dims, const void* adapter_w, const r
                           int32_t n_iterations, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev,
                           void* workspace, size_t workspace_bytes, void* stream);
 
-/* ---- Layer kinds of decoders with an fp32 residual stream (the Gitipel design; no counterpart in the reference) -----------
+/* ---- Layer kinds of decoders with an fp32 residual stream (the Gitipel and Gupitar designs; no counterpart in the reference) -----------
  * Rows of width channels are stored `ld` elements apart, ld = width rounded up to a multiple of 8 with zeros behind the true
  * width; heads likewise have head_dim elements, head_dim = dim rounded up to a multiple of 8 (the caller pads the weights).
  *
@@ -443,12 +443,88 @@ int raven_delta_rule(const float* z, int32_t ldz, const float* decay_logits, con
                      const float* a_bias, const float* norm, float* state, void* y, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t n_heads, int32_t dim, int32_t head_dim, float eps,
                      int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
 
+/* Latent attention: queries and keys come out of low-rank rows, and what a sequence keeps of a position is the normed key latent c
+ * [kv_rank] and one rotated key part [rot] for all heads.  Per head, with q = (q_n, q_r) and positions 0 <= i - j < window (window <= 0:
+ * every earlier position),
+ *     s_ij = scale (q_n . (W_uk c_j) + q_r . k_r,j),   o_i = sum_j softmax_j(s_ij) (W_uv c_j),   y = T(o * sigmoid(gate))
+ * Sizes with a true counterpart (q_dim of q_rank, kv_dim of kv_rank) are that size rounded up to a multiple of 8, zeros behind it; nope, rot
+ * and vdim are rounded up likewise.  The two halves of a rotation are stored side by side (elements 2 i and 2 i + 1 of a rotated
+ * part are the i-th pair), in the weights' rows and so in q and in the cache; angles [t_max, rot / 2, 2] holds (cos, sin) of every
+ * position and pair, (1, 0) behind the true pairs.
+ * Input rows z [B*S, ldz] (float when z_f32, else T): query latent [q_rank] | key latent [kv_rank] | rotated key part [rot] | gate
+ * [heads * vdim]; a layer that reads another layer's cache (own_kv = 0) has no middle two.
+ * raven_latent_rows: cq = T(RMSNorm(query latent) * q_norm) [B*S, q_rank] (cq NULL: not wanted) and, with own_kv, the rows' cache entries at
+ *   pos0 (or *pos_dev) + 0 .. S - 1.
+ * raven_latent_attention: q [B*S, heads * (nope + rot)] of T is W_uq cq (not rotated yet); the rows' own entries are in the cache.  Three
+ *   routes: bf16 chunks of 16 and more rows expand the visible latents to keys and values and run on the matrix cores; other bf16 rows
+ *   take W_uk over to the query and attend to the latents themselves, on the matrix cores too; fp32 rows do that on the vector units.
+ *   raven_latent_attention_workspace_bytes with the same pos0 or a larger one. */
+typedef struct raven_latent {
+    const void*  w_uq;    /* [heads * (nope + rot), q_rank], per head nope | rot                        */
+    const void*  w_uk_t;  /* [heads, kv_rank, nope]: W_uk of a head, transposed                         */
+    const void*  w_ukv;   /* [heads * nope + heads * vdim, kv_rank]: W_uk of all heads, W_uv of all heads */
+    const float* q_norm;  /* [q_rank]  */
+    const float* kv_norm; /* [kv_rank] */
+    float        scale, eps;
+    int32_t      heads, q_dim, q_rank, kv_dim, kv_rank, nope, rot, vdim, window, own_kv;
+} raven_latent;
+typedef struct raven_latent_cache {
+    void*        latent;  /* [batch, t_max, kv_rank] of T */
+    void*        rotated; /* [batch, t_max, rot] of T     */
+    const float* angles;  /* [t_max, rot / 2, 2]          */
+    int32_t      batch, t_max;
+} raven_latent_cache;
+int    raven_latent_rows(const raven_latent* l, const void* z, int32_t ldz, int32_t z_f32, const raven_latent_cache* cache, void* cq, int32_t B,
+                         int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t dtype, void* stream);
+size_t raven_latent_attention_workspace_bytes(const raven_latent* l, int32_t B, int32_t S, int32_t pos0, int32_t dtype);
+int    raven_latent_attention(const raven_latent* l, const void* q, const void* z, int32_t ldz, int32_t z_f32, const raven_latent_cache* cache,
+                              void* y, int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, int32_t dtype, void* workspace,
+                              size_t workspace_bytes, void* stream);
+
+/* Real-gated linear recurrent unit behind a causal convolution per channel.  z [B*S, 2 * width] of T holds v | x;
+ *     u_t = conv_bias + sum_j conv[j] x_(t - taps + 1 + j),   r = sigmoid(W_r u + b_r),   i = sigmoid(W_i u + b_i)    (W block-diagonal)
+ *     log a = -8 r softplus(lam),   S_t = a S_(t-1) + sqrt(1 - a^2) i u,   y = T(S gelu(v))      (gelu in its tanh form)
+ * gates [blocks, 2, block, block_ld] of T: per block the rows of W_r, then those of W_i, `block` = width / blocks true columns, block_ld the
+ * size rounded up to a multiple of 8; width is padded block by block: blocks * block_ld channels, all vectors and z likewise.
+ * ring [batch, taps, width] float carries the rows x (position p in row p mod taps), state [batch, width] float the recurrence; both count as
+ * zero before position 0.  u is rounded to T. */
+typedef struct raven_rglru {
+    const float* conv;       /* [taps, width]        */
+    const float* conv_bias;  /* [width]              */
+    const void*  gates;      /* [blocks, 2, block_ld, block_ld] */
+    const float* gate_bias;  /* [2, width]: b_r, b_i */
+    const float* softplus;   /* [width]: softplus(lam) */
+    int32_t      blocks, block_ld, taps, width;
+} raven_rglru;
+size_t raven_rglru_workspace_bytes(const raven_rglru* l, int32_t B, int32_t S, int32_t dtype);
+int    raven_rglru_forward(const raven_rglru* l, const void* z, float* ring, float* state, void* y, int32_t B, int32_t S, int32_t pos0,
+                           const int32_t* pos_dev, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
+
+/* Mixture of gated experts, added to the stream: x += sum over the `top` experts of largest score of E(s h) + sigmoid(g) E_shared(h), with
+ * s = sigmoid(router logit) of the expert (not renormalised; it scales the expert's input) and E(h) = W_down (silu(W_gate h) * (W_up h)).
+ * logits [M, logit_ld] float: one column per expert, then g (with a shared expert).  h [M, ld] of T, x [M, ld] float.
+ * Equal scores: the lower index wins.  Chunks run the experts as one grouped product, few rows (and fp32) row by row. */
+typedef struct raven_moe {
+    const void* router;      /* [logit_ld, ld]: a row per expert, the shared expert's gate, zeros */
+    const void* up;          /* [experts, 2 * ff, ld]: gate rows, then up rows */
+    const void* down;        /* [experts, ld, ff] */
+    const void* shared_up;   /* [2 * shared_ff, ld] or NULL */
+    const void* shared_down; /* [ld, shared_ff] */
+    int32_t     experts, top, ff, shared_ff, logit_ld;
+} raven_moe;
+size_t raven_moe_workspace_bytes(const raven_moe* m, int32_t M, int32_t ld, int32_t dtype);
+int    raven_moe_forward(const raven_moe* m, const void* h, const float* logits, float* x, int32_t M, int32_t ld, int32_t dtype, void* workspace, size_t workspace_bytes, void* stream);
+
 /* One pre-norm layer on the stream x [B*S, ld] (in place):
- *     h = norm1(x) [+ causal convolution];  x += mixer(h);  x += down(gelu(up(norm2(x))))      (up NULL: no feed-forward)
+ *     h = norm1(x) [+ causal convolution];  x += mixer(h);  x += ff(norm2(x))
  * mixer RAVEN_MIXER_ATTENTION: w_in = q | k rows [(heads + kv_heads) * head_dim, ld].  RAVEN_MIXER_GENERAL_DELTA: w_in = r | k | v | g | a
  * | low [5 * heads * head_dim + rank, ld] (rank a multiple of 8), w_decay = [heads * head_dim, rank]: decay logits =
- * w_decay tanh(low) + decay_bias.  w_out [ld, heads * head_dim], up [ff, ld], down [ld, ff].  Weights of T, vectors float. */
-enum { RAVEN_MIXER_ATTENTION = 0, RAVEN_MIXER_GENERAL_DELTA = 1 };
+ * w_decay tanh(low) + decay_bias.  RAVEN_MIXER_LATENT: `latent`, w_in = the rows of z, heads * head_dim = latent's heads * vdim.
+ * RAVEN_MIXER_RGLRU: `rglru`, w_in = v | x rows [2 * width, ld], in_bias [2 * width], heads * head_dim = width.
+ * w_out [ld, heads * head_dim].  ff: RAVEN_FF_GELU down gelu(up h) with up [ff, ld], down [ld, ff] (up NULL: no feed-forward); RAVEN_FF_SWIGLU the
+ * same with up [2 * ff, ld] (gate rows, up rows) and silu(gate) * up; RAVEN_FF_MOE `moe`.  Weights of T, vectors float. */
+enum { RAVEN_MIXER_ATTENTION = 0, RAVEN_MIXER_GENERAL_DELTA = 1, RAVEN_MIXER_LATENT = 2, RAVEN_MIXER_RGLRU = 3 };
+enum { RAVEN_FF_GELU = 0, RAVEN_FF_SWIGLU = 1, RAVEN_FF_MOE = 2 };
 typedef struct raven_mixer_layer {
     const float* norm1;
     const float* conv;        /* [taps, ld] or NULL */
@@ -463,19 +539,27 @@ typedef struct raven_mixer_layer {
     const void*  down;
     raven_score  score;
     int32_t      mixer, heads, kv_heads, dim, head_dim, rank, taps, ff;
+    const float* in_bias;     /* RAVEN_MIXER_RGLRU */
+    const raven_latent* latent; /* host structures */
+    const raven_rglru*  rglru;
+    const raven_moe*    moe;
+    int32_t      ff_kind;
 } raven_mixer_layer;
 typedef struct raven_stream_dims {
     int32_t width, ld;
     float   eps;
     int32_t dtype;
 } raven_stream_dims;
-/* What one run of a layer keeps of a batch of sequences: ring [B, taps, ld]; keys (attention) or state (delta rule). */
+/* What one run of a layer keeps of a batch of sequences: ring [B, taps, ld or width]; keys (attention), latents (latent attention; those of
+ * another layer when it reads from there) or state (delta rule, recurrent unit). */
 typedef struct raven_mixer_state {
-    float*          ring;
-    float*          state;
-    raven_key_cache keys;
+    float*             ring;
+    float*             state;
+    raven_key_cache    keys;
+    raven_latent_cache latent;
 } raven_mixer_state;
-size_t raven_mixer_layer_workspace_bytes(const raven_stream_dims* dims, const raven_mixer_layer* layer, int32_t B, int32_t S);
+/* pos0: position of the first row (or the largest it will have); only latent attention's need depends on it. */
+size_t raven_mixer_layer_workspace_bytes(const raven_stream_dims* dims, const raven_mixer_layer* layer, int32_t B, int32_t S, int32_t pos0);
 int    raven_mixer_layer_forward(const raven_stream_dims* dims, const raven_mixer_layer* layer, const raven_mixer_state* state, float* x,
                                  int32_t B, int32_t S, int32_t pos0, const int32_t* pos_dev, void* workspace, size_t workspace_bytes,
                                  void* stream);

@@ -21,8 +21,9 @@ from .adaptive import (  # noqa: F401
     get_adaptive_exit_evaluator,
 )
 from .cache import HuginnDynamicCache, HuginnStaticCache, MixerStateCache, RequestCaches, remap_step  # noqa: F401
-from .config import GitipelConfig, RavenConfig  # noqa: F401
-from .gitipel import GitipelForCausalLM, MixerDecodeRunner  # noqa: F401
+from .config import GitipelConfig, GupitarConfig, RavenConfig  # noqa: F401
+from .gitipel import GitipelForCausalLM  # noqa: F401
+from .gupitar import GupitarForCausalLM  # noqa: F401
 from .modeling import (  # noqa: F401
     CausalLMOutputRecurrentLatents,
     DecodeRunner,
@@ -32,12 +33,14 @@ from .modeling import (  # noqa: F401
 )
 from .paged import PagedDecoder  # noqa: F401
 from .registry import family_of, load_model  # noqa: F401
+from .stream_decoder import MixerDecodeRunner, StreamDecoderForCausalLM  # noqa: F401
 
 __all__ = [
     "hip", "HuginnDynamicCache", "HuginnStaticCache", "remap_step", "RavenConfig", "RavenForCausalLM", "DecodeRunner",
     "CausalLMOutputRecurrentLatents", "GenerationSettings", "precompute_freqs_cis", "adaptive", "vllm_binding",
     "PerIterationExitEvaluator", "NoOpExitEvaluator", "EntropyDiffExitEvaluator", "LatentDiffExitEvaluator",
     "KLExitEvaluator", "MinKLExitEvaluator", "ArgmaxStabilityExitEvaluator", "CosineExitEvaluator", "NumStepsGenerator",
-    "get_adaptive_exit_evaluator", "PagedDecoder", "GitipelConfig", "GitipelForCausalLM", "MixerDecodeRunner", "MixerStateCache",
+    "get_adaptive_exit_evaluator", "PagedDecoder", "GitipelConfig", "GitipelForCausalLM", "GupitarConfig",
+    "GupitarForCausalLM", "StreamDecoderForCausalLM", "MixerDecodeRunner", "MixerStateCache",
     "RequestCaches", "family_of", "load_model",
 ]

@@ -12,7 +12,8 @@ CSRC = os.path.join(PKG_DIR, "csrc")
 LIB_DIR = os.path.join(PKG_DIR, "lib")
 LIB_PATH = os.path.join(LIB_DIR, "libraven_hip.so")
 SOURCES = ["rmsnorm.hip", "gemm_skinny.hip", "gemm_splitk.hip", "gemm_tiled.hip", "gemv_decode.hip", "attention.hip", "attention_prefill.hip", "misc.hip", "exit_stats.hip", "compose.hip",
-           "tuning.hip", "norm_conv.hip", "attention_capped.hip", "delta_rule.hip", "compose_mixer.hip"]
+           "tuning.hip", "norm_conv.hip", "attention_capped.hip", "delta_rule.hip", "latent_attention.hip", "rglru.hip", "moe.hip",
+           "compose_mixer.hip"]
 
 HIPCC_FLAGS = [
     "--offload-arch=gfx950", "-O3", "-std=c++17", "-fPIC",

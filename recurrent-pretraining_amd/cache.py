@@ -461,9 +461,14 @@ class HuginnStaticCache(HuginnDynamicCache):
 
 
 class MixerStateCache:
-    """What a decoder with a list of mixers keeps of a batch of sequences that share their length: per layer RUN (a looped layer
-    has a state per pass) the last rows of the input convolution, and either the keys of every position or the recurrent state
-    matrices.  `plan` describes the runs: dicts with taps, ld, heads, head_dim and, for attention, kv_heads.
+    """What a decoder with a list of mixers keeps of a batch of sequences that share their length.  `plan` holds a dictionary per layer
+    RUN (a looped layer has a state per pass), with any of
+      taps, ld             the last rows of a convolution: a ring [batch, taps, ld] of floats
+      kv_heads, head_dim   the keys of every position
+      latent = (kp, rp)    the key latent and the rotated key part of every position, with
+      angles = (base, n)   the rotation's (cos, sin) of every position, n rotated dimensions, pair by pair
+      latent_from          another run, whose latents this one reads
+      state                the shape of a recurrent state (floats); heads and head_dim without kv_heads: [heads, head_dim, head_dim].
 
     Only the token count says what is in it: rows and states before position 0 are taken as zero by the kernels and keys past
     the length are never read, so a cache is given back and used again by resetting the count.  A recurrent state cannot be
@@ -480,9 +485,24 @@ class MixerStateCache:
         self.dtype: Optional[torch.dtype] = None
         self.rings: list = []
         self.keys: list = []      # per run [batch, kv_heads, t_max, head_dim], or None
-        self.states: list = []    # per run [batch, heads, head_dim, head_dim] float, or None
+        self.latents: list = []   # per run ([batch, t_max, kp], [batch, t_max, rp]), or None
+        self.states: list = []    # per run [batch, ...] float, or None
+        self.angles: dict = {}    # (base, n, rp) -> [t_max, rp] float
         self._structs: list = []
         self.generation = 0       # grows with every reallocation: captured launches hold pointers
+
+    @staticmethod
+    def _state_shape(p: dict):
+        if p.get("state") is not None:
+            return tuple(p["state"])
+        return None if p.get("kv_heads") or "heads" not in p else (p["heads"], p["head_dim"], p["head_dim"])
+
+    @staticmethod
+    def rotation_angles(base: float, n: int, rp: int, t_max: int, device) -> torch.Tensor:
+        """(cos, sin) of position * base^(-2 i / n) for pair i, [t_max, rp]; (1, 0) behind the n / 2 pairs."""
+        freq = base ** (-2.0 * torch.arange(n // 2, dtype=torch.float64) / n)
+        angle = torch.nn.functional.pad(torch.arange(t_max, dtype=torch.float64)[:, None] * freq, (0, (rp - n) // 2))
+        return torch.stack([angle.cos(), angle.sin()], -1).view(t_max, rp).float().to(device)
 
     def ensure(self, batch: int, t_needed: int, dtype: torch.dtype, device) -> None:
         """Room for t_needed positions of `batch` sequences; contents survive growth."""
@@ -501,22 +521,36 @@ class MixerStateCache:
             while new_t < t_needed:
                 new_t *= 2
         new_t = (new_t + 15) // 16 * 16  # whole cache lines per head, whatever the head size (a multiple of 8 elements)
-        old = self.keys if self.batch else None
-        keys = [torch.zeros(batch, p["kv_heads"], new_t, p["head_dim"], dtype=dtype, device=device) if p.get("kv_heads") else None
-                for p in self.plan]
-        if old is not None:
-            for k, o in zip(keys, old):
-                if k is not None:
-                    k[:, :, :o.shape[2]] = o
+        zeros = lambda *shape, dt=torch.float32: torch.zeros(*shape, dtype=dt, device=device)
+        keys = [zeros(batch, p["kv_heads"], new_t, p["head_dim"], dt=dtype) if p.get("kv_heads") else None for p in self.plan]
+        latents = [tuple(zeros(batch, new_t, n, dt=dtype) for n in p["latent"]) if p.get("latent") else None for p in self.plan]
+        if self.batch:
+            for new, old in zip(keys, self.keys):
+                if new is not None:
+                    new[:, :, :old.shape[2]] = old
+            for new, old in zip(latents, self.latents):
+                for n, o in zip(new or (), old or ()):
+                    n[:, :o.shape[1]] = o
         else:
-            self.rings = [torch.zeros(batch, p["taps"], p["ld"], dtype=torch.float32, device=device) for p in self.plan]
-            self.states = [None if p.get("kv_heads") else
-                           torch.zeros(batch, p["heads"], p["head_dim"], p["head_dim"], dtype=torch.float32, device=device) for p in self.plan]
-        self.keys, self.batch, self.t_max, self.dtype = keys, batch, new_t, dtype
-        self._structs = [hip.MixerState(r.data_ptr(), None if s is None else s.data_ptr(),
-                                        hip.KeyCache() if k is None else hip.KeyCache(k.data_ptr(), *[k.shape[i] for i in (0, 1, 3, 2)]))
-                         for r, s, k in zip(self.rings, self.states, self.keys)]
+            self.rings = [zeros(batch, p["taps"], p["ld"]) if p.get("taps") else None for p in self.plan]
+            shapes = [self._state_shape(p) for p in self.plan]
+            self.states = [None if s is None else zeros(batch, *s) for s in shapes]
+        self.keys, self.latents, self.batch, self.t_max, self.dtype = keys, latents, batch, new_t, dtype
+        self.angles = {key: self.rotation_angles(*key, new_t, device)
+                       for key in {(*p["angles"], p["latent"][1]) for p in self.plan if p.get("latent")}}
+        self._structs = [self._struct(run) for run in range(len(self.plan))]
         self.generation += 1
+
+    def _struct(self, run: int) -> "hip.MixerState":
+        ptr = lambda t: None if t is None else t.data_ptr()
+        k, source = self.keys[run], self.plan[run].get("latent_from", run)
+        keys = hip.KeyCache() if k is None else hip.KeyCache(k.data_ptr(), *[k.shape[i] for i in (0, 1, 3, 2)])
+        latent = hip.LatentCache()
+        if self.latents[source] is not None:
+            c, r = self.latents[source]
+            angles = self.angles[(*self.plan[source]["angles"], self.plan[source]["latent"][1])]
+            latent = hip.LatentCache(c.data_ptr(), r.data_ptr(), angles.data_ptr(), self.batch, self.t_max)
+        return hip.MixerState(ptr(self.rings[run]), ptr(self.states[run]), keys, latent)
 
     def native(self, run: int) -> "hip.MixerState":
         return self._structs[run]
@@ -532,7 +566,8 @@ class MixerStateCache:
 
     def get_memory_usage(self) -> float:
         """MiB allocated."""
-        return sum(t.nelement() * t.element_size() for group in (self.rings, self.keys, self.states) for t in group if t is not None) / 2 ** 20
+        held = [*self.rings, *self.keys, *self.states, *self.angles.values(), *(t for pair in self.latents if pair for t in pair)]
+        return sum(t.nelement() * t.element_size() for t in held if t is not None) / 2 ** 20
 
 
 class RequestCaches:

@@ -132,3 +132,64 @@ class GitipelConfig(PretrainedConfig):
             return [(i, None) for i in range(n)]
         inside = [(i, t) for t in range(loop["times"]) for i in range(loop["start"], loop["stop"])]
         return [(i, None) for i in range(loop["start"])] + inside + [(i, None) for i in range(loop["stop"], n)]
+
+
+class GupitarConfig(PretrainedConfig):
+    """Shape of a Gupitar decoder, with the field names of its `config.json`: a list of layers, each a mixer (latent attention or a real-gated
+    linear recurrent unit) with its sizes and a feed-forward (dense, a mixture of experts, or none).  Every size and constant comes
+    from here."""
+
+    model_type = "gupitar"
+    attribute_map = {"vocab_size": "vocab", "hidden_size": "width", "n_embd": "width"}
+
+    architecture: str = "Gupitar"
+    vocab: int = 256
+    width: int = 64
+    layers: list | None = None
+    norm: dict | None = None
+
+    def __post_init__(self, **kwargs):
+        for alias, field in self.attribute_map.items():
+            if kwargs.get(alias) is not None:
+                setattr(self, field, kwargs[alias])
+            kwargs.pop(alias, None)
+        kwargs.pop("model_type", None)
+        kwargs.pop("num_hidden_layers", None)
+        self.layers = [dict(x) for x in (self.layers or [])]
+        self.norm = self.norm or {"eps": 1e-6}
+        if self.architecture != "Gupitar":
+            raise ValueError(f"not a Gupitar configuration: architecture {self.architecture!r}")
+        for i, layer in enumerate(self.layers):
+            self._check_mixer(i, layer["type"], layer["mixer"])
+            mlp = layer.get("mlp")
+            if mlp is None or mlp["kind"] == "dense":
+                continue
+            if mlp["kind"] != "moe":
+                raise ValueError(f"layer {i}: unknown feed-forward {mlp['kind']!r}")
+            if not 1 <= mlp["router"]["top"] <= mlp["router"]["experts"]:
+                raise ValueError(f"layer {i}: top {mlp['router']['top']} of {mlp['router']['experts']} experts")
+        self.num_hidden_layers = len(self.layers)
+        kwargs["tie_word_embeddings"] = False
+        if self.dtype is None and kwargs.get("torch_dtype") is None:
+            self.dtype = "bfloat16"
+        super().__post_init__(**kwargs)
+
+    def _check_mixer(self, i: int, kind: str, m: dict) -> None:
+        if kind == "rglru":
+            if m["width"] % m["blocks"]:
+                raise ValueError(f"layer {i}: {m['blocks']} blocks over {m['width']} channels")
+            return
+        if kind != "latent_attention":
+            raise ValueError(f"layer {i}: unknown mixer {kind!r}")
+        if m["rot_dim"] % 2 or m["rot"]["dims"] != m["rot_dim"]:
+            raise ValueError(f"layer {i}: a rotation of {m['rot']['dims']} of {m['rot_dim']} rotated dimensions")
+        if m.get("mask") is not None and m["mask"]["size"] < 1:
+            raise ValueError(f"layer {i}: a window of {m['mask']['size']}")
+        source = m.get("kv_from")
+        if source is None:
+            return
+        if not 0 <= source < i or self.layers[source]["type"] != "latent_attention" or self.layers[source]["mixer"].get("kv_from") is not None:
+            raise ValueError(f"layer {i}: reads the latents of layer {source}, which must come earlier and have latents of its own")
+        other = self.layers[source]["mixer"]
+        if any(other[k] != m[k] for k in ("kv_rank", "rot_dim")) or other["rot"]["base"] != m["rot"]["base"]:
+            raise ValueError(f"layer {i}: kv_rank, rot_dim and rotation must equal those of layer {source}")

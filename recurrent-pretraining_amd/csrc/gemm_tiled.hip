@@ -63,6 +63,14 @@ struct TiledArgs {
     int out_f32;
     int tiles_m, tiles_n;
     raven_epilogue epi;    // EPI_FREE only (y and residual [M, ldy])
+    // Products of row groups with a weight matrix each (grouped_gemm): tile row t multiplies rows group_row[t] .. group_row[t] + BM - 1
+    // (below group_end[t]) with the matrix of group group_of[t]; group_of < 0: no such tile
+    struct Groups {
+        const int *group_of, *group_row, *group_end;
+        const int* x_row;        // row of x0 behind a row of the product, or null: the same
+        const float* x_scale;    // SwiGLU: factor of a row of x0, applied to its sums
+        int64_t w_stride;        // elements between two groups' matrices
+    } groups;
     int rope_on;           // the epilogue below instead of y
     // The product is a chunk's fused q | k | v rows (3 * nh * hd columns): instead of y, the epilogue adds the q / k bias,
     // rotates q and k (RoPE on adjacent pairs) and writes q to q_out and k, v to their cache rows -- what
@@ -154,7 +162,7 @@ __device__ __forceinline__ void store_tiles(const TiledArgs& a, const f32x4 (&ac
 
 // The accumulators of a workgroup laid down in LDS as the output tile (rows of BN_OUT columns, 16-byte unit u of row r at
 // position u ^ (r mod units per row)), between two workgroup barriers: the first because the K loop's stages are reused.
-template <int EPI, int TM, int TN, int WM, int WN>
+template <int EPI, int TM, int TN, int WM, int WN, bool GROUPED = false>
 __device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_n, int wave, int lane, unsigned lds_base) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
@@ -178,12 +186,15 @@ __device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&
         const int row = (wm * NB + tb) * 16 + l16;
         const unsigned row_addr = lds_base + row * RB + (q4 & 1) * 8;
         const int sw = row & (U - 1);
+        const float xs = GROUPED && SWIGLU ? a.groups.x_scale[min(row, a.M - 1)] : 1.f;
 #pragma unroll
         for (int t = 0; t < NT; ++t) {
             bf16 o[4];
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                if (SWIGLU) {
+                if (SWIGLU && GROUPED) {
+                    o[i] = from_f32<bf16>(silu_f32(acc[2 * t][tb][i] * xs) * (acc[2 * t + 1][tb][i] * xs));
+                } else if (SWIGLU) {
                     const float g = round_to<bf16>(acc[2 * t][tb][i]), u = round_to<bf16>(acc[2 * t + 1][tb][i]);
                     o[i] = from_f32<bf16>(round_to<bf16>(silu_f32(g)) * u);
                 } else if (is_free(EPI)) {
@@ -210,7 +221,7 @@ __device__ __forceinline__ void lay_tiles_lds(const TiledArgs& a, const f32x4 (&
 // residual is fetched the same way, before the tile is laid down, so that its latency hides behind the transposition.
 // 16-byte unit u of tile row r sits at position u ^ (r mod units per row): the 16 rows a store instruction spreads over
 // then fall on different banks.
-template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4, bool GROUPED = false>
 __device__ __forceinline__ void store_tiles_lds(const TiledArgs& a, const f32x4 (&acc)[2 * TN][2 * TM], int tile_m, int tile_n, int wave,
                                                 int lane, unsigned lds_base) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
@@ -230,7 +241,7 @@ __device__ __forceinline__ void store_tiles_lds(const TiledArgs& a, const f32x4 
         res[it] = u32x4{0, 0, 0, 0};
         if (EPI == EPI_PLAIN && a.residual && goff[it] >= 0) res[it] = *reinterpret_cast<const u32x4*>(a.residual + goff[it]);
     }
-    lay_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_n, wave, lane, lds_base);
+    lay_tiles_lds<EPI, TM, TN, WM, WN, GROUPED>(a, acc, tile_n, wave, lane, lds_base);
 #pragma unroll
     for (int it = 0; it < ITERS; ++it) {
         const int idx = (wave * ITERS + it) * 64 + lane;
@@ -336,7 +347,8 @@ __device__ __forceinline__ void store_tiles_rope(const TiledArgs& a, const f32x4
 
 __device__ __align__(16) unsigned int g_zero_piece[4];  // what a 16-byte piece past the end of K is loaded from
 
-template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
+// GROUPED: row groups with a weight matrix each (TiledArgs::groups); a tile works on a copy of the arguments cut to its group's rows
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4, bool GROUPED = false>
 __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32;
@@ -364,7 +376,20 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
     const int gsz = min(a.tiles_m - first_m, GROUP);
     const int in_band = logical - band * GROUP * a.tiles_n;
     const int tile_n = in_band / gsz;
-    const int tile_m = first_m + (in_band - tile_n * gsz);
+    int tile_m = first_m + (in_band - tile_n * gsz);
+    const int* x_row = nullptr;
+    if constexpr (GROUPED) {
+        const int g = a.groups.group_of[tile_m];
+        if (g < 0) return;
+        const int row = a.groups.group_row[tile_m];
+        a.M = a.groups.group_end[tile_m] - row;
+        a.w += g * a.groups.w_stride;
+        a.y = static_cast<char*>(a.y) + (int64_t)row * a.ldy * (a.out_f32 ? 4 : 2);
+        if (EPI == EPI_SWIGLU) a.groups.x_scale += row;
+        if (a.groups.x_row) x_row = a.groups.x_row + row;
+        else a.x0 += (int64_t)row * a.ldx;
+        tile_m = 0;
+    }
 
     const int lane = threadIdx.x & 63;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -388,6 +413,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
             else row = min(tile_n * BN + r, a.N - 1);
         } else {
             row = min(tile_m * BM + (r - BN), a.M - 1);
+            if (GROUPED && x_row) row = x_row[row];
         }
         goff[p] = (unsigned)row * ld2 + 2u * col8;
     }
@@ -567,7 +593,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
         }
     }
     if (a.out_f32) store_tiles<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
-    else store_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    else store_tiles_lds<EPI, TM, TN, WM, WN, GROUPED>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -804,26 +830,26 @@ int g_tiled_min_rows = 33;  // raven_set_tuning("gemm_tiled_min_rows"): fewest r
 int g_tiled_variant = 0;    // raven_set_tuning("gemm_tiled_variant"): 0 = by shape, 1 = 256 x 256 tiles, 2 = 128 x 128 tiles, 3 = 256 x 256 tiles by the eight-wave kernel
 int g_tiled_split_tail = 1; // raven_set_tuning("gemm_tiled_split_tail"): 0 = never hand the last round's tile columns to 128 x 128 tiles
 
-template <int EPI, int TM, int TN, int WM = 2, int WN = 4>
+template <int EPI, int TM, int TN, int WM = 2, int WN = 4, bool GROUPED = false>
 static int launch_tiled(TiledArgs a, hipStream_t s) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = WM * TM * 32, BN = WN * TN * 32, BN_OUT = SWIGLU ? BN / 2 : BN;
     constexpr size_t lds = (size_t)2 * (BM + BN) * 128;
     static bool attr_set = false;
     if (!attr_set) {
-        hipError_t e = hipFuncSetAttribute((const void*)gemm_tiled_kernel<EPI, TM, TN, WM, WN>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        hipError_t e = hipFuncSetAttribute((const void*)gemm_tiled_kernel<EPI, TM, TN, WM, WN, GROUPED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) {
             raven_host::set_error("gemm (tiled): hipFuncSetAttribute failed: %s", hipGetErrorString(e));
             return (int)e;
         }
         attr_set = true;
     }
-    a.tiles_m = (a.M + BM - 1) / BM;
+    if (!GROUPED) a.tiles_m = (a.M + BM - 1) / BM;
     a.tiles_n = (a.N + BN_OUT - 1) / BN_OUT;
     const int64_t n_tiles = (int64_t)a.tiles_m * a.tiles_n;
     RAVEN_REQUIRE(n_tiles < (1 << 28), "gemm (tiled): too many tiles (M=%d N=%d)", a.M, a.N);
     const unsigned grid = (unsigned)((n_tiles + 7) / 8 * 8);
-    gemm_tiled_kernel<EPI, TM, TN, WM, WN><<<dim3(grid), dim3(64 * WM * WN), lds, s>>>(a);
+    gemm_tiled_kernel<EPI, TM, TN, WM, WN, GROUPED><<<dim3(grid), dim3(64 * WM * WN), lds, s>>>(a);
     return raven_host::check_launch("gemm (tiled MFMA)");
 }
 
@@ -946,6 +972,26 @@ int tiled_gemm(const void* x0, const void* x1, const void* w, const void* residu
 int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi,
                     hipStream_t s) {
     return tiled_gemm_impl(x0, 0, x1, w, nullptr, y, M, N, K0, K1, 0, epi.out_f32, nullptr, s, &epi);
+}
+
+// Products of row groups (128 rows to a tile row): y[r] = x[x_row[r]] W_g^T, W_g = w + g * w_stride [N or 2N, K] of the group that row r of the
+// product belongs to.  swiglu: y = T(silu(s gate) * (s up)) with s = x_scale[r]; else y float.  n_tiles: entries of the three tile
+// tables (unused ones have group_of < 0); rows: rows of the product, x_rows: rows of x.
+int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, void* y, int rows, int N, int K, int swiglu, const int* group_of,
+                 const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s) {
+    RAVEN_REQUIRE(x && w && y && group_of && group_row && group_end && n_tiles > 0 && N > 0 && N % 8 == 0 && K > 0 && K % 8 == 0 && (!swiglu || x_scale),
+                  "gemm (grouped): bad arguments");
+    RAVEN_REQUIRE((int64_t)x_rows * K < (1ll << 31) && (int64_t)N * 2 * K < (1ll << 31) && (int64_t)rows * N < (1ll << 40), "gemm (grouped): too large");
+    TiledArgs a{};
+    a.w = static_cast<const bf16*>(w);
+    a.x0 = static_cast<const bf16*>(x);
+    a.y = y;
+    a.M = rows; a.N = N; a.K0 = K; a.out_f32 = !swiglu;
+    a.ldy = N; a.up_off = N; a.ldw = K; a.ldx = K;
+    a.tiles_m = n_tiles;
+    a.epi.scale = 1.f;
+    a.groups = TiledArgs::Groups{group_of, group_row, group_end, x_row, x_scale, w_stride};
+    return swiglu ? launch_tiled<EPI_SWIGLU, 2, 1, 2, 4, true>(a, s) : launch_tiled<EPI_FREE, 2, 1, 2, 4, true>(a, s);
 }
 
 // The same with the rows of x `ldx` elements apart (>= K, one segment): activations whose rows are padded to whole cache lines

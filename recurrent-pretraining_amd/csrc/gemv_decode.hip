@@ -307,7 +307,7 @@ static int launch_gemv1(Gemv1Args a, hipStream_t s) {
     } while (0)
     if (a.dim > 0) {  // PRO_STREAM
         RAVEN_REQUIRE(c <= 3, "gemv: K=%d is too long for the float-row norm prologue", a.K);
-        if constexpr (is_free(EPI)) {
+        if constexpr (is_free(EPI) || SWIGLU) {
             if (ppw > 1) gemv1_kernel<T, 3, EPI, PRO_STREAM, true><<<dim3(wgs), dim3(256), 0, s>>>(a);
             else gemv1_kernel<T, 3, EPI, PRO_STREAM, false><<<dim3(wgs), dim3(256), 0, s>>>(a);
         }
@@ -371,6 +371,12 @@ int gemv1_stream(const float* x, const float* norm, int dim, float eps, const vo
     Gemv1Args a{};
     a.w = w; a.x0 = x; a.norm_a = norm; a.y = y; a.N = N; a.K = K; a.k0 = K; a.ldw = K; a.epi = epi; a.dim = dim; a.eps = eps;
     return gemv1_free_dispatch(a, dtype, s);
+}
+// ... and with the SwiGLU epilogue: w [2 N, K], y [N] of T
+int gemv1_stream_swiglu(const float* x, const float* norm, int dim, float eps, const void* w, void* y, int N, int K, int dtype, hipStream_t s) {
+    Gemv1Args a{};
+    a.w = w; a.x0 = x; a.norm_a = norm; a.y = y; a.N = N; a.K = K; a.k0 = K; a.ldw = K; a.dim = dim; a.eps = eps;
+    return dtype == RAVEN_BF16 ? launch_gemv1<bf16, EPI_SWIGLU>(a, s) : launch_gemv1<float, EPI_SWIGLU>(a, s);
 }
 
 }  // namespace raven

@@ -58,10 +58,30 @@ class Score(C.Structure):
     _fields_ = [("scale", C.c_float), ("softcap", C.c_float), ("r1", C.c_void_p), ("r2", C.c_void_p)]
 
 
+class Latent(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("w_uq", "w_uk_t", "w_ukv", "q_norm", "kv_norm")] + [("scale", C.c_float), ("eps", C.c_float)] + [
+        (n, C.c_int32) for n in ("heads", "q_dim", "q_rank", "kv_dim", "kv_rank", "nope", "rot", "vdim", "window", "own_kv")]
+
+
+class LatentCache(C.Structure):
+    _fields_ = [("latent", C.c_void_p), ("rotated", C.c_void_p), ("angles", C.c_void_p), ("batch", C.c_int32), ("t_max", C.c_int32)]
+
+
+class Rglru(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("conv", "conv_bias", "gates", "gate_bias", "softplus")] + [
+        (n, C.c_int32) for n in ("blocks", "block_ld", "taps", "width")]
+
+
+class Moe(C.Structure):
+    _fields_ = [(n, C.c_void_p) for n in ("router", "up", "down", "shared_up", "shared_down")] + [
+        (n, C.c_int32) for n in ("experts", "top", "ff", "shared_ff", "logit_ld")]
+
+
 class MixerLayer(C.Structure):
     _fields_ = [(n, C.c_void_p) for n in ("norm1", "conv", "w_in", "w_decay", "decay_bias", "a_bias", "out_norm", "w_out", "norm2",
                                           "up", "down")] + [("score", Score)] + [
-        (n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "head_dim", "rank", "taps", "ff")]
+        (n, C.c_int32) for n in ("mixer", "heads", "kv_heads", "dim", "head_dim", "rank", "taps", "ff")] + [
+        ("in_bias", C.c_void_p), ("latent", C.POINTER(Latent)), ("rglru", C.POINTER(Rglru)), ("moe", C.POINTER(Moe)), ("ff_kind", C.c_int32)]
 
 
 class StreamDims(C.Structure):
@@ -69,12 +89,13 @@ class StreamDims(C.Structure):
 
 
 class MixerState(C.Structure):
-    _fields_ = [("ring", C.c_void_p), ("state", C.c_void_p), ("keys", KeyCache)]
+    _fields_ = [("ring", C.c_void_p), ("state", C.c_void_p), ("keys", KeyCache), ("latent", LatentCache)]
 
 
 PAGED_NHD, PAGED_HND = 0, 1
 ACT_NONE, ACT_GELU, ACT_TANH = 0, 1, 2
-MIXER_ATTENTION, MIXER_GENERAL_DELTA = 0, 1
+MIXER_ATTENTION, MIXER_GENERAL_DELTA, MIXER_LATENT, MIXER_RGLRU = 0, 1, 2, 3
+FF_GELU, FF_SWIGLU, FF_MOE = 0, 1, 2
 
 
 def _paged_dims(cache: torch.Tensor, layout: int):
@@ -150,7 +171,15 @@ SIGNATURES = {
     "raven_capped_attention": (C.c_int, [_VP, _VP, C.POINTER(KeyCache), C.POINTER(Score), _I32, _I32, _I32, _VP, _I32, _I32, _VP, _SZ, _VP]),
     "raven_delta_rule_workspace_bytes": (_SZ, [_I32, _I32, _I32, _I32]),
     "raven_delta_rule": (C.c_int, [_VP, _I32, _VP, _VP, _VP, _I32, _VP, _VP, _VP, _VP, _I32, _I32, _I32, _VP, _I32, _I32, _I32, _F, _I32, _VP, _SZ, _VP]),
-    "raven_mixer_layer_workspace_bytes": (_SZ, [C.POINTER(StreamDims), C.POINTER(MixerLayer), _I32, _I32]),
+    "raven_latent_rows": (C.c_int, [C.POINTER(Latent), _VP, _I32, _I32, C.POINTER(LatentCache), _VP, _I32, _I32, _I32, _VP, _I32, _VP]),
+    "raven_latent_attention_workspace_bytes": (_SZ, [C.POINTER(Latent), _I32, _I32, _I32, _I32]),
+    "raven_latent_attention": (C.c_int, [C.POINTER(Latent), _VP, _VP, _I32, _I32, C.POINTER(LatentCache), _VP, _I32, _I32, _I32, _VP, _I32, _VP, _SZ,
+                                         _VP]),
+    "raven_rglru_workspace_bytes": (_SZ, [C.POINTER(Rglru), _I32, _I32, _I32]),
+    "raven_rglru_forward": (C.c_int, [C.POINTER(Rglru), _VP, _VP, _VP, _VP, _I32, _I32, _I32, _VP, _I32, _VP, _SZ, _VP]),
+    "raven_moe_workspace_bytes": (_SZ, [C.POINTER(Moe), _I32, _I32, _I32]),
+    "raven_moe_forward": (C.c_int, [C.POINTER(Moe), _VP, _VP, _VP, _I32, _I32, _I32, _VP, _SZ, _VP]),
+    "raven_mixer_layer_workspace_bytes": (_SZ, [C.POINTER(StreamDims), C.POINTER(MixerLayer), _I32, _I32, _I32]),
     "raven_mixer_layer_forward": (C.c_int, [C.POINTER(StreamDims), C.POINTER(MixerLayer), C.POINTER(MixerState), _VP, _I32, _I32, _I32, _VP,
                                             _VP, _SZ, _VP]),
 }
@@ -740,8 +769,57 @@ def delta_rule(z, decay_logits, a_bias, norm, state, B, S, pos0, dim, eps, dtype
     return y
 
 
-def mixer_layer_workspace_bytes(dims: StreamDims, layer: MixerLayer, B: int, S: int) -> int:
-    return load().raven_mixer_layer_workspace_bytes(C.byref(dims), C.byref(layer), B, S)
+def latent_rows(desc: Latent, z, cache: LatentCache, B, S, pos0, dtype, want_cq=True, pos_dev=None):
+    """Normed query latents [B*S, q_rank] of rows z, and with desc.own_kv the rows' cache entries."""
+    cq = torch.empty(B * S, desc.q_rank, device=z.device, dtype=dtype) if want_cq else None
+    rc = load().raven_latent_rows(C.byref(desc), _ptr(z, "z"), z.shape[1], int(z.dtype == torch.float32), C.byref(cache), _ptr(cq, "cq"), B, S,
+                                  int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), dtype_code(dtype), _stream())
+    _check(rc, "raven_latent_rows")
+    return cq
+
+
+def latent_attention(desc: Latent, q, z, cache: LatentCache, B, S, pos0, pos_dev=None):
+    """q [B*S, heads * (nope + rot)], not rotated; the rows' cache entries are in place.  Returns [B*S, heads * vdim]."""
+    if q.shape != (B * S, desc.heads * (desc.nope + desc.rot)) or z.shape[0] != B * S:
+        raise RavenHipError("latent_attention: operand shapes do not fit together")
+    y = torch.empty(B * S, desc.heads * desc.vdim, device=q.device, dtype=q.dtype)
+    code = dtype_code(q.dtype)
+    ws = _workspace(load().raven_latent_attention_workspace_bytes(C.byref(desc), B, S, int(pos0), code), q.device)
+    rc = load().raven_latent_attention(C.byref(desc), _ptr(q, "q"), _ptr(z, "z"), z.shape[1], int(z.dtype == torch.float32), C.byref(cache), _ptr(y, "y"),
+                                       B, S, int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), code, _ptr(ws, "ws"), 0 if ws is None else ws.numel(),
+                                       _stream())
+    _check(rc, "raven_latent_attention")
+    return y
+
+
+def rglru(desc: Rglru, z, ring, state, B, S, pos0, pos_dev=None):
+    """z [B*S, 2 * width] (v | x); ring [B, taps, width] and state [B, width] float, updated in place.  Returns [B*S, width]."""
+    if z.shape != (B * S, 2 * desc.width) or ring.shape != (B, desc.taps, desc.width) or state.shape != (B, desc.width):
+        raise RavenHipError("rglru: operand shapes do not fit together")
+    y = torch.empty(B * S, desc.width, device=z.device, dtype=z.dtype)
+    code = dtype_code(z.dtype)
+    ws = _workspace(load().raven_rglru_workspace_bytes(C.byref(desc), B, S, code), z.device)
+    rc = load().raven_rglru_forward(C.byref(desc), _ptr(z, "z"), _ptr(ring, "ring", torch.float32), _ptr(state, "state", torch.float32), _ptr(y, "y"), B, S,
+                                    int(pos0), _ptr(pos_dev, "pos_dev", torch.int32), code, _ptr(ws, "ws"), 0 if ws is None else ws.numel(), _stream())
+    _check(rc, "raven_rglru_forward")
+    return y
+
+
+def moe(desc: Moe, h, logits, x):
+    """x [M, ld] float += the mixture over rows h [M, ld] with router logits [M, logit_ld] float; in place."""
+    M, ld = h.shape
+    if x.shape != h.shape or logits.shape != (M, desc.logit_ld):
+        raise RavenHipError("moe: operand shapes do not fit together")
+    code = dtype_code(h.dtype)
+    ws = _workspace(load().raven_moe_workspace_bytes(C.byref(desc), M, ld, code), h.device)
+    rc = load().raven_moe_forward(C.byref(desc), _ptr(h, "h"), _ptr(logits, "logits", torch.float32), _ptr(x, "x", torch.float32), M, ld, code,
+                                  _ptr(ws, "ws"), 0 if ws is None else ws.numel(), _stream())
+    _check(rc, "raven_moe_forward")
+    return x
+
+
+def mixer_layer_workspace_bytes(dims: StreamDims, layer: MixerLayer, B: int, S: int, pos0: int = 0) -> int:
+    return load().raven_mixer_layer_workspace_bytes(C.byref(dims), C.byref(layer), B, S, int(pos0))
 
 
 def mixer_layer(dims: StreamDims, layer: MixerLayer, state: MixerState, x, B, S, pos0, workspace, pos_dev=None):

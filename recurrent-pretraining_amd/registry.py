@@ -5,13 +5,15 @@ from __future__ import annotations
 from typing import Tuple
 
 from . import checkpoint
-from .config import GitipelConfig, RavenConfig
+from .config import GitipelConfig, GupitarConfig, RavenConfig
 from .gitipel import GitipelForCausalLM
+from .gupitar import GupitarForCausalLM
 from .modeling import RavenForCausalLM
 
 FAMILIES = {
     "huginn_raven": (RavenConfig, RavenForCausalLM),
     "gitipel": (GitipelConfig, GitipelForCausalLM),
+    "gupitar": (GupitarConfig, GupitarForCausalLM),
 }
 
 
