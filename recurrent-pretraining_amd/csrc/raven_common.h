@@ -115,11 +115,14 @@ __device__ __forceinline__ float wave_max(float v) {
 // with a copy of itself the pair holds rows (0,0,2,2) and (1,1,3,3) of 16 lanes, after v_permlane32_swap the two halves.
 __device__ __forceinline__ float max_over_quarters(float x) {
     typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
-    unsigned u = __builtin_bit_cast(unsigned, x);
+    // the pair's elements go through plain variables: __builtin_bit_cast of a vector's element reads element 0 whatever the index
+    const unsigned u = __builtin_bit_cast(unsigned, x);
     const u32x2 r = __builtin_amdgcn_permlane16_swap(u, u, false, false);
-    u = __builtin_bit_cast(unsigned, fmaxf(__builtin_bit_cast(float, r[0]), __builtin_bit_cast(float, r[1])));
-    const u32x2 q = __builtin_amdgcn_permlane32_swap(u, u, false, false);
-    return fmaxf(__builtin_bit_cast(float, q[0]), __builtin_bit_cast(float, q[1]));
+    const unsigned r0 = r[0], r1 = r[1];
+    const unsigned v = __builtin_bit_cast(unsigned, fmaxf(__builtin_bit_cast(float, r0), __builtin_bit_cast(float, r1)));
+    const u32x2 q = __builtin_amdgcn_permlane32_swap(v, v, false, false);
+    const unsigned q0 = q[0], q1 = q[1];
+    return fmaxf(__builtin_bit_cast(float, q0), __builtin_bit_cast(float, q1));
 }
 
 // x * sigmoid(x).  The reciprocal is the hardware's (1 ulp): its error vanishes in the bf16 rounding that follows and stays
