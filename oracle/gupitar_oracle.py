@@ -82,7 +82,8 @@ def latent_attention_mixer(h, w, p, m, eps, kept):
     q = latent_queries(h, w, p, m, eps)
     k = torch.cat([(c @ w[p + "uk"].T).view(T, H, m["dim"]), k_rot[:, None].expand(T, H, m["rot_dim"])], -1)
     v = (c @ w[p + "uv"].T).view(T, H, m["vdim"])
-    o = windowed_attention(q, k, v, m["scale"], m["mask"]["size"]).reshape(T, -1)
+    window = m["mask"]["size"] if m.get("mask") else T
+    o = windowed_attention(q, k, v, m["scale"], window).reshape(T, -1)
     return (o * torch.sigmoid(h @ w[p + "g"].T)) @ w[p + "o"].T
 
 
@@ -189,3 +190,67 @@ def greedy(cfg, w, prompt, n_new):
     for _ in range(n_new):
         ids.append(int(forward(cfg, w, torch.tensor(ids))[0][-1].argmax()))
     return ids[len(prompt):]
+
+
+def random_weights(cfg, seed, dtype=torch.float32, round_bf16=True):
+    """Weights of every tensor a configuration needs, scaled so that activations stay of order one; with round_bf16 the
+    values are representable in bfloat16."""
+    g = torch.Generator().manual_seed(seed)
+    D, V = cfg["width"], cfg["vocab"]
+    w = {}
+
+    def normal(name, *shape, std=None, mean=0.0):
+        std = (1.0 / math.sqrt(shape[-1])) if std is None else std
+        t = torch.randn(*shape, generator=g) * std + mean
+        w[name] = (t.bfloat16().float() if round_bf16 else t).to(dtype)
+
+    def gated(p, ff):
+        normal(p + "gate", ff, D)
+        normal(p + "up", ff, D)
+        normal(p + "down", D, ff)
+
+    normal("embed", V, D, std=1.0)
+    for n, spec in enumerate(cfg["layers"]):
+        p, m, mp = f"l{n}.", spec["mixer"], f"l{n}.mix."
+        normal(p + "norm1", D, std=0.2)
+        if spec["type"] == "latent_attention":
+            H = m["heads"]
+            normal(mp + "dq", m["q_rank"], D)
+            normal(mp + "dq.norm", m["q_rank"], std=0.2, mean=1.0)
+            normal(mp + "uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"], std=1.5 / math.sqrt(m["q_rank"]))
+            if m.get("kv_from") is None:
+                normal(mp + "dkv", m["kv_rank"] + m["rot_dim"], D)
+                normal(mp + "dkv.norm", m["kv_rank"], std=0.2, mean=1.0)
+            normal(mp + "uk", H * m["dim"], m["kv_rank"])
+            normal(mp + "uv", H * m["vdim"], m["kv_rank"])
+            normal(mp + "g", H * m["vdim"], D)
+            normal(mp + "o", D, H * m["vdim"], std=2.0 / math.sqrt(H * m["vdim"]))
+        else:
+            W, n_blocks = m["width"], m["blocks"]
+            size = W // n_blocks
+            for t in "yx":
+                normal(mp + t, W, D)
+                normal(mp + t + ".b", W, std=0.3)
+            normal(mp + "conv", W, m["conv"], std=0.6)
+            normal(mp + "conv.b", W, std=0.3)
+            for t in ("ra", "ri"):
+                normal(mp + t, n_blocks, size, size)
+                normal(mp + t + ".b", n_blocks, size, std=0.5)
+            normal(mp + "lam", W, std=2.0, mean=-4.0)  # decays from almost none to strong
+            normal(mp + "o", D, W, std=2.0 / math.sqrt(W))
+        mlp = spec.get("mlp")
+        if mlp is None:
+            continue
+        normal(p + "norm2", D, std=0.2)
+        if mlp["kind"] == "dense":
+            gated(p + "mlp.", mlp["ff"])
+            continue
+        normal(p + "mlp.router", mlp["router"]["experts"], D, std=1.5 / math.sqrt(D))
+        for e in range(mlp["router"]["experts"]):
+            gated(f"{p}mlp.e{e}.", mlp["expert"]["ff"])
+        if mlp.get("shared") is not None:
+            gated(p + "mlp.shared.", mlp["shared"]["ff"])
+            normal(p + "mlp.shared.sg", 1, D)
+    normal("final.norm", D, std=0.2)
+    normal("head", V, D)
+    return w
