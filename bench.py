@@ -68,9 +68,13 @@ def parse():
                     help="run only N launches of the dominant kernel plus one 256 MiB device copy (for rocprofv3 --pmc runs)")
     ap.add_argument("--gitipel", action="store_true",
                     help="prompt and decode throughput of the Gitipel family beside Raven blocks of equal size (another line; --width, --part)")
-    ap.add_argument("--width", type=int, action="append", default=None, metavar="D", help="with --gitipel: model widths (default 2048 and 4096)")
-    ap.add_argument("--part", default="all", choices=["all", "gitipel-prompt", "gitipel-decode", "raven-prompt", "raven-decode"],
-                    help="with --gitipel: one family and phase only (for rocprofv3 runs)")
+    ap.add_argument("--gupitar", action="store_true",
+                    help="the same of the Gupitar family beside Gitipel (another line; --width, --part)")
+    ap.add_argument("--width", type=int, action="append", default=None, metavar="D",
+                    help="with --gitipel / --gupitar: model widths (default 2048 and 4096)")
+    ap.add_argument("--part", default="all", choices=["all"] + [f"{m}-{p}" for m in ("gupitar", "gitipel", "raven") for p in ("prompt", "decode")],
+                    help="with --gitipel / --gupitar: one family and phase only (for rocprofv3 runs)")
+    ap.add_argument("--sequences", type=int, default=1, metavar="B", help="with --gitipel / --gupitar: sequences of a decode step")
     return ap.parse_args()
 
 
@@ -496,30 +500,93 @@ def raven_work(cfg, S, t_cached):
     return flops, 2 * (runs * (4 * D * D + ff) + 2 * 2 * D * D + D * cfg.vocab_size) + runs * 2 * 2 * D * t_cached
 
 
-def gitipel(args):
-    """Prompt (one sequence of 4096 tokens) and decode (one sequence, about 1024 positions cached, graph replay) of both families, timed
-    in turn in one process.  Random weights, random tokens."""
+def gupitar_shapes(width, vocab=32768):
+    """A Gupitar and a Gitipel configuration of one size: 12 layers (runs), feed-forwards of about 8 width^2 weights per token.  Gupitar: two
+    latent-attention layers (a window of 1024, every second one reading the latents of the one before) to one recurrent one; a dense
+    layer in front, then mixtures of 64 experts, 6 per token, and a shared one."""
+    heads = width // 128
+    kv = {"kv_rank": 512, "rot_dim": 64, "rot": {"base": 10000.0, "dims": 64}, "mask": {"size": 1024}}
+    ff = width // 8 * 3  # 3 width (6 + 1) ff = 7.9 width^2
+    mlp = {"kind": "moe", "router": {"experts": 64, "top": 6}, "expert": {"ff": ff}, "shared": {"ff": ff}}
+
+    def latent(i):
+        m = {"heads": heads, "dim": 128, "vdim": 128, "q_rank": 3 * width // 4, "scale": 192 ** -0.5, **kv}
+        if i % 3 == 1:
+            m["kv_from"] = i - 1
+        return {"type": "latent_attention", "mixer": m, "mlp": mlp}
+
+    unit = {"type": "rglru", "mixer": {"width": width, "blocks": width // 256, "conv": 4}, "mlp": mlp}
+    layers = [latent(i) if i % 3 != 2 else unit for i in range(12)]
+    layers[0] = {**layers[0], "mlp": {"kind": "dense", "ff": 8 * width // 3 // 64 * 64}}
+    return {"vocab": vocab, "width": width, "layers": layers, "norm": {"eps": 1e-6}}, gitipel_shapes(width, vocab)[0]
+
+
+def gupitar_work(cfg, S, t_cached, B=1):
+    """(flops of a prompt of S tokens with all its logits, bytes a decode step of B sequences reads with t_cached positions behind them;
+    experts of different sequences counted as different ones up to their number)."""
+    D = cfg["width"]
+    flops = weights = state = 0.0
+    for layer in cfg["layers"]:
+        m, f = layer["mixer"], layer["mlp"]
+        if layer["type"] == "latent_attention":
+            H, hd = m["heads"], m["dim"] + m["rot_dim"]
+            own = D * (m["kv_rank"] + m["rot_dim"]) if "kv_from" not in m else 0
+            w = D * m["q_rank"] + m["q_rank"] * H * hd + own + m["kv_rank"] * H * (m["dim"] + m["vdim"]) + 2 * D * H * m["vdim"]
+            win = min(m["mask"]["size"], S)
+            pairs = win * (win + 1) / 2 + (S - win) * win
+            flops += 2.0 * H * (hd + m["vdim"]) * pairs
+            state += B * 2 * (m["kv_rank"] + m["rot_dim"]) * min(t_cached, m["mask"]["size"])
+        else:
+            W = m["width"]
+            w = 3 * D * W + 2 * W * W // m["blocks"]
+            flops += 2.0 * S * m["conv"] * W
+            state += B * 2 * 4 * W
+        weights += w
+        flops += 2.0 * S * w
+        if f["kind"] == "dense":
+            ff = active = 3 * D * f["ff"]
+        else:
+            one, n = 3 * D * f["expert"]["ff"], f["router"]["experts"]
+            rest = 3 * D * f["shared"]["ff"] + D * n
+            active = f["router"]["top"] * one + rest
+            ff = one * n * (1 - (1 - f["router"]["top"] / n) ** B) + rest  # experts that B independent choices touch
+        weights += ff
+        flops += 2.0 * S * active
+    flops += 2.0 * S * D * cfg["vocab"]
+    return flops, 2 * (weights + D * cfg["vocab"]) + state
+
+
+def stream_families(args, names, shapes, title):
+    """Prompt (one sequence of 4096 tokens) and decode (args.sequences sequences, about 1024 positions cached, graph replay) of two
+    families of equal size, timed in turn in one process.  Random weights, random tokens."""
     import statistics
 
     import torch
     import __graft_entry__ as entry
     pkg = entry.import_package()
-    S, ctx, lines = 4096, 1024, {}
+    S, ctx, B, lines = 4096, 1024, args.sequences, {}
     for width in args.width or [2048, 4096]:
-        gcfg, rcfg = gitipel_shapes(width)
-        models = {}
-        if args.part == "all" or args.part.startswith("gitipel"):
-            models["gitipel"] = pkg.GitipelForCausalLM(pkg.GitipelConfig(**gcfg), device="cuda:0", dtype=torch.bfloat16)
-            models["gitipel"].init_weights(seed=0)
-        if args.part == "all" or args.part.startswith("raven"):
-            models["raven"] = pkg.RavenForCausalLM(pkg.RavenConfig(**rcfg), device="cuda:0", dtype=torch.bfloat16)
-            fill_synthetic(models["raven"])
-        ids = torch.randint(0, gcfg["vocab"], (1, S), generator=torch.Generator().manual_seed(1)).cuda()
-        work = {"gitipel": gitipel_work(gcfg, S, ctx), "raven": raven_work(models["raven"].config, S, ctx) if "raven" in models else None}
+        cfgs = dict(zip(names, shapes(width)))
+        models, work = {}, {}
+        for name, cfg in cfgs.items():
+            if args.part != "all" and not args.part.startswith(name):
+                continue
+            if name == "raven":
+                models[name] = pkg.RavenForCausalLM(pkg.RavenConfig(**cfg), device="cuda:0", dtype=torch.bfloat16)
+                fill_synthetic(models[name])
+                work[name] = raven_work(models[name].config, S, ctx)
+            else:
+                config, family = pkg.family_of({"model_type": name})
+                models[name] = family(config(**cfg), device="cuda:0", dtype=torch.bfloat16)
+                models[name].init_weights(seed=0)
+                work[name] = gitipel_work(cfg, S, ctx) if name == "gitipel" else gupitar_work(cfg, S, ctx, B)
+        vocab = 32768
+        ids = torch.randint(0, vocab, (1, S), generator=torch.Generator().manual_seed(1)).cuda()
+        rows = torch.randint(0, vocab, (B, ctx), generator=torch.Generator().manual_seed(2)).cuda()
         runs, rec = {}, {}
         for name, m in models.items():
             cache, dcache = m.new_cache(S), m.new_cache(ctx + 256)
-            kw = {} if name == "gitipel" else {"num_steps": 2, "init_scale": 0.0}
+            kw = {"num_steps": 2, "init_scale": 0.0} if name == "raven" else {}
 
             def prompt(m=m, cache=cache, kw=kw):
                 cache.reset()
@@ -527,10 +594,10 @@ def gitipel(args):
 
             def decode(n, m=m, dcache=dcache, kw=kw, box={}):
                 if "runner" not in box:
-                    m.forward(input_ids=ids[:, :ctx - 64], past_key_values=dcache, use_cache=True, **kw)
-                    box["runner"] = m.decode_runner(dcache, 1, 2, greedy=True, use_graph=True)
-                for _ in range(n):
-                    box["runner"].step(ids[0, :1], None, 0.0)
+                    m.forward(input_ids=rows[:, :ctx - 64], past_key_values=dcache, use_cache=True, **kw)
+                    box["runner"] = m.decode_runner(dcache, B, 2, greedy=True, use_graph=True)
+                for i in range(n):
+                    box["runner"].step(rows[:, i], None, 0.0)
 
             runs[name] = (prompt, decode)
 
@@ -559,13 +626,21 @@ def gitipel(args):
                     r["prompt"] = {"ms": round(t, 3), "tokens_per_s": round(S / t * 1e3), "tflops": round(flops / t / 1e9, 1),
                                    "of_mfma_peak": round(flops / t / 1e9 / MFMA_PEAK_TFLOPS, 4)}
                 else:
-                    r["decode"] = {"ms": round(t, 4), "tokens_per_s": round(1e3 / t, 1), "gb_per_s": round(nbytes / t / 1e6, 1),
+                    r["decode"] = {"ms": round(t, 4), "tokens_per_s": round(B * 1e3 / t, 1), "gb_per_s": round(nbytes / t / 1e6, 1),
                                    "of_hbm_peak": round(nbytes / t / 1e6 / HBM_PEAK_GBS, 4)}
         lines[str(width)] = rec
-        del models, runs
+        del models, runs, prompt, decode, m, cache, dcache
         torch.cuda.empty_cache()
-    print(json.dumps({"metric": "Gitipel beside Raven blocks of equal size: one sequence, 4096-token prompt / decode at 1024 positions",
+    print(json.dumps({"metric": f"{title}: one sequence, 4096-token prompt / decode of {B} sequence{'s' if B > 1 else ''} at 1024 positions",
                       "dtype": "bf16", "data": "synthetic", "n_gpus": 1, "layer_runs": 12, "by_width": lines}))
+
+
+def gitipel(args):
+    stream_families(args, ("gitipel", "raven"), gitipel_shapes, "Gitipel beside Raven blocks of equal size")
+
+
+def gupitar(args):
+    stream_families(args, ("gupitar", "gitipel"), gupitar_shapes, "Gupitar beside Gitipel of equal size")
 
 
 def event_time_ms(fn, reps, warm=3):
@@ -653,6 +728,9 @@ def main():
         return
     if args.gitipel:
         gitipel(args)
+        return
+    if args.gupitar:
+        gupitar(args)
         return
     if args.gpus != 1:
         print("bench.py measures one GPU: the decode path has no multi-GPU part (run with --gpus 1)", file=sys.stderr)

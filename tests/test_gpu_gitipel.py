@@ -203,6 +203,22 @@ def test_attention_far_key_stands_out(pkg, dtype, how):
 
 
 @DT
+@pytest.mark.parametrize("cap", [0.0, 300.0])
+def test_attention_reference_follows_every_lane(pkg, dtype, cap):
+    """Without a small cap, scores far apart inside a tile, the largest at each of its places in turn."""
+    T, H, d = 128, 2, 32
+    g = torch.Generator().manual_seed(4)
+    q, k = torch.randn(T, H, d, generator=g), torch.randn(T, 1, d, generator=g)
+    for i in range(64, T):
+        q[i] = 40 * k[i - 64]
+    q, k = q.to(dtype).float(), k.to(dtype).float()
+    want = O.attention(q.double(), k.double(), 0.2, cap if cap else 1e9, torch.zeros(H).double(), torch.zeros(H).double())
+    for cuts in ([T], [64] + [1] * 64):
+        got = run_attention(pkg, q, k, pkg.hip.make_score(0.2, cap), cuts, dtype)
+        assert torch.isfinite(got).all() and G.rel(got, want) < (1e-4 if dtype == F32 else 2e-2), cuts
+
+
+@DT
 def test_attention_long_cache_split_over_workgroups(pkg, dtype):
     """Decode rows over a few thousand positions, with the position on the device and a larger bound by value."""
     T, H, Gk, d = 3000, 4, 2, 48

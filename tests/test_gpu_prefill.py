@@ -397,3 +397,21 @@ def test_bench_prefill_iteration_runs_through_the_c_abi(pkg):
         cur = nxt
     assert torch.equal(cur, outs[0][0]) and torch.equal(kd, outs[0][1]) and torch.equal(vd, outs[0][2])
     assert torch.isfinite(cur.float()).all()
+
+
+@pytest.mark.parametrize("hd", [64, 96, 128])
+def test_prefill_attention_reference_follows_every_lane(pkg, hd):
+    """Scores far apart inside a tile, the largest at each of its places in turn: the running reference must see all of them."""
+    S, nh, dt = 128, 2, torch.bfloat16
+    g = torch.Generator().manual_seed(hd)
+    k, v, q = (torch.randn(1, nh, S, hd, generator=g) for _ in range(3))
+    for i in range(64, S):
+        q[0, :, i] = 40 * k[0, :, i - 64]  # its score is about 40 sqrt(hd), the others' a small part of that
+    q, k, v = q.to(dt), k.to(dt), v.to(dt)
+    kc, vc = k[None].cuda(), v[None].cuda()
+    cache = pkg.hip.make_cache(kc, vc)
+    rows = q.transpose(1, 2).reshape(S, nh * hd).contiguous().cuda()
+    got = pkg.hip.prefill_attention(rows, cache, 0, 1, S, 0, nh, hd).float().cpu().view(S, nh, hd)
+    want = torch.nn.functional.scaled_dot_product_attention(q.double(), k.double(), v.double(), is_causal=True)[0].transpose(0, 1)
+    assert torch.isfinite(got).all()
+    assert (got - want).abs().max() < 5e-2
