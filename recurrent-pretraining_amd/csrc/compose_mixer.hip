@@ -19,13 +19,15 @@ RAVEN_WEAK decltype(raven_latent_attention_workspace_bytes) raven_latent_attenti
 RAVEN_WEAK decltype(raven_rglru_workspace_bytes) raven_rglru_workspace_bytes;
 RAVEN_WEAK decltype(raven_rglru_forward) raven_rglru_forward;
 RAVEN_WEAK decltype(raven_moe_workspace_bytes) raven_moe_workspace_bytes;
-RAVEN_WEAK decltype(raven_moe_forward) raven_moe_forward;
 }
 
 namespace raven {
 
 RAVEN_WEAK int latent_attention(const raven_latent* l, const void* q, const void* z, int ldz, int z_f32, const raven_latent_cache* cache, void* y, int B,
                                 int S, int pos0, const int* pos_dev, int append, int dtype, void* workspace, size_t workspace_bytes, hipStream_t s);
+
+RAVEN_WEAK int moe_forward(const raven_moe* m, const void* h, const float* norm, int dim, float eps, const float* logits, float* x, int M, int ld, int dtype,
+                           void* workspace, size_t workspace_bytes, hipStream_t s);
 
 bool gemv1_stream_fits(int K, int dtype);
 int gemv1_stream(const float* x, const float* norm, int dim, float eps, const void* w, void* y, int N, int K, const raven_epilogue& epi, int dtype,
@@ -116,7 +118,7 @@ static int check_mixer_layer(const char* who, const raven_stream_dims* d, const 
     }
     RAVEN_REQUIRE(l->ff_kind >= RAVEN_FF_GELU && l->ff_kind <= RAVEN_FF_MOE, "%s: unknown feed-forward %d", who, l->ff_kind);
     if (l->ff_kind == RAVEN_FF_MOE) {
-        RAVEN_REQUIRE(&raven_moe_forward, "%s: this build lacks the mixture of experts", who);
+        RAVEN_REQUIRE(&raven_moe_workspace_bytes && &moe_forward, "%s: this build lacks the mixture of experts", who);
         RAVEN_REQUIRE(l->moe && l->moe->router && l->norm2, "%s: bad mixture of experts", who);
     } else {
         RAVEN_REQUIRE((l->up == nullptr) == (l->down == nullptr) && (l->up == nullptr || (l->norm2 && l->ff > 0 && l->ff % 8 == 0)),
@@ -205,9 +207,9 @@ extern "C" int raven_mixer_layer_forward(const raven_stream_dims* dims, const ra
     if (int rc = product(w.y, l.w_out, x, ld, inner, RAVEN_ACT_NONE, nullptr, x, 1)) return rc;
 
     if (l.ff_kind == RAVEN_FF_MOE) {
-        if (int rc = raven_norm_conv(x, l.norm2, nullptr, nullptr, w.h, B, S, dims->width, ld, 1, dims->eps, pos0, pos_dev, dt, stream)) return rc;
-        if (int rc = product(w.h, l.moe->router, w.logits, l.moe->logit_ld, ld, RAVEN_ACT_NONE, nullptr, nullptr, 1)) return rc;
-        return raven_moe_forward(l.moe, w.h, w.logits, x, M, ld, dt, w.ff_ws, w.ff_ws_bytes, stream);
+        // (one row: the norm rides in the router's product and again in the experts' first one; else it lies in w.h)
+        if (int rc = normed_product(l.norm2, l.moe->router, w.logits, l.moe->logit_ld, RAVEN_ACT_NONE, nullptr, 1)) return rc;
+        return moe_forward(l.moe, one_row ? nullptr : w.h, l.norm2, dims->width, dims->eps, w.logits, x, M, ld, dt, w.ff_ws, w.ff_ws_bytes, s);
     }
     if (!l.up) return 0;
     if (l.ff_kind == RAVEN_FF_SWIGLU) {

@@ -975,7 +975,7 @@ int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int 
 }
 
 // Products of row groups (128 rows to a tile row): y[r] = x[x_row[r]] W_g^T, W_g = w + g * w_stride [N or 2N, K] of the group that row r of the
-// product belongs to.  swiglu: y = T(silu(s gate) * (s up)) with s = x_scale[r]; else y float.  n_tiles: entries of the three tile
+// product belongs to.  swiglu: y = T(silu(s gate) * (s up)) with s = x_scale[r]; else y = T(sums).  n_tiles: entries of the three tile
 // tables (unused ones have group_of < 0); rows: rows of the product, x_rows: rows of x.
 int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, void* y, int rows, int N, int K, int swiglu, const int* group_of,
                  const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s) {
@@ -986,7 +986,7 @@ int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, voi
     a.w = static_cast<const bf16*>(w);
     a.x0 = static_cast<const bf16*>(x);
     a.y = y;
-    a.M = rows; a.N = N; a.K0 = K; a.out_f32 = !swiglu;
+    a.M = rows; a.N = N; a.K0 = K; a.out_f32 = 0;
     a.ldy = N; a.up_off = N; a.ldw = K; a.ldx = K;
     a.tiles_m = n_tiles;
     a.epi.scale = 1.f;

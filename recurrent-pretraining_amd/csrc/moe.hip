@@ -2,9 +2,9 @@
 //     x += sum over the chosen experts of W_down ( silu(s W_gate h) * (s W_up h) )  +  sigmoid(g) W_down' ( silu(W_gate' h) * (W_up' h) )
 // s = sigmoid(router logit): the factor of an expert's input is applied to the sums of its first two products, which is the same.
 //
-// Few rows (and fp32): one launch forms the gated activations of a row's experts and of the shared one side by side, one launch
-// multiplies them by the down matrices and adds to the stream.  Both pick the row's experts themselves from its logits -- a handful of
-// wave reductions -- so no routing launch stands in between.
+// Few rows (and fp32): moe_up_kernel forms the gated activations of a row's experts and of the shared one side by side, moe_down_kernel
+// multiplies them by the down matrices and adds to the stream.  The first picks the row's experts itself from its logits -- a handful
+// of wave reductions -- so no routing launch stands in between; for a single row it also takes the norm of the stream as a prologue.
 // bf16 chunks: the rows are sorted by expert (moe_pick_kernel, moe_sort_kernel) and the experts run as one grouped product on the
 // matrix cores (gemm_tiled.hip), rows gathered through the sorted list; every (token, expert) pair has a slot of its own, and
 // moe_combine_kernel adds a token's slots and its shared expert to the stream in a fixed order.
@@ -17,11 +17,15 @@ int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, voi
                  const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s);
 
 constexpr int kMaxExperts = 1024, kMaxTop = 32, kSlotRows = 128;
+constexpr int kPickRows = 64;  // tokens a workgroup of the two sorting kernels owns
 
 struct MoeArgs {
     const void *h, *up, *down, *shared_up, *shared_down;
     const float* logits;
     float* x;
+    const float* norm;      // h null (one row): the norm of x that gives it, with its true width and eps
+    int dim;
+    float eps;
     void* act;              // few rows: [M, top * ff + shared_ff] of T
     int M, ld, ldl, experts, top, ff, sff;
     // chunks
@@ -32,7 +36,8 @@ struct MoeArgs {
     float* slot_scale;      // [M * top]
     int *group_of, *group_row, *group_end;
     int n_tiles;
-    const float* y;         // [M * top, ld]
+    int* block_count;       // [ceil(M / kPickRows), experts]: pairs of a workgroup's tokens
+    const bf16* y;          // [M * top, ld]
     const float* ys;        // [M, ld] or null
 };
 
@@ -70,44 +75,61 @@ __device__ __forceinline__ void pick_experts(const float* logits, int experts, i
 }
 
 // ---- few rows --------------------------------------------------------------------------------------------
-// 16 (gate, up) row pairs per workgroup, 16 lanes to a pair, over the concatenation of the row's experts and the shared one
+// A wave per (gate, up) row pair, over the concatenation of the row's experts and the shared one
 template <typename T>
 __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
-    constexpr int E = Chunk<T>::N;
+    constexpr int E = Chunk<T>::N, U = 4;
     extern __shared__ __align__(16) unsigned char smem_raw[];
     T* xs = reinterpret_cast<T*>(smem_raw);  // [ld]
     __shared__ int idx[kMaxTop];
-    __shared__ float score[kMaxTop];
-    const int m = blockIdx.y, nc = a.ld / E, total = a.top * a.ff + a.sff;
-    for (int i = threadIdx.x; i < nc; i += 256) store_chunk(xs + i * E, load_chunk(static_cast<const T*>(a.h) + (int64_t)m * a.ld + i * E));
-    if (threadIdx.x < 64) pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, idx, score);
+    __shared__ float score[kMaxTop], red[4];
+    const int m = blockIdx.y, nc = a.ld / E, total = a.top * a.ff + a.sff, lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+    if (a.h) {
+        for (int i = threadIdx.x; i < nc; i += 256) store_chunk(xs + i * E, load_chunk(static_cast<const T*>(a.h) + (int64_t)m * a.ld + i * E));
+    }
+    if (wave == 0) pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, idx, score);
+    if (!a.h) {
+        const float* x = a.x + (int64_t)m * a.ld;
+        float ss = 0.f;
+        for (int i = 4 * threadIdx.x; i < a.ld; i += 1024) {
+            const f32x4 v = load4(x + i);
+            ss += v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3];
+        }
+        ss = wave_sum(ss);
+        if (lane == 0) red[wave] = ss;
+        __syncthreads();
+        const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)a.dim + a.eps);
+        for (int i = 4 * threadIdx.x; i < a.ld; i += 1024) store4(xs + i, load4(x + i) * inv * load4(a.norm + i));
+    }
     __syncthreads();
-    const int p = blockIdx.x * 16 + (threadIdx.x >> 4), pp = min(p, total - 1), c16 = threadIdx.x & 15;
-    const bool shared = pp >= a.top * a.ff;
-    const int slot = shared ? 0 : pp / a.ff, r = shared ? pp - a.top * a.ff : pp - slot * a.ff;
+    if (blockIdx.x == 0 && (int)threadIdx.x < a.top) a.pick[(int64_t)m * a.top + threadIdx.x] = idx[threadIdx.x];
+    const int p = blockIdx.x * 4 + wave;
+    if (p >= total) return;
+    const bool shared = p >= a.top * a.ff;
+    const int slot = shared ? 0 : p / a.ff, r = shared ? p - a.top * a.ff : p - slot * a.ff;
     const T* g = shared ? static_cast<const T*>(a.shared_up) + (int64_t)r * a.ld
                         : static_cast<const T*>(a.up) + ((int64_t)idx[slot] * 2 * a.ff + r) * a.ld;
     const T* u = g + (int64_t)(shared ? a.sff : a.ff) * a.ld;
     float sg = 0.f, su = 0.f;
-    for (int c0 = c16; c0 < nc; c0 += 64) {
-        Chunk<T> vg[4], vu[4];
+    for (int c0 = lane; c0 < nc; c0 += 64 * U) {
+        Chunk<T> vg[U], vu[U];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            const int c = min(c0 + 16 * j, nc - 1);
+        for (int j = 0; j < U; ++j) {
+            const int c = min(c0 + 64 * j, nc - 1);
             vg[j] = load_chunk_stream(g + c * E);
             vu[j] = load_chunk_stream(u + c * E);
         }
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
-            if (c0 + 16 * j >= nc) break;
-            const Chunk<T> x = load_chunk(xs + (c0 + 16 * j) * E);
+        for (int j = 0; j < U; ++j) {
+            if (c0 + 64 * j >= nc) break;
+            const Chunk<T> x = load_chunk(xs + (c0 + 64 * j) * E);
             sg = dot_chunk(vg[j], x, sg);
             su = dot_chunk(vu[j], x, su);
         }
     }
-    sg = row16_sum(sg);
-    su = row16_sum(su);
-    if (c16 != 0 || p >= total) return;
+    sg = wave_sum(sg);
+    su = wave_sum(su);
+    if (lane != 0) return;
     const float s = shared ? 1.f : score[slot];
     float v = silu_f32(s * sg) * (s * su);
     if (shared) v *= sigmoid_f32(a.logits[(int64_t)m * a.ldl + a.experts]);
@@ -117,13 +139,11 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
 // a wave per output channel: its row of every chosen down matrix and of the shared one, as one long row
 template <typename T>
 __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
-    constexpr int E = Chunk<T>::N, U = 8;
-    __shared__ int idx[kMaxTop];
-    __shared__ float score[kMaxTop];
-    const int m = blockIdx.y, n = min((int)(blockIdx.x * 4 + (threadIdx.x >> 6)), a.ld - 1), lane = threadIdx.x & 63;
-    const bool real = (int)(blockIdx.x * 4 + (threadIdx.x >> 6)) < a.ld;
-    if (threadIdx.x < 64) pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, idx, score);
-    __syncthreads();
+    constexpr int E = Chunk<T>::N, U = 6;
+    const int m = blockIdx.y, n = blockIdx.x * 4 + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+    if (n >= a.ld) return;
+    const int* pick = a.pick + (int64_t)m * a.top;
+    const float x = a.x[(int64_t)m * a.ld + n];
     const int nf = a.ff / E, nr = a.top * nf, nc = nr + a.sff / E;
     const T* act = static_cast<const T*>(a.act) + (int64_t)m * nc * E;
     const T* down = static_cast<const T*>(a.down);
@@ -131,39 +151,68 @@ __global__ __launch_bounds__(256) void moe_down_kernel(MoeArgs a) {
     float sum = 0.f;
     for (int c0 = lane; c0 < nc; c0 += 64 * U) {
         Chunk<T> w[U], v[U];
+        int e[U];
 #pragma unroll
         for (int j = 0; j < U; ++j) {
             const int c = min(c0 + 64 * j, nc - 1);
-            const T* row = c < nr ? down + ((int64_t)idx[c / nf] * a.ld + n) * a.ff + (c % nf) * E : sdown + (int64_t)n * a.sff + (c - nr) * E;
-            w[j] = load_chunk_stream(row);
             v[j] = load_chunk(act + c * E);
+            e[j] = c < nr ? pick[c / nf] : 0;
+        }
+#pragma unroll
+        for (int j = 0; j < U; ++j) {
+            const int c = min(c0 + 64 * j, nc - 1);
+            w[j] = load_chunk_stream(c < nr ? down + ((int64_t)e[j] * a.ld + n) * a.ff + (c % nf) * E : sdown + (int64_t)n * a.sff + (c - nr) * E);
         }
 #pragma unroll
         for (int j = 0; j < U; ++j)
             if (c0 + 64 * j < nc) sum = dot_chunk(w[j], v[j], sum);
     }
     sum = wave_sum(sum);
-    if (lane == 0 && real) a.x[(int64_t)m * a.ld + n] += sum;
+    if (lane == 0) a.x[(int64_t)m * a.ld + n] = x + sum;
 }
 
 // ---- chunks ----------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void moe_pick_kernel(MoeArgs a) {
-    const int m = blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (m >= a.M) return;
-    pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, a.pick + (int64_t)m * a.top, a.pick_scale + (int64_t)m * a.top);
+// Both sorting kernels give kPickRows tokens to a workgroup.  The first picks their experts (a wave per token in turn) and counts
+// its pairs per expert; the second adds the counts up -- every workgroup for itself: they are few --, so that it knows where each
+// expert's rows start and which of them are its own, and puts its pairs there.  Inside a workgroup's share of an expert the order is
+// whatever the counters give: no result depends on it.
+__global__ __launch_bounds__(1024) void moe_pick_kernel(MoeArgs a) {
+    __shared__ int count[kMaxExperts];
+    const int m0 = blockIdx.x * kPickRows, wave = threadIdx.x >> 6;
+    for (int e = threadIdx.x; e < a.experts; e += 1024) count[e] = 0;
+    __syncthreads();
+    for (int i = wave; i < kPickRows && m0 + i < a.M; i += 16) {
+        const int64_t m = m0 + i;
+        pick_experts(a.logits + m * a.ldl, a.experts, a.top, a.pick + m * a.top, a.pick_scale + m * a.top);
+        // lane 0 wrote the picks and reads them back
+        if ((threadIdx.x & 63) == 0)
+            for (int k = 0; k < a.top; ++k) atomicAdd(&count[a.pick[m * a.top + k]], 1);
+    }
+    __syncthreads();
+    for (int e = threadIdx.x; e < a.experts; e += 1024) a.block_count[(int64_t)blockIdx.x * a.experts + e] = count[e];
 }
 
-// One workgroup sorts the (token, expert) pairs by expert and lays out the tile rows of the grouped product.  The order of an expert's
-// rows is whatever the counters give: no result depends on it.
 __global__ __launch_bounds__(1024) void moe_sort_kernel(MoeArgs a) {
-    __shared__ int count[kMaxExperts], next[kMaxExperts], wave_sums[2][16];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pairs = a.M * a.top;
-    count[tid] = 0;
+    __shared__ int before[kMaxExperts], total[kMaxExperts], wave_sums[2][16];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, blocks = gridDim.x, me = blockIdx.x;
+    before[tid] = total[tid] = 0;
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) atomicAdd(&count[a.pick[i]], 1);
+    const int counts = blocks * a.experts;
+    for (int i0 = tid; i0 < counts; i0 += 4096) {
+        int v[4];
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[j] = i0 + 1024 * j < counts ? a.block_count[i0 + 1024 * j] : 0;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            if (v[j] == 0) continue;
+            const int i = i0 + 1024 * j, b = i / a.experts, e = i - b * a.experts;
+            atomicAdd(&total[e], v[j]);
+            if (b < me) atomicAdd(&before[e], v[j]);
+        }
+    }
     __syncthreads();
     // running sums over the experts of rows and of tile rows
-    const int rows = tid < a.experts ? count[tid] : 0, tiles = (rows + kSlotRows - 1) / kSlotRows;
+    const int rows = total[tid], tiles = (rows + kSlotRows - 1) / kSlotRows;
     int r = rows, t = tiles;
 #pragma unroll
     for (int d = 1; d < 64; d <<= 1) {
@@ -183,18 +232,21 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(MoeArgs a) {
         t += wave_sums[1][w];
     }
     const int first = r - rows, first_tile = t - tiles;
-    next[tid] = first;
-    for (int i = 0; i < tiles; ++i) {
-        a.group_of[first_tile + i] = tid;
-        a.group_row[first_tile + i] = first + i * kSlotRows;
-        a.group_end[first_tile + i] = min(first + (i + 1) * kSlotRows, first + rows);
+    before[tid] += first;  // where this workgroup's rows of expert tid start
+    if (me == 0) {
+        for (int i = 0; i < tiles; ++i) {
+            a.group_of[first_tile + i] = tid;
+            a.group_row[first_tile + i] = first + i * kSlotRows;
+            a.group_end[first_tile + i] = min(first + (i + 1) * kSlotRows, first + rows);
+        }
+        int used = 0;
+        for (int w = 0; w < 16; ++w) used += wave_sums[1][w];
+        for (int i = used + tid; i < a.n_tiles; i += 1024) a.group_of[i] = -1;
     }
-    int used = 0;
-    for (int w = 0; w < 16; ++w) used += wave_sums[1][w];
-    for (int i = used + tid; i < a.n_tiles; i += 1024) a.group_of[i] = -1;
     __syncthreads();
-    for (int i = tid; i < pairs; i += 1024) {
-        const int slot = atomicAdd(&next[a.pick[i]], 1);
+    const int lo = me * kPickRows * a.top, hi = min(a.M, (me + 1) * kPickRows) * a.top;
+    for (int i = lo + tid; i < hi; i += 1024) {
+        const int slot = atomicAdd(&before[a.pick[i]], 1);
         a.slot_of[i] = slot;
         a.slot_row[slot] = i / a.top;
         a.slot_scale[slot] = a.pick_scale[i];
@@ -207,7 +259,14 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(MoeArgs a) {
     if (i >= (int64_t)a.M * per) return;
     const int m = (int)(i / per), c = 4 * (int)(i % per);
     f32x4 x = load4(a.x + (int64_t)m * a.ld + c);
-    for (int k = 0; k < a.top; ++k) x += load4(a.y + (int64_t)a.slot_of[m * a.top + k] * a.ld + c);
+    for (int k0 = 0; k0 < a.top; k0 += 4) {
+        f32x4 v[4];
+#pragma unroll
+        for (int k = 0; k < 4; ++k) v[k] = load4(a.y + (int64_t)a.slot_of[m * a.top + min(k0 + k, a.top - 1)] * a.ld + c);
+#pragma unroll
+        for (int k = 0; k < 4; ++k)
+            if (k0 + k < a.top) x += v[k];
+    }
     if (a.ys) x += load4(a.ys + (int64_t)m * a.ld + c) * sigmoid_f32(a.logits[(int64_t)m * a.ldl + a.experts]);
     store4(a.x + (int64_t)m * a.ld + c, x);
 }
@@ -218,8 +277,9 @@ static bool moe_grouped(const raven_moe* m, int M, int dtype) {
 }
 
 struct MoeChunk {
-    int *pick, *slot_of, *slot_row, *group_of, *group_row, *group_end;
-    float *pick_scale, *slot_scale, *y, *ys;
+    int *pick, *slot_of, *slot_row, *group_of, *group_row, *group_end, *block_count;
+    bf16* y;
+    float *pick_scale, *slot_scale, *ys;
     char *act, *sact, *lin;
     size_t lin_bytes;
     int n_tiles;
@@ -235,6 +295,7 @@ static size_t carve_moe(const raven_moe* m, int M, int ld, int dtype, char* base
     MoeChunk c{};
     if (!moe_grouped(m, M, dtype)) {
         c.act = take((size_t)M * (m->top * (size_t)m->ff + m->shared_ff) * es);
+        c.pick = (int*)take(pairs * 4);
     } else {
         c.n_tiles = (int)(pairs / kSlotRows) + m->experts;
         c.pick = (int*)take(pairs * 4);
@@ -245,8 +306,9 @@ static size_t carve_moe(const raven_moe* m, int M, int ld, int dtype, char* base
         c.group_of = (int*)take((size_t)c.n_tiles * 4);
         c.group_row = (int*)take((size_t)c.n_tiles * 4);
         c.group_end = (int*)take((size_t)c.n_tiles * 4);
+        c.block_count = (int*)take((size_t)((M + kPickRows - 1) / kPickRows) * m->experts * 4);
         c.act = take(pairs * m->ff * es);
-        c.y = (float*)take(pairs * ld * sizeof(float));
+        c.y = (bf16*)take(pairs * ld * sizeof(bf16));
         if (m->shared_up) {
             c.sact = take((size_t)M * m->shared_ff * es);
             c.ys = (float*)take((size_t)M * ld * sizeof(float));
@@ -272,7 +334,7 @@ static int run_moe_rows(const MoeArgs& a, hipStream_t s) {
     const size_t lds = (size_t)a.ld * sizeof(T);
     RAVEN_REQUIRE(lds <= 64 * 1024 - 1024, "moe: rows of %d channels do not fit the LDS", a.ld);
     const int total = a.top * a.ff + a.sff;
-    moe_up_kernel<T><<<dim3((total + 15) / 16, a.M), dim3(256), lds, s>>>(a);
+    moe_up_kernel<T><<<dim3((total + 3) / 4, a.M), dim3(256), lds, s>>>(a);
     moe_down_kernel<T><<<dim3((a.ld + 3) / 4, a.M), dim3(256), 0, s>>>(a);
     return raven_host::check_launch("moe (rows)");
 }
@@ -284,30 +346,31 @@ extern "C" size_t raven_moe_workspace_bytes(const raven_moe* m, int32_t M, int32
     return raven::carve_moe(m, M, ld, dtype, nullptr, nullptr);
 }
 
-extern "C" int raven_moe_forward(const raven_moe* m, const void* h, const float* logits, float* x, int32_t M, int32_t ld, int32_t dtype,
-                                 void* workspace, size_t workspace_bytes, void* stream) {
-    using namespace raven;
+namespace raven {
+// h null (one row): moe_up_kernel norms the row of x itself
+int moe_forward(const raven_moe* m, const void* h, const float* norm, int dim, float eps, const float* logits, float* x, int M, int ld, int dtype,
+                void* workspace, size_t workspace_bytes, hipStream_t s) {
     if (const int rc = check_moe("moe", m, M, ld, dtype)) return rc;
     if (M == 0) return 0;
-    RAVEN_REQUIRE(m->up && m->down && h && logits && x, "moe: null pointer");
+    RAVEN_REQUIRE(m->up && m->down && (h || (norm && M == 1)) && logits && x, "moe: null pointer");
     RAVEN_REQUIRE(workspace && ((uintptr_t)workspace & 255) == 0 && carve_moe(m, M, ld, dtype, nullptr, nullptr) <= workspace_bytes,
                   "moe: workspace of %zu bytes is too small or unaligned", workspace_bytes);
     MoeChunk c;
     carve_moe(m, M, ld, dtype, static_cast<char*>(workspace), &c);
-    hipStream_t s = static_cast<hipStream_t>(stream);
     MoeArgs a{};
     a.h = h; a.up = m->up; a.down = m->down; a.shared_up = m->shared_up; a.shared_down = m->shared_down;
-    a.logits = logits; a.x = x; a.act = c.act;
+    a.logits = logits; a.x = x; a.act = c.act; a.norm = norm; a.dim = dim; a.eps = eps; a.pick = c.pick;
     a.M = M; a.ld = ld; a.ldl = m->logit_ld; a.experts = m->experts; a.top = m->top; a.ff = m->ff; a.sff = m->shared_ff;
     if (!moe_grouped(m, M, dtype)) {
         RAVEN_REQUIRE(M <= 65535, "moe: %d rows in one call", M);
         return dtype == RAVEN_BF16 ? run_moe_rows<bf16>(a, s) : run_moe_rows<float>(a, s);
     }
-    const int pairs = M * m->top;
-    a.pick = c.pick; a.pick_scale = c.pick_scale; a.slot_of = c.slot_of; a.slot_row = c.slot_row; a.slot_scale = c.slot_scale;
-    a.group_of = c.group_of; a.group_row = c.group_row; a.group_end = c.group_end; a.n_tiles = c.n_tiles; a.y = c.y; a.ys = c.ys;
-    moe_pick_kernel<<<dim3((M + 3) / 4), dim3(256), 0, s>>>(a);
-    moe_sort_kernel<<<dim3(1), dim3(1024), 0, s>>>(a);
+    const int pairs = M * m->top, blocks = (M + kPickRows - 1) / kPickRows;
+    a.pick_scale = c.pick_scale; a.slot_of = c.slot_of; a.slot_row = c.slot_row; a.slot_scale = c.slot_scale;
+    a.group_of = c.group_of; a.group_row = c.group_row; a.group_end = c.group_end; a.n_tiles = c.n_tiles; a.block_count = c.block_count;
+    a.y = c.y; a.ys = c.ys;
+    moe_pick_kernel<<<dim3(blocks), dim3(1024), 0, s>>>(a);
+    moe_sort_kernel<<<dim3(blocks), dim3(1024), 0, s>>>(a);
     if (const int rc = raven_host::check_launch("moe (sort)")) return rc;
     if (const int rc = grouped_gemm(h, M, m->up, (int64_t)2 * m->ff * ld, c.act, pairs, m->ff, ld, 1, c.group_of, c.group_row, c.group_end, c.n_tiles, c.slot_row,
                                     c.slot_scale, s)) return rc;
@@ -316,9 +379,16 @@ extern "C" int raven_moe_forward(const raven_moe* m, const void* h, const float*
     if (m->shared_up) {
         raven_epilogue e{};
         e.scale = 1.f; e.out_f32 = 1;
-        if (const int rc = raven_linear(h, nullptr, m->shared_up, nullptr, c.sact, M, m->shared_ff, ld, 0, 1, 0, dtype, c.lin, c.lin_bytes, stream)) return rc;
-        if (const int rc = raven_linear_epilogue(c.sact, nullptr, m->shared_down, c.ys, M, ld, m->shared_ff, 0, &e, dtype, c.lin, c.lin_bytes, stream)) return rc;
+        if (const int rc = raven_linear(h, nullptr, m->shared_up, nullptr, c.sact, M, m->shared_ff, ld, 0, 1, 0, dtype, c.lin, c.lin_bytes, s)) return rc;
+        if (const int rc = raven_linear_epilogue(c.sact, nullptr, m->shared_down, c.ys, M, ld, m->shared_ff, 0, &e, dtype, c.lin, c.lin_bytes, s)) return rc;
     }
     moe_combine_kernel<<<dim3((unsigned)(((int64_t)M * (ld / 4) + 255) / 256)), dim3(256), 0, s>>>(a);
     return raven_host::check_launch("moe (combine)");
+}
+}  // namespace raven
+
+extern "C" int raven_moe_forward(const raven_moe* m, const void* h, const float* logits, float* x, int32_t M, int32_t ld, int32_t dtype,
+                                 void* workspace, size_t workspace_bytes, void* stream) {
+    RAVEN_REQUIRE(h || M == 0, "moe: null pointer");
+    return raven::moe_forward(m, h, nullptr, 0, 0.f, logits, x, M, ld, dtype, workspace, workspace_bytes, static_cast<hipStream_t>(stream));
 }

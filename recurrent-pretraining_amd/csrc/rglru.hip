@@ -34,10 +34,22 @@ __device__ __forceinline__ float gelu_tanh_f32(float z) {
     return z / (1.0f + expf(-2.0f * x));
 }
 
-// log a and the input term of one channel from the gates' sums
+// log a and the input term of one channel from the gates' sums.  float: the library's functions.  bf16 operands: hardware exp2 and
+// reciprocal (1 ulp), and 1 - exp(-t) by its series where the subtraction would lose digits (the first term left out is 1.5e-7 of the sum).
+template <typename T>
 __device__ __forceinline__ void gate_terms(float zr, float zi, float softplus, float u, float* la, float* in) {
-    *la = -8.0f * sigmoid_f32(zr) * softplus;
-    *in = sqrtf(-expm1f(2.0f * *la)) * sigmoid_f32(zi) * u;
+    if constexpr (sizeof(T) == 4) {
+        *la = -8.0f * sigmoid_f32(zr) * softplus;
+        *in = sqrtf(-expm1f(2.0f * *la)) * sigmoid_f32(zi) * u;
+    } else {
+        const float log2e = 1.4426950408889634f;
+        const float r = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-log2e * zr)), i = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-log2e * zi));
+        const float t = 16.0f * r * softplus;
+        const float series = t * (1.0f + t * (-0.5f + t * (1.f / 6.f + t * (-1.f / 24.f + t * (1.f / 120.f - t * (1.f / 720.f))))));
+        const float gain2 = t < 0.3f ? series : 1.0f - __builtin_amdgcn_exp2f(-log2e * t);
+        *la = -0.5f * t;
+        *in = __builtin_amdgcn_sqrtf(gain2) * i * u;
+    }
 }
 
 // x of channel group c (4 channels) at position pos0 + s, s < 0: from the ring
@@ -55,14 +67,31 @@ __device__ __forceinline__ f32x4 conv_at(const RglruArgs& a, int b, int pos0, in
     return o;
 }
 
-template <typename T>
+// kConvRows rows and 4 channels per thread
+constexpr int kConvRows = 8;
+template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void rglru_conv_kernel(RglruArgs a) {
-    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
-    const int per = a.W / 4;
-    if (i >= (int64_t)a.M * per) return;
-    const int m = (int)(i / per), c = (int)(i % per);
+    const int c = blockIdx.x * 256 + threadIdx.x, b = blockIdx.z, s0 = blockIdx.y * kConvRows;
+    if (c >= a.W / 4) return;
     const int pos0 = a.pos_dev ? *a.pos_dev : a.pos0;
-    store4(static_cast<T*>(a.u) + (int64_t)m * a.W + 4 * c, conv_at<T>(a, m / a.S, pos0, m % a.S, c));
+    T* u = static_cast<T*>(a.u) + (int64_t)b * a.S * a.W + 4 * c;
+    if constexpr (TAPS == 0) {  // any number of taps
+        for (int s = s0; s < min(s0 + kConvRows, a.S); ++s) store4(u + (int64_t)s * a.W, conv_at<T>(a, b, pos0, s, c));
+    } else {
+        f32x4 x[kConvRows + TAPS - 1], w[TAPS];
+        const f32x4 bias = load4(a.conv_bias + 4 * c);
+#pragma unroll
+        for (int t = 0; t < TAPS; ++t) w[t] = load4(a.conv + (int64_t)t * a.W + 4 * c);
+#pragma unroll
+        for (int i = 0; i < kConvRows + TAPS - 1; ++i) x[i] = past_x<T>(a, b, pos0, min(s0 - TAPS + 1 + i, a.S - 1), c);
+#pragma unroll
+        for (int i = 0; i < kConvRows; ++i) {
+            f32x4 o = bias;
+#pragma unroll
+            for (int t = 0; t < TAPS; ++t) o += w[t] * x[i + t];
+            if (s0 + i < a.S) store4(u + (int64_t)(s0 + i) * a.W, o);
+        }
+    }
 }
 
 // Gates of RB rows and 16 channels of a block on the vector units: 16 lanes to a channel
@@ -97,58 +126,82 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(RglruArgs a) {
         const float sr = row16_sum(zr[b]), si = row16_sum(zi[b]);
         if (c16 != 0 || r >= a.bl || m0 + b >= a.M) continue;
         const int64_t at = (int64_t)(m0 + b) * a.W + ch;
-        gate_terms(sr + a.gate_bias[ch], si + a.gate_bias[a.W + ch], a.softplus[ch], to_f32(xs[b * a.bl + rr]), a.la + at, a.in + at);
+        gate_terms<T>(sr + a.gate_bias[ch], si + a.gate_bias[a.W + ch], a.softplus[ch], to_f32(xs[b * a.bl + rr]), a.la + at, a.in + at);
     }
 }
 
-// bf16 chunks: 64 token rows x 32 channels of a block per workgroup (32 rows of W_r and the 32 of W_i: a lane that ends up with
-// a channel's r has its i too).  A wave owns 16 token rows; fragments come straight from global memory (a block's matrices are
-// read by every row tile: L2), the products' K is one block.
+// bf16 chunks: 128 token rows x 32 channels of a block per workgroup (32 rows of W_r and the 32 of W_i: a lane that ends up with
+// a channel's r has its i too).  A wave owns 32 token rows; the matrices' rows are staged through LDS once per workgroup, 128 columns
+// at a time, the token rows come straight from global memory, requested one step ahead.
 __global__ __launch_bounds__(256) void rglru_gates_mfma_kernel(RglruArgs a) {
     typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
+    constexpr int KC = 128, PITCH = KC + 8;
+    __shared__ __align__(16) bf16 ws[64][PITCH];  // W_r rows c0 .. +31, W_i rows c0 .. +31
     const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, q4 = lane >> 4;
-    const int blk = blockIdx.x / a.parts, c0 = (blockIdx.x % a.parts) * 32, m0 = blockIdx.y * 64 + wave * 16;
+    const int blk = blockIdx.x / a.parts, c0 = (blockIdx.x % a.parts) * 32, m0 = blockIdx.y * 128 + wave * 32;
     const bf16* W = static_cast<const bf16*>(a.gates) + (int64_t)blk * 2 * a.bl * a.bl;
-    const bf16* u = static_cast<const bf16*>(a.u) + (int64_t)min(m0 + l16, a.M - 1) * a.W + blk * a.bl;
-    const bf16* w[4];  // W_r rows c0 .. +15, +16 .. +31, then W_i
+    const u32x4 zero = {0, 0, 0, 0};
+    const bf16* u[2];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) w[t] = W + ((int64_t)(t >> 1) * a.bl + min(c0 + 16 * (t & 1) + l16, a.bl - 1)) * a.bl;
-    f32x4 acc[4];
+    for (int r = 0; r < 2; ++r) u[r] = static_cast<const bf16*>(a.u) + (int64_t)min(m0 + 16 * r + l16, a.M - 1) * a.W + blk * a.bl;
+    f32x4 acc[2][4];
 #pragma unroll
-    for (int t = 0; t < 4; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    for (int k = 0; k < a.bl; k += 32) {
-        const int d = k + 8 * q4;
-        const bool ok = d < a.bl;
-        const int at = ok ? d : 0;
-        const u32x4 zero = {0, 0, 0, 0};
-        const u32x4 x = *reinterpret_cast<const u32x4*>(u + at);
-        u32x4 v[4];
+    for (int r = 0; r < 2; ++r)
 #pragma unroll
-        for (int t = 0; t < 4; ++t) v[t] = *reinterpret_cast<const u32x4*>(w[t] + at);
-        const bf16x8 xf = __builtin_bit_cast(bf16x8, ok ? x : zero);
+        for (int t = 0; t < 4; ++t) acc[r][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int k0 = 0; k0 < a.bl; k0 += KC) {
+        u32x4 x[2][KC / 32];
 #pragma unroll
-        for (int t = 0; t < 4; ++t)
-            acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, ok ? v[t] : zero), xf, acc[t], 0, 0, 0);
+        for (int r = 0; r < 2; ++r)
+#pragma unroll
+            for (int j = 0; j < KC / 32; ++j) {
+                const int d = k0 + 32 * j + 8 * q4;
+                x[r][j] = *reinterpret_cast<const u32x4*>(u[r] + (d < a.bl ? d : 0));
+                if (d >= a.bl) x[r][j] = zero;
+            }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 64 * (KC / 8) / 256; ++i) {
+            const int p = threadIdx.x + 256 * i, row = p / (KC / 8), d = k0 + (p % (KC / 8)) * 8;
+            const bf16* src = W + ((int64_t)(row >> 5) * a.bl + min(c0 + (row & 31), a.bl - 1)) * a.bl;
+            const u32x4 v = *reinterpret_cast<const u32x4*>(src + (d < a.bl ? d : 0));
+            *reinterpret_cast<u32x4*>(&ws[row][(p % (KC / 8)) * 8]) = d < a.bl ? v : zero;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int j = 0; j < KC / 32; ++j)
+#pragma unroll
+            for (int t = 0; t < 4; ++t) {
+                const bf16x8 wf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(&ws[16 * t + l16][32 * j + 8 * q4]));
+#pragma unroll
+                for (int r = 0; r < 2; ++r) {
+                    const u32x4 xv = x[r][j];
+                    acc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, __builtin_bit_cast(bf16x8, xv), acc[r][t], 0, 0, 0);
+                }
+            }
     }
-    const int m = m0 + l16;
-    if (m >= a.M) return;
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
         const int c = c0 + 16 * t + 4 * q4;  // four channels; bl is a multiple of 8
         if (c >= a.bl) continue;
         const int ch = blk * a.bl + c;
         const f32x4 br = load4(a.gate_bias + ch), bi = load4(a.gate_bias + a.W + ch), sp = load4(a.softplus + ch);
-        const f32x4 uu = load4(static_cast<const bf16*>(a.u) + (int64_t)m * a.W + ch);
-        f32x4 la, in;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            float x, y;
-            gate_terms(acc[t][i] + br[i], acc[2 + t][i] + bi[i], sp[i], uu[i], &x, &y);
-            la[i] = x;
-            in[i] = y;
+        for (int r = 0; r < 2; ++r) {
+            const int m = m0 + 16 * r + l16;
+            if (m >= a.M) continue;
+            const f32x4 uu = load4(static_cast<const bf16*>(a.u) + (int64_t)m * a.W + ch);
+            f32x4 la, in;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                float x, y;
+                gate_terms<bf16>(acc[r][t][i] + br[i], acc[r][2 + t][i] + bi[i], sp[i], uu[i], &x, &y);
+                la[i] = x;
+                in[i] = y;
+            }
+            store4(a.la + (int64_t)m * a.W + ch, la);
+            store4(a.in + (int64_t)m * a.W + ch, in);
         }
-        store4(a.la + (int64_t)m * a.W + ch, la);
-        store4(a.in + (int64_t)m * a.W + ch, in);
     }
 }
 
@@ -175,16 +228,17 @@ __global__ __launch_bounds__(64) void rglru_carry_kernel(RglruArgs a) {
     const int pos0 = a.pos_dev ? *a.pos_dev : a.pos0;
     float S = pos0 > 0 ? a.state[(int64_t)b * a.W + ch] : 0.f;
     const int64_t base = (int64_t)b * a.pieces * a.W + ch;
-    for (int p0 = 0; p0 < a.pieces; p0 += 8) {
-        float sum[8], end[8];
+    constexpr int U = 32;
+    for (int p0 = 0; p0 < a.pieces; p0 += U) {
+        float sum[U], end[U];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
+        for (int i = 0; i < U; ++i) {
             const int64_t at = base + (int64_t)min(p0 + i, max(a.pieces - 2, 0)) * a.W;
             sum[i] = a.sum[at];
             end[i] = a.end[at];
         }
 #pragma unroll
-        for (int i = 0; i < 8; ++i) {
+        for (int i = 0; i < U; ++i) {
             if (p0 + i >= a.pieces) break;
             a.carry[base + (int64_t)(p0 + i) * a.W] = S;
             S = expf(sum[i]) * S + end[i];
@@ -258,7 +312,7 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(RglruArgs a) {
     zi = row16_sum(zi);
     if (c16 != 0 || r >= a.bl) return;
     float la, in;
-    gate_terms(zr + a.gate_bias[ch], zi + a.gate_bias[a.W + ch], a.softplus[ch], to_f32(xs[rr]), &la, &in);
+    gate_terms<T>(zr + a.gate_bias[ch], zi + a.gate_bias[a.W + ch], a.softplus[ch], to_f32(xs[rr]), &la, &in);
     const float S = expf(la) * old + in;
     a.state[(int64_t)b * a.W + ch] = S;
     a.ring[((int64_t)b * a.taps + pos % a.taps) * a.W + ch] = x;  // not one of the rows the convolution reads
@@ -293,12 +347,14 @@ static int run_rglru(RglruArgs a, int B, hipStream_t s) {
         rglru_step_kernel<T><<<dim3(a.blocks * a.parts, B), dim3(256), lds, s>>>(a);
         return raven_host::check_launch("rglru (step)");
     }
-    rglru_conv_kernel<T><<<dim3((unsigned)(((int64_t)a.M * (a.W / 4) + 255) / 256)), dim3(256), 0, s>>>(a);
+    const dim3 conv_grid((a.W / 4 + 255) / 256, (a.S + kConvRows - 1) / kConvRows, B);
+    if (a.taps == 4) rglru_conv_kernel<T, 4><<<conv_grid, dim3(256), 0, s>>>(a);
+    else rglru_conv_kernel<T, 0><<<conv_grid, dim3(256), 0, s>>>(a);
     bool done = false;
     if constexpr (sizeof(T) == 2) {
         if (a.M >= 16) {
             a.parts = (a.bl + 31) / 32;
-            rglru_gates_mfma_kernel<<<dim3(a.blocks * a.parts, (a.M + 63) / 64), dim3(256), 0, s>>>(a);
+            rglru_gates_mfma_kernel<<<dim3(a.blocks * a.parts, (a.M + 127) / 128), dim3(256), 0, s>>>(a);
             done = true;
         }
     }
