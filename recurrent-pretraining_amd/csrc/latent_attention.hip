@@ -118,18 +118,21 @@ __global__ __launch_bounds__(256) void latent_out_kernel(LatentArgs a) {
     T* xs = reinterpret_cast<T*>(smem_raw);  // [RB][kp]
     const int h = blockIdx.x / a.rows_out, part = blockIdx.x % a.rows_out, m0 = blockIdx.y * RB;
     const int ld = a.kp + 4;
-#pragma unroll
-    for (int b = 0; b < RB; ++b) {
+    {
+        // RB 4: a wave per row; RB 1: the four waves share the row's columns
+        static_assert(RB == 1 || RB == 4, "rows per workgroup");
+        const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, b = RB == 4 ? wave : 0;
         const int m = min(m0 + b, a.M - 1);
         const float* p = a.part + ((int64_t)m * a.H + h) * a.splits * ld;
         // lane n holds range n (at most 64); some range always holds a position
-        const int mine = min((int)(threadIdx.x & 63), a.splits - 1);
+        const int mine = min(lane, a.splits - 1);
         const float ref = p[(int64_t)mine * ld + a.kp], sum = p[(int64_t)mine * ld + a.kp + 1];
         const float top = wave_max(ref);
-        const float w = (int)(threadIdx.x & 63) < a.splits ? soft_exp<T>(ref - top) : 0.f;
+        const float w = lane < a.splits ? soft_exp<T>(ref - top) : 0.f;
         const float f = w / wave_sum(w * sum);
-        for (int i0 = 0; i0 < a.kp; i0 += 1024) {  // uniform trip count: every lane takes part in the exchanges
-            const int i = i0 + 4 * threadIdx.x;
+        constexpr int STEP = RB == 4 ? 256 : 1024;
+        for (int i0 = 0; i0 < a.kp; i0 += STEP) {  // uniform trip count: every lane takes part in the exchanges
+            const int i = i0 + 4 * (RB == 4 ? lane : (int)threadIdx.x);
             const int at = min(i, a.kp - 4);
             f32x4 o = {0.f, 0.f, 0.f, 0.f};
             for (int s0 = 0; s0 < a.splits; s0 += 8) {
@@ -293,6 +296,198 @@ __global__ __launch_bounds__(256) void latent_rows_attention_kernel(LatentArgs a
             out[a.kp + 1] = sl[0][n] * f[0] + sl[1][n] * f[1] + sl[2][n] * f[2] + sl[3][n] * f[3];
         }
     }
+}
+
+// ------------------------------------------------------------------------------------------------
+// The same on the matrix cores (bf16): the query rows are the heads.  A workgroup takes RG groups of 16 of a sequence's S * H rows and
+// walks its range in tiles of 64 positions; one staged tile [64][kp + rp] serves both products.  Scores: wave w multiplies positions
+// 16 w .. + 15 with every row.  The four exchange their maxima and weights through LDS.  Weighted sum: wave w owns every fourth tile of 16
+// latent channels, read through the transposing loads; the weights are picked up in the key order those deliver.
+// ------------------------------------------------------------------------------------------------
+constexpr int kLsKeys = 64;
+
+template <int KS, int NTW, int RG>
+__global__ __launch_bounds__(256) void latent_step_kernel(LatentArgs a) {
+    constexpr int PITCH = KS * 32 + 16, CPR = KS * 4, NKC = kLsKeys * CPR / 256, PP = kLsKeys + 8;
+    static_assert(kLsKeys * CPR % 256 == 0, "staging shape");
+    typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
+    typedef unsigned int u32x2 __attribute__((ext_vector_type(2)));
+    typedef short s16x4 __attribute__((ext_vector_type(4)));
+    extern __shared__ __align__(16) unsigned char smem_raw[];
+    bf16(*sk)[PITCH] = reinterpret_cast<bf16(*)[PITCH]>(smem_raw);
+    __shared__ __align__(16) bf16 sp[16 * RG][PP];
+    __shared__ float smx[4][16 * RG];
+    const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, q4 = lane >> 4;
+    const int b = blockIdx.z, r0 = blockIdx.y * 16 * RG, n_rows = a.S * a.H, ld = a.kp + a.rp;
+    const int pos0 = min(a.pos_dev ? *a.pos_dev : a.pos0, a.t_max - a.S);
+    const int window = a.window > 0 ? a.window : 0x40000000;
+    const int first = max(0, pos0 - window + 1), end = pos0 + a.S;
+    const int span = (end - first + a.splits - 1) / a.splits;
+    const int lo = first + (int)blockIdx.x * span, hi = min(end, lo + span);
+    const bf16* lat = static_cast<const bf16*>(a.latent) + (int64_t)b * a.t_max * a.kp;
+    const bf16* rot = static_cast<const bf16*>(a.rotated) + (int64_t)b * a.t_max * a.rp;
+
+    u32x4 reg[NKC];
+    auto fetch = [&](int kt) {
+#pragma unroll
+        for (int i = 0; i < NKC; ++i) {
+            const int c = threadIdx.x + 256 * i, d = (c % CPR) * 8;
+            const int64_t p = min(kt + c / CPR, hi - 1);
+            const u32x4 v = *reinterpret_cast<const u32x4*>(d < a.kp ? lat + p * a.kp + d : d < ld ? rot + p * a.rp + (d - a.kp) : lat + p * a.kp);
+            reg[i] = d < ld ? v : u32x4{0, 0, 0, 0};
+        }
+    };
+    if (lo < hi) fetch(lo);
+    bf16x8 qf[RG][KS];
+    int my_pos[RG];
+#pragma unroll
+    for (int g = 0; g < RG; ++g) {
+        const int row = min(r0 + 16 * g + l16, n_rows - 1);
+        my_pos[g] = pos0 + row / a.H;
+        const bf16* qp = static_cast<const bf16*>(a.qa) + ((int64_t)b * n_rows + row) * ld;
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            const int d = 32 * ks + 8 * q4;
+            const u32x4 v = *reinterpret_cast<const u32x4*>(qp + (d < ld ? d : 0));
+            qf[g][ks] = __builtin_bit_cast(bf16x8, d < ld ? v : u32x4{0, 0, 0, 0});
+        }
+    }
+    f32x4 o[RG][NTW], osum[RG];
+    float ref[RG];
+#pragma unroll
+    for (int g = 0; g < RG; ++g) {
+        ref[g] = -INFINITY;
+        osum[g] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int n = 0; n < NTW; ++n) o[g][n] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    bf16x8 ones;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) ones[e] = static_cast<bf16>(1.0f);
+    const float in_scale = a.scale * 1.4426950408889634f;
+    const int n_tiles = (a.kp + 15) / 16;
+
+    for (int kt = lo; kt < hi; kt += kLsKeys) {
+#pragma unroll
+        for (int i = 0; i < NKC; ++i) {
+            const int c = threadIdx.x + 256 * i;
+            *reinterpret_cast<u32x4*>(&sk[c / CPR][(c % CPR) * 8]) = reg[i];
+        }
+        __syncthreads();
+        if (kt + kLsKeys < hi) fetch(kt + kLsKeys);
+        f32x4 sc[RG];
+#pragma unroll
+        for (int g = 0; g < RG; ++g) sc[g] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int ks = 0; ks < KS; ++ks) {
+            const bf16x8 kf = __builtin_bit_cast(bf16x8, *reinterpret_cast<const u32x4*>(&sk[16 * wave + l16][32 * ks + 8 * q4]));
+#pragma unroll
+            for (int g = 0; g < RG; ++g) sc[g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[g][ks], sc[g], 0, 0, 0);
+        }
+        // lane: positions kt + 16 wave + 4 q4 + (0 .. 3) of row l16
+        const int p0 = kt + 16 * wave + 4 * q4;
+#pragma unroll
+        for (int g = 0; g < RG; ++g) {
+            float mx = -INFINITY;
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const bool seen = p0 + v < hi && (unsigned)(my_pos[g] - p0 - v) < (unsigned)window;
+                sc[g][v] = seen ? sc[g][v] * in_scale : -INFINITY;
+                mx = fmaxf(mx, sc[g][v]);
+            }
+            mx = max_over_quarters(mx);
+            if (q4 == 0) smx[wave][16 * g + l16] = mx;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int g = 0; g < RG; ++g) {
+            const int r = 16 * g + l16;
+            const float top = fmaxf(ref[g], fmaxf(fmaxf(smx[0][r], smx[1][r]), fmaxf(smx[2][r], smx[3][r])));
+            const float m = top == -INFINITY ? 0.f : top;
+            bf16 w[4];
+#pragma unroll
+            for (int v = 0; v < 4; ++v) w[v] = from_f32<bf16>(__builtin_amdgcn_exp2f(sc[g][v] - m));
+            *reinterpret_cast<u32x2*>(&sp[r][16 * wave + 4 * q4]) = *reinterpret_cast<const u32x2*>(w);
+            const float corr = __builtin_amdgcn_exp2f(ref[g] - m);  // 0 while nothing has been seen
+            ref[g] = top;
+#pragma unroll
+            for (int v = 0; v < 4; ++v) {
+                const float cv = __shfl(corr, 4 * q4 + v, 64);
+                osum[g][v] *= cv;
+#pragma unroll
+                for (int n = 0; n < NTW; ++n) o[g][n][v] *= cv;
+            }
+        }
+        __syncthreads();
+#pragma unroll
+        for (int c = 0; c < 2; ++c) {
+            bf16x8 pf[RG];
+#pragma unroll
+            for (int g = 0; g < RG; ++g) {  // keys 32 c + 4 q4 + (0 .. 3) and 16 further
+                const u32x2 p_lo = *reinterpret_cast<const u32x2*>(&sp[16 * g + l16][32 * c + 4 * q4]);
+                const u32x2 p_hi = *reinterpret_cast<const u32x2*>(&sp[16 * g + l16][32 * c + 16 + 4 * q4]);
+                const u32x4 both = {p_lo[0], p_lo[1], p_hi[0], p_hi[1]};
+                pf[g] = __builtin_bit_cast(bf16x8, both);
+                osum[g] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[g], ones, osum[g], 0, 0, 0);
+            }
+#pragma unroll
+            for (int n = 0; n < NTW; ++n) {
+                const int col = 16 * min(wave + 4 * n, n_tiles - 1);
+                const bf16* src = &sk[32 * c + 4 * q4 + (l16 >> 2)][col + 4 * (l16 & 3)];
+                const s16x4 v_lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4 __attribute__((address_space(3)))*)(src));
+                const s16x4 v_hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((s16x4 __attribute__((address_space(3)))*)(src + 16 * PITCH));
+                const bf16x8 vf = __builtin_bit_cast(bf16x8, __builtin_shufflevector(v_lo, v_hi, 0, 1, 2, 3, 4, 5, 6, 7));
+#pragma unroll
+                for (int g = 0; g < RG; ++g) o[g][n] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(pf[g], vf, o[g][n], 0, 0, 0);
+            }
+        }
+        __syncthreads();
+    }
+    // lane: rows 4 q4 + v, channel l16 of each of the wave's tiles
+#pragma unroll
+    for (int g = 0; g < RG; ++g)
+#pragma unroll
+        for (int v = 0; v < 4; ++v) {
+            const int row = r0 + 16 * g + 4 * q4 + v;
+            const float m = __shfl(ref[g], 4 * q4 + v, 64);
+            if (row >= n_rows) continue;
+            float* out = a.part + (((int64_t)b * n_rows + row) * a.splits + blockIdx.x) * (a.kp + 4);
+#pragma unroll
+            for (int n = 0; n < NTW; ++n) {
+                const int col = 16 * (wave + 4 * n) + l16;
+                if (col < a.kp) out[col] = o[g][n][v];
+            }
+            if (wave == 0 && l16 == 0) {
+                out[a.kp] = m == -INFINITY ? m : m * 0.69314718055994531f;  // natural units
+                out[a.kp + 1] = osum[g][v];
+            }
+        }
+}
+
+template <int KS, int NTW, int RG>
+static int launch_step(const LatentArgs& a, hipStream_t s) {
+    const size_t lds = (size_t)kLsKeys * (KS * 32 + 16) * sizeof(bf16);
+    if (lds > 32 * 1024) {
+        static bool attr_set = false;
+        if (!attr_set) {
+            const hipError_t e = hipFuncSetAttribute((const void*)latent_step_kernel<KS, NTW, RG>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            if (e != hipSuccess) {
+                raven_host::set_error("latent_attention: hipFuncSetAttribute failed: %s", hipGetErrorString(e));
+                return (int)e;
+            }
+            attr_set = true;
+        }
+    }
+    const int groups = (a.S * a.H + 16 * RG - 1) / (16 * RG);
+    latent_step_kernel<KS, NTW, RG><<<dim3(a.splits, groups, a.M / a.S), dim3(256), lds, s>>>(a);
+    return raven_host::check_launch("latent_attention (step)");
+}
+// rows of 16 heads per workgroup: 2 once a sequence has more than 16 (head, row) pairs
+static bool step_fits(int kp, int rp) { return kp <= 512 && kp + rp <= 576; }
+static int run_step(const LatentArgs& a, hipStream_t s) {
+    const bool two = a.S * a.H > 16;
+    if (a.kp <= 256 && a.kp + a.rp <= 320) return two ? launch_step<10, 4, 2>(a, s) : launch_step<10, 4, 1>(a, s);
+    return two ? launch_step<18, 8, 2>(a, s) : launch_step<18, 8, 1>(a, s);
 }
 
 // ------------------------------------------------------------------------------------------------
@@ -530,20 +725,23 @@ static bool expands(const raven_latent* l, int S, int pos0, const int* pos_dev, 
     return *n_rows <= 64 * S;  // a short chunk behind a very long visible past reads the latents as they are
 }
 
+constexpr int kRowHeads = 4;  // heads a workgroup of the vector kernel takes
+
 // position ranges per row: enough workgroups for the chip, at least 64 positions each
-static int latent_splits(int rows, int H, int per_wg, int visible) {
-    const int64_t wgs = (int64_t)rows * ((H + per_wg - 1) / per_wg);
-    int64_t n = (512 + wgs - 1) / wgs;
+static int latent_splits(const raven_latent* l, int B, int S, int dtype, int visible) {
+    const bool step = dtype == RAVEN_BF16 && step_fits(l->kv_rank, l->rot);
+    const int rg = S * l->heads > 16 ? 32 : 16;
+    const int64_t wgs = step ? (int64_t)B * ((S * l->heads + rg - 1) / rg) : (int64_t)B * S * ((l->heads + kRowHeads - 1) / kRowHeads);
+    int64_t n = ((step ? 256 : 512) + wgs - 1) / wgs;
     if (n > (visible + 63) / 64) n = (visible + 63) / 64;
     if (n > 32) n = 32;
     return n < 1 ? 1 : (int)n;
 }
-static int visible_positions(const raven_latent* l, int pos0, int S) {
+static int visible_positions(const raven_latent* l, int pos0, int S) {  // by a sequence's S rows together
     const int all = pos0 + S;
-    return l->window > 0 && l->window < all ? l->window : all;
+    return l->window > 0 && l->window + S - 1 < all ? l->window + S - 1 : all;
 }
 
-constexpr int kRowHeads = 4;
 template <typename T, int CJ>
 static int launch_rows_attention(const LatentArgs& a, hipStream_t s) {
     const size_t lds = (((size_t)kRowHeads * (a.kp + a.rp) * sizeof(T) + 15) & ~(size_t)15) + (size_t)4 * kRowHeads * a.kp * sizeof(float);
@@ -572,7 +770,8 @@ static int run_absorbed(LatentArgs a, hipStream_t s) {
     if (const int rc = raven_host::check_launch("latent_attention (absorb)")) return rc;
     const int pieces = (a.kp / Chunk<T>::N + 63) / 64;
     int rc;
-    if (pieces <= 1) rc = launch_rows_attention<T, 1>(a, s);
+    if (sizeof(T) == 2 && step_fits(a.kp, a.rp)) rc = run_step(a, s);
+    else if (pieces <= 1) rc = launch_rows_attention<T, 1>(a, s);
     else if (pieces <= 2) rc = launch_rows_attention<T, 2>(a, s);
     else rc = launch_rows_attention<T, 4>(a, s);
     if (rc) return rc;
@@ -639,7 +838,7 @@ extern "C" size_t raven_latent_attention_workspace_bytes(const raven_latent* l, 
     using namespace raven;
     if (check_latent("latent_attention_workspace_bytes", l, nullptr, B, S, pos0, dtype) || B == 0 || S == 0) return 0;
     const size_t es = raven_host::elt_size(dtype), M = (size_t)B * S;
-    const size_t part = M * l->heads * latent_splits((int)M, l->heads, kRowHeads, 1 << 30) * (l->kv_rank + 4) * sizeof(float);
+    const size_t part = M * l->heads * latent_splits(l, B, S, dtype, 1 << 30) * (l->kv_rank + 4) * sizeof(float);
     const size_t absorbed = raven_host::align_up(M * l->heads * (l->kv_rank + l->rot) * es) + raven_host::align_up(part);
     int k0, n_rows;
     if (!expands(l, S, pos0, nullptr, dtype, &k0, &n_rows)) return absorbed;
@@ -686,7 +885,7 @@ int latent_attention(const raven_latent* l, const void* q, const void* z, int ld
     }
     RAVEN_REQUIRE(a.M <= 65535, "latent_attention: %d x %d rows in one call of the absorbed route", B, S);
     a.append = append && l->own_kv;
-    a.splits = latent_splits(a.M, a.H, kRowHeads, visible_positions(l, pos0, S));
+    a.splits = latent_splits(l, B, S, dtype, visible_positions(l, pos0, S));
     const size_t qa = raven_host::align_up((size_t)a.M * a.H * (a.kp + a.rp) * es);
     RAVEN_REQUIRE(qa + (size_t)a.M * a.H * a.splits * (a.kp + 4) * sizeof(float) <= workspace_bytes, "latent_attention: workspace of %zu bytes is too small",
                   workspace_bytes);

@@ -17,7 +17,7 @@ int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, voi
                  const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s);
 
 constexpr int kMaxExperts = 1024, kMaxTop = 32, kSlotRows = 128;
-constexpr int kPickRows = 64;  // tokens a workgroup of the two sorting kernels owns
+constexpr int kPickRows = 32;  // tokens a workgroup of the two sorting kernels owns
 
 struct MoeArgs {
     const void *h, *up, *down, *shared_up, *shared_down;
@@ -41,8 +41,8 @@ struct MoeArgs {
     const float* ys;        // [M, ld] or null
 };
 
-// one wave: the `top` experts of largest logit (lower index first among equals), each with its score, in every lane's view of idx / score
-__device__ __forceinline__ void pick_experts(const float* logits, int experts, int top, int* idx, float* score) {
+// one wave: the `top` experts of largest logit (lower index first among equals); lane k holds the k-th one and its score
+__device__ __forceinline__ void pick_experts(const float* logits, int experts, int top, int& mine, float& score) {
     const int lane = threadIdx.x & 63;
     float v[kMaxExperts / 64];
 #pragma unroll
@@ -50,6 +50,8 @@ __device__ __forceinline__ void pick_experts(const float* logits, int experts, i
         v[j] = -INFINITY;
         if (64 * j < experts && lane + 64 * j < experts) v[j] = logits[lane + 64 * j];
     }
+    mine = 0;
+    float logit = 0.f;
     for (int k = 0; k < top; ++k) {
         float best = -INFINITY;
         int at = 0x7fffffff;
@@ -64,14 +66,15 @@ __device__ __forceinline__ void pick_experts(const float* logits, int experts, i
 #pragma unroll
         for (int d = 1; d < 64; d <<= 1) who = min(who, __shfl_xor(who, d, 64));
         who = min(who, experts - 1);  // all logits NaN: still an expert
-        if (lane == 0) {
-            idx[k] = who;
-            score[k] = sigmoid_f32(m);
+        if (lane == k) {
+            mine = who;
+            logit = m;
         }
 #pragma unroll
         for (int j = 0; j < kMaxExperts / 64; ++j)
             if (lane + 64 * j == who) v[j] = -INFINITY;
     }
+    score = sigmoid_f32(logit);
 }
 
 // ---- few rows --------------------------------------------------------------------------------------------
@@ -87,7 +90,16 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
     if (a.h) {
         for (int i = threadIdx.x; i < nc; i += 256) store_chunk(xs + i * E, load_chunk(static_cast<const T*>(a.h) + (int64_t)m * a.ld + i * E));
     }
-    if (wave == 0) pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, idx, score);
+    if (wave == 0) {
+        int e;
+        float s;
+        pick_experts(a.logits + (int64_t)m * a.ldl, a.experts, a.top, e, s);
+        if (lane < a.top) {
+            idx[lane] = e;
+            score[lane] = s;
+            if (blockIdx.x == 0) a.pick[(int64_t)m * a.top + lane] = e;
+        }
+    }
     if (!a.h) {
         const float* x = a.x + (int64_t)m * a.ld;
         float ss = 0.f;
@@ -102,7 +114,6 @@ __global__ __launch_bounds__(256) void moe_up_kernel(MoeArgs a) {
         for (int i = 4 * threadIdx.x; i < a.ld; i += 1024) store4(xs + i, load4(x + i) * inv * load4(a.norm + i));
     }
     __syncthreads();
-    if (blockIdx.x == 0 && (int)threadIdx.x < a.top) a.pick[(int64_t)m * a.top + threadIdx.x] = idx[threadIdx.x];
     const int p = blockIdx.x * 4 + wave;
     if (p >= total) return;
     const bool shared = p >= a.top * a.ff;
@@ -183,10 +194,15 @@ __global__ __launch_bounds__(1024) void moe_pick_kernel(MoeArgs a) {
     __syncthreads();
     for (int i = wave; i < kPickRows && m0 + i < a.M; i += 16) {
         const int64_t m = m0 + i;
-        pick_experts(a.logits + m * a.ldl, a.experts, a.top, a.pick + m * a.top, a.pick_scale + m * a.top);
-        // lane 0 wrote the picks and reads them back
-        if ((threadIdx.x & 63) == 0)
-            for (int k = 0; k < a.top; ++k) atomicAdd(&count[a.pick[m * a.top + k]], 1);
+        const int lane = threadIdx.x & 63;
+        int e;
+        float s;
+        pick_experts(a.logits + m * a.ldl, a.experts, a.top, e, s);
+        if (lane < a.top) {
+            a.pick[m * a.top + lane] = e;
+            a.pick_scale[m * a.top + lane] = s;
+            atomicAdd(&count[e], 1);
+        }
     }
     __syncthreads();
     for (int e = threadIdx.x; e < a.experts; e += 1024) a.block_count[(int64_t)blockIdx.x * a.experts + e] = count[e];
