@@ -347,6 +347,20 @@ __device__ __forceinline__ void store_tiles_rope(const TiledArgs& a, const f32x4
 
 __device__ __align__(16) unsigned int g_zero_piece[4];  // what a 16-byte piece past the end of K is loaded from
 
+// Cuts the arguments to the rows and the matrix of tile row tile_m's group; false: no such tile
+__device__ __forceinline__ bool enter_group(TiledArgs& a, int tile_m, const int*& x_row) {
+    const int g = a.groups.group_of[tile_m];
+    if (g < 0) return false;
+    const int row = a.groups.group_row[tile_m];
+    a.M = a.groups.group_end[tile_m] - row;
+    a.w += g * a.groups.w_stride;
+    a.y = static_cast<char*>(a.y) + (int64_t)row * a.ldy * (a.out_f32 ? 4 : 2);
+    if (a.groups.x_scale) a.groups.x_scale += row;
+    if (a.groups.x_row) x_row = a.groups.x_row + row;
+    else a.x0 += (int64_t)row * a.ldx;
+    return true;
+}
+
 // GROUPED: row groups with a weight matrix each (TiledArgs::groups); a tile works on a copy of the arguments cut to its group's rows
 template <int EPI, int TM, int TN, int WM = 2, int WN = 4, bool GROUPED = false>
 __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
@@ -379,15 +393,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
     int tile_m = first_m + (in_band - tile_n * gsz);
     const int* x_row = nullptr;
     if constexpr (GROUPED) {
-        const int g = a.groups.group_of[tile_m];
-        if (g < 0) return;
-        const int row = a.groups.group_row[tile_m];
-        a.M = a.groups.group_end[tile_m] - row;
-        a.w += g * a.groups.w_stride;
-        a.y = static_cast<char*>(a.y) + (int64_t)row * a.ldy * (a.out_f32 ? 4 : 2);
-        if (EPI == EPI_SWIGLU) a.groups.x_scale += row;
-        if (a.groups.x_row) x_row = a.groups.x_row + row;
-        else a.x0 += (int64_t)row * a.ldx;
+        if (!enter_group(a, tile_m, x_row)) return;
         tile_m = 0;
     }
 
@@ -612,7 +618,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_tiled_kernel(TiledArgs a) {
 //     of step k + 1 have landed, and its slice 0 is read under the last products.  A request has between 1.4 and 2.4
 //     steps to land.
 // Same products in the same order per accumulator as the eight-wave kernel: bit-identical results.
-template <int EPI>
+template <int EPI, bool GROUPED = false>
 __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int TM = 4, TN = 4, WM = 2, WN = 2;
@@ -632,7 +638,12 @@ __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
     const int gsz = min(a.tiles_m - first_m, GROUP);
     const int in_band = logical - band * GROUP * a.tiles_n;
     const int tile_n = in_band / gsz;
-    const int tile_m = first_m + (in_band - tile_n * gsz);
+    int tile_m = first_m + (in_band - tile_n * gsz);
+    const int* x_row = nullptr;
+    if constexpr (GROUPED) {
+        if (!enter_group(a, tile_m, x_row)) return;
+        tile_m = 0;
+    }
 
     const int lane = threadIdx.x & 63;
     const int wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
@@ -652,7 +663,9 @@ __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
         if (SWIGLU) row_w = min(tile_n * BN_OUT + (r >> 5) * 16 + (r & 15), a.N - 1) + ((r & 16) ? a.up_off : 0);
         else row_w = min(tile_n * BN + r, a.N - 1);
         goff_w[p] = (unsigned)row_w * (2u * a.ldw) + 2u * colp[p & 1];
-        goff_x[p] = (unsigned)min(tile_m * BM + r, a.M - 1) * (2u * a.ldx) + 2u * colp[p & 1];
+        int row_x = min(tile_m * BM + r, a.M - 1);
+        if (GROUPED && x_row) row_x = x_row[row_x];
+        goff_x[p] = (unsigned)row_x * (2u * a.ldx) + 2u * colp[p & 1];
     }
     const char* const zero = reinterpret_cast<const char*>(g_zero_piece);
     const char* const w0 = reinterpret_cast<const char*>(a.w);
@@ -800,29 +813,29 @@ __global__ __launch_bounds__(256) void gemm_ring_kernel(TiledArgs a) {
         }
     }
     if (a.out_f32) store_tiles<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wm, wn, l16, q4);
-    else store_tiles_lds<EPI, TM, TN, WM, WN>(a, acc, tile_m, tile_n, wave, lane, lds_base);
+    else store_tiles_lds<EPI, TM, TN, WM, WN, GROUPED>(a, acc, tile_m, tile_n, wave, lane, lds_base);
 }
 
-template <int EPI>
+template <int EPI, bool GROUPED = false>
 static int launch_ring(TiledArgs a, hipStream_t s) {
     constexpr bool SWIGLU = EPI == EPI_SWIGLU;
     constexpr int BM = 256, BN_OUT = SWIGLU ? 128 : 256;
     constexpr size_t lds = 5 * 32768;
     static bool attr_set = false;
     if (!attr_set) {
-        hipError_t e = hipFuncSetAttribute((const void*)gemm_ring_kernel<EPI>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        hipError_t e = hipFuncSetAttribute((const void*)gemm_ring_kernel<EPI, GROUPED>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) {
             raven_host::set_error("gemm (ring): hipFuncSetAttribute failed: %s", hipGetErrorString(e));
             return (int)e;
         }
         attr_set = true;
     }
-    a.tiles_m = (a.M + BM - 1) / BM;
+    if (!GROUPED) a.tiles_m = (a.M + BM - 1) / BM;
     a.tiles_n = (a.N + BN_OUT - 1) / BN_OUT;
     const int64_t n_tiles = (int64_t)a.tiles_m * a.tiles_n;
     RAVEN_REQUIRE(n_tiles < (1 << 28), "gemm (ring): too many tiles (M=%d N=%d)", a.M, a.N);
     const unsigned grid = (unsigned)((n_tiles + 7) / 8 * 8);
-    gemm_ring_kernel<EPI><<<dim3(grid), dim3(256), lds, s>>>(a);
+    gemm_ring_kernel<EPI, GROUPED><<<dim3(grid), dim3(256), lds, s>>>(a);
     return raven_host::check_launch("gemm (ring MFMA)");
 }
 
@@ -974,11 +987,11 @@ int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int 
     return tiled_gemm_impl(x0, 0, x1, w, nullptr, y, M, N, K0, K1, 0, epi.out_f32, nullptr, s, &epi);
 }
 
-// Products of row groups (128 rows to a tile row): y[r] = x[x_row[r]] W_g^T, W_g = w + g * w_stride [N or 2N, K] of the group that row r of the
+// Products of row groups (tile_rows = 128 or 256 rows to a tile row): y[r] = x[x_row[r]] W_g^T, W_g = w + g * w_stride [N or 2N, K] of the group that row r of the
 // product belongs to.  swiglu: y = T(silu(s gate) * (s up)) with s = x_scale[r]; else y = T(sums).  n_tiles: entries of the three tile
 // tables (unused ones have group_of < 0); rows: rows of the product, x_rows: rows of x.
 int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, void* y, int rows, int N, int K, int swiglu, const int* group_of,
-                 const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s) {
+                 const int* group_row, const int* group_end, int n_tiles, int tile_rows, const int* x_row, const float* x_scale, hipStream_t s) {
     RAVEN_REQUIRE(x && w && y && group_of && group_row && group_end && n_tiles > 0 && N > 0 && N % 8 == 0 && K > 0 && K % 8 == 0 && (!swiglu || x_scale),
                   "gemm (grouped): bad arguments");
     RAVEN_REQUIRE((int64_t)x_rows * K < (1ll << 31) && (int64_t)N * 2 * K < (1ll << 31) && (int64_t)rows * N < (1ll << 40), "gemm (grouped): too large");
@@ -991,6 +1004,7 @@ int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, voi
     a.tiles_m = n_tiles;
     a.epi.scale = 1.f;
     a.groups = TiledArgs::Groups{group_of, group_row, group_end, x_row, x_scale, w_stride};
+    if (tile_rows == 256) return swiglu ? launch_ring<EPI_SWIGLU, true>(a, s) : launch_ring<EPI_FREE, true>(a, s);
     return swiglu ? launch_tiled<EPI_SWIGLU, 2, 1, 2, 4, true>(a, s) : launch_tiled<EPI_FREE, 2, 1, 2, 4, true>(a, s);
 }
 

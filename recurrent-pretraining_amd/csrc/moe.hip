@@ -14,9 +14,10 @@
 namespace raven {
 
 int grouped_gemm(const void* x, int x_rows, const void* w, int64_t w_stride, void* y, int rows, int N, int K, int swiglu, const int* group_of,
-                 const int* group_row, const int* group_end, int n_tiles, const int* x_row, const float* x_scale, hipStream_t s);
+                 const int* group_row, const int* group_end, int n_tiles, int tile_rows, const int* x_row, const float* x_scale, hipStream_t s);
 
-constexpr int kMaxExperts = 1024, kMaxTop = 32, kSlotRows = 128;
+constexpr int kMaxExperts = 1024, kMaxTop = 32;
+constexpr int kBigTileRows = 320;  // rows per expert from which the grouped products take 256-row tiles
 constexpr int kPickRows = 32;  // tokens a workgroup of the two sorting kernels owns
 
 struct MoeArgs {
@@ -35,7 +36,7 @@ struct MoeArgs {
     int *slot_row;          // [M * top]: token of a slot
     float* slot_scale;      // [M * top]
     int *group_of, *group_row, *group_end;
-    int n_tiles;
+    int n_tiles, tile_rows;
     int* block_count;       // [ceil(M / kPickRows), experts]: pairs of a workgroup's tokens
     const bf16* y;          // [M * top, ld]
     const float* ys;        // [M, ld] or null
@@ -228,7 +229,7 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(MoeArgs a) {
     }
     __syncthreads();
     // running sums over the experts of rows and of tile rows
-    const int rows = total[tid], tiles = (rows + kSlotRows - 1) / kSlotRows;
+    const int rows = total[tid], tiles = (rows + a.tile_rows - 1) / a.tile_rows;
     int r = rows, t = tiles;
 #pragma unroll
     for (int d = 1; d < 64; d <<= 1) {
@@ -252,8 +253,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(MoeArgs a) {
     if (me == 0) {
         for (int i = 0; i < tiles; ++i) {
             a.group_of[first_tile + i] = tid;
-            a.group_row[first_tile + i] = first + i * kSlotRows;
-            a.group_end[first_tile + i] = min(first + (i + 1) * kSlotRows, first + rows);
+            a.group_row[first_tile + i] = first + i * a.tile_rows;
+            a.group_end[first_tile + i] = min(first + (i + 1) * a.tile_rows, first + rows);
         }
         int used = 0;
         for (int w = 0; w < 16; ++w) used += wave_sums[1][w];
@@ -298,7 +299,7 @@ struct MoeChunk {
     float *pick_scale, *slot_scale, *ys;
     char *act, *sact, *lin;
     size_t lin_bytes;
-    int n_tiles;
+    int n_tiles, tile_rows;
 };
 static size_t carve_moe(const raven_moe* m, int M, int ld, int dtype, char* base, MoeChunk* out) {
     const size_t es = raven_host::elt_size(dtype), pairs = (size_t)M * m->top;
@@ -313,7 +314,9 @@ static size_t carve_moe(const raven_moe* m, int M, int ld, int dtype, char* base
         c.act = take((size_t)M * (m->top * (size_t)m->ff + m->shared_ff) * es);
         c.pick = (int*)take(pairs * 4);
     } else {
-        c.n_tiles = (int)(pairs / kSlotRows) + m->experts;
+        // 256-row tiles (twice the speed per row) once an expert fills most of two of them on average
+        c.tile_rows = pairs >= (size_t)kBigTileRows * m->experts ? 256 : 128;
+        c.n_tiles = (int)(pairs / c.tile_rows) + m->experts;
         c.pick = (int*)take(pairs * 4);
         c.pick_scale = (float*)take(pairs * 4);
         c.slot_of = (int*)take(pairs * 4);
@@ -383,14 +386,14 @@ int moe_forward(const raven_moe* m, const void* h, const float* norm, int dim, f
     }
     const int pairs = M * m->top, blocks = (M + kPickRows - 1) / kPickRows;
     a.pick_scale = c.pick_scale; a.slot_of = c.slot_of; a.slot_row = c.slot_row; a.slot_scale = c.slot_scale;
-    a.group_of = c.group_of; a.group_row = c.group_row; a.group_end = c.group_end; a.n_tiles = c.n_tiles; a.block_count = c.block_count;
+    a.group_of = c.group_of; a.group_row = c.group_row; a.group_end = c.group_end; a.n_tiles = c.n_tiles; a.tile_rows = c.tile_rows; a.block_count = c.block_count;
     a.y = c.y; a.ys = c.ys;
     moe_pick_kernel<<<dim3(blocks), dim3(1024), 0, s>>>(a);
     moe_sort_kernel<<<dim3(blocks), dim3(1024), 0, s>>>(a);
     if (const int rc = raven_host::check_launch("moe (sort)")) return rc;
-    if (const int rc = grouped_gemm(h, M, m->up, (int64_t)2 * m->ff * ld, c.act, pairs, m->ff, ld, 1, c.group_of, c.group_row, c.group_end, c.n_tiles, c.slot_row,
+    if (const int rc = grouped_gemm(h, M, m->up, (int64_t)2 * m->ff * ld, c.act, pairs, m->ff, ld, 1, c.group_of, c.group_row, c.group_end, c.n_tiles, c.tile_rows, c.slot_row,
                                     c.slot_scale, s)) return rc;
-    if (const int rc = grouped_gemm(c.act, pairs, m->down, (int64_t)ld * m->ff, c.y, pairs, ld, m->ff, 0, c.group_of, c.group_row, c.group_end, c.n_tiles, nullptr,
+    if (const int rc = grouped_gemm(c.act, pairs, m->down, (int64_t)ld * m->ff, c.y, pairs, ld, m->ff, 0, c.group_of, c.group_row, c.group_end, c.n_tiles, c.tile_rows, nullptr,
                                     nullptr, s)) return rc;
     if (m->shared_up) {
         raven_epilogue e{};

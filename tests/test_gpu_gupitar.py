@@ -321,6 +321,27 @@ def test_mixture(pkg, dtype, M, D, E, top, ff, shared):
     assert Dp == D or stream[:, D:].abs().max() == 0
 
 
+@pytest.mark.parametrize("M,D,E,top,ff", [(900, 96, 2, 1, 136), (700, 64, 3, 3, 264), (1100, 264, 1, 1, 72)])
+def test_mixture_in_large_tiles(pkg, M, D, E, top, ff):
+    """Enough rows per expert for the 256-row tiles, a last tile cut short, experts of unequal share; every row against a dense sum."""
+    cfg = G.config(D, 8, [G.rglru(8, 1, 1, G.moe(E, top, ff))])
+    w = O.random_weights(cfg, E)
+    model = pkg.GupitarForCausalLM(pkg.GupitarConfig(**cfg), device="cuda", dtype=BF16)
+    model.load_state_dict(w)
+    g = torch.Generator().manual_seed(M)
+    h = torch.randn(M, D, generator=g).to(BF16)
+    logits = torch.full((M, model.layers[0].moe.logit_ld), 1e9)
+    logits[:, :E] = torch.randn(M, E, generator=g) + torch.arange(E) * 0.5
+    x = torch.randn(M, D, generator=g) * 10
+    stream = x.clone().cuda()
+    pkg.hip.moe(model.layers[0].moe, h.cuda(), logits.cuda(), stream)
+    s, want = torch.sigmoid(logits[:, :E].double()), torch.zeros(M, D).double()
+    chosen = torch.zeros(M, E).scatter(1, s.topk(top, 1).indices, 1.0)
+    for e in range(E):
+        want += chosen[:, e:e + 1] * O.gated_mlp(s[:, e:e + 1] * h.double(), {k: t.double() for k, t in w.items()}, f"l0.mlp.e{e}.")
+    assert (stream.cpu().double() - x - want).abs().max() < 2e-2 * max(1.0, want.abs().max().item())
+
+
 @DT
 @pytest.mark.parametrize("M", [1, 20])
 def test_mixture_prefers_the_lower_index_among_equals(pkg, dtype, M):
