@@ -321,7 +321,8 @@ __global__ __launch_bounds__(256) void latent_step_kernel(LatentArgs a) {
     const int b = blockIdx.z, r0 = blockIdx.y * 16 * RG, n_rows = a.S * a.H, ld = a.kp + a.rp;
     const int pos0 = min(a.pos_dev ? *a.pos_dev : a.pos0, a.t_max - a.S);
     const int window = a.window > 0 ? a.window : 0x40000000;
-    const int first = max(0, pos0 - window + 1), end = pos0 + a.S;
+    // the positions that these rows see
+    const int first = max(0, pos0 + r0 / a.H - window + 1), end = pos0 + min(r0 + 16 * RG - 1, n_rows - 1) / a.H + 1;
     const int span = (end - first + a.splits - 1) / a.splits;
     const int lo = first + (int)blockIdx.x * span, hi = min(end, lo + span);
     const bf16* lat = static_cast<const bf16*>(a.latent) + (int64_t)b * a.t_max * a.kp;
@@ -762,8 +763,8 @@ static int launch_rows_attention(const LatentArgs& a, hipStream_t s) {
 
 template <typename T, typename Z, int RB>
 static int run_absorbed(LatentArgs a, hipStream_t s) {
-    // weight rows per workgroup: 16 for a few token rows (latency), 64 for many
-    a.per_wg = a.M <= 2 ? 1 : 4;
+    // weight rows per workgroup: 16 for one or two token rows (latency), more for more
+    a.per_wg = a.M <= 2 ? 1 : a.M <= 64 ? 2 : 4;
     const int rows = 16 * a.per_wg, blocks = (a.M + RB - 1) / RB;
     a.rows_out = (a.kp + rows - 1) / rows;
     absorb_kernel<T, Z, RB><<<dim3(a.H * a.rows_out + (a.append ? 1 : 0), blocks), dim3(256), (size_t)RB * a.np * sizeof(T), s>>>(a);
