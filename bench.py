@@ -470,8 +470,8 @@ def gitipel_shapes(width, vocab=32768):
     return gitipel, raven
 
 
-def gitipel_work(cfg, S, t_cached):
-    """(flops of a prompt of S tokens with all its logits, bytes a decode step reads with t_cached positions behind it)."""
+def gitipel_work(cfg, S, t_cached, B=1):
+    """(flops of a prompt of S tokens with all its logits, bytes a decode step of B sequences reads with t_cached positions behind them)."""
     D = cfg["width"]
     flops = weights = state = 0.0
     for i, t in [(i, None) for i in (0, 1)] + [(i, t) for t in (0, 1) for i in (2, 3, 4, 5)] + [(i, None) for i in (6, 7)]:
@@ -491,13 +491,13 @@ def gitipel_work(cfg, S, t_cached):
         flops += 2.0 * S * w
     weights += 2 * 2 * D * D
     flops += 2 * 2.0 * S * 2 * D * D + 2.0 * S * D * cfg["vocab"]
-    return flops, 2 * (weights + D * cfg["vocab"]) + state
+    return flops, 2 * (weights + D * cfg["vocab"]) + B * state
 
 
-def raven_work(cfg, S, t_cached):
+def raven_work(cfg, S, t_cached, B=1):
     D, ff, runs = cfg.n_embd, 3 * cfg.n_embd * cfg.intermediate_size, 12
     flops = runs * (2.0 * S * (4 * D * D + ff) + 4.0 * D * S * (S + 1) / 2) + 2 * 2.0 * S * 2 * D * D + 2.0 * S * D * cfg.vocab_size
-    return flops, 2 * (runs * (4 * D * D + ff) + 2 * 2 * D * D + D * cfg.vocab_size) + runs * 2 * 2 * D * t_cached
+    return flops, 2 * (runs * (4 * D * D + ff) + 2 * 2 * D * D + D * cfg.vocab_size) + B * runs * 2 * 2 * D * t_cached
 
 
 def gupitar_shapes(width, vocab=32768):
@@ -574,12 +574,12 @@ def stream_families(args, names, shapes, title):
             if name == "raven":
                 models[name] = pkg.RavenForCausalLM(pkg.RavenConfig(**cfg), device="cuda:0", dtype=torch.bfloat16)
                 fill_synthetic(models[name])
-                work[name] = raven_work(models[name].config, S, ctx)
+                work[name] = raven_work(models[name].config, S, ctx, B)
             else:
                 config, family = pkg.family_of({"model_type": name})
                 models[name] = family(config(**cfg), device="cuda:0", dtype=torch.bfloat16)
                 models[name].init_weights(seed=0)
-                work[name] = gitipel_work(cfg, S, ctx) if name == "gitipel" else gupitar_work(cfg, S, ctx, B)
+                work[name] = (gitipel_work if name == "gitipel" else gupitar_work)(cfg, S, ctx, B)
         vocab = 32768
         ids = torch.randint(0, vocab, (1, S), generator=torch.Generator().manual_seed(1)).cuda()
         rows = torch.randint(0, vocab, (B, ctx), generator=torch.Generator().manual_seed(2)).cuda()

@@ -44,6 +44,7 @@ struct GemmArgs {
     int row_stride;        // mfma: 1 = a tile is 16 neighbouring weight rows, 2 = every second row (see mfma_kernel)
     int line_aligned;      // mfma: the rows of a tile all start at the same offset inside a 128-byte line
     raven_epilogue epi;    // EPI_FREE only (residual and y already offset to the pass)
+    int ldy;               // EPI_FREE only: elements between two rows of y and residual
     int rows_per_unit;     // mfma, ragged variants: weight rows (per side for SwiGLU) a workgroup owns; its last tile is partly empty
 };
 
@@ -85,7 +86,7 @@ __device__ __forceinline__ Chunk<T> load_weight(const T* p) {
 template <typename T, int EPI = EPI_PLAIN>
 __device__ __forceinline__ void store_out(const GemmArgs& a, int m, int n, float acc) {
     if (is_free(EPI)) {
-        store_free<T, EPI>(a.epi, a.y, (int64_t)m * a.N + n, n, acc);
+        store_free<T, EPI>(a.epi, a.y, (int64_t)m * a.ldy + n, n, acc);
         return;
     }
     float r = round_to<T>(acc);
@@ -240,6 +241,13 @@ __global__ __launch_bounds__(256) void mfma_kernel(GemmArgs a) {
     const int ln = lane & 15, kq = lane >> 4;
     const int K = a.K;
     const int rs = a.row_stride;
+    if constexpr (is_free(EPI)) {  // gemm_narrow_free: a grid row per 16 * MT rows of X
+        const int64_t m0 = (int64_t)blockIdx.y * 16 * MT;
+        a.M -= (int)m0;
+        a.x0 = static_cast<const bf16*>(a.x0) + m0 * a.k0;
+        a.y = static_cast<char*>(a.y) + m0 * a.ldy * (a.epi.out_f32 ? 4 : 2);
+        if (a.epi.residual) a.epi.residual += m0 * a.ldy;
+    }
     // a group is rs units: with rs = 2 the even unit takes the even rows of the group's tiles, the odd unit the odd rows
     const int group = rs == 2 ? blockIdx.x >> 1 : blockIdx.x;
     const int parity = rs == 2 ? blockIdx.x & 1 : 0;
@@ -591,11 +599,36 @@ int gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int
               hipStream_t s) {
     GemmArgs a{};
     a.w = w; a.x0 = x0; a.x1 = x1; a.y = y;
-    a.M = M; a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.out_f32 = epi.out_f32; a.epi = epi;
+    a.M = M; a.N = N; a.K = K0 + K1; a.k0 = K0; a.k1 = K1; a.out_f32 = epi.out_f32; a.epi = epi; a.ldy = N;
     switch (EPI_FREE + epi.act) {
         case EPI_FREE_GELU: return run_gemm<EPI_FREE_GELU>(a, dtype, s);
         case EPI_FREE_TANH: return run_gemm<EPI_FREE_TANH>(a, dtype, s);
         default: return run_gemm<EPI_FREE>(a, dtype, s);
+    }
+}
+
+// Many rows against a matrix of at most 128 rows, where 128 x 128 tiles would leave most of the chip idle: 32 x 32 pieces of the output,
+// K split over a workgroup's waves.  ldy: row pitch of y and the residual.
+bool gemm_narrow_fits(int M, int N, int K, int dtype) {
+    return dtype == RAVEN_BF16 && M > 128 && M <= 8192 && N <= 128 && N % 16 == 0 && K % 32 == 0 && K >= 256;
+}
+template <int EPI>
+static int launch_narrow(GemmArgs a, hipStream_t s) {
+    const int pitch = a.K * 2, n_tiles16 = a.N / 16;
+    a.row_stride = (pitch % 128 == 64 && a.N % 32 == 0) ? 2 : 1;
+    a.line_aligned = (pitch * a.row_stride) % 128 == 0;
+    const int rs = a.row_stride, groups = (n_tiles16 + 2 * rs - 1) / (2 * rs) * rs;
+    mfma_kernel<2, 2, EPI><<<dim3(groups, (a.M + 31) / 32), dim3(256), 0, s>>>(a);
+    return raven_host::check_launch("mfma gemm (narrow)");
+}
+int gemm_narrow_free(const void* x, const void* w, void* y, int ldy, int M, int N, int K, const raven_epilogue& epi, hipStream_t s) {
+    GemmArgs a{};
+    a.w = w; a.x0 = x; a.y = y;
+    a.M = M; a.N = N; a.K = K; a.k0 = K; a.out_f32 = epi.out_f32; a.epi = epi; a.ldy = ldy;
+    switch (EPI_FREE + epi.act) {
+        case EPI_FREE_GELU: return launch_narrow<EPI_FREE_GELU>(a, s);
+        case EPI_FREE_TANH: return launch_narrow<EPI_FREE_TANH>(a, s);
+        default: return launch_narrow<EPI_FREE>(a, s);
     }
 }
 

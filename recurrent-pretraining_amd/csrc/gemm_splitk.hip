@@ -35,6 +35,9 @@ int tiled_gemm_free(const void* x0, const void* x1, const void* w, void* y, int 
 int gemm_free(const void* x0, const void* x1, const void* w, void* y, int M, int N, int K0, int K1, const raven_epilogue& epi, int dtype,
               hipStream_t s);
 
+bool gemm_narrow_fits(int M, int N, int K, int dtype);
+int gemm_narrow_free(const void* x, const void* w, void* y, int ldy, int M, int N, int K, const raven_epilogue& epi, hipStream_t s);
+
 constexpr int kNsPitch = 136;  // bf16 elements per LDS row: 128 + 8 (272 bytes)
 typedef unsigned int u32x4 __attribute__((ext_vector_type(4)));
 
@@ -449,6 +452,7 @@ extern "C" int raven_linear_epilogue(const void* x0, const void* x1, const void*
     RAVEN_REQUIRE(((uintptr_t)epi->residual & 15) == 0 && ((uintptr_t)epi->bias & 15) == 0, "linear_epilogue: residual and bias must be 16-byte aligned");
     RAVEN_REQUIRE(!epi->residual || epi->out_f32, "linear_epilogue: a residual needs a float output");
     hipStream_t s = static_cast<hipStream_t>(stream);
+    if (K1 == 0 && gemm_narrow_fits(M, N, K0, dtype)) return gemm_narrow_free(x0, w, y, N, M, N, K0, *epi, s);
     if (M >= g_tiled_min_rows && tiled_gemm_fits(M, N, K0, K1, dtype)) return tiled_gemm_free(x0, x1, w, y, M, N, K0, K1, *epi, s);
     // the same choice between the kernels with and without a K split as raven_linear
     const bool split = dtype == RAVEN_BF16 && M > g_linear_min_rows && N % 16 == 0 && K0 % 32 == 0 && K1 % 32 == 0 && workspace != nullptr &&

@@ -50,6 +50,9 @@
 
 namespace raven {
 
+bool gemm_narrow_fits(int M, int N, int K, int dtype);
+int gemm_narrow_free(const void* x, const void* w, void* y, int ldy, int M, int N, int K, const raven_epilogue& epi, hipStream_t s);
+
 struct TiledArgs {
     const bf16* w;         // [N or 2N, K0 + K1]
     const bf16* x0;        // [M, K0]
@@ -970,8 +973,10 @@ static int tiled_gemm_impl(const void* x0, int ldx, const void* x1, const void* 
         tail.rope.col0 = n_big;
         if (tail.epi.bias) tail.epi.bias += n_big;
         if (tail.epi.residual) tail.epi.residual += n_big;
-        const int rc = launch(head, true);
-        return rc ? rc : launch(tail, false);
+        if (const int rc = launch(head, true)) return rc;
+        if (epi && a.K1 == 0 && a.ldx == K0 && a.ldw == K0 && gemm_narrow_fits(M, tail.N, K0, RAVEN_BF16))
+            return gemm_narrow_free(tail.x0, tail.w, tail.y, tail.ldy, M, tail.N, K0, tail.epi, s);
+        return launch(tail, false);
     }
     return launch(a, big);
 }

@@ -55,6 +55,30 @@ def test_linear_epilogue(pkg, dtype, M, N, K0, K1):
         assert ((got - want).abs() <= (2e-5 if dtype == F32 else want.abs() * 2 ** -8 + 1e-4)).all()
 
 
+@pytest.mark.parametrize("M,N,K", [(129, 16, 256), (700, 80, 2048), (1000, 128, 288), (333, 64, 1056), (8192, 96, 512)])
+def test_linear_epilogue_of_narrow_matrices(pkg, M, N, K):
+    """Many rows against a few matrix rows; K with and without whole cache lines per row."""
+    g = torch.Generator(device="cuda").manual_seed(N)
+    x, w = torch.randn(M, K, generator=g, device="cuda").to(BF16), (torch.randn(N, K, generator=g, device="cuda") / K ** 0.5).to(BF16)
+    bias, res = torch.randn(N, generator=g, device="cuda"), torch.randn(M, N, generator=g, device="cuda")
+    want = torch.nn.functional.linear(x.float(), w.float())
+    assert (pkg.hip.linear_epilogue(x, w, bias=bias, residual=res, scale=0.5) - (0.5 * want + bias + res)).abs().max() < 1e-4
+    got = pkg.hip.linear_epilogue(x, w, bias=bias, act=pkg.hip.ACT_TANH, out_f32=False).float()
+    assert ((got - torch.tanh(want + bias)).abs() <= 2 ** -8 + 1e-4).all()
+
+
+def test_linear_epilogue_narrow_rest_behind_large_tiles(pkg):
+    """4096 x 4160: a round of 256 x 256 tiles and 64 columns more, which write into the same rows."""
+    g = torch.Generator(device="cuda").manual_seed(5)
+    M, N, K = 4096, 4160, 256
+    x, w = torch.randn(M, K, generator=g, device="cuda").to(BF16), (torch.randn(N, K, generator=g, device="cuda") / K ** 0.5).to(BF16)
+    bias, res = torch.randn(N, generator=g, device="cuda"), torch.randn(M, N, generator=g, device="cuda")
+    want = torch.nn.functional.linear(x.float(), w.float())
+    assert (pkg.hip.linear_epilogue(x, w, bias=bias, residual=res) - (want + bias + res)).abs().max() < 1e-4
+    got, ref = pkg.hip.linear_epilogue(x, w, bias=bias, out_f32=False).float(), want + bias
+    assert ((got - ref).abs() <= ref.abs() * 2 ** -8 + 1e-4).all()
+
+
 @pytest.mark.parametrize("M,N,K", [(4096, 2048, 96), (4200, 4096, 64), (16384, 1160, 128)])
 def test_linear_epilogue_large_tiles(pkg, M, N, K):
     """Shapes that take the 256 x 256 tiles, also with the last tile columns handed to small tiles."""
