@@ -1,4 +1,4 @@
-"""The Gupitar decoder: pre-norm layers over an fp32 residual stream, norms stored around zero, each layer with one of two mixers --
+"""The Gupitar decoder: pre-norm layers over an fp32 residual stream (norm weights as distances from one), each with one of two mixers --
 windowed attention over low-rank key latents with a rotated part shared by all heads and an output gate, where a layer may read
 another layer's latents, or a real-gated linear recurrent unit behind a short convolution -- and a gated feed-forward: dense, or a mixture
 of experts with sigmoid scores on the experts' inputs and an optional gated shared expert."""

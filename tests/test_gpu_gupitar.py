@@ -92,7 +92,7 @@ def inputs(T, H, dim, rot, vdim, kr, seed=0, q_scale=1.0):
             torch.randn(T, H, dim + rot, generator=g) * q_scale)
 
 
-SHAPES = [(2, 16, 8, 16, 24, 20), (3, 10, 6, 13, 27, 33), (8, 64, 32, 64, 128, 100), (5, 32, 64, 72, 136, 64), (16, 128, 64, 128, 512, 70),
+SHAPES = [(2, 16, 8, 16, 24, 20), (3, 10, 6, 13, 27, 33), (6, 64, 32, 56, 120, 100), (5, 32, 64, 72, 136, 64), (16, 128, 64, 128, 512, 70),
           (1, 24, 2, 40, 1016, 1), (4, 200, 40, 120, 64, 5), (2, 56, 8, 136, 40, 500)]
 
 
@@ -114,7 +114,7 @@ def test_attention_prompts_portions_and_decoding(pkg, dtype, H, dim, rot, vdim, 
 
 @DT
 @pytest.mark.parametrize("how", ["prompt", "decoded", "portions", "short portions"])
-@pytest.mark.parametrize("window", [64, 96, 130])
+@pytest.mark.parametrize("window", [64, 90, 130])
 def test_attention_keys_at_the_edges_of_a_window(pkg, dtype, window, how):
     """Single keys that dominate their query: just inside the window, just outside, and at tile borders."""
     T, H, dim, rot, vdim, kr = 420, 2, 32, 8, 32, 32
@@ -294,7 +294,7 @@ def test_recurrent_unit_of_several_sequences(pkg, dtype):
 # ---- mixture of experts alone --------------------------------------------------------------------------
 @DT
 @pytest.mark.parametrize("M", [1, 2, 9, 40, 300])
-@pytest.mark.parametrize("D,E,top,ff,shared", [(50, 5, 2, 11, 9), (64, 3, 3, 24, None), (96, 70, 8, 40, 56), (136, 12, 1, 200, 64), (72, 300, 4, 16, 8)])
+@pytest.mark.parametrize("D,E,top,ff,shared", [(50, 5, 2, 11, 9), (64, 3, 3, 24, None), (96, 70, 8, 40, 56), (136, 11, 1, 200, 64), (72, 300, 4, 16, 8)])
 def test_mixture(pkg, dtype, M, D, E, top, ff, shared):
     cfg = G.config(D, 8, [G.rglru(8, 1, 1, G.moe(E, top, ff, shared))])
     w = O.random_weights(cfg, E)
